@@ -69,12 +69,13 @@ __device__ __forceinline__ float am_column_max(float v) {
 
 // One block of 32 keys for the NT column tiles of a wave: scores, online softmax, P*V.
 // Scores and the running maximum are kept in the base-2 domain (score * scale * log2 e), so the
-// exponential is one v_exp_f32; sums and accumulators are float.  Masking is skipped when every
+// exponential is one v_exp_f32; sums and accumulators are float.  CAP: the scores are bent by a cap first
+// (tl_capped; scale2 is then its factor into the exponent and cap2 the cap in the base-2 domain).  Masking is skipped when every
 // key of the block is visible to every column of the wave, the rescaling of the accumulator when
 // no running maximum moved.
-template <int DC, int NT>
+template <int DC, int NT, bool CAP>
 __device__ __forceinline__ void am_block(const uint4* kf0, const uint4* kf1, const uint4* vf, const uint4 (*qf)[DC],
-                                         const int* p_col, const int* lo_col, int first, int kb, int g, float scale2,
+                                         const int* p_col, const int* lo_col, int first, int kb, int g, float scale2, float cap2,
                                          float* m_run, float* l_run, f32x4 (*acc)[DC * 2]) {
     constexpr int DB = DC * 2;
     const int key_base = kb + 8 * g;
@@ -89,8 +90,8 @@ __device__ __forceinline__ void am_block(const uint4* kf0, const uint4* kf1, con
         float sv[8];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            sv[i] = st0[i] * scale2;
-            sv[4 + i] = st1[i] * scale2;
+            sv[i] = CAP ? tl_capped(st0[i], scale2, cap2) : st0[i] * scale2;
+            sv[4 + i] = CAP ? tl_capped(st1[i], scale2, cap2) : st1[i] * scale2;
         }
         const bool edge = (kb + 31 > p_col[j]) || (kb < lo_col[j]);
         if (__any(edge)) {
@@ -142,13 +143,13 @@ __device__ __forceinline__ int am_page_index(int k, int bs, int bs_shift) {
     return bs_shift >= 0 ? k >> bs_shift : k / bs;
 }
 
-template <int DC, int NT>
+template <int DC, int NT, bool CAP>
 __global__ __launch_bounds__(256) void attn_mfma_kernel(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int32_t* __restrict__ tables, int NB, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_start, bf16_t* __restrict__ out, int out_stride, float* __restrict__ ws_o,
     float* __restrict__ ws_ml, int nq, int nkv, int bs, int bs_shift, TlMask mask, float scale, int nsplit,
-    int split_blocks, const int32_t* __restrict__ seq_list, int skip_single, int sink) {
+    int split_blocks, const int32_t* __restrict__ seq_list, int skip_single, const float* __restrict__ sinks, float softcap) {
     constexpr int D = DC * 32;
     constexpr int DB = D / 16;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -159,7 +160,8 @@ __global__ __launch_bounds__(256) void attn_mfma_kernel(
     const int widx = blockIdx.z * (blockDim.x >> 6) + wave;    // one to four waves per work-group
     const int tg = widx / nsplit, sp = widx - tg * nsplit;
     const int G = nq / nkv;
-    const float scale2 = scale * AM_LOG2E;
+    const float scale2 = CAP ? 2.0f * AM_LOG2E * scale / softcap : scale * AM_LOG2E;   // see am_block
+    const float cap2 = softcap * AM_LOG2E;
     const int r0 = q_start[s];
     const int n = q_start[s + 1] - r0;
     const int start = ctx_start[s];
@@ -270,7 +272,7 @@ __global__ __launch_bounds__(256) void attn_mfma_kernel(
         const int b_next = i_next < n_head ? ha + i_next : bb + (i_next - n_head);
         AM_LOAD_BLOCK(b_next, kn0, kn1, vn)
 
-        am_block<DC, NT>(kf0, kf1, vf, qf, p_col, lo_col, mask.first, kb, g, scale2, m_run, l_run, acc);
+        am_block<DC, NT, CAP>(kf0, kf1, vf, qf, p_col, lo_col, mask.first, kb, g, scale2, cap2, m_run, l_run, acc);
 #pragma unroll
         for (int dc = 0; dc < DC; ++dc) {
             kf0[dc] = kn0[dc];
@@ -289,7 +291,7 @@ __global__ __launch_bounds__(256) void attn_mfma_kernel(
         l_tot += __shfl_xor(l_tot, 16, TL_WAVE);
         l_tot += __shfl_xor(l_tot, 32, TL_WAVE);
         if (nsplit == 1) {
-            if (sink) l_tot += exp2f(-m_run[j]);             // the sink: a key of score 0 without a value
+            if (sinks) l_tot += exp2f(sinks[head_col[j]] * AM_LOG2E - m_run[j]);   // the head's sink: a key without a value
             const float inv = 1.0f / l_tot;
             bf16_t* op = out + (size_t)row_col[j] * out_stride + (size_t)head_col[j] * D + 4 * g;
 #pragma unroll
@@ -321,10 +323,10 @@ __global__ __launch_bounds__(256) void attn_mfma_kernel(
 // take the same unit of 16 consecutive rows, are spread over all banks (at_k_swizzle, at_v_swizzle).
 // All score tiles first, then the softmax of each column tile, then all P*V products, so that key
 // fragments are dead before value fragments are read: few registers are live at once.
-template <int DC, int NT>
+template <int DC, int NT, bool CAP>
 __device__ __forceinline__ void am_block_lds(const uint4* kt, const uint4* vt, int kx, int vx, int half,
                                              const uint4 (*qf)[DC], const int* p_col, const int* lo_col, int first, int kb,
-                                             int c, int g, float scale2, float* m_run, float* l_run, f32x4 (*acc)[DC * 2]) {
+                                             int c, int g, float scale2, float cap2, float* m_run, float* l_run, f32x4 (*acc)[DC * 2]) {
     constexpr int DB = DC * 2;
     constexpr int UPK = DC * 4;
     const int key_base = kb + 8 * g;
@@ -347,8 +349,8 @@ __device__ __forceinline__ void am_block_lds(const uint4* kt, const uint4* vt, i
         float sv[8];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            sv[i] = st0[j][i] * scale2;
-            sv[4 + i] = st1[j][i] * scale2;
+            sv[i] = CAP ? tl_capped(st0[j][i], scale2, cap2) : st0[j][i] * scale2;
+            sv[4 + i] = CAP ? tl_capped(st1[j][i], scale2, cap2) : st1[j][i] * scale2;
         }
         const bool edge = (kb + 31 > p_col[j]) || (kb < lo_col[j]);
         if (__any(edge)) {
@@ -406,9 +408,9 @@ __device__ __forceinline__ void am_block_lds(const uint4* kt, const uint4* vt, i
 // argument, and the LDS reads ahead of the products that use them: the key fragments of two
 // 32-wide slices of the head are in flight while the products of the slice before run, the value
 // fragments of the first 32 keys while the softmax is computed.
-template <int DC>
+template <int DC, bool CAP>
 __device__ __forceinline__ void am_tile_lds(const uint4* kt, const uint4* vt, int kx, int vx, const uint4* qf,
-                                            int p_col, int lo_col, int first, int kb, int c, int g, float scale2,
+                                            int p_col, int lo_col, int first, int kb, int c, int g, float scale2, float cap2,
                                             float& m_run, float& l_run, f32x4* acc) {
     constexpr int DB = DC * 2;
     constexpr int UPK = DC * 4;
@@ -453,7 +455,7 @@ __device__ __forceinline__ void am_tile_lds(const uint4* kt, const uint4* vt, in
 #pragma unroll
     for (int r = 0; r < 4; ++r)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) sv[4 * r + i] = st[r][i];
+        for (int i = 0; i < 4; ++i) sv[4 * r + i] = CAP ? tl_capped(st[r][i], scale2, cap2) : st[r][i];
     const bool edge = (kb + 63 > p_col) || (kb < lo_col);
     if (__any(edge)) {
 #pragma unroll
@@ -467,13 +469,13 @@ __device__ __forceinline__ void am_tile_lds(const uint4* kt, const uint4* vt, in
     float bmax = am_max3(am_max3(am_max3(sv[0], sv[1], sv[2]), am_max3(sv[3], sv[4], sv[5]), sv[6]),
                          am_max3(am_max3(sv[7], sv[8], sv[9]), am_max3(sv[10], sv[11], sv[12]), sv[13]), am_max3(sv[14], sv[15], sv[15]));
     bmax = am_column_max(bmax);
-    bmax *= scale2;                                          // the scale is positive: the order is the same
+    if (!CAP) bmax *= scale2;                                // the scale is positive: the order is the same
     const bool moved = bmax > m_run + AM_LAZY;               // also the first keys: -inf + AM_LAZY is -inf
     const float m_new = moved ? bmax : m_run;
     const float neg_m = (m_new == -INFINITY) ? 0.f : -m_new;
     float pr[16];
 #pragma unroll
-    for (int i = 0; i < 16; ++i) pr[i] = __builtin_amdgcn_exp2f(__builtin_fmaf(sv[i], scale2, neg_m));
+    for (int i = 0; i < 16; ++i) pr[i] = __builtin_amdgcn_exp2f(CAP ? sv[i] + neg_m : __builtin_fmaf(sv[i], scale2, neg_m));
     const float psum = (((pr[0] + pr[1]) + (pr[2] + pr[3])) + ((pr[4] + pr[5]) + (pr[6] + pr[7]))) +
                        (((pr[8] + pr[9]) + (pr[10] + pr[11])) + ((pr[12] + pr[13]) + (pr[14] + pr[15])));
     uint4 pf[2];
@@ -559,12 +561,12 @@ __device__ __forceinline__ void at_load_to_lds(const void* g, void* lds_base) {
 // work-group per CU (a short portion behind a long context), where the longest walk sets the time and
 // a lone work-group leaves part of its CU unused.  The chains share the barrier, so they pass a
 // tile's phases together and gain less than two work-groups that drift apart would: 10 to 17%.
-template <int DC, int NT, int WAVES, int CH>
+template <int DC, int NT, int WAVES, int CH, bool CAP>
 __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int32_t* __restrict__ tables, int NB, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_start, bf16_t* __restrict__ out, int out_stride, int S, int nq, int nkv, int bs,
-    int bs_shift, TlMask mask, float scale, int skip_single, int sink) {
+    int bs_shift, TlMask mask, float scale, int skip_single, const float* __restrict__ sinks, float softcap) {
     constexpr int THREADS = CH * WAVES * 64;
     constexpr int WCOLS = NT * 16;                       // columns of a wave; WAVES * WCOLS = 128 per work-group
     constexpr int D = DC * 32;
@@ -587,7 +589,8 @@ __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
     const int c = lane & 15, g = lane >> 4;
     const int kvh = blockIdx.x;                            // fastest: the heads of a group start together
     const int G = nq / nkv;
-    const float scale2 = scale * AM_LOG2E;
+    const float scale2 = CAP ? 2.0f * AM_LOG2E * scale / softcap : scale * AM_LOG2E;   // see am_block
+    const float cap2 = softcap * AM_LOG2E;
     // Which (sequence, group of 128 columns) this work-group owns: the grid has one work-group per
     // group that exists (a step mixes a long prompt portion with many one-token sequences, and a
     // grid of sequences x most groups would be nearly all empty work-groups).  Within a sequence
@@ -741,13 +744,13 @@ __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
         const uint4* vt = vs + cur * TILE;                                                                    \
         if (NT == 1 && (T) * AT_KEYS + 32 <= wk_hi && (T) * AT_KEYS + 31 >= wk_lo) {                          \
             /* both halves hold keys of the wave: the whole tile at once */                                   \
-            am_tile_lds<DC>(kt, vt, kx, vx, qf[0], p_col[0], lo_col[0], first_key, (T) * AT_KEYS, c, g, scale2,   \
+            am_tile_lds<DC, CAP>(kt, vt, kx, vx, qf[0], p_col[0], lo_col[0], first_key, (T) * AT_KEYS, c, g, scale2, cap2, \
                             m_run[0], l_run[0], acc[0]);                                                      \
         } else {                                                                                              \
             _Pragma("unroll") for (int half = 0; half < 2; ++half) {                                          \
                 const int kb = (T) * AT_KEYS + half * 32;                                                     \
                 if (kb > wk_hi || (kb + 31 < wk_lo && kb >= first_key)) continue; /* the same for the whole wave */ \
-                am_block_lds<DC, NT>(kt, vt, kx, vx, half, qf, p_col, lo_col, first_key, kb, c, g, scale2, m_run, l_run, acc); \
+                am_block_lds<DC, NT, CAP>(kt, vt, kx, vx, half, qf, p_col, lo_col, first_key, kb, c, g, scale2, cap2, m_run, l_run, acc); \
             }                                                                                                 \
         }                                                                                                     \
     }
@@ -826,7 +829,7 @@ __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
         float l_tot = l_run[j];
         l_tot += __shfl_xor(l_tot, 16, TL_WAVE);
         l_tot += __shfl_xor(l_tot, 32, TL_WAVE);
-        if (sink) l_tot += exp2f(-m_run[j]);                 // the sink: a key of score 0 without a value
+        if (sinks) l_tot += exp2f(sinks[head_col[j]] * AM_LOG2E - m_run[j]);       // the head's sink: a key without a value
         const float inv = 1.0f / l_tot;
         bf16_t* op = out + (size_t)row_col[j] * out_stride + (size_t)head_col[j] * D + 4 * g;
 #pragma unroll
@@ -859,7 +862,7 @@ template <int AM_MERGE_THREADS>
 __global__ __launch_bounds__(AM_MERGE_THREADS) void attn_merge_kernel(
     const float* __restrict__ ws_o, const float* __restrict__ ws_ml, const int32_t* __restrict__ pos,
     bf16_t* __restrict__ out, int out_stride, int nq, int D, int nsplit, int split_blocks, TlMask mask,
-    const int32_t* __restrict__ seq_list, const int32_t* __restrict__ q_start, int sink) {
+    const int32_t* __restrict__ seq_list, const int32_t* __restrict__ q_start, const float* __restrict__ sinks) {
     __shared__ float wgt[AM_MAX_SPLITS];
     __shared__ float red_m[AM_MERGE_THREADS / 64], red_l[AM_MERGE_THREADS / 64];
     __shared__ float4 part[AM_MERGE_THREADS];
@@ -922,7 +925,7 @@ __global__ __launch_bounds__(AM_MERGE_THREADS) void attn_merge_kernel(
     float L = red_l[0];
 #pragma unroll
     for (int w = 1; w < AM_MERGE_THREADS / 64; ++w) L += red_l[w];
-    if (sink) L += exp2f(-M);                                // the sink: a key of score 0 without a value
+    if (sinks) L += exp2f(sinks[h] * AM_LOG2E - M);          // the head's sink: a key without a value
     float4 o4 = zero4;
 #pragma unroll
     for (int k = 0; k < AM_MERGE_AHEAD; ++k) {
@@ -961,18 +964,22 @@ static void launch_attn(int NT, dim3 grid, int wg_waves, hipStream_t stream, con
                         const bf16_t* vc, const int32_t* tables, int NB, const int32_t* q_start,
                         const int32_t* ctx_start, bf16_t* out, int out_stride, float* ws_o, float* ws_ml, int nq, int nkv,
                         int bs, TlMask mask, float scale, int nsplit, int split_blocks, const int32_t* seq_list,
-                        int skip_single, int sink) {
+                        int skip_single, const float* sinks, float softcap) {
     int bs_shift = -1;                               // pages of a power of two of tokens: a shift finds the page
     if ((bs & (bs - 1)) == 0)
         for (bs_shift = 0; (1 << bs_shift) < bs;) ++bs_shift;
-    if (NT == 1)
-        hipLaunchKernelGGL((attn_mfma_kernel<DC, 1>), grid, dim3(64 * wg_waves), 0, stream, q, q_stride, kc, vc, tables, NB, q_start,
-                           ctx_start, out, out_stride, ws_o, ws_ml, nq, nkv, bs, bs_shift, mask, scale, nsplit,
-                           split_blocks, seq_list, skip_single, sink);
-    else
-        hipLaunchKernelGGL((attn_mfma_kernel<DC, 2>), grid, dim3(64 * wg_waves), 0, stream, q, q_stride, kc, vc, tables, NB, q_start,
-                           ctx_start, out, out_stride, ws_o, ws_ml, nq, nkv, bs, bs_shift, mask, scale, nsplit,
-                           split_blocks, seq_list, skip_single, sink);
+#define AM_GO(NTV, CAPV)                                                                                                         \
+    hipLaunchKernelGGL((attn_mfma_kernel<DC, NTV, CAPV>), grid, dim3(64 * wg_waves), 0, stream, q, q_stride, kc, vc, tables, NB, \
+                       q_start, ctx_start, out, out_stride, ws_o, ws_ml, nq, nkv, bs, bs_shift, mask, scale, nsplit,           \
+                       split_blocks, seq_list, skip_single, sinks, softcap)
+    if (NT == 1) {
+        if (softcap > 0.f) AM_GO(1, true);
+        else AM_GO(1, false);
+    } else {
+        if (softcap > 0.f) AM_GO(2, true);
+        else AM_GO(2, false);
+    }
+#undef AM_GO
 }
 
 // q: bfloat16 [T, >= nq*d] (row stride q_stride); k_cache [pages, page, nkv, d]; v_cache
@@ -989,14 +996,15 @@ static void launch_attn(int NT, dim3 grid, int wg_waves, hipStream_t stream, con
 // computed, with split keys, and the workspace then holds n_list rows instead of T), and one
 // with skip_single != 0, which leaves sequences of one token out.
 // total_groups128: the sum over the sequences of ceil(n_s * G / 128), that kernel's grid.
-// sink != 0: one is added to the softmax's denominator (a key of score 0 that has no value).
+// sinks: a float per query head (null: none): exp(sinks[h]) is added to head h's softmax denominator (a key that has no
+// value; neither scaled nor capped).  softcap > 0: scores are bent, score -> softcap tanh(score / softcap).
 // window, chunk, keep_first: which keys a token sees (TlMask).
 extern "C" int tl_attention_mfma(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                  const int32_t* tables, int NB, const int32_t* q_start, const int32_t* ctx_start,
                                  const int32_t* pos, void* out, int out_stride, float* ws_o, float* ws_ml, int T, int S,
                                  int nq, int nkv, int d, int bs, int window, float scale, int NT, int max_tile_groups,
                                  int nsplit, int split_blocks, int shared, int total_groups128,
-                                 const int32_t* seq_list, int n_list, int skip_single, int sink, int keep_first, int chunk,
+                                 const int32_t* seq_list, int n_list, int skip_single, const float* sinks, float softcap, int keep_first, int chunk,
                                  hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && S >= 0 && nq > 0 && nkv > 0 && NB > 0, "tl_attention_mfma: bad sizes T=%d S=%d nq=%d nkv=%d NB=%d", T, S, nq, nkv, NB);
     TL_CHECK_ARG(nq % nkv == 0, "tl_attention_mfma: %d query heads are not a multiple of %d key/value heads", nq, nkv);
@@ -1004,6 +1012,7 @@ extern "C" int tl_attention_mfma(const void* q, int q_stride, const void* k_cach
     TL_CHECK_ARG(bs >= 8 && bs % 8 == 0, "tl_attention_mfma: page size %d must be a multiple of 8", bs);
     TL_CHECK_ARG(NT == 1 || NT == 2, "tl_attention_mfma: NT=%d must be 1 or 2", NT);
     TL_CHECK_ARG(window >= 0 && keep_first >= 0 && chunk >= 0, "tl_attention_mfma: negative window, chunk or kept first keys");
+    TL_CHECK_ARG(softcap >= 0.f, "tl_attention_mfma: negative cap %g", (double)softcap);
     const TlMask mask{window, chunk, keep_first};
     TL_CHECK_ARG(nsplit >= 1 && nsplit <= AM_MAX_SPLITS && max_tile_groups >= 1,
                  "tl_attention_mfma: bad split count %d (at most %d) or group count", nsplit, AM_MAX_SPLITS);
@@ -1041,45 +1050,47 @@ extern "C" int tl_attention_mfma(const void* q, int q_stride, const void* k_cach
         dim3 sgrid(nkv, (unsigned)total_groups128, 1);
         const int chains = (shared == 2 && at_lds_bytes(d / 32, NB, S, 2) <= 160 * 1024) ? 2 : 1;
         const size_t lds = at_lds_bytes(d / 32, NB, S, chains);
-#define TL_TILE_CASE(DCV)                                                                                             \
+#define TL_TILE_CASE(DCV) do { if (softcap > 0.f) TL_TILE_GO(DCV, true); else TL_TILE_GO(DCV, false); } while (0)
+#define TL_TILE_GO(DCV, CAPV)                                                                                         \
     do {                                                                                                              \
         if (chains == 2)                                                                                              \
-            hipLaunchKernelGGL((attn_tile_kernel<DCV, AT_NT, 8 / AT_NT, 2>), sgrid, dim3(2 * 64 * 8 / AT_NT), lds,    \
+            hipLaunchKernelGGL((attn_tile_kernel<DCV, AT_NT, 8 / AT_NT, 2, CAPV>), sgrid, dim3(2 * 64 * 8 / AT_NT), lds,    \
                                stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride, \
-                               S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sink);                                 \
+                               S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap);                                 \
         else                                                                                                          \
-            hipLaunchKernelGGL((attn_tile_kernel<DCV, AT_NT, 8 / AT_NT, 1>), sgrid, dim3(64 * 8 / AT_NT), lds,        \
+            hipLaunchKernelGGL((attn_tile_kernel<DCV, AT_NT, 8 / AT_NT, 1, CAPV>), sgrid, dim3(64 * 8 / AT_NT), lds,        \
                                stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride, \
-                               S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sink);                                 \
+                               S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap);                                 \
     } while (0)
         if (d == 32) TL_TILE_CASE(1);
         else if (d == 64) TL_TILE_CASE(2);
         else TL_TILE_CASE(4);
+#undef TL_TILE_GO
 #undef TL_TILE_CASE
         TL_CHECK_LAUNCH("tl_attention_mfma tiles");
         return 0;
     }
     if (d == 32)
         launch_attn<1>(NT, grid, wg_waves, stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride,
-                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sink);
+                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap);
     else if (d == 64)
         launch_attn<2>(NT, grid, wg_waves, stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride,
-                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sink);
+                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap);
     else if (d == 128)
         launch_attn<4>(NT, grid, wg_waves, stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride,
-                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sink);
+                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap);
     else
         launch_attn<8>(NT, grid, wg_waves, stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride,
-                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sink);
+                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap);
     TL_CHECK_LAUNCH("tl_attention_mfma");
     if (nsplit > 1) {
         const int merge_rows = seq_list ? n_list : T;
         if (nsplit > 32)
             hipLaunchKernelGGL(attn_merge_kernel<256>, dim3(merge_rows, nq), dim3(256), 0, stream, ws_o, ws_ml, pos,
-                               (bf16_t*)out, out_stride, nq, d, nsplit, split_blocks, mask, seq_list, q_start, sink);
+                               (bf16_t*)out, out_stride, nq, d, nsplit, split_blocks, mask, seq_list, q_start, sinks);
         else
             hipLaunchKernelGGL(attn_merge_kernel<128>, dim3(merge_rows, nq), dim3(128), 0, stream, ws_o, ws_ml, pos,
-                               (bf16_t*)out, out_stride, nq, d, nsplit, split_blocks, mask, seq_list, q_start, sink);
+                               (bf16_t*)out, out_stride, nq, d, nsplit, split_blocks, mask, seq_list, q_start, sinks);
         TL_CHECK_LAUNCH("tl_attention_mfma merge");
     }
     return 0;

@@ -161,13 +161,14 @@ __device__ __forceinline__ void t32_weighted_sum(const uint4* vt, const int* vof
 // by more than T32_LAZY, so probabilities stay below 2^T32_LAZY and the accumulator is rescaled in
 // few tiles instead of most.  Sums and accumulators stay relative to the same running maximum, so
 // the result is the same.
+template <bool CAP>
 __device__ __forceinline__ float t32_softmax(const t32_f32x16* sc, bool edge, int p_col, int lo_col, int first, int kb, int h,
-                                             float scale2, float& m_run, float& l_run, uint4* pf) {
+                                             float scale2, float cap2, float& m_run, float& l_run, uint4* pf) {
     float sv[32];
 #pragma unroll
     for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int r = 0; r < 16; ++r) sv[16 * t + r] = sc[t][r];
+        for (int r = 0; r < 16; ++r) sv[16 * t + r] = CAP ? tl_capped(sc[t][r], scale2, cap2) : sc[t][r];
     if (edge) {                                              // some key of the tile is hidden from some column of the wave
 #pragma unroll
         for (int x = 0; x < 32; ++x) {
@@ -183,13 +184,13 @@ __device__ __forceinline__ float t32_softmax(const t32_f32x16* sc, bool edge, in
     float bmax = t32_max3(t32_max3(mx[0], mx[1], mx[2]), t32_max3(mx[3], mx[4], mx[5]), t32_max3(mx[6], mx[7], mx[8]));
     bmax = t32_max3(bmax, mx[9], mx[10]);
     bmax = t32_halves_max(bmax);
-    bmax *= scale2;                                          // the scale is positive: the order is the same
+    if (!CAP) bmax *= scale2;                                // the scale is positive: the order is the same
     const bool moved = bmax > m_run + T32_LAZY;              // also the first keys: -inf + T32_LAZY is -inf
     const float m_new = moved ? bmax : m_run;
     const float neg_m = (m_new == -INFINITY) ? 0.f : -m_new;
     float pr[32];
 #pragma unroll
-    for (int x = 0; x < 32; ++x) pr[x] = __builtin_amdgcn_exp2f(__builtin_fmaf(sv[x], scale2, neg_m));
+    for (int x = 0; x < 32; ++x) pr[x] = __builtin_amdgcn_exp2f(CAP ? sv[x] + neg_m : __builtin_fmaf(sv[x], scale2, neg_m));
     float ps[8];
 #pragma unroll
     for (int x = 0; x < 8; ++x) ps[x] = (pr[4 * x] + pr[4 * x + 1]) + (pr[4 * x + 2] + pr[4 * x + 3]);
@@ -215,12 +216,12 @@ __device__ __forceinline__ float t32_softmax(const t32_f32x16* sc, bool edge, in
 // [S, NB]; q_start [S + 1]; ctx_start [S]; out [T, nq * D] (row stride out_stride).  Grid: (nkv,
 // sum over the sequences of ceil(n_s * G / (32 WAVES))): one work-group per group of columns that
 // exists.  bs = 2^bs_shift >= 8.  skip_single: sequences of one token belong to another launch.
-template <int DC, int WAVES>
+template <int DC, int WAVES, bool CAP>
 __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int32_t* __restrict__ tables, int NB, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_start, bf16_t* __restrict__ out, int out_stride, int S, int nq, int nkv, int bs,
-    int bs_shift, TlMask mask, float scale, int skip_single, int sink) {
+    int bs_shift, TlMask mask, float scale, int skip_single, const float* __restrict__ sinks, float softcap) {
     constexpr int THREADS = WAVES * 64;
     constexpr int WGC = WAVES * 32;           // columns of a work-group
     constexpr int D = DC * 32, KS = D / 16, DT = D / 32;
@@ -239,7 +240,9 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
     const int n32 = lane & 31, h = lane >> 5;
     const int kvh = blockIdx.x;                            // fastest: the heads of a group start together
     const int G = nq / nkv;
-    const float scale2 = scale * T32_LOG2E;
+    // capped scores: the factor into tl_capped's exponent, and the cap in the base-2 domain
+    const float scale2 = CAP ? 2.0f * T32_LOG2E * scale / softcap : scale * T32_LOG2E;
+    const float cap2 = softcap * T32_LOG2E;
     // Which (sequence, group of WGC columns) this work-group owns.  Within a sequence the groups
     // with the most keys (the last columns) come first.
     for (int i = tid; i <= S; i += THREADS) qst[i] = q_start[i];
@@ -404,7 +407,7 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
             t32_f32x16 sc[2];
             uint4 pf[4];
             t32_scores<DC>(ks + cur * TILE, koff, qf, sc);
-            const float factor = t32_softmax(sc, edge, p_col, lo_col, mask.first, kb, h, scale2, m_run, l_run, pf);
+            const float factor = t32_softmax<CAP>(sc, edge, p_col, lo_col, mask.first, kb, h, scale2, cap2, m_run, l_run, pf);
             if (__any(factor != 1.0f)) {                     // some column's maximum moved
 #pragma unroll
                 for (int m = 0; m < DT; ++m)
@@ -423,8 +426,8 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
 #undef T32_TILE_AT
 
     if (!valid) return;
-    // with a sink one is added to the denominator: a key of score 0 that has no value
-    const float inv = 1.0f / (t32_halves_sum(l_run) + (sink ? exp2f(-m_run) : 0.f));
+    // the head's sink: a key that has no value
+    const float inv = 1.0f / (t32_halves_sum(l_run) + (sinks ? exp2f(sinks[head] * T32_LOG2E - m_run) : 0.f));
     // register r of row tile m is dim 32 m + 8 (r / 4) + 4 h + r % 4: four consecutive dims per store
     bf16_t* op = out + (size_t)row_out * out_stride + (size_t)head * D + 4 * h;
 #pragma unroll
@@ -458,7 +461,8 @@ extern "C" int tl_attention_tile32_columns(int waves) { return 32 * waves; }
 extern "C" int tl_attention_tile32(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                    const int32_t* tables, int NB, const int32_t* q_start, const int32_t* ctx_start,
                                    void* out, int out_stride, int T, int S, int nq, int nkv, int d, int bs, int window,
-                                   float scale, int waves, int total_groups, int skip_single, int sink, int keep_first,
+                                   float scale, int waves, int total_groups, int skip_single, const float* sinks,
+                                   float softcap, int keep_first,
                                    int chunk, hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && S >= 0 && nq > 0 && nkv > 0 && NB > 0, "tl_attention_tile32: bad sizes T=%d S=%d nq=%d nkv=%d NB=%d", T, S, nq, nkv, NB);
     TL_CHECK_ARG(nq % nkv == 0, "tl_attention_tile32: %d query heads are not a multiple of %d key/value heads", nq, nkv);
@@ -472,7 +476,7 @@ extern "C" int tl_attention_tile32(const void* q, int q_stride, const void* k_ca
                  "tl_attention_tile32: %d key/value heads or %d column groups are more than a launch takes", nkv, total_groups);
     TL_CHECK_ARG(scale > 0.f, "tl_attention_tile32: the score scale %g must be positive", (double)scale);
     TL_CHECK_ARG((uint64_t)nkv * d * 2 * 8 < (1ull << 31), "tl_attention_tile32: a cache slot of %d heads is too wide", nkv);
-    TL_CHECK_ARG(window >= 0 && chunk >= 0 && keep_first >= 0, "tl_attention_tile32: negative window, chunk or kept first keys");
+    TL_CHECK_ARG(window >= 0 && chunk >= 0 && keep_first >= 0 && softcap >= 0.f, "tl_attention_tile32: negative window, chunk, kept first keys or cap");
     if (T == 0 || S == 0 || total_groups == 0) return 0;
     const TlMask mask{window, chunk, keep_first};
     int bs_shift = 0;
@@ -480,13 +484,15 @@ extern "C" int tl_attention_tile32(const void* q, int q_stride, const void* k_ca
     const size_t lds = t32_lds_bytes(d, NB, S);
     dim3 grid(nkv, (unsigned)total_groups, 1);
     const bf16_t *qq = (const bf16_t*)q, *kk = (const bf16_t*)k_cache, *vv = (const bf16_t*)v_cache;
-#define T32_LAUNCH(DCV, WV)                                                                                             \
-    hipLaunchKernelGGL((attn_tile32_kernel<DCV, WV>), grid, dim3(64 * WV), lds, stream, qq, q_stride, kk, vv, tables, NB, \
-                       q_start, ctx_start, (bf16_t*)out, out_stride, S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sink)
+#define T32_LAUNCH(DCV, WV) do { if (softcap > 0.f) T32_GO(DCV, WV, true); else T32_GO(DCV, WV, false); } while (0)
+#define T32_GO(DCV, WV, CAPV)                                                                                           \
+    hipLaunchKernelGGL((attn_tile32_kernel<DCV, WV, CAPV>), grid, dim3(64 * WV), lds, stream, qq, q_stride, kk, vv, tables, NB, \
+                       q_start, ctx_start, (bf16_t*)out, out_stride, S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap)
     if (d == 64 && waves == 4) T32_LAUNCH(2, 4);
     else if (d == 64) T32_LAUNCH(2, 8);
     else if (waves == 4) T32_LAUNCH(4, 4);
     else T32_LAUNCH(4, 8);
+#undef T32_GO
 #undef T32_LAUNCH
     TL_CHECK_LAUNCH("tl_attention_tile32");
     return 0;

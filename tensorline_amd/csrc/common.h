@@ -128,6 +128,17 @@ __host__ __device__ __forceinline__ int tl_mask_lo(const TlMask& k, int p) {
 // a key below lo is hidden unless it is one of the kept first keys
 __device__ __forceinline__ bool tl_mask_hides(const TlMask& k, int key, int lo) { return key < lo && key >= k.first; }
 
+// ---- scores bent by a cap ------------------------------------------------------------------------
+// cap * tanh(score / cap), in the units the caller keeps scores in: raw is the bare product of query and
+// key, to_exp = 2 log2(e) * scale / cap turns it into the exponent of e^(2 score / cap) = 2^(raw to_exp), and
+// cap_out is the cap in the caller's units (times log2 e where scores are exponents of two).  tanh(y) =
+// 1 - 2 / (1 + e^(2 y)): one exponential and one reciprocal, exact limits at both ends (an infinite or zero
+// exponential gives cap_out and -cap_out), an absolute error of the order of cap times the float's precision.
+__device__ __forceinline__ float tl_capped(float raw, float to_exp, float cap_out) {
+    const float e = __builtin_amdgcn_exp2f(raw * to_exp);
+    return __builtin_fmaf(-2.0f * cap_out, __builtin_amdgcn_rcpf(1.0f + e), cap_out);
+}
+
 // ---- host side -----------------------------------------------------------------------------
 // Every C entry point returns 0 on success.  On failure it returns a non-zero code and leaves a
 // message that tl_last_error() hands out; nothing is launched in that case.

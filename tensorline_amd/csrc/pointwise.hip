@@ -605,6 +605,26 @@ extern "C" int tl_diff_combine(const void* a, int lda, void* out, int dtype, int
     return 0;
 }
 
+// ---- a block of columns in the other storage type --------------------------------------------------------------
+template <typename O>
+__global__ void cast_rows_kernel(const float* __restrict__ in, int ldi, O* __restrict__ out, int T, int n) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= (size_t)T * n) return;
+    out[i] = tl_from_float<O>(in[(i / n) * ldi + i % n]);
+}
+
+// in float [T, >= n] (row stride ldi), out [T, n] float or bfloat16
+extern "C" int tl_cast_rows(const float* in, int ldi, void* out, int out_dtype, int T, int n, hipStream_t stream) {
+    TL_CHECK_ARG(T >= 0 && n > 0 && ldi >= n, "tl_cast_rows: bad sizes");
+    if (T == 0) return 0;
+    dim3 grid((unsigned)(((size_t)T * n + 255) / 256)), block(256);
+    if (out_dtype == TL_F32) hipLaunchKernelGGL(cast_rows_kernel<float>, grid, block, 0, stream, in, ldi, (float*)out, T, n);
+    else if (out_dtype == TL_BF16) hipLaunchKernelGGL(cast_rows_kernel<bf16_t>, grid, block, 0, stream, in, ldi, (bf16_t*)out, T, n);
+    else return tl_fail("tl_cast_rows: unknown dtype %d", out_dtype);
+    TL_CHECK_LAUNCH("tl_cast_rows");
+    return 0;
+}
+
 // ---- gated activations of a fused gate/up projection --------------------------------------------------------
 // gu [T, 2F] (gate columns first): out = act(gate) * up; kind 0: act = silu, kind 1: act = the tanh form of
 // gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))).  float arithmetic.
@@ -631,13 +651,16 @@ extern "C" int tl_glu(const void* gu, int in_dtype, void* out, int out_dtype, in
     return 0;
 }
 
-// ---- queries and keys normed per head, neighbouring pairs turned, the cache write ---------------------------
+// ---- queries and keys normed per head, pairs turned, the cache write ------------------------------------------
 // proj float [T, ldp] = [q: H*d | k: G*d | v: G*dv] (biases added already; no v columns with v_from_k).
 // Per token, for every query head and key head:
 //   * the head's d values are divided by their root mean square (eps inside the root) and multiplied by a
-//     weight per dimension that all heads share (wq [d], wk [d]; null: no norm);
-//   * then the pairs (2i, 2i + 1), i < rot / 2, are turned by the angle pos * freq[i], cosine and sine both
-//     times `mag` (freq null or rot 0: no rotation); the angle, its cosine and sine are float;
+//     weight per dimension that all heads share (wq [d], wk [d]) with norm 1, by that root mean square alone with
+//     norm 2 (no weights; as a rotation with mag 1 leaves a head's sum of squares as it is, norming ahead of the
+//     rotation and behind it are then the same), and left as they are with norm 0;
+//   * then the pairs (2i, 2i + 1), or with `halves` the pairs (i, i + rot / 2), i < rot / 2, are turned by the angle
+//     pos * freq[i], cosine and sine both times `mag` (freq null or rot 0: no rotation); the angle, its cosine and
+//     sine are float;
 //   * q goes to q_out [T, H*D], every head padded with zeros from d to D; k into the cache at `slot`
 //     ([pages, page, G, D], zeros from d to D); v with a page's tokens innermost ([pages, G, D, page], zeros
 //     from dv to D).  With v_from_k the values are the keys as projected: before norm and rotation.
@@ -648,7 +671,7 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
     const float* __restrict__ proj, int ldp, const int32_t* __restrict__ pos, const float* __restrict__ wq,
     const float* __restrict__ wk, float eps, const float* __restrict__ freq, float mag, int rot,
     const int32_t* __restrict__ slots, T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache, int H, int G,
-    int d, int dv, int D, int page, int v_from_k) {
+    int d, int dv, int D, int page, int v_from_k, int norm, int halves) {
     __shared__ float cs[128], sn[128];
     const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const float* row = proj + (size_t)t * ldp;
@@ -668,28 +691,33 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
         const int n = (is_q || is_k) ? d : dv;                   // the values the head has
         const float* x = row + (is_q ? head * d : is_k ? H * d + head * d : (H + G) * d + head * dv);
         float raw[4], y[4];
+        // the dimensions of the lane's two pairs: neighbours, or with `halves` those rot / 2 apart among the turned ones
+        int ca[2], cb[2];
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
-            const int c = 2 * (lane + 64 * j);
-            raw[2 * j] = c < n ? x[c] : 0.f;
-            raw[2 * j + 1] = c + 1 < n ? x[c + 1] : 0.f;
+            const int i = lane + 64 * j;
+            const bool apart = halves && (is_q || is_k) && 2 * i < rot;
+            ca[j] = apart ? i : 2 * i;
+            cb[j] = apart ? i + (rot >> 1) : 2 * i + 1;
+            raw[2 * j] = ca[j] < n ? x[ca[j]] : 0.f;
+            raw[2 * j + 1] = cb[j] < n ? x[cb[j]] : 0.f;
         }
         if (!is_q && slot < 0) continue;                         // nothing to write for this token (the same for the wave)
-        const float* w = is_q ? wq : is_k ? wk : nullptr;
+        const float* w = norm == 1 ? (is_q ? wq : is_k ? wk : nullptr) : nullptr;
         float rstd = 1.0f;
-        if (w) {
+        if (norm && (is_q || is_k)) {
             const float ss = tl_wave_sum(raw[0] * raw[0] + raw[1] * raw[1] + raw[2] * raw[2] + raw[3] * raw[3]);
             rstd = 1.0f / sqrtf(ss / (float)n + eps);
         }
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
-            const int i = lane + 64 * j, c = 2 * i;
-            float a = raw[2 * j], b = raw[2 * j + 1];
+            const int i = lane + 64 * j;
+            float a = raw[2 * j] * rstd, b = raw[2 * j + 1] * rstd;
             if (w) {
-                a = c < n ? a * rstd * w[c] : 0.f;
-                b = c + 1 < n ? b * rstd * w[c + 1] : 0.f;
+                a = ca[j] < n ? a * w[ca[j]] : 0.f;
+                b = cb[j] < n ? b * w[cb[j]] : 0.f;
             }
-            if ((is_q || is_k) && c + 1 < rot) {
+            if ((is_q || is_k) && 2 * i + 1 < rot) {
                 const float ra = a * cs[i] - b * sn[i], rb = b * cs[i] + a * sn[i];
                 a = ra;
                 b = rb;
@@ -701,7 +729,7 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
         for (int j = 0; j < 2; ++j) {
 #pragma unroll
             for (int e = 0; e < 2; ++e) {
-                const int c = 2 * (lane + 64 * j) + e;
+                const int c = e ? cb[j] : ca[j];
                 if (c >= D) continue;
                 const T o = tl_from_float<T>(y[2 * j + e]);       // zeros beyond the head's values
                 if (is_q) {
@@ -720,12 +748,13 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
 extern "C" int tl_head_norm_rotate_store(const float* proj, int ldp, const int32_t* pos, const float* wq, const float* wk,
                                          float eps, const float* freq, float mag, int rot, const int32_t* slots, void* q_out,
                                          void* k_cache, void* v_cache, int dtype, int T, int H, int G, int d, int dv, int D,
-                                         int page, int v_from_k, hipStream_t stream) {
+                                         int page, int v_from_k, int norm, int halves, hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && H > 0 && G >= 0 && d > 0 && dv > 0 && D >= d && D >= dv && D <= 256 && page > 0,
                  "tl_head_norm_rotate_store: bad sizes H=%d G=%d d=%d dv=%d D=%d", H, G, d, dv, D);
     TL_CHECK_ARG(rot >= 0 && rot % 2 == 0 && rot <= d && (rot == 0 || freq), "tl_head_norm_rotate_store: %d turned dimensions of %d", rot, d);
     TL_CHECK_ARG(!v_from_k || dv == d, "tl_head_norm_rotate_store: values that are the keys have the keys' size");
-    TL_CHECK_ARG((wq == nullptr) == (wk == nullptr), "tl_head_norm_rotate_store: queries and keys are normed together or not at all");
+    TL_CHECK_ARG(norm >= 0 && norm <= 2 && (norm == 1) == (wq != nullptr) && (norm == 1) == (wk != nullptr),
+                 "tl_head_norm_rotate_store: queries and keys are normed together or not at all, with weights in form 1");
     TL_CHECK_ARG(ldp >= (H + G) * d + (v_from_k ? 0 : G * dv), "tl_head_norm_rotate_store: the projection's rows are too short");
     TL_CHECK_ARG(G == 0 || (slots && k_cache && v_cache), "tl_head_norm_rotate_store: keys need their cache");
     if (T == 0) return 0;
@@ -733,7 +762,7 @@ extern "C" int tl_head_norm_rotate_store(const float* proj, int ldp, const int32
     TL_CHECK_ARG(grid.y <= 65535, "tl_head_norm_rotate_store: too many heads");
 #define GO(TT)                                                                                                         \
     hipLaunchKernelGGL(head_norm_rotate_store_kernel<TT>, grid, block, 0, stream, proj, ldp, pos, wq, wk, eps, freq, mag, \
-                       rot, slots, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, H, G, d, dv, D, page, v_from_k)
+                       rot, slots, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, H, G, d, dv, D, page, v_from_k, norm, halves)
     if (dtype == TL_F32) GO(float);
     else if (dtype == TL_BF16) GO(bf16_t);
     else return tl_fail("tl_head_norm_rotate_store: unknown dtype %d", dtype);

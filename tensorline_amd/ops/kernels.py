@@ -177,6 +177,51 @@ def _branch_norm_add(x, branch: NormedBranch, weight, eps, out_dtype, rows):
     return out
 
 
+@dataclass
+class ScaledBranches:
+    """Residual branches that join the stream together, with one factor: stands for ``mult * (y1 + y2)`` (``y2`` may
+    be None), still to be added.  The norm that reads the stream next adds it in its own pass
+    (:func:`add_layernorm`)."""
+    y1: torch.Tensor                 # float32 [T, H]
+    y2: torch.Tensor | None
+    mult: float
+
+
+def add_scaled_branches(x: torch.Tensor, branches: ScaledBranches) -> None:
+    """``x += branches.mult * (branches.y1 + branches.y2)`` in place, nothing else."""
+    add_layernorm(x, branches, None, None, 0.0, None)
+
+
+def add_layernorm(x: torch.Tensor, residual: "torch.Tensor | ScaledBranches | None", weight: torch.Tensor | None,
+                  bias: torch.Tensor | None, eps: float, out_dtype: torch.dtype | None,
+                  rows: torch.Tensor | None = None) -> torch.Tensor | None:
+    """Without ``rows``: ``x += residual`` in place (float32), returns ``(x - mean) / sqrt(variance + eps) * weight +
+    bias`` with the mean and the variance (the mean of the squared deviations) of each row.  With ``rows``: the norm of
+    ``x[rows] + residual[rows]``, ``x`` left alone.  ``residual`` may be :class:`ScaledBranches`.  Without ``weight``:
+    only the sum, and None is returned."""
+    if residual is not None and not isinstance(residual, ScaledBranches):
+        residual = ScaledBranches(residual, None, 1.0)
+    y1, y2, mult = (residual.y1, residual.y2, residual.mult) if residual is not None else (None, None, 1.0)
+    _on_gpu(x, y1, y2, weight, bias, rows)
+    _check(x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(), "add_layernorm: x must be contiguous float32 [T, H]")
+    T, H = x.shape
+    for y in (y1, y2):
+        if y is not None:
+            _check(y.dtype == torch.float32 and y.is_contiguous() and tuple(y.shape) == (T, H),
+                   "add_layernorm: a branch must be contiguous float32 of x's shape")
+    out, n = None, T
+    if weight is not None:
+        _f32(weight, "add_layernorm weight", H)
+        _f32(bias, "add_layernorm bias", H)
+        if rows is not None:
+            _i32(rows, "rows")
+            n = rows.numel()
+        out = torch.empty(n, H, dtype=out_dtype, device=x.device)
+    _call("tl_add_layernorm", _ptr(x), _ptr(y1), _ptr(y2), ctypes.c_float(mult), _ptr(weight), _ptr(bias), ctypes.c_float(eps),
+          _ptr(out), _code(out, "add_layernorm out") if out is not None else F32, _ptr(rows), n, H, _stream())
+    return out
+
+
 def add_rmsnorm(x: torch.Tensor, residual: "torch.Tensor | ShareSum | None", weight: torch.Tensor, eps: float,
                 out_dtype: torch.dtype, rows: torch.Tensor | None = None,
                 out: torch.Tensor | None = None) -> torch.Tensor:
@@ -803,7 +848,8 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     q_start: torch.Tensor | None = None, ctx_start: torch.Tensor | None = None, plan=None,
                     path: str | None = None, split_keys: int | None = None,
                     single_seqs: torch.Tensor | None = None, route_singles: bool | None = None,
-                    sink: bool = False, keep_first: int = 0, chunk: int = 0) -> torch.Tensor:
+                    sink: torch.Tensor | None = None, keep_first: int = 0, chunk: int = 0,
+                    softcap: float = 0.0) -> torch.Tensor:
     """Causal attention of each token over the cached keys of its sequence.
 
     ``q``: [T, >= nq*d] with the query heads in the first nq*d columns (row stride free);
@@ -813,8 +859,10 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     limits a token at position p to keys [p - window + 1, p]; ``chunk`` > 0 to the keys from the last
     multiple of ``chunk`` at or below p on (positions count from the start of the sequence); with
     ``keep_first`` > 0 the first ``keep_first`` keys of the sequence stay in sight wherever those ranges
-    begin.  ``sink`` adds one to the softmax's
-    denominator (a key of score 0 that has no value): ``p_j = exp(s_j) / (1 + sum exp(s))``.  Returns [T, nq*d].
+    begin.  ``softcap`` > 0 bends the
+    scores: ``softcap * tanh(s / softcap)``.  ``sink`` (float32 [nq]) adds ``exp(sink_h)`` to the denominator of head h's
+    softmax, a key that has no value (its logit is neither scaled nor capped): ``p_j = exp(s_j) / (exp(sink_h) + sum
+    exp(s))``.  Returns [T, nq*d].
 
     bfloat16 with a head size of 32, 64 or 128 and pages of a multiple of 8 tokens runs on the
     matrix cores; that kernel works per sequence and needs ``q_start`` [S+1], ``ctx_start`` [S]
@@ -832,7 +880,10 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     estimated to be faster (``_singles_get_own_launch``), split like a decode step of that many
     sequences, and the launch for the portions leaves them out.  ``route_singles`` forces that
     on or off."""
-    _on_gpu(q, k_cache, v_cache, tables, seq_of_token, pos, out, q_start, ctx_start)
+    _on_gpu(q, k_cache, v_cache, tables, seq_of_token, pos, out, q_start, ctx_start, sink)
+    if sink is not None:
+        _f32(sink, "paged_attention sink", num_heads)
+    cap = ctypes.c_float(softcap)
     T = q.shape[0]
     _check(q.dim() == 2 and q.stride(1) == 1 and q.shape[1] >= num_heads * head_dim, "paged_attention: bad query layout")
     _check_caches(k_cache, v_cache, q.dtype, num_kv_heads, head_dim, "paged_attention")
@@ -875,7 +926,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                       _ptr(q_start), _ptr(ctx_start), _ptr(pos), _ptr(out), o_stride, _ptr(ws[:n_o]), _ptr(ws[n_o:]), T, S,
                       num_heads, num_kv_heads, head_dim, page, int(window), ctypes.c_float(scale), nt1,
                       -(-G // (16 * nt1)), nsplit, max(split_len // 32, 1), 0, 0, _ptr(single_seqs), len(singles), 0,
-                      int(bool(sink)), keep_first, chunk, _stream())
+                      _ptr(sink), cap, keep_first, chunk, _stream())
                 skip_single = 1
         q_lens = [n for n in plan.q_lens if n > 1] if skip_single else plan.q_lens
         nt = 1 if plan.max_query_len * G <= 16 or head_dim == 256 else 2
@@ -907,14 +958,14 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
             total = sum(-(-n * G // cols) for n in q_lens) + pads
             _call("tl_attention_tile32", _ptr(q), q_stride, _ptr(k_cache), _ptr(v_cache), _ptr(tables), tables.shape[1],
                   _ptr(q_start), _ptr(ctx_start), _ptr(out), o_stride, T, S, num_heads, num_kv_heads, head_dim, page,
-                  int(window), ctypes.c_float(scale), waves, total, skip_single, int(bool(sink)), keep_first, chunk, _stream())
+                  int(window), ctypes.c_float(scale), waves, total, skip_single, _ptr(sink), cap, keep_first, chunk, _stream())
             return out
         _call("tl_attention_mfma", _ptr(q), q_stride, _ptr(k_cache), _ptr(v_cache), _ptr(tables), tables.shape[1],
               _ptr(q_start), _ptr(ctx_start), _ptr(pos), _ptr(out), o_stride, _ptr(ws_o), _ptr(ws_ml), T, S, num_heads,
               num_kv_heads, head_dim, page, int(window), ctypes.c_float(scale), nt, max_groups, nsplit, split_blocks,
               0 if path == "mfma-direct" else _tile16_chains(total128, num_kv_heads, path, plan.max_context), total128,
               _ptr(None), 0,
-              skip_single, int(bool(sink)), keep_first, chunk, _stream())
+              skip_single, _ptr(sink), cap, keep_first, chunk, _stream())
         return out
     # The any-shape kernel tiles each sequence's tokens: it needs the first row of every sequence and the
     # most tokens one of them brings.  The engine has both; a bare call derives them from seq_of_token.
@@ -947,7 +998,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
             ws = torch.empty(T * num_heads * nsplit * (head_dim + 2), dtype=torch.float32, device=q.device)
     _call("tl_attention_generic", _ptr(q), q_stride, _ptr(k_cache), _ptr(v_cache), _ptr(tables), tables.shape[1],
           _ptr(q_start), _ptr(pos), _ptr(out), o_stride, _code(q, "paged_attention"), T, S, max(max_query_len, 1), num_heads,
-          num_kv_heads, head_dim, page, int(window), ctypes.c_float(scale), nsplit, split_len, _ptr(ws), int(bool(sink)),
+          num_kv_heads, head_dim, page, int(window), ctypes.c_float(scale), nsplit, split_len, _ptr(ws), _ptr(sink), cap,
           keep_first, chunk, _stream())
     return out
 
@@ -1048,6 +1099,16 @@ def add_cast(x: torch.Tensor, residual: torch.Tensor | None, out_dtype: torch.dt
                "add_cast: the residual must be float32 of x's shape")
     out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
     _call("tl_add_cast", _ptr(x), _ptr(residual), _ptr(out), _code(out, "add_cast out"), ctypes.c_longlong(x.numel()), _stream())
+    return out
+
+
+def cast_rows(x: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """A float32 [T, n] matrix (may be a block of columns of a wider one) in ``out_dtype``, contiguous."""
+    _on_gpu(x)
+    _check(x.dtype == torch.float32 and x.dim() == 2 and x.stride(1) == 1, "cast_rows: the input must be float32 [T, n]")
+    T, n = x.shape
+    out = torch.empty(T, n, dtype=out_dtype, device=x.device)
+    _call("tl_cast_rows", _ptr(x), x.stride(0) if T > 1 else max(n, x.stride(0)), _ptr(out), _code(out, "cast_rows out"), T, n, _stream())
     return out
 
 
@@ -1325,6 +1386,158 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, ctx, st
 
 
 # ---------------------------------------------------------------------------------------------
+# Recurrences in chunks of a step's rows: the delta rule and the selective scan
+CHUNK_TOKENS = 64          # tokens per chunk in both kernels
+CHUNKED_FROM = 33          # steps whose sequences bring at most this many tokens less one walk token by token
+
+
+@dataclass
+class SequenceChunks:
+    """How the sequences of a step are cut into chunks of ``CHUNK_TOKENS`` rows, each from its first row of the step:
+    ``seq`` and ``row`` (int32 [n]) hold a chunk's sequence and its first row, ``first`` (int32 [S + 1]) a sequence's first
+    chunk."""
+    seq: torch.Tensor
+    row: torch.Tensor
+    first: torch.Tensor
+
+    @property
+    def count(self) -> int:
+        return self.seq.numel()
+
+
+def chunk_vectors(facts) -> dict[str, list[int]]:
+    """The index vectors of :class:`SequenceChunks` for a step's shape, for the step's upload; none for a step that walks."""
+    if facts.decode_only or facts.max_query_len < CHUNKED_FROM:
+        return {}
+    seq, row, first, at = [], [], [0], 0
+    lens = list(facts.q_lens) + [1] * (facts.num_seqs - len(facts.q_lens))      # padding sequences bring one token
+    for s, n in enumerate(lens):
+        for lo in range(0, n, CHUNK_TOKENS):
+            seq.append(s)
+            row.append(at + lo)
+        at += n
+        first.append(len(seq))
+    return {"chunks.seq": seq, "chunks.row": row, "chunks.first": first}
+
+
+def step_chunks(ctx) -> SequenceChunks | None:
+    """The chunks uploaded with the step, or None: then its tokens are walked one after another."""
+    seq = ctx.extra.get("chunks.seq")
+    return None if seq is None else SequenceChunks(seq, ctx.extra["chunks.row"], ctx.extra["chunks.first"])
+
+
+def _check_chunks(chunks: SequenceChunks, num_seqs: int, who: str) -> None:
+    _on_gpu(chunks.seq, chunks.row, chunks.first)
+    _i32(chunks.seq, who + " chunk sequences")
+    _i32(chunks.row, who + " chunk rows", chunks.count)
+    _i32(chunks.first, who + " first chunks", num_seqs + 1)
+
+
+def conv_unit(x: torch.Tensor, taps: torch.Tensor, ctx, state: torch.Tensor, offset: int, unit: int, n_unit: int,
+              n_scaled: int, scale: float, eps: float = 1e-6) -> torch.Tensor:
+    """A short causal convolution per channel and SiLU, as :func:`causal_conv` without bias (``x`` float32 [T, C], ``taps``
+    float32 [K, C], a tap's weights for all channels in a row; the last K - 1 inputs at ``state[slot, offset :]``).  The
+    channels lie in units of ``unit``: the first ``n_unit`` units are then divided by ``sqrt(sum of squares + eps)``, the first
+    ``n_scaled`` of those also multiplied by ``scale``.  Returns float32 [T, C]."""
+    _on_gpu(x, taps, state)
+    T, C = x.shape
+    K = taps.shape[0]
+    _check(x.dtype == torch.float32 and x.stride(1) == 1, "conv_unit: the input must be float32 [T, C]")
+    _check(taps.dim() == 2 and taps.shape[1] == C and 1 <= K <= CONV_MAX_TAPS, f"conv_unit: taps must be [up to {CONV_MAX_TAPS}, C]")
+    _f32(taps, "conv_unit taps")
+    _check(offset + (K - 1) * C <= state.shape[1], "conv_unit: the kept inputs do not fit the state")
+    kept, stride = _state_ptr(state, offset)
+    out = torch.empty(T, C, dtype=torch.float32, device=x.device)
+    _call("tl_conv_unit", _ptr(x), x.stride(0) if T > 1 else max(C, x.stride(0)), _ptr(taps), kept, ctypes.c_longlong(stride),
+          _ptr(ctx.state_slots), _ptr(ctx.seq_of_token), _ptr(ctx.q_start), _ptr(out), C, T, ctx.num_seqs, C, K, int(unit),
+          int(n_unit), int(n_scaled), ctypes.c_float(scale), ctypes.c_float(eps),
+          2 if ctx.facts.decode_only and T == ctx.num_seqs else 1, _stream())
+    return out
+
+
+def delta_takes_key_dim(dk: int) -> bool:
+    return 0 < dk <= 256
+
+
+def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b: torch.Tensor, a: torch.Tensor, rate_log: torch.Tensor,
+               step_bias: torch.Tensor | None, ctx, state: torch.Tensor, heads: int, dk: int, dv: int, share: int = 1,
+               state_offset: int = 0, chunks: SequenceChunks | None = None) -> torch.Tensor:
+    """The gated delta rule per sequence and head, with S [dk, dv] in the sequence's slot (kept transposed: ``state[slot,
+    state_offset : state_offset + heads * dv * dk]``, float32, renewed in place): with ``beta = sigmoid(b)`` and ``g = exp(-exp(
+    rate_log) softplus(a + step_bias))`` per token and head, ``S <- g S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q``.
+
+    ``q``, ``k`` float32 [T, heads / share * dk] as they enter the rule (the ``share`` consecutive heads of a group read the
+    same), ``v`` [T, heads * dv], ``b``, ``a`` [T, heads]; all may be column blocks of wider matrices.  With ``chunks`` (and
+    ``dk`` up to 128) the step's rows are taken in chunks: the same sums in another order.  Returns float32 [T, heads * dv]."""
+    _on_gpu(q, k, v, b, a, rate_log, step_bias, state)
+    T = q.shape[0]
+    share = int(share)
+    _check(share >= 1 and heads % share == 0, f"delta_rule: {heads} heads do not share queries in groups of {share}")
+    for name, t, n in (("q", q, heads // share * dk), ("k", k, heads // share * dk), ("v", v, heads * dv), ("b", b, heads), ("a", a, heads)):
+        _check(t.dtype == torch.float32 and t.dim() == 2 and t.stride(1) == 1 and tuple(t.shape) == (T, n),
+               f"delta_rule: {name} must be float32 [T, {n}]")
+    _f32(rate_log, "delta_rule rate_log", heads)
+    if step_bias is not None:
+        _f32(step_bias, "delta_rule step_bias", heads)
+    _check(state_offset + heads * dk * dv <= state.shape[1], "delta_rule: the state of a request is too small")
+    st, stride = _state_ptr(state, state_offset)
+    out = torch.empty(T, heads * dv, dtype=torch.float32, device=q.device)
+    ld = lambda t: t.stride(0) if T > 1 else max(t.shape[1], t.stride(0))
+    head = (_ptr(q), ld(q), _ptr(k), ld(k), _ptr(v), ld(v), _ptr(b), ld(b), _ptr(a), ld(a), _ptr(rate_log), _ptr(step_bias), share, st,
+            ctypes.c_longlong(stride), _ptr(ctx.state_slots), _ptr(ctx.q_start))
+    if chunks is not None and library().tl_delta_chunked_takes(dk, dv):
+        _check_chunks(chunks, ctx.num_seqs, "delta_rule")
+        fn = library().tl_delta_chunked_workspace
+        fn.restype = ctypes.c_longlong
+        ws = torch.empty(chunks.count * heads * fn(dk, dv), dtype=torch.float32, device=q.device)
+        _call("tl_delta_chunked", *head, _ptr(chunks.seq), _ptr(chunks.row), _ptr(chunks.first), _ptr(ws), _ptr(out), heads * dv,
+              ctx.num_seqs, chunks.count, heads, dk, dv, _stream())
+        return out
+    _call("tl_delta_walk", *head, _ptr(out), heads * dv, ctx.num_seqs, heads, dk, dv, _stream())
+    return out
+
+
+SELECTIVE_SCAN_MAX_STATE = 256
+
+
+def selective_scan(dt_raw: torch.Tensor, dt_bias: torch.Tensor | None, x: torch.Tensor, z: torch.Tensor, bc: torch.Tensor,
+                   a2: torch.Tensor, skip: torch.Tensor, ctx, state: torch.Tensor, offset: int,
+                   chunks: SequenceChunks | None = None) -> torch.Tensor:
+    """Mamba's selective scan per sequence, channel and state, with its gate: ``dt = softplus(dt_raw + dt_bias)``, ``S[c, n] <-
+    exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n``, result ``(sum_n S[c, n] C_n + skip_c x_c) * silu(z_c)`` in x's dtype.
+
+    ``dt_raw``, ``z`` float32 [T, inner], ``x`` [T, inner] float32 or bfloat16, ``bc`` float32 [T, 2 N] = [B | C] (all may be column
+    blocks of wider matrices), ``a2`` float32 [N, inner] = ``A^T log2(e)``, ``skip`` float32 [inner].  S lives at ``state[slot, offset
+    : offset + N * inner]`` as [N, inner].  With ``chunks`` the step's rows are taken in chunks, all at once."""
+    _on_gpu(dt_raw, dt_bias, x, z, bc, a2, skip, state)
+    T, inner = x.shape
+    N = a2.shape[0]
+    for name, t, n in (("dt", dt_raw, inner), ("z", z, inner), ("[B | C]", bc, 2 * N)):
+        _check(t.dtype == torch.float32 and t.dim() == 2 and t.stride(1) == 1 and tuple(t.shape) == (T, n),
+               f"selective_scan: {name} must be float32 [T, {n}]")
+    _check(x.stride(1) == 1 and tuple(a2.shape) == (N, inner) and N <= SELECTIVE_SCAN_MAX_STATE, "selective_scan: bad x or A")
+    _f32(a2, "selective_scan A")
+    _f32(skip, "selective_scan D", inner)
+    if dt_bias is not None:
+        _f32(dt_bias, "selective_scan dt bias", inner)
+    _check(offset + N * inner <= state.shape[1], "selective_scan: the state of a request is too small")
+    st, stride = _state_ptr(state, offset)
+    out = torch.empty(T, inner, dtype=x.dtype, device=x.device)
+    ld = lambda t: t.stride(0) if T > 1 else max(t.shape[1], t.stride(0))
+    ws_s = ws_dt = None
+    if chunks is not None:
+        _check_chunks(chunks, ctx.num_seqs, "selective_scan")
+        ws_s = torch.empty(chunks.count * N * inner, dtype=torch.float32, device=x.device)
+        ws_dt = torch.empty(chunks.count * inner, dtype=torch.float32, device=x.device)
+    seq, row, first = (chunks.seq, chunks.row, chunks.first) if chunks is not None else (None, None, None)
+    _call("tl_selective_scan", _ptr(dt_raw), ld(dt_raw), _ptr(dt_bias), _ptr(x), ld(x), _ptr(z), ld(z), _ptr(bc), ld(bc), _ptr(a2),
+          _ptr(skip), st, ctypes.c_longlong(stride), _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(seq), _ptr(row), _ptr(first),
+          _ptr(ws_s), _ptr(ws_dt), _ptr(out), _code(x, "selective_scan"), inner, ctx.num_seqs,
+          chunks.count if chunks is not None else 0, inner, N, _stream())
+    return out
+
+
+# ---------------------------------------------------------------------------------------------
 # Routed experts
 ROUTER_WEIGHTINGS = {"softmax_top": 0, "sigmoid": 1, "softmax_all": 2, "sigmoid_grouped": 3}
 
@@ -1503,12 +1716,13 @@ def qk_norm_store(proj: torch.Tensor, pos: torch.Tensor, q_weight: torch.Tensor 
 def head_norm_rotate_store(proj: torch.Tensor, pos: torch.Tensor, q_weight: torch.Tensor | None, k_weight: torch.Tensor | None,
                            eps: float, freq: torch.Tensor | None, mag: float, k_cache: torch.Tensor, v_cache: torch.Tensor,
                            slots: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, values_from_keys: bool,
-                           out_dtype: torch.dtype) -> torch.Tensor:
+                           out_dtype: torch.dtype, plain_norm: bool = False, halves: bool = False) -> torch.Tensor:
     """What lies between a fused q/k(/v) projection and attention, in one pass per token.  ``proj`` float32 [T,
     heads*dim + kv_heads*dim (+ kv_heads*vdim)] (biases added).  Every query head and key head is RMS-normed over
-    its ``dim`` values with a weight per dimension that all heads share (float32 [dim]; both None: no norm), then
-    neighbouring pairs (2i, 2i + 1) of its first ``2 len(freq)`` dimensions are turned by ``pos * freq[i]``, cosine and
-    sine times ``mag`` (``freq`` None: no rotation).  Keys and values go into the cache pages at ``slots`` (``k_cache``
+    its ``dim`` values with a weight per dimension that all heads share (float32 [dim]; both None: no norm, or with
+    ``plain_norm`` a norm without weights), then neighbouring pairs (2i, 2i + 1) of its first ``2 len(freq)`` dimensions, or
+    with ``halves`` the pairs (i, i + len(freq)), are turned by ``pos * freq[i]``, cosine and sine times ``mag`` (``freq``
+    None: no rotation).  A norm without weights comes to the same ahead of a rotation and behind it.  Keys and values go into the cache pages at ``slots`` (``k_cache``
     [pages, page, kv_heads, D], ``v_cache`` [pages, kv_heads, D, page]), heads padded with zeros to D.
     ``values_from_keys``: there are no value columns; a key head's values are its keys as projected, before norm and
     rotation.  Returns the queries [T, heads * D] in ``out_dtype``."""
@@ -1523,6 +1737,7 @@ def head_norm_rotate_store(proj: torch.Tensor, pos: torch.Tensor, q_weight: torc
     _i32(pos, "pos", T)
     _i32(slots, "slots", T)
     _check((q_weight is None) == (k_weight is None), "head_norm_rotate_store: queries and keys are normed together or not at all")
+    _check(not (plain_norm and (q_weight is not None or mag != 1.0)), "head_norm_rotate_store: a norm without weights has no weights, and a rotation of magnitude 1")
     if q_weight is not None:
         _f32(q_weight, "head_norm_rotate_store q weight", dim)
         _f32(k_weight, "head_norm_rotate_store k weight", dim)
@@ -1535,7 +1750,7 @@ def head_norm_rotate_store(proj: torch.Tensor, pos: torch.Tensor, q_weight: torc
     _call("tl_head_norm_rotate_store", _ptr(proj), proj.stride(0) if T > 1 else proj.shape[1], _ptr(pos), _ptr(q_weight),
           _ptr(k_weight), ctypes.c_float(eps), _ptr(freq), ctypes.c_float(mag), rot, _ptr(slots), _ptr(q), _ptr(k_cache),
           _ptr(v_cache), _code(q, "head_norm_rotate_store"), T, heads, kv_heads, dim, vdim, D, page,
-          1 if values_from_keys else 0, _stream())
+          1 if values_from_keys else 0, 1 if q_weight is not None else 2 if plain_norm else 0, 1 if halves else 0, _stream())
     return q
 
 

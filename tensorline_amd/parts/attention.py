@@ -152,7 +152,7 @@ class NormedAttention(Part):
     * ``q_temp`` = {coef, every} or None: the query at position p is multiplied by
       ``1 + coef * ln(floor((p + 1) / every) + 1)``;
     * ``sink``: one is added to the softmax's denominator, ``p_j = exp(s_j) / (1 + sum exp(s))``: a key
-      of score 0 that has no value;
+      of score 0 that has no value (the same for every head; nothing is learned);
     * ``window``: a token sees the last ``window`` keys only (0: all).
 
     Tensors under the prefix: q, k, v (with ``.b`` where ``bias``), q.norm, k.norm, o.  Projection
@@ -175,7 +175,8 @@ class NormedAttention(Part):
         self.scale, self.eps, self.window = float(scale), float(eps), int(window or 0)
         if self.scale <= 0.0:
             raise ValueError(f"{prefix}: the score scale {scale} must be positive")
-        self.qk_norm, self.sink = bool(qk_norm), bool(sink)
+        self.qk_norm = bool(qk_norm)
+        self.sink = torch.zeros(self.heads, dtype=torch.float32, device=device) if sink else None
         self.temp_coef = float(q_temp["coef"]) if q_temp else 0.0
         self.temp_every = int(q_temp["every"]) if q_temp else 0
         if q_temp and self.temp_every <= 0:

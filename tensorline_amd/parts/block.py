@@ -201,3 +201,50 @@ class SandwichBlock:
             return branch
         kernels.add_normed_branch(x, branch)
         return None
+
+
+@register_block("parallel_branches")
+class ParallelBranchesBlock:
+    """One norm ahead of both branches, which run side by side on its output and join the stream together:
+
+        h = norm1(x);  x <- x + m * (mixer(h) + ffn(h))
+
+    with the factor ``m`` = ``LayerSpec.branch_scale``; the feed-forward may be absent.  The branches' outputs are not
+    added at once: they are handed on as :class:`tensorline_amd.ops.kernels.ScaledBranches`, and the norm that reads
+    the stream next adds both in its own pass.  Where whoever runs next does not take that form
+    (``after.scaled_branches``), the block adds them itself and leaves nothing."""
+
+    def __init__(self, spec: LayerSpec, hidden_size: int, dtype, device):
+        common = dict(hidden_size=hidden_size, dtype=dtype, device=device)
+        self.spec = spec
+        self.scale = float(spec.branch_scale)
+        if spec.feed_forward_norm is not None:
+            raise ValueError(f"{spec.prefix}: both branches read the one norm: there is no norm for the feed-forward")
+        self.norm = build_part("norm", spec.mixer_norm, layer_prefix=spec.prefix, **common)
+        self.mixer = build_part("mixer", spec.mixer, layer_prefix=spec.prefix, **common)
+        self.feed_forward = None
+        if spec.feed_forward is not None:
+            self.feed_forward = build_part("feed_forward", spec.feed_forward, layer_prefix=spec.prefix, **common)
+
+    def parts(self) -> list[Part]:
+        return [p for p in (self.norm, self.mixer, self.feed_forward) if p is not None]
+
+    def cache_need(self):
+        fn = getattr(self.mixer, "cache_need", None)
+        return fn() if fn is not None else None
+
+    def state_need(self):
+        fn = getattr(self.mixer, "state_need", None)
+        return fn() if fn is not None else None
+
+    def intake(self) -> Intake:
+        return Intake(scaled_branches=bool(getattr(self.norm, "adds_scaled_branches", False)))
+
+    def forward(self, x: torch.Tensor, carry, ctx, cache, after: Intake | None = None):
+        h = self.norm.forward(x, carry)
+        y = self.mixer.forward(h, ctx, cache)
+        branches = kernels.ScaledBranches(y, self.feed_forward.forward(h, ctx) if self.feed_forward is not None else None, self.scale)
+        if after is not None and after.scaled_branches:
+            return branches
+        kernels.add_scaled_branches(x, branches)
+        return None

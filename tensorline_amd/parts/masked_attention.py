@@ -7,16 +7,21 @@ designs combine around it:
   ``c`` at or below p on, positions counted from the start of the sequence; None: all of them;
 * ``values``: "proj" (a value projection ``v`` of ``vdim`` per key head) or "keys": there is no value projection,
   a key head's values are its keys as projected (with bias), before norm and rotation;
-* ``qk_norm``: every query and key head is RMS-normed over its ``dim`` values with a weight per dimension that all
-  heads share (``q.norm``, ``k.norm`` [dim]), before rotation;
-* ``rot`` = {dims, base, scaling or None}: neighbouring pairs (2i, 2i + 1) of a head's first ``dims`` dimensions are
-  turned by ``pos * f_i``, ``f_i = base^(-2i / dims)`` (blended YaRN's way with ``scaling``); None: positions do not
-  enter the scores;
+* ``qk_norm``: True: every query and key head is RMS-normed over its ``dim`` values with a weight per dimension that
+  all heads share (``q.norm``, ``k.norm`` [dim]), before rotation; "plain": the same without weights, which is the same
+  before the rotation and after it; False: no norm;
+* ``rot`` = {dims, base, scaling or None, layout}: neighbouring pairs (2i, 2i + 1) of a head's first ``dims``
+  dimensions (``layout`` "pairs", the default) or the pairs (i, i + dims / 2) ("halves") are turned by ``pos * f_i``,
+  ``f_i = base^(-2i / dims)`` (with ``scaling`` blended YaRN's way or in Llama 3.1's bands, see
+  ``rotary.rotation_frequencies``); None: positions do not enter the scores;
+* ``softcap``: a score s becomes ``softcap * tanh(s / softcap)`` ahead of the softmax; None: it stays;
+* ``sink``: a learned number per query head (``sink`` [heads]) whose exponential joins the softmax's denominator: a key
+  without value, in sight of every token, whose logit is neither scaled nor capped;
 * ``gate``: "head": head h's output is multiplied by ``sigmoid(W_g h)_h`` (``g`` [heads, width]); "column": every
   output column by its own gate (``g`` [heads * vdim, width]); None.  The gate reads the mixer's input;
 * ``bias``: q, k (and v) carry biases (``.b``).
 
-Tensors under the prefix: q, k, (v), (g), o, (q.norm, k.norm).  One fused product gives q | k | (v) | (gate) in
+Tensors under the prefix: q, k, (v), (g), o, (q.norm, k.norm), (sink).  One fused product gives q | k | (v) | (gate) in
 float32; one kernel does everything between it and attention (norms, rotation, the cache writes); attention runs
 on the framework's paged kernels, which know the masks; the cache manager is told what may be given back while the
 request lives (the pages a window or a chunk has passed, but never those of the kept first keys).
@@ -29,7 +34,7 @@ from tensorline_amd.ops import kernels
 from tensorline_amd.parts.attention import PagedAttention
 from tensorline_amd.parts.base import Linear, Part, TensorGetter, fuse_linears
 from tensorline_amd.parts.registry import register_mixer
-from tensorline_amd.parts.rotary import yarn_frequencies
+from tensorline_amd.parts.rotary import rotation_frequencies
 from tensorline_amd.parts.spec import CacheNeed, TensorDecl, keys_and_values
 
 MASK_KINDS = ("window", "chunk")
@@ -51,8 +56,9 @@ def read_mask(prefix: str, mask: dict | None) -> tuple[int, int, int]:
 @register_mixer("masked_attention")
 class MaskedAttention(Part):
     def __init__(self, hidden_size, prefix, dtype, device, heads: int, kv_heads: int, dim: int, scale: float,
-                 vdim: int | None = None, values: str = "proj", mask: dict | None = None, qk_norm: bool = False,
-                 eps: float = 1e-6, rot: dict | None = None, gate: str | None = None, bias: bool = False):
+                 vdim: int | None = None, values: str = "proj", mask: dict | None = None, qk_norm: bool | str = False,
+                 eps: float = 1e-6, rot: dict | None = None, gate: str | None = None, bias: bool = False,
+                 softcap: float | None = None, sink: bool = False):
         super().__init__(hidden_size, prefix, dtype, device)
         self.heads, self.kv_heads, self.dim = int(heads), int(kv_heads), int(dim)
         self.vdim = self.dim if vdim is None else int(vdim)
@@ -71,13 +77,27 @@ class MaskedAttention(Part):
         if self.scale <= 0.0:
             raise ValueError(f"{prefix}: the score scale {scale} must be positive")
         self.window, self.keep_first, self.chunk = read_mask(prefix, mask)
-        self.qk_norm, self.gate = bool(qk_norm), gate
-        self.freq, self.mag = None, 1.0
+        if qk_norm not in (True, False, "plain"):
+            raise ValueError(f"{prefix}: qk_norm {qk_norm!r} must be True, False or 'plain'")
+        self.plain_norm = qk_norm == "plain"
+        self.qk_norm, self.gate = qk_norm is True, gate
+        self.softcap = float(softcap) if softcap else 0.0
+        if self.softcap < 0.0:
+            raise ValueError(f"{prefix}: the score cap {softcap} must be positive")
+        self.sink_name = prefix + "sink" if sink else None
+        self.sink: torch.Tensor | None = None
+        self.freq, self.mag, self.halves = None, 1.0, False
         if rot:
             dims = int(rot["dims"])
             if dims <= 0 or dims % 2 or dims > self.dim:
                 raise ValueError(f"{prefix}: rot.dims {dims} must be even and within the head size {self.dim}")
-            freq, self.mag = yarn_frequencies(dims, float(rot["base"]), rot.get("scaling"))
+            layout = rot.get("layout", "pairs")
+            if layout not in ("pairs", "halves"):
+                raise ValueError(f"{prefix}: rot.layout {layout!r} must be 'pairs' or 'halves'")
+            self.halves = layout == "halves"
+            freq, self.mag = rotation_frequencies(dims, float(rot["base"]), rot.get("scaling"))
+            if self.plain_norm and self.mag != 1.0:
+                raise ValueError(f"{prefix}: a norm without weights goes with a rotation that keeps lengths")
             self.freq = freq.to(device)
         mk = lambda s, n_in, n_out, b: Linear(prefix + s, n_in, n_out, b, weight_name=prefix + s, bias_name=prefix + s + ".b")
         self._projs = [mk("q", hidden_size, self.heads * self.dim, bias), mk("k", hidden_size, self.kv_heads * self.dim, bias)]
@@ -98,6 +118,8 @@ class MaskedAttention(Part):
         if self.qk_norm:
             out[self.prefix + "q.norm"] = TensorDecl((self.dim,), "one_plus_normal", 0.1, "float32")
             out[self.prefix + "k.norm"] = TensorDecl((self.dim,), "one_plus_normal", 0.1, "float32")
+        if self.sink_name:
+            out[self.sink_name] = TensorDecl((self.heads,), "normal", 1.0, "float32")
         return out
 
     def load(self, get: TensorGetter) -> None:
@@ -123,9 +145,11 @@ class MaskedAttention(Part):
         self.o_proj.prepare()
         if self.qk_norm:
             self.q_norm, self.k_norm = get(self.prefix + "q.norm"), get(self.prefix + "k.norm")
+        if self.sink_name:
+            self.sink = get(self.sink_name)
 
     def weight_tensors(self):
-        return self.qkv.tensors_kept() + self.o_proj.tensors_kept() + [t for t in (self.q_norm, self.k_norm, self.freq) if t is not None]
+        return self.qkv.tensors_kept() + self.o_proj.tensors_kept() + [t for t in (self.q_norm, self.k_norm, self.freq, self.sink) if t is not None]
 
     def library_products(self):
         return [(lin.weight, torch.float32) for lin in (self.qkv, self.o_proj) if lin.weight is not None]
@@ -145,11 +169,11 @@ class MaskedAttention(Part):
         proj = self.qkv(h, out_dtype=torch.float32)
         q = kernels.head_norm_rotate_store(proj, ctx.pos, self.q_norm, self.k_norm, self.eps, self.freq, self.mag, keys, values,
                                            cache.slots, self.heads, self.kv_heads, self.dim, self.vdim, self.values_from_keys,
-                                           self.dtype)
+                                           self.dtype, plain_norm=self.plain_norm, halves=self.halves)
         o = kernels.paged_attention(q, keys, values, cache.tables, ctx.seq_of_token, ctx.pos, self.heads, self.kv_heads,
                                     self.kernel_dim, self.scale, window=self.window, keep_first=self.keep_first,
                                     chunk=self.chunk, q_start=ctx.q_start, ctx_start=ctx.ctx_start, plan=ctx.facts,
-                                    single_seqs=ctx.extra.get("attention.single_seqs"))
+                                    single_seqs=ctx.extra.get("attention.single_seqs"), sink=self.sink, softcap=self.softcap)
         if self.gate:
             kernels.head_gate(o, proj[:, self.qkv_cols:self.qkv_cols + self.gate_cols], self.gate_cols)
         return self.o_proj(o, out_dtype=torch.float32)

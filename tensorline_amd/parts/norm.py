@@ -1,4 +1,4 @@
-"""Norms, fused with the residual add that precedes them: RMSNorm and Dynamic Tanh.
+"""Norms, fused with the residual add that precedes them: RMSNorm, layer norm and Dynamic Tanh.
 
 ``h = forward(x, residual)`` does ``x += residual`` on the float32 residual stream (in place)
 and returns ``x / sqrt(mean(x^2) + eps) * weight`` in the activation dtype.  Sum of squares,
@@ -49,6 +49,35 @@ class RMSNorm(Part):
 
     def forward(self, x: torch.Tensor, residual=None, rows: torch.Tensor | None = None) -> torch.Tensor:
         return kernels.add_rmsnorm(x, residual, self.weight, self.eps, self.dtype, rows=rows)
+
+
+@register_norm("layernorm")
+class LayerNorm(Part):
+    """``(x - mean) / sqrt(variance + eps) * weight + bias`` over the row, the variance being the mean of the squared
+    deviations.  Tensors: ``name`` (weight), ``name + ".b"``.  Same interface as the RMS norm; the residual may
+    also be :class:`tensorline_amd.ops.kernels.ScaledBranches`, added in the same pass.  It takes a mean off
+    before it divides, so no product can carry it as one factor per row: no ``deferrable``."""
+
+    def __init__(self, hidden_size, prefix, dtype, device, eps: float, name: str = "weight"):
+        super().__init__(hidden_size, prefix, dtype, device)
+        self.eps = float(eps)
+        self.name = prefix + name
+        self.weight = self.bias = None
+
+    def tensors(self):
+        return {self.name: TensorDecl((self.hidden_size,), "one_plus_normal", 0.1, "float32"),
+                self.name + ".b": TensorDecl((self.hidden_size,), "normal", 0.1, "float32")}
+
+    def load(self, get: TensorGetter) -> None:
+        self.weight, self.bias = get(self.name), get(self.name + ".b")
+
+    def weight_tensors(self):
+        return [self.weight, self.bias]
+
+    adds_scaled_branches = True    # ``forward`` takes a kernels.ScaledBranches as the residual
+
+    def forward(self, x: torch.Tensor, residual=None, rows: torch.Tensor | None = None) -> torch.Tensor:
+        return kernels.add_layernorm(x, residual, self.weight, self.bias, self.eps, self.dtype, rows=rows)
 
 
 @register_norm("dyt")

@@ -1,8 +1,9 @@
 """Mixers that keep a matrix state per head and request instead of a cache of tokens.
 
-Both run on one kernel (``kernels.linear_recurrence``): the state S [heads, key dim, value dim]
+The first ones run on one kernel (``kernels.linear_recurrence``): the state S [heads, key dim, value dim]
 lives in float32 in the request's state slot, starts at zero, and is carried from token to token
 and from step to step; a prompt portion is walked token by token in the order of the sequence.
+``ssd``, ``gated_delta`` and ``selective_scan`` take prompt portions in chunks of tokens instead.
 
 ``lightning_attention``: linear attention with a fixed decay per head.  With q = silu(W_q h), k =
 silu(W_k h), v = silu(W_v h):  S_t = decay_h S_(t-1) + k_t v_t^T,  o_t = S_t^T q_t;  the heads'
@@ -17,6 +18,8 @@ a weight and the gate silu(W_g mix_g), then projected.  The previous token's inp
 state: it sits behind S in the request's slot.
 """
 from __future__ import annotations
+
+import math
 
 import torch
 
@@ -319,3 +322,181 @@ class RealGatedLRU(Part):
         kernels.batched_linear(u.view(T, nb, bw), self.gates, g)
         o = kernels.gated_scan(g, self.bias_r, self.bias_i, u, proj[:, :W], self.lam, self.c, ctx, cache.state, 0, self.dtype)
         return self.o_proj(o, out_dtype=torch.float32)
+
+
+@register_mixer("gated_delta")
+class GatedDeltaRule(Part):
+    """The mixer of Gated DeltaNet (Yang, Kautz and Hatamizadeh, "Gated Delta Networks: Improving Mamba2 with Delta Rule").
+    Parameters: ``heads`` (value heads), ``kv_heads`` (query/key heads; value head h reads number ``h // (heads /
+    kv_heads)``), ``dim`` (query/key size), ``vdim``, ``conv`` (taps), ``eps`` of the output norm, ``unit_eps`` inside the
+    root of the unit vectors' length.  q, k and v each pass a causal convolution per channel and SiLU;  q and k are made
+    unit vectors per head, q also times ``dim^(-1/2)``;  beta = sigmoid(W_b h), g = exp(-exp(A_log) softplus(W_a h +
+    dt_bias)) per head;  S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q;  each head's o is divided by its root
+    mean square, times ``norm`` [vdim] that all heads share, times silu(W_g h), and projected.  The request's slot keeps S
+    of every head (transposed, [heads, vdim, dim]) and, behind it, the convolutions' last ``conv`` - 1 inputs.  Everything
+    between the projections and the output norm's result is float32 whatever the engine's dtype.  Tensors under the
+    prefix: q, q.conv, k, k.conv, v, v.conv, b, a, A_log, dt_bias, g, norm, o."""
+
+    def __init__(self, hidden_size, prefix, dtype, device, heads: int, kv_heads: int, dim: int, vdim: int, conv: int,
+                 eps: float = 1e-6, unit_eps: float = 1e-6):
+        super().__init__(hidden_size, prefix, dtype, device)
+        self.heads, self.kv_heads, self.dim, self.vdim = int(heads), int(kv_heads), int(dim), int(vdim)
+        self.taps, self.eps, self.unit_eps = int(conv), float(eps), float(unit_eps)
+        if min(self.heads, self.kv_heads, self.dim, self.vdim) <= 0 or self.heads % self.kv_heads:
+            raise ValueError(f"{prefix}: {heads} value heads of {vdim} do not share {kv_heads} query/key heads of {dim}")
+        if not kernels.delta_takes_key_dim(self.dim):
+            raise ValueError(f"{prefix}: a key size of {dim} per head is not served: the delta rule kernels take up to 256")
+        if not 1 <= self.taps <= kernels.CONV_MAX_TAPS:
+            raise ValueError(f"{prefix}: a convolution of {conv} taps is not served (1 to {kernels.CONV_MAX_TAPS})")
+        self.qk, self.vs = self.kv_heads * self.dim, self.heads * self.vdim
+        self.conv_channels = 2 * self.qk + self.vs
+        mk = lambda s, n_in, n_out: Linear(prefix + s, n_in, n_out, False, weight_name=prefix + s)
+        self._parts = [mk("q", hidden_size, self.qk), mk("k", hidden_size, self.qk), mk("v", hidden_size, self.vs),
+                       mk("g", hidden_size, self.vs), mk("b", hidden_size, self.heads), mk("a", hidden_size, self.heads)]
+        self.proj: Linear | None = None
+        self.o_proj = mk("o", self.vs, hidden_size)
+        self.conv_w = self.rate_log = self.dt_bias = self.norm_w = None
+
+    def tensors(self):
+        out = {}
+        for lin in self._parts + [self.o_proj]:
+            out.update(lin.tensors())
+        p = self.prefix
+        for s, n in (("q", self.qk), ("k", self.qk), ("v", self.vs)):
+            out[f"{p}{s}.conv"] = TensorDecl((n, self.taps), "normal", 0.4, "float32")
+        out[p + "A_log"] = TensorDecl((self.heads,), "normal", 1.0, "float32")
+        out[p + "dt_bias"] = TensorDecl((self.heads,), "normal", 1.0, "float32")
+        out[p + "norm"] = TensorDecl((self.vdim,), "one_plus_normal", 0.1, "float32")
+        return out
+
+    def load(self, get: TensorGetter) -> None:
+        p = self.prefix
+        for lin in self._parts + [self.o_proj]:
+            lin.load(get)
+        parts = list(self._parts)
+        spare = -sum(lin.out_features for lin in parts) % 8
+        if spare:                                  # rows of zeros at the end: the product's rows start at 16-byte borders
+            pad = Linear(p + "pad", self.hidden_size, spare, False)
+            pad.weight = parts[0].weight.new_zeros(spare, self.hidden_size)
+            parts.append(pad)
+        self.proj = fuse_linears(p + "qkvgba", parts)
+        for lin in self._parts:
+            lin.weight = None
+        self.o_proj.prepare()
+        # a tap's weights for all channels in a row
+        self.conv_w = torch.cat([get(f"{p}{s}.conv") for s in "qkv"]).t().contiguous()
+        self.rate_log, self.dt_bias = get(p + "A_log"), get(p + "dt_bias")
+        self.norm_w = get(p + "norm").repeat(self.heads).contiguous()
+
+    def weight_tensors(self):
+        return self.proj.tensors_kept() + self.o_proj.tensors_kept() + [self.conv_w, self.rate_log, self.dt_bias, self.norm_w]
+
+    def library_products(self):
+        return [(lin.weight, torch.float32) for lin in (self.proj, self.o_proj) if lin is not None and lin.weight is not None]
+
+    def cache_need(self):
+        return None
+
+    def state_need(self):
+        return StateNeed((self.vs * self.dim + (self.taps - 1) * self.conv_channels,), "float32")
+
+    step_vectors = staticmethod(kernels.chunk_vectors)
+
+    def input_linear(self) -> Linear:
+        return self.proj
+
+    def forward(self, h, ctx, cache):
+        return self.forward_projected(self.proj(h, out_dtype=torch.float32), ctx, cache)
+
+    def forward_projected(self, proj, ctx, cache):
+        """``proj`` float32 [T, q | k | v | g | b | a (| padding)]; rows may be strided."""
+        H, C, vs = self.heads, self.conv_channels, self.vs
+        qkv = kernels.conv_unit(proj[:, :C], self.conv_w, ctx, cache.state, vs * self.dim, self.dim, 2 * self.kv_heads,
+                                self.kv_heads, self.dim ** -0.5, self.unit_eps)
+        gate, b, a = proj[:, C:C + vs], proj[:, C + vs:C + vs + H], proj[:, C + vs + H:C + vs + 2 * H]
+        o = kernels.delta_rule(qkv[:, :self.qk], qkv[:, self.qk:2 * self.qk], qkv[:, 2 * self.qk:], b, a, self.rate_log,
+                               self.dt_bias, ctx, cache.state, H, self.dim, self.vdim, share=H // self.kv_heads,
+                               chunks=kernels.step_chunks(ctx))
+        y = kernels.gated_group_norm(o, self.norm_w, gate, self.vdim, self.eps, "silu", self.dtype)
+        return self.o_proj(y, out_dtype=torch.float32)
+
+
+@register_mixer("selective_scan")
+class SelectiveScan(Part):
+    """The mixer of Mamba (Gu and Dao, "Mamba: Linear-Time Sequence Modeling with Selective State Spaces").  Parameters:
+    ``inner`` (channels), ``state`` (N states per channel), ``dt_rank``, ``conv`` (taps).  W_in h = [x: inner | z: inner];  x
+    passes a causal convolution per channel (with bias) and SiLU;  W_x x = [low: dt_rank | B: N | C: N];  dt =
+    softplus(W_dt low + bias) per channel, A = -exp(A_log) [inner, N];  S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,
+    y_c = sum_n S[c, n] C_n + D_c x_c;  y * silu(z) is projected.  The request's slot keeps S ([N, inner]) and, behind it,
+    the convolution's last ``conv`` - 1 inputs.  Projections and the convolution leave x in the engine's dtype; the steps,
+    the decays, the state and the gate are float32.  Tensors under the prefix: in, conv, conv.b, x, dt, dt.b, A_log, D, o."""
+
+    def __init__(self, hidden_size, prefix, dtype, device, inner: int, state: int, dt_rank: int, conv: int):
+        super().__init__(hidden_size, prefix, dtype, device)
+        self.inner, self.N, self.rank, self.taps = int(inner), int(state), int(dt_rank), int(conv)
+        if min(self.inner, self.N, self.rank) <= 0 or self.N > kernels.SELECTIVE_SCAN_MAX_STATE:
+            raise ValueError(f"{prefix}: {inner} channels of {state} states are not served (up to {kernels.SELECTIVE_SCAN_MAX_STATE} states)")
+        if not 1 <= self.taps <= kernels.CONV_MAX_TAPS:
+            raise ValueError(f"{prefix}: a convolution of {conv} taps is not served (1 to {kernels.CONV_MAX_TAPS})")
+        mk = lambda s, n_in, n_out: Linear(prefix + s, n_in, n_out, False, weight_name=prefix + s)
+        self.proj = mk("in", hidden_size, 2 * self.inner)
+        self.x_proj = mk("x", self.inner, self.rank + 2 * self.N)
+        self.dt_proj = mk("dt", self.rank, self.inner)
+        self.o_proj = mk("o", self.inner, hidden_size)
+        self.conv_w = self.conv_b = self.dt_bias = self.a2 = self.skip = None
+
+    def _linears(self):
+        return [self.proj, self.x_proj, self.dt_proj, self.o_proj]
+
+    def tensors(self):
+        out = {}
+        for lin in self._linears():
+            out.update(lin.tensors())
+        p = self.prefix
+        out[p + "conv"] = TensorDecl((self.inner, self.taps), "normal", 0.4, "float32")
+        out[p + "conv.b"] = TensorDecl((self.inner,), "normal", 0.1, "float32")
+        out[p + "dt.b"] = TensorDecl((self.inner,), "normal", 1.0, "float32")
+        out[p + "A_log"] = TensorDecl((self.inner, self.N), "normal", 1.0, "float32")
+        out[p + "D"] = TensorDecl((self.inner,), "one_plus_normal", 0.3, "float32")
+        return out
+
+    def load(self, get: TensorGetter) -> None:
+        p = self.prefix
+        for lin in self._linears():
+            lin.load(get)
+            lin.prepare()
+        self.conv_w, self.conv_b, self.dt_bias, self.skip = get(p + "conv"), get(p + "conv.b"), get(p + "dt.b"), get(p + "D")
+        # the scan takes powers of two: A log2(e), a state's values for all channels in a row
+        self.a2 = (-torch.exp(get(p + "A_log").double()) * math.log2(math.e)).t().to(torch.float32).contiguous()
+
+    def weight_tensors(self):
+        return [t for lin in self._linears() for t in lin.tensors_kept()] + [self.conv_w, self.conv_b, self.dt_bias, self.a2, self.skip]
+
+    def library_products(self):
+        return [(lin.weight, torch.float32) for lin in self._linears() if lin.weight is not None]
+
+    def cache_need(self):
+        return None
+
+    def state_need(self):
+        return StateNeed((self.N * self.inner + (self.taps - 1) * self.inner,), "float32")
+
+    step_vectors = staticmethod(kernels.chunk_vectors)
+
+    def input_linear(self) -> Linear:
+        return self.proj
+
+    def forward(self, h, ctx, cache):
+        return self.forward_projected(self.proj(h, out_dtype=torch.float32), ctx, cache)
+
+    def forward_projected(self, proj, ctx, cache):
+        """``proj`` float32 [T, x | z]; rows may be strided."""
+        f32 = torch.float32
+        x = kernels.causal_conv(proj[:, :self.inner], self.conv_w, self.conv_b, ctx, cache.state, self.N * self.inner, act="silu",
+                                out_dtype=self.dtype)
+        low = self.x_proj(x, out_dtype=f32)
+        dt_in = low[:, :self.rank] if self.dtype == f32 else kernels.cast_rows(low[:, :self.rank], self.dtype)
+        dt = self.dt_proj(dt_in, out_dtype=f32)
+        y = kernels.selective_scan(dt, self.dt_bias, x, proj[:, self.inner:2 * self.inner], low[:, self.rank:], self.a2, self.skip,
+                                   ctx, cache.state, 0, chunks=kernels.step_chunks(ctx))
+        return self.o_proj(y, out_dtype=f32)

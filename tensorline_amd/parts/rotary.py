@@ -63,6 +63,33 @@ class NoPosition:
             kernels.rope_store(qkv, pos, None, num_heads, num_kv_heads, head_dim, k_cache, v_cache, slots, bias)
 
 
+def band_frequencies(dims: int, base: float, scaling: dict | None) -> torch.Tensor:
+    """Rotation frequencies of ``dims / 2`` pairs, stretched by wavelength bands the way Llama 3.1 does it, as
+    float32 (computed in float64 and rounded once).
+
+    f_i = base^(-2i / dims).  With ``scaling`` = {factor, low, high, original}, a wave turns n_i = original f_i /
+    (2 pi) times over ``original`` positions: waves of more than ``high`` turns keep f_i, waves of fewer than
+    ``low`` turns get f_i / factor, and in between the kept share is s = (n_i - low) / (high - low):
+    (1 - s) f_i / factor + s f_i."""
+    import math
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims)
+    if scaling:
+        factor, low, high = float(scaling["factor"]), float(scaling["low"]), float(scaling["high"])
+        turns = float(scaling["original"]) * f / (2.0 * math.pi)
+        kept = ((turns - low) / (high - low)).clamp(0.0, 1.0) if high != low else (turns > high).to(torch.float64)
+        f = (1.0 - kept) * f / factor + kept * f
+    return f.to(torch.float32)
+
+
+def rotation_frequencies(dims: int, base: float, scaling: dict | None) -> tuple[torch.Tensor, float]:
+    """(frequencies, the factor on cosine and sine) for any of the known scalings, told apart by their keys:
+    ``fast`` / ``slow``: :func:`yarn_frequencies`; ``low`` / ``high``: :func:`band_frequencies`; None: none."""
+    if scaling and "low" in scaling:
+        return band_frequencies(dims, base, scaling), 1.0
+    return yarn_frequencies(dims, base, scaling)
+
+
 def yarn_frequencies(dims: int, base: float, scaling: dict | None) -> tuple[torch.Tensor, float]:
     """Rotation frequencies of ``dims / 2`` pairs with YaRN scaling, as float32 (computed in float64
     and rounded once), and the factor that multiplies cosine and sine.

@@ -50,7 +50,8 @@ class LayerSpec:
     feed_forward_norm: PartSpec | None
     block: str = "prenorm"            # the arrangement of the parts
     token_input: PartSpec | None = None   # a per-layer input from the token ids, for blocks that take one
-    # for blocks that norm a branch's output before it joins the stream: those norms, and the factor on the normed output
+    # for blocks that norm a branch's output before it joins the stream: those norms; branch_scale is the factor on what
+    # joins the stream, for blocks that have one
     mixer_post_norm: PartSpec | None = None
     feed_forward_post_norm: PartSpec | None = None
     branch_scale: float = 1.0
@@ -71,10 +72,12 @@ class Intake:
     norm's input as ``tensorline_amd.ops.kernels.NormedRows``.  ``share_sums``: its first norm adds a
     product left in its shares of K (``tensorline_amd.ops.kernels.ShareSum``).  ``normed_branch``: its
     first norm adds a branch output that is still to be normed and scaled
-    (``tensorline_amd.ops.kernels.NormedBranch``)."""
+    (``tensorline_amd.ops.kernels.NormedBranch``).  ``scaled_branches``: its first norm adds up to two branch outputs with
+    one factor (``tensorline_amd.ops.kernels.ScaledBranches``)."""
     normed_rows_for: tuple | None = None
     share_sums: bool = False
     normed_branch: bool = False
+    scaled_branches: bool = False
 
 
 @dataclass(frozen=True)
