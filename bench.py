@@ -566,6 +566,49 @@ def make_kabulix_twin(size: str):
         rope_theta=10000.0, rms_norm_eps=1e-6, tie_word_embeddings=False, max_position_embeddings=32768))
 
 
+# ---- the Taluvik design beside the dense decoder at equal size ----------------------------------------
+# Layer sizes that resemble real models of its kinds: a delta-rule layer with key and value heads of 128, twice as many
+# value heads as query/key heads; a selective scan with an inner width of two and 16 states; chunked attention with heads
+# of 128 in groups of four, whole heads rotated, capped scores (chunks of ``--reach`` tokens, beyond the contexts measured
+# unless asked for, so that attention does the dense model's work); a GELU feed-forward of three widths beside each.  Four
+# layers (delta, scan, attention, delta), each with weights of its own.  ``dense`` has the same width, layers, vocabulary
+# and attention heads, and a SwiGLU that makes the layers' weights as many as the design's.
+TALUVIK_SIZES = {
+    "w1024": dict(width=1024, heads=8),
+    "w2048": dict(width=2048, heads=16),
+    "w4096": dict(width=4096, heads=32),
+}
+
+
+def make_taluvik_config(size: str, reach: int = 4096):
+    from tensorline_amd.config import TaluvikConfig
+    z = TALUVIK_SIZES[size]
+    W, H = z["width"], z["heads"]
+    delta = {"heads": H, "kv_heads": H // 2, "dim": 128, "vdim": 128, "conv": 4}
+    scan = {"inner": 2 * W, "state": 16, "dt_rank": W // 16, "conv": 4}
+    attention = {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+                 "mask": {"size": reach},
+                 "rot": {"dims": 128, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    ff = {"kind": "dense", "ff": 3 * W}
+    layers = [{"type": "delta", "mixer": delta, "mlp": ff}, {"type": "mamba1", "mixer": scan, "mlp": ff},
+              {"type": "attention", "mixer": attention, "mlp": ff}, {"type": "delta", "mixer": delta, "mlp": ff}]
+    return TaluvikConfig.from_dict({"architecture": "Taluvik", "vocab": HYBRID_VOCAB, "width": W, "norm": {"eps": 1e-5},
+                                    "embedding": {"scale": 1.0}, "residual_mult": 0.5, "layers": layers})
+
+
+def make_taluvik_twin(size: str):
+    from tensorline_amd.config import Qwen2Config
+    z = TALUVIK_SIZES[size]
+    W = z["width"]
+    # mixers, in squares of the width: delta 4, scan 6 + its small matrices, attention 2.5, delta 4; dense attention 2.5
+    extra = (4.0 + 6.0 + 2 * (W // 16 + 32) / W + W / 16 * 2 / W + 2.5 + 4.0) / 4 - 2.5
+    inter = int(W * (3 + extra / 3)) // 128 * 128
+    return Qwen2Config.from_dict(dict(
+        architectures=["Qwen2ForCausalLM"], vocab_size=HYBRID_VOCAB, hidden_size=W, intermediate_size=inter,
+        num_hidden_layers=4, num_attention_heads=z["heads"], num_key_value_heads=max(1, z["heads"] // 4), head_dim=128,
+        rope_theta=10000.0, rms_norm_eps=1e-6, tie_word_embeddings=False, max_position_embeddings=32768))
+
+
 def profile_step(llm, entries_of, seed: int) -> dict:
     """Event time of every kernel of one eager step, summed per entry point (milliseconds), after a
     warm-up step of the same shape."""
@@ -596,8 +639,8 @@ def profile_step(llm, entries_of, seed: int) -> dict:
 
 def bench_hybrid(args, design: str = "samovik") -> int:
     """Prefill and decode throughput of a design at real layer sizes (``samovik``: HYBRID_SIZES, ``tumitar``:
-    TUMITAR_SIZES, ``zeganex``: ZEGANEX_SIZES, ``kabulix``: KABULIX_SIZES) beside the dense decoder at equal size, and each step's time by kernel.  One JSON line;
-    the default benchmark is not run."""
+    TUMITAR_SIZES, ``zeganex``: ZEGANEX_SIZES, ``kabulix``: KABULIX_SIZES, ``taluvik``: TALUVIK_SIZES)
+    beside the dense decoder at equal size, and each step's time by kernel.  One JSON line; the default benchmark is not run."""
     import torch
     table, make, make_twin, model_text = {
         "samovik": (HYBRID_SIZES, make_hybrid_config, make_dense_twin,
@@ -612,7 +655,11 @@ def bench_hybrid(args, design: str = "samovik") -> int:
         "kabulix": (KABULIX_SIZES, (lambda size: make_kabulix_config(size, args.reach)), make_kabulix_twin,
                     "Kabulix layer sizes (4 layers: windowed attention with kept first tokens + dense, latent attention + experts, "
                     "windowed attention + experts, chunked attention + experts; windows and chunks of %d tokens) beside Qwen2 "
-                    "layers of equal width (4 layers)" % args.reach)}[design]
+                    "layers of equal width (4 layers)" % args.reach),
+        "taluvik": (TALUVIK_SIZES, (lambda size: make_taluvik_config(size, args.reach)), make_taluvik_twin,
+                    "Taluvik layer sizes (4 layers: delta rule, selective scan, chunked attention with capped scores and sinks, delta "
+                    "rule, a dense feed-forward beside each; chunks of %d tokens) beside Qwen2 layers of equal width and weights "
+                    "(4 layers)" % args.reach)}[design]
 
     from tensorline_amd import LLM
     from tensorline_amd.engine.batch import StepEntry
@@ -707,7 +754,10 @@ def main() -> int:
     ap.add_argument("--kabulix", action="store_true",
                     help="the same for the Kabulix design (windowed attention with kept first tokens, latent attention, chunked "
                          "attention, experts chosen within groups beside a gated shared expert)")
-    ap.add_argument("--reach", type=int, default=4096, help="with --kabulix: tokens of its windows and chunks")
+    ap.add_argument("--taluvik", action="store_true",
+                    help="the same for the Taluvik design (gated delta rule, selective scan, chunked attention with capped scores "
+                         "and sinks, both branches of a layer side by side)")
+    ap.add_argument("--reach", type=int, default=4096, help="with --kabulix and --taluvik: tokens of the windows and chunks")
     ap.add_argument("--hybrid-sizes", default="", help="which of w1024,w2048,w4096 (default: all)")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -723,6 +773,8 @@ def main() -> int:
         return bench_hybrid(args, "zeganex")
     if args.kabulix:
         return bench_hybrid(args, "kabulix")
+    if args.taluvik:
+        return bench_hybrid(args, "taluvik")
 
     import torch
 

@@ -373,12 +373,13 @@ def test_product_adds_into_the_residual_and_prepares_the_next_norm(M, N, Kd):
 
 def _attention_case(dtype, nq, nkv, d, bs, lens, q_lens=None, window=0, seed=0, spike=False, path=None, split_keys=None,
                     route_singles=None, pool_pages=None, spike_at=None, sink=False, spike_gain=4.0, score_shift=0.0,
-                    keep_first=0, chunk=0):
+                    keep_first=0, chunk=0, softcap=0.0):
     """Sequences of context ``lens``; the last ``q_lens[i]`` positions of each are queries.
     pool_pages: the sequences' pages are the last ones of a pool of that many.  ``spike``: the key
     at position 1 (or at ``spike_at(position of the query)``, if that is a key at all) is made to
     match its query, so that it dominates the sum if it is seen.  ``score_shift``: the first dimension of
-    every key and query is set so that it takes that much off every score."""
+    every key and query is set so that it takes that much off every score.  ``sink``: True for a logit of 0 in every head, or
+    the heads' logits; ``softcap``: scores bent by that cap."""
     torch.manual_seed(seed)
     S = len(lens)
     q_lens = q_lens or [1] * S
@@ -423,14 +424,15 @@ def _attention_case(dtype, nq, nkv, d, bs, lens, q_lens=None, window=0, seed=0, 
     plan = StepFacts(max_context=max(lens), max_query_len=max(q_lens), decode_only=max(q_lens) == 1,
                      num_seqs=S, q_lens=list(q_lens), starts=[n - ql for n, ql in zip(lens, q_lens)])
     single_seqs = None
+    logits = None if sink is False else torch.zeros(nq) if sink is True else torch.as_tensor(sink, dtype=torch.float32)
     if K().one_token_sequences(plan):
         single_seqs = torch.tensor(K().one_token_sequences(plan), dtype=torch.int32, device=DEV)
     out = K().paged_attention(q, kc, vc, tables, torch.tensor(seq_of, dtype=torch.int32, device=DEV),
                               torch.tensor(pos, dtype=torch.int32, device=DEV), nq, nkv, d, d ** -0.5, window=window,
                               q_start=torch.tensor(qs, dtype=torch.int32, device=DEV),
                               ctx_start=torch.tensor(plan.starts, dtype=torch.int32, device=DEV), plan=plan,
-                              path=path, split_keys=split_keys, single_seqs=single_seqs, route_singles=route_singles, sink=sink,
-                              keep_first=keep_first, chunk=chunk)
+                              path=path, split_keys=split_keys, single_seqs=single_seqs, route_singles=route_singles,
+                              sink=None if logits is None else logits.to(DEV), keep_first=keep_first, chunk=chunk, softcap=softcap)
     if pool_pages:
         kc, vc, tables = kc[first:], vc[first:], tables - first
     kf, vf = kc.double().cpu().view(-1, nkv, d), vc.double().cpu().permute(0, 3, 1, 2).reshape(-1, nkv, d)
@@ -441,8 +443,8 @@ def _attention_case(dtype, nq, nkv, d, bs, lens, q_lens=None, window=0, seed=0, 
         keys = torch.arange(n)
         rows = tcpu[s][keys // bs] * bs + keys % bs
         qs = q[t0:t0 + ql].double().cpu().view(ql, nq, d)
-        if keep_first or chunk:
-            want[t0:t0 + ql] = _masked_attention(qs, kf[rows], vf[rows], d ** -0.5, n - ql, window, keep_first, chunk)
+        if keep_first or chunk or softcap or (logits is not None and bool(logits.any())):
+            want[t0:t0 + ql] = _masked_attention(qs, kf[rows], vf[rows], d ** -0.5, n - ql, window, keep_first, chunk, softcap, logits)
         else:
             want[t0:t0 + ql] = plain.causal_attention(qs, kf[rows], vf[rows], d ** -0.5, window=window, q_offset=n - ql, sink=sink)
         t0 += ql
@@ -639,9 +641,10 @@ def test_attention_one_token_sequences_beside_prompt_portions(heads, d, bs):
     assert torch.equal(short[0], unrouted[0])                 # short contexts stay with the portions
 
 
-def _masked_attention(q, k, v, scale, q_offset, window, keep_first, chunk):
+def _masked_attention(q, k, v, scale, q_offset, window, keep_first, chunk, softcap=0.0, logits=None):
     """q [n, nq, d] at positions q_offset.., k and v [keys, nkv, d]: the query at position i sees key j <= i if it
-    lies in the window (i - j < window) or among the first ``keep_first`` keys, and (with ``chunk``) in i's chunk."""
+    lies in the window (i - j < window) or among the first ``keep_first`` keys, and (with ``chunk``) in i's chunk.
+    ``softcap`` bends the scores, ``logits`` [nq] are one more entry of each head's softmax, without a value."""
     n, nq, d = q.shape
     nkv = k.shape[1]
     i = (q_offset + torch.arange(n)).view(n, 1)
@@ -655,7 +658,12 @@ def _masked_attention(q, k, v, scale, q_offset, window, keep_first, chunk):
     for h in range(nq):
         g = h // (nq // nkv)
         s = (q[:, h] @ k[:, g].T) * scale
-        out[:, h] = torch.softmax(s.masked_fill(~seen, float("-inf")), dim=1) @ v[:, g]
+        if softcap:
+            s = softcap * torch.tanh(s / softcap)
+        s = s.masked_fill(~seen, float("-inf"))
+        if logits is not None:
+            s = torch.cat((s, torch.full((n, 1), float(logits[h]), dtype=torch.float64)), dim=1)
+        out[:, h] = torch.softmax(s, dim=1)[:, :k.shape[0]] @ v[:, g]
     return out
 
 
@@ -942,3 +950,33 @@ def test_attention_with_a_sink_in_every_kernel(case, gain):
     torch.testing.assert_close(got, want, atol=tol, rtol=tol)
     if gain == 0:
         assert (got - without).norm() > 0.1 * without.norm(), "the sink changed nothing where it must"
+
+
+@pytest.mark.parametrize("case", range(len(SINK_CASES)))
+@pytest.mark.parametrize("gain", [0.0, 4.0])
+def test_capped_scores_and_a_sink_per_head_in_every_kernel(case, gain):
+    """``s -> cap tanh(s / cap)``, then ``p_j = exp(s_j) / (exp(sink_h) + sum exp(s))`` with a logit of each head's own, from
+    one that vanishes to one that outweighs every key: in every kernel and through every merge.  With one key made to
+    match its query the uncapped score would be tens; capped it is not, so a cap that is left out shows."""
+    dtype, nq, nkv, d, bs, lens, q_lens, window, path, split = SINK_CASES[case]
+    logits = torch.linspace(-6.0, 9.0, nq) if nq > 1 else torch.tensor([2.0])
+    kw = dict(window=window, seed=case + 50, spike=gain > 0, path=path, split_keys=split, spike_gain=gain or 4.0, sink=logits)
+    got, want = _attention_case(dtype, nq, nkv, d, bs, lens, q_lens, softcap=2.5, **kw)
+    tol = 1e-5 if dtype == torch.float32 else 2e-2
+    torch.testing.assert_close(got, want, atol=tol, rtol=tol)
+    uncapped, want = _attention_case(dtype, nq, nkv, d, bs, lens, q_lens, softcap=0.0, **kw)
+    torch.testing.assert_close(uncapped, want, atol=tol, rtol=tol)
+    if gain:
+        assert (got - uncapped).norm() > 0.1 * uncapped.norm(), "the cap changed nothing where it must"
+
+
+@pytest.mark.parametrize("path,dtype", MASK_PATHS)
+def test_capped_scores_with_chunks_in_portions_and_one_token_steps(path, dtype):
+    logits = torch.tensor([-1.0, 3.0, 0.5, 6.0])
+    for lens, q_lens in (([160, 99, 300, 9], [60, 1, 200, 9]), ([120, 333, 64], None)):
+        if q_lens is None and path in ("mfma-tile16", "mfma-tile16x2", "mfma-tile32"):
+            continue
+        for chunk in (50, 64, 7):
+            got, want = _attention_case(dtype, 4, 2, 64, 16, lens, q_lens, seed=chunk, spike=True, path=path, chunk=chunk, spike_gain=6.0,
+                                        spike_at=lambda p: (p // chunk) * chunk, softcap=9.0, sink=logits)
+            torch.testing.assert_close(got, want, **tol(dtype, 3e-5, 2e-2))
