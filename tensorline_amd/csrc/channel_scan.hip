@@ -462,19 +462,19 @@ extern "C" int tl_conv_rotate_store(const float* proj, int ldp, const float* tap
 
 // ---- convolution and SiLU of the rows a recurrence reads, heads made unit vectors --------------------------------
 // x float [T, >= C] (row stride ldx): every channel goes through its short causal convolution (taps [K, C], a tap's weights
-// for all channels in a row, the last tap the current token's, no bias; kept inputs as in tl_causal_conv) and SiLU.  The
+// for all channels in a row, the last tap the current token's, bias [C] or none; kept inputs as in tl_causal_conv) and SiLU.  The
 // channels lie in units of `unit` (a head of queries or keys); the first n_unit units are then divided by
-// sqrt(sum of squares + eps), and the first n_scaled of those multiplied by `scale`.  out float [T, >= C].
+// sqrt(sum of squares + eps), and the first n_scaled of those multiplied by `scale`.  out float or bfloat16 [T, >= C].
 //
 // A wave takes a run of TB tokens of 64 / LPU units, LPU = 2^lpu lanes to a unit, four neighbouring channels to a lane;
 // the run's rows are asked for at once and every row is read once, the inputs of the taps before it moving along in
 // registers (KT of them, weights ahead of the first of K taps being zero).  shift != 0 (steps of one token per sequence):
 // the lane also renews what the slot keeps of its channels.
-template <int TB, int KT>
+template <int TB, int KT, typename O>
 __global__ __launch_bounds__(256) void conv_unit_kernel(
-    const float* __restrict__ x, int ldx, const float* __restrict__ taps, float* __restrict__ kept, long long state_stride,
+    const float* __restrict__ x, int ldx, const float* __restrict__ taps, const float* __restrict__ bias, float* __restrict__ kept, long long state_stride,
     const int32_t* __restrict__ state_slots, const int32_t* __restrict__ seq_of_token, const int32_t* __restrict__ q_start,
-    float* __restrict__ out, int ldo, int T, int C, int K, int unit, int n_unit, int n_scaled, float scale, float eps, int lpu,
+    O* __restrict__ out, int ldo, int T, int C, int K, int unit, int n_unit, int n_scaled, float scale, float eps, int lpu,
     int vec, int shift) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int u = ((blockIdx.y * 4 + wave) << (6 - lpu)) + (lane >> lpu);
@@ -491,17 +491,19 @@ __global__ __launch_bounds__(256) void conv_unit_kernel(
         if (live > 3) r.w = row[c0 + 3];
         return r;
     };
-    auto store = [&](float* row, float4 v) {
+    auto store = [&](auto* row, float4 v) {
+        using E = __typeof__(*row);
         if (vec && live == 4) {
-            *reinterpret_cast<float4*>(row + c0) = v;
+            crs_store4<E>(row + c0, v);
             return;
         }
-        if (live > 0) row[c0] = v.x;
-        if (live > 1) row[c0 + 1] = v.y;
-        if (live > 2) row[c0 + 2] = v.z;
-        if (live > 3) row[c0 + 3] = v.w;
+        if (live > 0) row[c0] = tl_from_float<E>(v.x);
+        if (live > 1) row[c0 + 1] = tl_from_float<E>(v.y);
+        if (live > 2) row[c0 + 2] = tl_from_float<E>(v.z);
+        if (live > 3) row[c0 + 3] = tl_from_float<E>(v.w);
     };
     float4 w[KT], hist[KT], xs[TB];
+    const float4 b4 = bias ? load(bias) : make_float4(0.f, 0.f, 0.f, 0.f);
 #pragma unroll
     for (int j = 0; j < KT; ++j)
         w[j] = j >= KT - K ? load(taps + (size_t)(j - (KT - K)) * C) : make_float4(0.f, 0.f, 0.f, 0.f);
@@ -530,7 +532,7 @@ __global__ __launch_bounds__(256) void conv_unit_kernel(
             for (int j = 0; j < KT - 1; ++j) hist[j] = hist[j + 1];
         }
         hist[KT - 1] = xs[tt];
-        float4 y = make_float4(0.f, 0.f, 0.f, 0.f);
+        float4 y = b4;
 #pragma unroll
         for (int j = 0; j < KT; ++j) {
             y.x = __builtin_fmaf(w[j].x, hist[j].x, y.x);
@@ -542,13 +544,15 @@ __global__ __launch_bounds__(256) void conv_unit_kernel(
         y.y = y.y / (1.0f + expf(-y.y));
         y.z = y.z / (1.0f + expf(-y.z));
         y.w = y.w / (1.0f + expf(-y.w));
-        // channels that do not exist are zero; the sum is formed by every lane and used by the units that are normed
-        float ss = (y.x * y.x + y.y * y.y) + (y.z * y.z + y.w * y.w);
-        for (int off = 1; off < (1 << lpu); off <<= 1) ss += __shfl_xor(ss, off, TL_WAVE);
-        if (u < n_unit) {
-            float f = 1.0f / sqrtf(ss + eps);
-            if (u < n_scaled) f *= scale;
-            y.x *= f, y.y *= f, y.z *= f, y.w *= f;
+        if (n_unit > 0) {
+            // channels that do not exist are zero (those units have no bias); every lane forms the sum of its unit
+            float ss = (y.x * y.x + y.y * y.y) + (y.z * y.z + y.w * y.w);
+            for (int off = 1; off < (1 << lpu); off <<= 1) ss += __shfl_xor(ss, off, TL_WAVE);
+            if (u < n_unit) {
+                float f = 1.0f / sqrtf(ss + eps);
+                if (u < n_scaled) f *= scale;
+                y.x *= f, y.y *= f, y.z *= f, y.w *= f;
+            }
         }
         store(out + (size_t)t * ldo, y);
         if (shift) {
@@ -560,27 +564,30 @@ __global__ __launch_bounds__(256) void conv_unit_kernel(
 }
 
 // `update` as in tl_causal_conv.  unit: at most 256 channels.
-extern "C" int tl_conv_unit(const float* x, int ldx, const float* taps, float* kept, long long state_stride,
-                            const int32_t* state_slots, const int32_t* seq_of_token, const int32_t* q_start, float* out, int ldo,
-                            int T, int S, int C, int K, int unit, int n_unit, int n_scaled, float scale, float eps, int update,
+extern "C" int tl_conv_unit(const float* x, int ldx, const float* taps, const float* bias, float* kept, long long state_stride,
+                            const int32_t* state_slots, const int32_t* seq_of_token, const int32_t* q_start, void* out, int out_dtype,
+                            int ldo, int T, int S, int C, int K, int unit, int n_unit, int n_scaled, float scale, float eps, int update,
                             hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && S >= 0 && C > 0 && K >= 1 && K <= CS_MAX_TAPS, "tl_conv_unit: bad sizes C=%d taps=%d (at most %d)", C, K, CS_MAX_TAPS);
     TL_CHECK_ARG(unit > 0 && unit <= 256 && n_unit >= 0 && (long long)n_unit * unit <= C && n_scaled >= 0 && n_scaled <= n_unit,
                  "tl_conv_unit: %d units of %d channels (at most 256) do not fit %d channels", n_unit, unit, C);
     TL_CHECK_ARG(ldx >= C && ldo >= C && state_stride >= (long long)(K - 1) * C, "tl_conv_unit: rows or the kept inputs are too short");
+    TL_CHECK_ARG(!bias || n_unit == 0, "tl_conv_unit: units that are normed have no bias");
     TL_CHECK_ARG(update != 2 || T == S, "tl_conv_unit: the one-launch form is for steps of one token per sequence");
     if (T == 0 || S == 0) return 0;
     int lpu = 0;
     while ((4 << lpu) < unit) ++lpu;                               // lanes to a unit: 2^lpu of four channels
     const int vec = (unit % 4 == 0 && C % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 && state_stride % 4 == 0 && (uintptr_t)x % 16 == 0 &&
-                     (uintptr_t)taps % 16 == 0 && (uintptr_t)kept % 16 == 0 && (uintptr_t)out % 16 == 0) ? 1 : 0;
+                     (uintptr_t)taps % 16 == 0 && (uintptr_t)bias % 16 == 0 && (uintptr_t)kept % 16 == 0 && (uintptr_t)out % 16 == 0) ? 1 : 0;
     const int units = tl_ceil_div(C, unit), per_group = 4 << (6 - lpu);
     const int shift = update == 2 ? 1 : 0, few = T <= 64;
     TL_CHECK_ARG(tl_ceil_div(units, per_group) <= 65535 && S <= 65535, "tl_conv_unit: too many channels or sequences for one launch");
-#define GO(TB, KT)                                                                                                                   \
-    hipLaunchKernelGGL((conv_unit_kernel<TB, KT>), dim3(tl_ceil_div(T, TB), tl_ceil_div(units, per_group)), dim3(256), 0, stream, x, ldx, \
-                       taps, kept, state_stride, state_slots, seq_of_token, q_start, out, ldo, T, C, K, unit, n_unit, n_scaled, scale, \
-                       eps, lpu, vec, shift)
+    TL_CHECK_ARG(out_dtype == TL_F32 || out_dtype == TL_BF16, "tl_conv_unit: unknown dtype %d", out_dtype);
+#define GO_TYPE(TB, KT, OT)                                                                                                          \
+    hipLaunchKernelGGL((conv_unit_kernel<TB, KT, OT>), dim3(tl_ceil_div(T, TB), tl_ceil_div(units, per_group)), dim3(256), 0, stream, x, \
+                       ldx, taps, bias, kept, state_stride, state_slots, seq_of_token, q_start, (OT*)out, ldo, T, C, K, unit, n_unit, \
+                       n_scaled, scale, eps, lpu, vec, shift)
+#define GO(TB, KT) do { if (out_dtype == TL_BF16) GO_TYPE(TB, KT, bf16_t); else GO_TYPE(TB, KT, float); } while (0)
     if (few) {
         if (K <= 4) GO(1, 4);
         else GO(1, CS_MAX_TAPS);
@@ -589,6 +596,7 @@ extern "C" int tl_conv_unit(const float* x, int ldx, const float* taps, float* k
         else GO(8, CS_MAX_TAPS);
     }
 #undef GO
+#undef GO_TYPE
     TL_CHECK_LAUNCH("tl_conv_unit");
     if (update == 1 && K > 1) {
         hipLaunchKernelGGL(causal_conv_keep_kernel, dim3(tl_ceil_div(C, 256), S), dim3(256), 0, stream, x, ldx, kept, state_stride,

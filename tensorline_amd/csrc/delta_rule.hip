@@ -17,10 +17,9 @@
 //
 //     is a triangular system (I + A) U = diag(beta) (V - diag(exp c) K S_0), A_ts = beta_t exp(c_t - c_s) (k_t . k_s):
 //       1. delta_prepare_kernel solves it for both right-hand sides, U_0 = (I + A)^-1 diag(beta) V and W = (I + A)^-1
-//          diag(beta exp c) K, per chunk and head, all chunks at once;
-//       2. delta_states_kernel walks the chunks of a sequence: U = U_0 - W S_0, S_L = exp(c_L) S_0 + sum_s exp(c_L - c_s)
-//          k_s u_s^T, a work-group per head and 16 value columns, leaving U and every chunk's S_0 in the workspace;
-//       3. delta_outputs_kernel: o_t = exp(c_t) S_0^T q_t + sum_(s <= t) exp(c_t - c_s) (q_t . k_s) u_s, all chunks at once.
+//          diag(beta exp c) K, and forms what else a chunk needs of its keys and queries, all chunks at once;
+//       2. delta_states_kernel walks the chunks of a sequence, a work-group per head and 16 value columns: U = U_0 - W S_0,
+//          o_t = exp(c_t) S_0^T q_t + sum_(s <= t) exp(c_t - c_s) (q_t . k_s) u_s, S_L = exp(c_L) S_0 + sum_s exp(c_L - c_s) k_s u_s^T.
 //     The sums c are double and only their differences (never positive) become float, so that a chunk of strong decays
 //     costs no digits between weak ones.  Products run on the float matrix instruction (v_mfma_f32_16x16x4_f32).
 //
@@ -191,7 +190,7 @@ __device__ __forceinline__ dr_f32x4 dr_mfma4(float4 a, float4 w, dr_f32x4 acc) {
     return acc;
 }
 
-// cs[t] = ln g_1 + .. + ln g_t for the chunk's n tokens (constant beyond), by the first wave, in both kernels that need it
+// cs[t] = ln g_1 + .. + ln g_t for the chunk's n tokens (constant beyond), by the first wave
 __device__ __forceinline__ void dr_log_decays(const float* __restrict__ a, int lda, int t0, int n, int h, float rate, float bias,
                                               double* cs) {
     const int tid = threadIdx.x;
@@ -223,108 +222,176 @@ __device__ __forceinline__ void dr_fill_keys(const float* __restrict__ kh, int l
     }
 }
 
-// Per (head, chunk): U_0 [DR_L][dv], W [DR_L][DP], the decayed keys transposed [DP][DR_L] and exp(c_L).  The system is
-// solved by forward substitution, a thread per column of the right-hand sides, its 64 unknowns in registers, a row of A
-// read from LDS by all threads at once.
+// Per (head, chunk): U_0, W [DR_L][DP], the decayed keys transposed [DP][DR_L], the outputs' matrix M_ts = exp(c_t - c_s) (q_t .
+// k_s), s <= t [DR_L][DR_L], exp(c_t) and exp(c_L).  The system is solved in blocks of 16 tokens: the diagonal blocks I + A_ii
+// are inverted by substitution (a lane per column), then X_i = (I + A_ii)^-1 (R_i - sum_(j < i) A_ij X_j) runs on the matrix
+// instruction, 16 columns of a right-hand side at a time: what it leaves in a lane is in the layout it reads its second
+// operand in, so solved blocks are used as they are.  U_0 is kept in that layout, [16 columns][16 tokens][lane][4].
 template <int DP>
 __global__ __launch_bounds__(DR_THREADS) void delta_prepare_kernel(
-    const float* __restrict__ k, int ldk, const float* __restrict__ v, int ldv, const float* __restrict__ b, int ldb,
-    const float* __restrict__ a, int lda, const float* __restrict__ rate_log, const float* __restrict__ step_bias, int share,
-    const int32_t* __restrict__ q_start, const int32_t* __restrict__ chunk_seq, const int32_t* __restrict__ chunk_row,
-    float* __restrict__ ws_u0, float* __restrict__ ws_w, float* __restrict__ ws_kt, float* __restrict__ ws_dec, int H, int dk,
-    int dv, int vec) {
-    constexpr int LDK = DP + 4;
-    extern __shared__ __attribute__((aligned(16))) float dr_smem[];
-    float* Ks = dr_smem;                         // [DR_L][LDK]
-    float* As = Ks + DR_L * LDK;                 // [DR_L][DR_LDA]: A, zeros on and above the diagonal
-    double* cs = reinterpret_cast<double*>(As + DR_L * DR_LDA);   // [DR_L]
-    float* bet = reinterpret_cast<float*>(cs + DR_L);             // [DR_L]
+    const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk, const float* __restrict__ v, int ldv,
+    const float* __restrict__ b, int ldb, const float* __restrict__ a, int lda, const float* __restrict__ rate_log,
+    const float* __restrict__ step_bias, int share, const int32_t* __restrict__ q_start, const int32_t* __restrict__ chunk_seq,
+    const int32_t* __restrict__ chunk_row, float* __restrict__ ws_u0, float* __restrict__ ws_w, float* __restrict__ ws_kt,
+    float* __restrict__ ws_m, float* __restrict__ ws_in, float* __restrict__ ws_dec, int H, int dk, int dv, int vec) {
+    constexpr int LDK = DP + 4, NB = DR_L / 16, LDI = 20;
+    __shared__ __attribute__((aligned(16))) float Ks[DR_L * LDK];
+    __shared__ __attribute__((aligned(16))) float As[DR_L * DR_LDA];      // zeros on and above the diagonal
+    __shared__ __attribute__((aligned(16))) float Ti[NB * 16 * LDI];      // the inverted diagonal blocks
+    __shared__ double cs[DR_L];
+    __shared__ float bet[DR_L], bin[DR_L];                                // beta_t, beta_t exp(c_t); zero beyond the chunk
     const int h = blockIdx.x, c = blockIdx.y, tid = threadIdx.x;
     const int t0 = chunk_row[c], n = min(DR_L, q_start[chunk_seq[c] + 1] - t0);
     const size_t at = (size_t)c * H + h;
+    const int lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
+    float4 qf[DP / 16];
+    {
+        const int tt = wave * 16 + li;
+        const float* qr = q + (size_t)(t0 + (tt < n ? tt : 0)) * ldq + (size_t)(h / share) * dk;
+#pragma unroll
+        for (int kk = 0; kk < DP / 16; ++kk)
+            qf[kk] = tt < n ? dr_load4(qr, 16 * kk + 4 * lg, dk, vec) : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
     dr_log_decays(a, lda, t0, n, h, expf(rate_log[h]), step_bias ? step_bias[h] : 0.f, cs);
-    if (tid < DR_L) bet[tid] = tid < n ? dr_sigmoid(b[(size_t)(t0 + tid) * ldb + h]) : 0.f;
+    if (tid < DR_L) {
+        const float beta = tid < n ? dr_sigmoid(b[(size_t)(t0 + tid) * ldb + h]) : 0.f;
+        const float in = expf((float)cs[tid]);
+        bet[tid] = beta;
+        bin[tid] = beta * in;
+        ws_in[at * DR_L + tid] = in;
+    }
     dr_fill_keys<DP>(k + (size_t)(h / share) * dk, ldk, t0, n, dk, vec, Ks);
     __syncthreads();
-    const int lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
     {
-        dr_f32x4 acc[DR_L / 16];
+        dr_f32x4 ka[NB], qa[NB];
 #pragma unroll
-        for (int sb = 0; sb < DR_L / 16; ++sb) acc[sb] = dr_f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int sb = 0; sb < NB; ++sb) ka[sb] = qa[sb] = dr_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int kk = 0; kk < DP / 16; ++kk) {
-            const float4 af = *reinterpret_cast<const float4*>(&Ks[(wave * 16 + li) * LDK + kk * 16 + 4 * lg]);
+            const float4 kf = *reinterpret_cast<const float4*>(&Ks[(wave * 16 + li) * LDK + kk * 16 + 4 * lg]);
 #pragma unroll
-            for (int sb = 0; sb < DR_L / 16; ++sb)
-                if (sb <= wave)
-                    acc[sb] = dr_mfma4(af, *reinterpret_cast<const float4*>(&Ks[(sb * 16 + li) * LDK + kk * 16 + 4 * lg]), acc[sb]);
+            for (int sb = 0; sb < NB; ++sb)
+                if (sb <= wave) {
+                    const float4 other = *reinterpret_cast<const float4*>(&Ks[(sb * 16 + li) * LDK + kk * 16 + 4 * lg]);
+                    ka[sb] = dr_mfma4(kf, other, ka[sb]);
+                    qa[sb] = dr_mfma4(qf[kk], other, qa[sb]);
+                }
         }
+        float* M = ws_m + at * (DR_L * DR_L);
 #pragma unroll
-        for (int sb = 0; sb < DR_L / 16; ++sb)
+        for (int sb = 0; sb < NB; ++sb)
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int t = wave * 16 + 4 * lg + e, ss = sb * 16 + li;
-                As[t * DR_LDA + ss] = ss < t ? bet[t] * expf((float)(cs[t] - cs[ss])) * acc[sb][e] : 0.f;
+                const float f = ss <= t ? expf((float)(cs[t] - cs[ss])) : 0.f;
+                As[t * DR_LDA + ss] = ss < t ? bet[t] * f * ka[sb][e] : 0.f;
+                M[t * DR_L + ss] = f * qa[sb][e];
             }
     }
     // the decayed keys, transposed, and the chunk's whole decay
     const double c_end = cs[n - 1];
-    for (int idx = tid; idx < DP * DR_L; idx += DR_THREADS) {
-        const int i = idx >> 6, tt = idx & 63;
-        ws_kt[at * (DP * DR_L) + idx] = tt < n ? expf((float)(c_end - cs[tt])) * Ks[tt * LDK + i] : 0.f;
-    }
+    const float out_of = lane < n ? expf((float)(c_end - cs[lane])) : 0.f;        // a thread's token is the same in every pass
+#pragma unroll 8
+    for (int i = wave; i < DP; i += DR_THREADS / 64) ws_kt[at * (DP * DR_L) + i * DR_L + lane] = out_of * Ks[lane * LDK + i];
     if (tid == 0) ws_dec[at] = expf((float)c_end);
     __syncthreads();
-    const int cols = dv + DP;
-    for (int col = tid; col < cols; col += DR_THREADS) {
-        float X[DR_L];
-        if (col < dv) {
-            const float* vc = v + (size_t)t0 * ldv + (size_t)h * dv + col;
+    {
+        float x[16];
 #pragma unroll
-            for (int t = 0; t < DR_L; ++t) X[t] = vc[(size_t)(t < n ? t : n - 1) * ldv];      // beyond the chunk beta is zero
+        for (int i = 0; i < 16; ++i) {
+            float sum = 0.f;
 #pragma unroll
-            for (int t = 0; t < DR_L; ++t) X[t] *= bet[t];
+            for (int m4 = 0; m4 < (i + 3) / 4; ++m4) {
+                const float4 r = *reinterpret_cast<const float4*>(&As[(wave * 16 + i) * DR_LDA + wave * 16 + 4 * m4]);
+                sum = __builtin_fmaf(r.x, x[4 * m4], sum);
+                if (4 * m4 + 1 < i) sum = __builtin_fmaf(r.y, x[4 * m4 + 1], sum);
+                if (4 * m4 + 2 < i) sum = __builtin_fmaf(r.z, x[4 * m4 + 2], sum);
+                if (4 * m4 + 3 < i) sum = __builtin_fmaf(r.w, x[4 * m4 + 3], sum);
+            }
+            x[i] = (i == li ? 1.0f : 0.f) - sum;
+            if (lg == 0) Ti[(wave * 16 + i) * LDI + li] = x[i];
+        }
+    }
+    __syncthreads();
+    float4 af[NB][NB];                                                     // A_ij below the diagonal, the inverses on it
+#pragma unroll
+    for (int i = 0; i < NB; ++i)
+#pragma unroll
+        for (int j = 0; j <= i; ++j)
+            af[i][j] = j < i ? *reinterpret_cast<const float4*>(&As[(i * 16 + li) * DR_LDA + j * 16 + 4 * lg])
+                             : *reinterpret_cast<const float4*>(&Ti[(i * 16 + li) * LDI + 4 * lg]);
+    const int vt = (dv + 15) >> 4, tiles = vt + DP / 16;
+    for (int ct = wave; ct < tiles; ct += DR_THREADS / 64) {
+        dr_f32x4 X[NB];
+        if (ct < vt) {
+            const int j = ct * 16 + li;
+            const float* vc = v + (size_t)t0 * ldv + (size_t)h * dv + (j < dv ? j : dv - 1);
+#pragma unroll
+            for (int i = 0; i < NB; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int t = 16 * i + 4 * lg + e;
+                    X[i][e] = vc[(size_t)(t < n ? t : n - 1) * ldv];       // beyond the chunk beta is zero
+                }
+#pragma unroll
+            for (int i = 0; i < NB; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) X[i][e] *= bet[16 * i + 4 * lg + e];
         } else {
 #pragma unroll
-            for (int t = 0; t < DR_L; ++t) X[t] = bet[t] * expf((float)cs[t]) * Ks[t * LDK + col - dv];
+            for (int i = 0; i < NB; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) X[i][e] = bin[16 * i + 4 * lg + e] * Ks[(16 * i + 4 * lg + e) * LDK + (ct - vt) * 16 + li];
         }
 #pragma unroll
-        for (int t = 1; t < DR_L; ++t) {
-            float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
+        for (int i = 0; i < NB; ++i) {
+            dr_f32x4 r = X[i];
+            if (i > 0) {
+                dr_f32x4 acc = dr_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int m = 0; m < (t + 3) / 4; ++m) {           // entries on and above the diagonal are zero
-                const float4 r = *reinterpret_cast<const float4*>(&As[t * DR_LDA + 4 * m]);
-                s.x = __builtin_fmaf(r.x, X[4 * m], s.x);
-                s.y = __builtin_fmaf(r.y, X[4 * m + 1], s.y);
-                s.z = __builtin_fmaf(r.z, X[4 * m + 2], s.z);
-                s.w = __builtin_fmaf(r.w, X[4 * m + 3], s.w);
+                for (int j = 0; j < i; ++j) acc = dr_mfma4(af[i][j], make_float4(X[j][0], X[j][1], X[j][2], X[j][3]), acc);
+                r -= acc;
             }
-            X[t] -= (s.x + s.y) + (s.z + s.w);
+            X[i] = dr_mfma4(af[i][i], make_float4(r[0], r[1], r[2], r[3]), dr_f32x4{0.f, 0.f, 0.f, 0.f});
         }
-        float* dst = col < dv ? ws_u0 + at * (size_t)(DR_L * dv) + col : ws_w + at * (DR_L * DP) + (col - dv);
-        const int ld = col < dv ? dv : DP;
+        if (ct < vt) {
+            float4* dst = reinterpret_cast<float4*>(ws_u0 + at * (size_t)(vt * 16 * DR_L)) + (size_t)ct * NB * 64 + lane;
 #pragma unroll
-        for (int t = 0; t < DR_L; ++t) dst[(size_t)t * ld] = X[t];
+            for (int i = 0; i < NB; ++i) dst[i * 64] = make_float4(X[i][0], X[i][1], X[i][2], X[i][3]);
+        } else {
+            float* dst = ws_w + at * (DR_L * DP) + (ct - vt) * 16 + li;
+#pragma unroll
+            for (int i = 0; i < NB; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) dst[(16 * i + 4 * lg + e) * DP] = X[i][e];
+        }
     }
 }
 
-// The chunks of a sequence in order, for one head and 16 value columns.  S lives in registers in the layout the matrix
-// instruction leaves results in, wave w holding the blocks of 16 key rows w and w + 4, and goes through LDS (as does U) in
-// the layout it reads operands in, which is the same: [block][lane group][lane] of four values.  The next chunk's operands
-// are on their way in registers while a chunk is computed.
+// The chunks of a sequence in order, for one head and 16 value columns: U = U_0 - W S, the outputs exp(c_t) S^T q_t + M U, S <-
+// exp(c_L) S + (decayed keys)^T U.  S lives in registers in the layout the matrix instruction leaves results in, wave w
+// holding the blocks of 16 key rows w and w + 4, and goes through LDS (as does U) in the layout it reads operands in, which
+// is the same: [block][lane group][lane] of four values.  Wave w has tokens 16 w .. 16 w + 15 of U and of the outputs.  A
+// step's operands are asked for as soon as the step before has used its own, into the same registers.
 template <int NK>
 __global__ __launch_bounds__(DR_THREADS) void delta_states_kernel(
-    const float* __restrict__ ws_u0, const float* __restrict__ ws_w, const float* __restrict__ ws_kt,
-    const float* __restrict__ ws_dec, float* __restrict__ ws_s, float* __restrict__ ws_ut, float* __restrict__ state,
-    long long state_stride, const int32_t* __restrict__ state_slots, const int32_t* __restrict__ seq_chunk, int H, int dk, int dv) {
+    const float* __restrict__ q, int ldq, const float* __restrict__ ws_u0, const float* __restrict__ ws_w,
+    const float* __restrict__ ws_kt, const float* __restrict__ ws_m, const float* __restrict__ ws_in,
+    const float* __restrict__ ws_dec, int share, float* __restrict__ state, long long state_stride,
+    const int32_t* __restrict__ state_slots, const int32_t* __restrict__ q_start, const int32_t* __restrict__ seq_chunk,
+    float* __restrict__ out, int ldo, int H, int dk, int dv, int vec) {
     constexpr int DP = NK * 16, NT = (NK + 3) / 4;
     __shared__ float4 Sl[NK * 64], Ul[4 * 64];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
-    const int j = blockIdx.x * 16 + li, h = blockIdx.y, s = blockIdx.z;
+    // heads vary fastest: with heads a multiple of 8, the column blocks of a head, which read the same W, keys and M, lie on one
+    // XCD and share its L2
+    const int j = blockIdx.y * 16 + li, h = blockIdx.x, s = blockIdx.z;
     const int c0 = seq_chunk[s], c1 = seq_chunk[s + 1];
     if (c1 <= c0) return;
+    const int row0 = q_start[s], row1 = q_start[s + 1], vt = (dv + 15) >> 4;
     const bool col_ok = j < dv;
     float* st = state + (size_t)state_slots[s] * state_stride + ((size_t)h * dv + (col_ok ? j : 0)) * dk;
+    const float* qh = q + (size_t)(h / share) * dk;
     dr_f32x4 S[NT];
 #pragma unroll
     for (int m = 0; m < NT; ++m) {
@@ -332,67 +399,88 @@ __global__ __launch_bounds__(DR_THREADS) void delta_states_kernel(
 #pragma unroll
         for (int e = 0; e < 4; ++e) S[m][e] = (col_ok && wave + 4 * m < NK && i + e < dk) ? st[i + e] : 0.f;
     }
-    float4 wf[NK], kf[NT][4];
-    float u0[4], dec;
-    auto fetch = [&](int c, float4 (&W)[NK], float4 (&K)[NT][4], float (&U)[4], float& D) {
-        const size_t at = (size_t)c * H + h;
-        const float* w = ws_w + at * (DR_L * DP) + (wave * 16 + li) * DP + 4 * lg;
+    float4 wf[NK], qf[NK], kf[NT][4], mf[4], u0, in;
+    float dec;
+    auto fetch_w = [&](int c) {
+        const float* w = ws_w + ((size_t)c * H + h) * (DR_L * DP) + (wave * 16 + li) * DP + 4 * lg;
 #pragma unroll
-        for (int kk = 0; kk < NK; ++kk) W[kk] = *reinterpret_cast<const float4*>(w + 16 * kk);
+        for (int kk = 0; kk < NK; ++kk) wf[kk] = *reinterpret_cast<const float4*>(w + 16 * kk);
+    };
+    auto fetch_u = [&](int c) {
+        const size_t at = (size_t)c * H + h;
+        u0 = reinterpret_cast<const float4*>(ws_u0 + at * (size_t)(vt * 16 * DR_L))[((size_t)blockIdx.y * 4 + wave) * 64 + lane];
+        in = *reinterpret_cast<const float4*>(ws_in + at * DR_L + wave * 16 + 4 * lg);
+        dec = ws_dec[at];
+    };
+    auto fetch_q = [&](int c) {
+        int t = row0 + (c - c0) * DR_L + wave * 16 + li;
+        t = t < row1 ? t : row1 - 1;                          // rows beyond the sequence are computed and not written
+        const float* qr = qh + (size_t)t * ldq;
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) qf[kk] = dr_load4(qr, 16 * kk + 4 * lg, dk, vec);
+    };
+    auto fetch_k = [&](int c) {
+        const float* kt = ws_kt + ((size_t)c * H + h) * (DP * DR_L) + 4 * lg;
 #pragma unroll
         for (int m = 0; m < NT; ++m) {
             const int it = wave + 4 * m < NK ? wave + 4 * m : NK - 1;
-            const float* kt = ws_kt + at * (DP * DR_L) + (it * 16 + li) * DR_L + 4 * lg;
 #pragma unroll
-            for (int kk = 0; kk < 4; ++kk) K[m][kk] = *reinterpret_cast<const float4*>(kt + 16 * kk);
+            for (int kk = 0; kk < 4; ++kk) kf[m][kk] = *reinterpret_cast<const float4*>(kt + (it * 16 + li) * DR_L + 16 * kk);
         }
-        const float* up = ws_u0 + at * (size_t)(DR_L * dv) + (size_t)(wave * 16 + 4 * lg) * dv + (col_ok ? j : 0);
+        const float* mm = ws_m + ((size_t)c * H + h) * (DR_L * DR_L) + (wave * 16 + li) * DR_L + 4 * lg;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) U[e] = up[(size_t)e * dv];
-        D = ws_dec[at];
+        for (int kk = 0; kk < 4; ++kk) mf[kk] = *reinterpret_cast<const float4*>(mm + 16 * kk);
     };
-    fetch(c0, wf, kf, u0, dec);
+    fetch_w(c0);
+    fetch_u(c0);
+    fetch_q(c0);
+    fetch_k(c0);
     for (int c = c0; c < c1; ++c) {
-        const size_t at = (size_t)c * H + h;
+        const int cn = c + 1 < c1 ? c + 1 : c;
 #pragma unroll
-        for (int m = 0; m < NT; ++m) {
-            const int it = wave + 4 * m;
-            if (it < NK) {
-                const float4 mine = make_float4(S[m][0], S[m][1], S[m][2], S[m][3]);
-                Sl[(it * 4 + lg) * 16 + li] = mine;
-                if (col_ok) *reinterpret_cast<float4*>(ws_s + at * (size_t)(dv * DP) + (size_t)j * DP + it * 16 + 4 * lg) = mine;
-            }
-        }
+        for (int m = 0; m < NT; ++m)
+            if (wave + 4 * m < NK) Sl[((wave + 4 * m) * 4 + lg) * 16 + li] = make_float4(S[m][0], S[m][1], S[m][2], S[m][3]);
         __syncthreads();
-        float4 wn[NK], kn[NT][4];
-        float un[4], dn;
-        fetch(c + 1 < c1 ? c + 1 : c, wn, kn, un, dn);
-        dr_f32x4 p0 = dr_f32x4{0.f, 0.f, 0.f, 0.f}, p1 = p0;
+        float4 sf[NK];
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) sf[kk] = Sl[(kk * 4 + lg) * 16 + li];
+        dr_f32x4 p0 = dr_f32x4{0.f, 0.f, 0.f, 0.f}, p1 = p0, y0 = p0, y1 = p0;
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
-            if (kk & 1) p1 = dr_mfma4(wf[kk], Sl[(kk * 4 + lg) * 16 + li], p1);
-            else p0 = dr_mfma4(wf[kk], Sl[(kk * 4 + lg) * 16 + li], p0);
+            if (kk & 1) p1 = dr_mfma4(wf[kk], sf[kk], p1);
+            else p0 = dr_mfma4(wf[kk], sf[kk], p0);
         }
-        const float4 U = make_float4(u0[0] - (p0[0] + p1[0]), u0[1] - (p0[1] + p1[1]), u0[2] - (p0[2] + p1[2]), u0[3] - (p0[3] + p1[3]));
-        Ul[(wave * 4 + lg) * 16 + li] = U;
-        if (col_ok) *reinterpret_cast<float4*>(ws_ut + at * (size_t)(dv * DR_L) + (size_t)j * DR_L + wave * 16 + 4 * lg) = U;
+        fetch_w(cn);
+        Ul[(wave * 4 + lg) * 16 + li] = make_float4(u0.x - (p0[0] + p1[0]), u0.y - (p0[1] + p1[1]), u0.z - (p0[2] + p1[2]), u0.w - (p0[3] + p1[3]));
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) {
+            if (kk & 1) y1 = dr_mfma4(qf[kk], sf[kk], y1);
+            else y0 = dr_mfma4(qf[kk], sf[kk], y0);
+        }
+        fetch_q(cn);
+        dr_f32x4 y = y0 + y1;
+        y[0] *= in.x, y[1] *= in.y, y[2] *= in.z, y[3] *= in.w;
+        const float dec_now = dec;
+        fetch_u(cn);
         __syncthreads();
+        float4 uf[4];
 #pragma unroll
-        for (int m = 0; m < NT; ++m)
-            if (wave + 4 * m < NK) {
-                S[m] *= dec;
+        for (int kk = 0; kk < 4; ++kk) uf[kk] = Ul[(kk * 4 + lg) * 16 + li];
 #pragma unroll
-                for (int kk = 0; kk < 4; ++kk) S[m] = dr_mfma4(kf[m][kk], Ul[(kk * 4 + lg) * 16 + li], S[m]);
-            }
+        for (int m = 0; m < NT; ++m) S[m] *= dec_now;
 #pragma unroll
-        for (int kk = 0; kk < NK; ++kk) wf[kk] = wn[kk];
+        for (int kk = 0; kk < 4; ++kk) {
 #pragma unroll
-        for (int m = 0; m < NT; ++m)
+            for (int m = 0; m < NT; ++m) S[m] = dr_mfma4(kf[m][kk], uf[kk], S[m]);
+            if (kk <= wave) y = dr_mfma4(mf[kk], uf[kk], y);
+        }
+        fetch_k(cn);
+        if (col_ok) {
+            const int t = row0 + (c - c0) * DR_L + wave * 16 + 4 * lg;
 #pragma unroll
-            for (int kk = 0; kk < 4; ++kk) kf[m][kk] = kn[m][kk];
-#pragma unroll
-        for (int e = 0; e < 4; ++e) u0[e] = un[e];
-        dec = dn;
+            for (int e = 0; e < 4; ++e)
+                if (t + e < row1) out[(size_t)(t + e) * ldo + (size_t)h * dv + j] = y[e];
+        }
     }
 #pragma unroll
     for (int m = 0; m < NT; ++m) {
@@ -403,110 +491,14 @@ __global__ __launch_bounds__(DR_THREADS) void delta_states_kernel(
     }
 }
 
-// Per (head, chunk): wave w owns tokens 16 w .. 16 w + 15.  The chunk's matrix exp(c_t - c_s) (q_t . k_s), s <= t, goes
-// through LDS within the wave; the entering state and U are read in operand layout straight from the workspace.
-template <int NK>
-__global__ __launch_bounds__(DR_THREADS) void delta_outputs_kernel(
-    const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk, const float* __restrict__ a, int lda,
-    const float* __restrict__ rate_log, const float* __restrict__ step_bias, int share, const int32_t* __restrict__ q_start,
-    const int32_t* __restrict__ chunk_seq, const int32_t* __restrict__ chunk_row, const float* __restrict__ ws_s,
-    const float* __restrict__ ws_ut, float* __restrict__ out, int ldo, int H, int dk, int dv, int vec) {
-    constexpr int DP = NK * 16, LDK = DP + 4;
-    extern __shared__ __attribute__((aligned(16))) float dr_smem[];
-    float* Ks = dr_smem;                         // [DR_L][LDK]
-    float* Ms = Ks + DR_L * LDK;                 // [DR_L][DR_LDA]
-    double* cs = reinterpret_cast<double*>(Ms + DR_L * DR_LDA);
-    const int h = blockIdx.x, c = blockIdx.y, tid = threadIdx.x;
-    const int t0 = chunk_row[c], n = min(DR_L, q_start[chunk_seq[c] + 1] - t0);
-    const size_t at = (size_t)c * H + h;
-    const int lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
-    float4 qf[NK];
-    {
-        const int tt = wave * 16 + li;
-        const float* qr = q + (size_t)(t0 + (tt < n ? tt : 0)) * ldq + (size_t)(h / share) * dk;
-#pragma unroll
-        for (int kk = 0; kk < NK; ++kk)
-            qf[kk] = tt < n ? dr_load4(qr, 16 * kk + 4 * lg, dk, vec) : make_float4(0.f, 0.f, 0.f, 0.f);
-    }
-    dr_log_decays(a, lda, t0, n, h, expf(rate_log[h]), step_bias ? step_bias[h] : 0.f, cs);
-    dr_fill_keys<DP>(k + (size_t)(h / share) * dk, ldk, t0, n, dk, vec, Ks);
-    __syncthreads();
-    if (wave * 16 >= n) return;                  // no barrier follows
-    {
-        dr_f32x4 acc[DR_L / 16];
-#pragma unroll
-        for (int sb = 0; sb < DR_L / 16; ++sb) acc[sb] = dr_f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int kk = 0; kk < NK; ++kk) {
-#pragma unroll
-            for (int sb = 0; sb < DR_L / 16; ++sb)
-                if (sb <= wave)
-                    acc[sb] = dr_mfma4(qf[kk], *reinterpret_cast<const float4*>(&Ks[(sb * 16 + li) * LDK + kk * 16 + 4 * lg]), acc[sb]);
-        }
-#pragma unroll
-        for (int sb = 0; sb < DR_L / 16; ++sb)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int t = wave * 16 + 4 * lg + e, ss = sb * 16 + li;
-                Ms[t * DR_LDA + ss] = ss <= t ? acc[sb][e] * expf((float)(cs[t] - cs[ss])) : 0.f;
-            }
-    }
-    // Ms rows of this wave are written and read by this wave only; LDS operations of a wave complete in order
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-    float4 mf[DR_L / 16];
-#pragma unroll
-    for (int sb = 0; sb < DR_L / 16; ++sb) mf[sb] = *reinterpret_cast<const float4*>(&Ms[(wave * 16 + li) * DR_LDA + sb * 16 + 4 * lg]);
-    const float into = expf((float)cs[wave * 16 + li]);      // the factor on the entering state, for this lane's row
-#pragma unroll
-    for (int kk = 0; kk < NK; ++kk) qf[kk].x *= into, qf[kk].y *= into, qf[kk].z *= into, qf[kk].w *= into;
-    const float* S0 = ws_s + at * (size_t)(dv * DP);          // [dv][DP]
-    const float* UT = ws_ut + at * (size_t)(dv * DR_L);       // [dv][DR_L]
-    for (int j0 = 0; j0 < dv; j0 += 32) {
-        float4 sf[2][NK], uf[2][DR_L / 16];
-#pragma unroll
-        for (int x = 0; x < 2; ++x) {
-            const int j = j0 + 16 * x + li, jc = j < dv ? j : dv - 1;
-#pragma unroll
-            for (int kk = 0; kk < NK; ++kk) sf[x][kk] = *reinterpret_cast<const float4*>(S0 + (size_t)jc * DP + 16 * kk + 4 * lg);
-#pragma unroll
-            for (int sb = 0; sb < DR_L / 16; ++sb)
-                if (sb <= wave) uf[x][sb] = *reinterpret_cast<const float4*>(UT + (size_t)jc * DR_L + 16 * sb + 4 * lg);
-        }
-        dr_f32x4 y[2];
-        y[0] = y[1] = dr_f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int kk = 0; kk < NK; ++kk)
-#pragma unroll
-            for (int x = 0; x < 2; ++x) y[x] = dr_mfma4(qf[kk], sf[x][kk], y[x]);
-#pragma unroll
-        for (int sb = 0; sb < DR_L / 16; ++sb)
-            if (sb <= wave) {
-#pragma unroll
-                for (int x = 0; x < 2; ++x) y[x] = dr_mfma4(mf[sb], uf[x][sb], y[x]);
-            }
-#pragma unroll
-        for (int x = 0; x < 2; ++x) {
-            const int j = j0 + 16 * x + li;
-            if (j >= dv) continue;
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int t = wave * 16 + 4 * lg + e;
-                if (t < n) out[(size_t)(t0 + t) * ldo + (size_t)h * dv + j] = y[x][e];
-            }
-        }
-    }
-}
-
 static int dr_padded_keys(int dk) { return dk <= 16 ? 16 : dk <= 32 ? 32 : dk <= 64 ? 64 : 128; }
 
 extern "C" int tl_delta_chunked_takes(int dk, int dv) { return dk > 0 && dk <= 128 && dv > 0 ? 1 : 0; }
 extern "C" int tl_delta_chunk_tokens() { return DR_L; }
 // floats of workspace per chunk and head
 extern "C" long long tl_delta_chunked_workspace(int dk, int dv) {
-    const long long DP = dr_padded_keys(dk);
-    return 2LL * DR_L * dv + 2LL * DR_L * DP + (long long)dv * DP + 4;
+    const long long DP = dr_padded_keys(dk), DV = (dv + 15) / 16 * 16;
+    return 2LL * DR_L * DP + DV * DR_L + DR_L * DR_L + DR_L + 4;
 }
 
 // The operands of tl_delta_walk.  chunk_seq, chunk_row [NC]: a chunk's sequence and its first row of the step (a sequence's
@@ -525,26 +517,24 @@ extern "C" int tl_delta_chunked(const float* q, int ldq, const float* k, int ldk
     if (S == 0 || NC == 0) return 0;
     TL_CHECK_ARG(ws && (uintptr_t)ws % 16 == 0 && chunk_seq && chunk_row && seq_chunk, "tl_delta_chunked: the workspace (16-byte aligned) or the chunk tables are missing");
     const int vec = ((uintptr_t)q % 16 == 0 && (uintptr_t)k % 16 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && dk % 4 == 0) ? 1 : 0;
-    const int DP = dr_padded_keys(dk);
+    const int DP = dr_padded_keys(dk), DV = (dv + 15) / 16 * 16;
     const size_t nh = (size_t)NC * H;
-    float* ws_w = ws;                            // pieces that are read in 16-byte units first
+    float* ws_w = ws;
     float* ws_kt = ws_w + nh * DR_L * DP;
-    float* ws_s = ws_kt + nh * DR_L * DP;
-    float* ws_ut = ws_s + nh * dv * DP;
-    float* ws_u0 = ws_ut + nh * dv * DR_L;
-    float* ws_dec = ws_u0 + nh * dv * DR_L;
-    const size_t lds = sizeof(float) * (DR_L * (DP + 4) + DR_L * DR_LDA + DR_L) + sizeof(double) * DR_L;
-#define GO(NK)                                                                                                                   \
-    do {                                                                                                                         \
-        hipLaunchKernelGGL(delta_prepare_kernel<16 * NK>, dim3(H, NC), dim3(DR_THREADS), lds, stream, k, ldk, v, ldv, b, ldb, a, lda, \
-                           rate_log, step_bias, share, q_start, chunk_seq, chunk_row, ws_u0, ws_w, ws_kt, ws_dec, H, dk, dv, vec); \
-        TL_CHECK_LAUNCH("tl_delta_chunked prepare");                                                                             \
-        hipLaunchKernelGGL(delta_states_kernel<NK>, dim3(tl_ceil_div(dv, 16), H, S), dim3(DR_THREADS), 0, stream, ws_u0, ws_w, ws_kt, \
-                           ws_dec, ws_s, ws_ut, state, state_stride, state_slots, seq_chunk, H, dk, dv);                          \
-        TL_CHECK_LAUNCH("tl_delta_chunked states");                                                                              \
-        hipLaunchKernelGGL(delta_outputs_kernel<NK>, dim3(H, NC), dim3(DR_THREADS), lds, stream, q, ldq, k, ldk, a, lda, rate_log,  \
-                           step_bias, share, q_start, chunk_seq, chunk_row, ws_s, ws_ut, out, ldo, H, dk, dv, vec);               \
-        TL_CHECK_LAUNCH("tl_delta_chunked outputs");                                                                             \
+    float* ws_m = ws_kt + nh * DR_L * DP;
+    float* ws_u0 = ws_m + nh * DR_L * DR_L;
+    float* ws_in = ws_u0 + nh * DV * DR_L;
+    float* ws_dec = ws_in + nh * DR_L;
+#define GO(NK)                                                                                                                     \
+    do {                                                                                                                           \
+        hipLaunchKernelGGL(delta_prepare_kernel<16 * NK>, dim3(H, NC), dim3(DR_THREADS), 0, stream, q, ldq, k, ldk, v, ldv, b, ldb, a, lda, \
+                           rate_log, step_bias, share, q_start, chunk_seq, chunk_row, ws_u0, ws_w, ws_kt, ws_m, ws_in, ws_dec, H, dk, \
+                           dv, vec);                                                                                                \
+        TL_CHECK_LAUNCH("tl_delta_chunked prepare");                                                                               \
+        hipLaunchKernelGGL(delta_states_kernel<NK>, dim3(H, tl_ceil_div(dv, 16), S), dim3(DR_THREADS), 0, stream, q, ldq, ws_u0, ws_w, \
+                           ws_kt, ws_m, ws_in, ws_dec, share, state, state_stride, state_slots, q_start, seq_chunk, out, ldo, H, dk, dv, \
+                           vec);                                                                                                    \
+        TL_CHECK_LAUNCH("tl_delta_chunked states");                                                                                \
     } while (0)
     if (DP == 16) GO(1);
     else if (DP == 32) GO(2);

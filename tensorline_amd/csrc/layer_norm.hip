@@ -3,7 +3,7 @@
 //     x[r] += mult * (y1[r] + y2[r])
 //     out[r] = (x[r] - mean) / sqrt(mean((x[r] - mean)^2) + eps) * w + b
 //
-// y1 and y2 may each be absent.  With `rows`: out only, for the sums at rows[r]; x is left as it is.  Without w:
+// y1 and y2 may each be absent, and each may come in shares (the K shares of a product, added in ascending order first).  With `rows`: out only, for the sums at rows[r]; x is left as it is.  Without w:
 // the sum only.  Everything is float; the deviations are taken from the row's own mean, never from a difference of
 // two large sums.
 #include "common.h"
@@ -19,21 +19,38 @@ __device__ __forceinline__ void ln_store4(bf16_t* p, float4 v) {
     *reinterpret_cast<uint2*>(p) = u;
 }
 
+// A branch: null, or `parts` shares of it `stride` elements apart.
+struct LnBranch {
+    const float* y;
+    int parts;
+    long long stride;
+};
+__device__ __forceinline__ float ln_branch(const LnBranch& b, size_t i) {
+    float v = b.y[i];
+    for (int p = 1; p < b.parts; ++p) v += b.y[i + p * b.stride];
+    return v;
+}
+__device__ __forceinline__ float4 ln_branch4(const LnBranch& b, size_t i) {
+    float4 v = ln_load4(b.y + i);
+    for (int p = 1; p < b.parts; ++p) {
+        const float4 e = ln_load4(b.y + i + p * b.stride);
+        v.x += e.x, v.y += e.y, v.z += e.z, v.w += e.w;
+    }
+    return v;
+}
+
 // Any row length: a thread walks its columns three times.
 template <typename O>
-__global__ __launch_bounds__(1024) void add_layernorm_kernel(float* __restrict__ x, const float* __restrict__ y1,
-                                                             const float* __restrict__ y2, float mult, const float* __restrict__ w,
+__global__ __launch_bounds__(1024) void add_layernorm_kernel(float* __restrict__ x, LnBranch b1, LnBranch b2, float mult, const float* __restrict__ w,
                                                              const float* __restrict__ b, float eps, O* __restrict__ out,
                                                              const int32_t* __restrict__ rows, int H) {
     __shared__ float red[16];
     const int r = blockIdx.x;
     const size_t src = rows ? (size_t)rows[r] : (size_t)r;
     float* xr = x + src * H;
-    const float* y1r = y1 ? y1 + src * H : nullptr;
-    const float* y2r = y2 ? y2 + src * H : nullptr;
     auto value = [&](int c) {
         float v = xr[c];
-        if (y1r) v += mult * (y2r ? y1r[c] + y2r[c] : y1r[c]);
+        if (b1.y) v += mult * (b2.y ? ln_branch(b1, src * H + c) + ln_branch(b2, src * H + c) : ln_branch(b1, src * H + c));
         return v;
     };
     float sum = 0.f;
@@ -49,15 +66,14 @@ __global__ __launch_bounds__(1024) void add_layernorm_kernel(float* __restrict__
     const float rstd = 1.0f / sqrtf(ss / (float)H + eps);
     for (int c = threadIdx.x; c < H; c += blockDim.x) {
         const float v = value(c);
-        if (!rows && y1r) xr[c] = v;
+        if (!rows && b1.y) xr[c] = v;
         if (w) out[(size_t)r * H + c] = tl_from_float<O>((v - mean) * rstd * w[c] + b[c]);
     }
 }
 
 // H a multiple of 4 and at most 16384: one pass over memory, 16-byte accesses, the row in registers meanwhile.
 template <typename O>
-__global__ __launch_bounds__(1024) void add_layernorm_vec_kernel(float* __restrict__ x, const float* __restrict__ y1,
-                                                                 const float* __restrict__ y2, float mult,
+__global__ __launch_bounds__(1024) void add_layernorm_vec_kernel(float* __restrict__ x, LnBranch b1, LnBranch b2, float mult,
                                                                  const float* __restrict__ w, const float* __restrict__ b, float eps,
                                                                  O* __restrict__ out, const int32_t* __restrict__ rows, int H) {
     __shared__ float red[16];
@@ -72,10 +88,10 @@ __global__ __launch_bounds__(1024) void add_layernorm_vec_kernel(float* __restri
         const int c4 = threadIdx.x + i * blockDim.x;
         if (c4 < n4) {
             float4 a = ln_load4(xr + 4 * c4);
-            if (y1) {
-                float4 p = ln_load4(y1 + src * H + 4 * c4);
-                if (y2) {
-                    const float4 q = ln_load4(y2 + src * H + 4 * c4);
+            if (b1.y) {
+                float4 p = ln_branch4(b1, src * H + 4 * c4);
+                if (b2.y) {
+                    const float4 q = ln_branch4(b2, src * H + 4 * c4);
                     p.x += q.x, p.y += q.y, p.z += q.z, p.w += q.w;
                 }
                 a.x += mult * p.x, a.y += mult * p.y, a.z += mult * p.z, a.w += mult * p.w;
@@ -115,21 +131,26 @@ __global__ __launch_bounds__(1024) void add_layernorm_vec_kernel(float* __restri
     }
 }
 
-// x float [n, H] (rows: [>= every row + 1, H]); y1, y2 float of x's shape or null (y2 only beside y1); w, b float [H]
+// x float [n, H] (rows: [>= every row + 1, H]); y1, y2 float of x's shape or null (y2 only beside y1), in parts1 and parts2
+// shares stride1 and stride2 elements apart; w, b float [H]
 // and out [n_rows, H] float or bfloat16, or all three null: the sum only.
-extern "C" int tl_add_layernorm(float* x, const float* y1, const float* y2, float mult, const float* w, const float* b, float eps,
+extern "C" int tl_add_layernorm(float* x, const float* y1, int parts1, long long stride1, const float* y2, int parts2,
+                                long long stride2, float mult, const float* w, const float* b, float eps,
                                 void* out, int out_dtype, const int32_t* rows, int n_rows, int H, hipStream_t stream) {
     TL_CHECK_ARG(n_rows >= 0 && H > 0 && eps >= 0.f, "tl_add_layernorm: bad sizes rows=%d H=%d", n_rows, H);
     TL_CHECK_ARG((w == nullptr) == (out == nullptr) && (w == nullptr) == (b == nullptr) && (rows == nullptr || w != nullptr),
                  "tl_add_layernorm: a norm needs weight, bias and output, and rows a norm");
     TL_CHECK_ARG(y1 || !y2, "tl_add_layernorm: a second branch without a first");
+    TL_CHECK_ARG(parts1 >= 1 && parts1 <= 64 && parts2 >= 1 && parts2 <= 64 && (parts1 == 1 || stride1 > 0) && (parts2 == 1 || stride2 > 0),
+                 "tl_add_layernorm: bad shares %d, %d", parts1, parts2);
+    const LnBranch b1{y1, parts1, stride1}, b2{y2, parts2, stride2};
     if (n_rows == 0) return 0;
-    const bool vec = H % 4 == 0 && H <= 1024 * 4 * LN_VPT;
+    const bool vec = H % 4 == 0 && H <= 1024 * 4 * LN_VPT && (parts1 == 1 || stride1 % 4 == 0) && (parts2 == 1 || stride2 % 4 == 0);
     int threads = (((vec ? H / 4 : H) + 63) / 64) * 64;
     if (threads > 1024) threads = 1024;
     if (vec && threads > 256 && n_rows >= 512) threads = H / 4 <= 256 * LN_VPT ? 256 : threads;   // many rows: several float4 per thread
     dim3 grid(n_rows), block(threads);
-#define TL_LN(KERNEL, OT) hipLaunchKernelGGL(KERNEL<OT>, grid, block, 0, stream, x, y1, y2, mult, w, b, eps, (OT*)out, rows, H)
+#define TL_LN(KERNEL, OT) hipLaunchKernelGGL(KERNEL<OT>, grid, block, 0, stream, x, b1, b2, mult, w, b, eps, (OT*)out, rows, H)
     if (out_dtype == TL_BF16) {
         if (vec) TL_LN(add_layernorm_vec_kernel, bf16_t);
         else TL_LN(add_layernorm_kernel, bf16_t);

@@ -172,12 +172,78 @@ __global__ void gated_group_norm_kernel(const float* __restrict__ o, int ldo, co
     }
 }
 
+// Groups of a multiple of four columns, up to 1024: 2^lpg lanes of a wave to a group, up to four pieces of four columns to a
+// lane, so that small groups share a wave and every access is 16 bytes.  The same sums per group whatever else runs.
+template <typename O>
+__global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(const float* __restrict__ o, int ldo, const float* __restrict__ weight,
+                                                                   const float* __restrict__ gate, int ldg, O* __restrict__ out, int N,
+                                                                   int group, float eps, int gate_act, int lpg, int groups) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int t = blockIdx.x, g = ((blockIdx.y * 4 + wave) << (6 - lpg)) + (lane >> lpg);
+    const int l = lane & ((1 << lpg) - 1), step = 4 << lpg;
+    const bool live = g < groups;
+    const float* row = o + (size_t)t * ldo + (size_t)(live ? g : 0) * group;
+    const float* grow = gate + (size_t)t * ldg + (size_t)(live ? g : 0) * group;
+    float4 v[4], z[4];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int c = 4 * l + i * step;
+        v[i] = z[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (c < group) {
+            v[i] = *reinterpret_cast<const float4*>(row + c);
+            z[i] = *reinterpret_cast<const float4*>(grow + c);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        if (gate_act == 2) {
+            v[i].x *= pw_silu(z[i].x), v[i].y *= pw_silu(z[i].y), v[i].z *= pw_silu(z[i].z), v[i].w *= pw_silu(z[i].w);
+        }
+        ss += (v[i].x * v[i].x + v[i].y * v[i].y) + (v[i].z * v[i].z + v[i].w * v[i].w);
+    }
+    for (int off = 1; off < (1 << lpg); off <<= 1) ss += __shfl_xor(ss, off, TL_WAVE);
+    const float rstd = 1.0f / sqrtf(ss / (float)group + eps);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int c = 4 * l + i * step;
+        if (!live || c >= group) continue;
+        const float4 w = *reinterpret_cast<const float4*>(weight + (size_t)g * group + c);
+        float r[4] = {v[i].x * rstd * w.x, v[i].y * rstd * w.y, v[i].z * rstd * w.z, v[i].w * rstd * w.w};
+        const float zz[4] = {z[i].x, z[i].y, z[i].z, z[i].w};
+        O* dst = out + (size_t)t * N + (size_t)g * group + c;
+        uint32_t bits[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            if (gate_act != 2) r[e] *= gate_act == 0 ? pw_sigmoid(zz[e]) : pw_silu(zz[e]);
+            bits[e] = sizeof(O) == 2 ? (uint32_t)tl_f2bf_bits(r[e]) : 0u;
+        }
+        if (sizeof(O) == 2) *reinterpret_cast<uint2*>(dst) = make_uint2(bits[0] | (bits[1] << 16), bits[2] | (bits[3] << 16));
+        else *reinterpret_cast<float4*>(dst) = make_float4(r[0], r[1], r[2], r[3]);
+    }
+}
+
 extern "C" int tl_gated_group_norm(const float* o, int ldo, const float* weight, const float* gate, int ldg, void* out,
                                    int out_dtype, int T, int N, int group, float eps, int gate_act, hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && N > 0 && group > 0 && N % group == 0 && ldo >= N && ldg >= N, "tl_gated_group_norm: bad sizes");
     if (T == 0) return 0;
     const int groups = N / group;
     TL_CHECK_ARG(groups <= 65535, "tl_gated_group_norm: %d groups are more than a launch takes", groups);
+    if (group % 4 == 0 && group <= 1024 && ldo % 4 == 0 && ldg % 4 == 0 && (uintptr_t)o % 16 == 0 && (uintptr_t)gate % 16 == 0 &&
+        (uintptr_t)weight % 16 == 0 && (uintptr_t)out % 16 == 0) {
+        int lpg = 0;
+        while (lpg < 6 && (4 << lpg) < group) ++lpg;
+        dim3 vgrid(T, tl_ceil_div(groups, 4 << (6 - lpg)));
+        if (out_dtype == TL_F32)
+            hipLaunchKernelGGL(gated_group_norm_vec_kernel<float>, vgrid, dim3(256), 0, stream, o, ldo, weight, gate, ldg, (float*)out, N,
+                               group, eps, gate_act, lpg, groups);
+        else if (out_dtype == TL_BF16)
+            hipLaunchKernelGGL(gated_group_norm_vec_kernel<bf16_t>, vgrid, dim3(256), 0, stream, o, ldo, weight, gate, ldg, (bf16_t*)out, N,
+                               group, eps, gate_act, lpg, groups);
+        else return tl_fail("tl_gated_group_norm: unknown dtype %d", out_dtype);
+        TL_CHECK_LAUNCH("tl_gated_group_norm");
+        return 0;
+    }
     dim3 grid(T, groups), block(group >= 256 ? 256 : 64 * tl_ceil_div(group, 64));
     if (out_dtype == TL_F32)
         hipLaunchKernelGGL(gated_group_norm_kernel<float>, grid, block, 0, stream, o, ldo, weight, gate, ldg, (float*)out, N, group, eps, gate_act);
@@ -637,9 +703,38 @@ __global__ void glu_kernel(const I* __restrict__ gu, O* __restrict__ out, int T,
     out[i] = tl_from_float<O>((kind == 1 ? pw_gelu_tanh(g) : g * pw_sigmoid(g)) * u);
 }
 
+// bfloat16 in and out with F a multiple of 8: 16 bytes of gate and of up per thread.  1/2 (1 + tanh(y)) is the sigmoid of
+// 2 y, so either gate is z times a sigmoid.
+__global__ __launch_bounds__(256) void glu_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __restrict__ out, int F, int kind) {
+    const int i8 = blockIdx.y * blockDim.x + threadIdx.x;
+    if (i8 * 8 >= F) return;
+    const bf16_t* row = gu + (size_t)blockIdx.x * 2 * F;
+    const uint4 gv = *reinterpret_cast<const uint4*>(row + i8 * 8);
+    const uint4 uv = *reinterpret_cast<const uint4*>(row + F + i8 * 8);
+    const uint32_t gw[4] = {gv.x, gv.y, gv.z, gv.w}, uw[4] = {uv.x, uv.y, uv.z, uv.w};
+    auto gate = [&](float z) {
+        const float y2 = kind == 1 ? 2.0f * 0.7978845608028654f * (z + 0.044715f * z * z * z) : z;
+        return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * y2));
+    };
+    uint32_t ow[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+        const float o0 = gate(__uint_as_float(gw[k] << 16)) * __uint_as_float(uw[k] << 16);
+        const float o1 = gate(__uint_as_float(gw[k] & 0xffff0000u)) * __uint_as_float(uw[k] & 0xffff0000u);
+        ow[k] = (uint32_t)tl_f2bf_bits(o0) | ((uint32_t)tl_f2bf_bits(o1) << 16);
+    }
+    *reinterpret_cast<uint4*>(out + (size_t)blockIdx.x * F + i8 * 8) = make_uint4(ow[0], ow[1], ow[2], ow[3]);
+}
+
 extern "C" int tl_glu(const void* gu, int in_dtype, void* out, int out_dtype, int T, int F, int kind, hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && F > 0 && (kind == 0 || kind == 1), "tl_glu: bad sizes or unknown activation %d", kind);
     if (T == 0) return 0;
+    if (in_dtype == TL_BF16 && out_dtype == TL_BF16 && F % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+        tl_ceil_div(F, 2048) <= 65535) {
+        hipLaunchKernelGGL(glu_bf16x8_kernel, dim3(T, tl_ceil_div(F, 2048)), dim3(256), 0, stream, (const bf16_t*)gu, (bf16_t*)out, F, kind);
+        TL_CHECK_LAUNCH("tl_glu");
+        return 0;
+    }
     dim3 grid((unsigned)(((size_t)T * F + 255) / 256)), block(256);
 #define GO(I, O) hipLaunchKernelGGL((glu_kernel<I, O>), grid, block, 0, stream, (const I*)gu, (O*)out, T, F, kind)
     if (in_dtype == TL_F32 && out_dtype == TL_F32) GO(float, float);
@@ -664,14 +759,16 @@ extern "C" int tl_glu(const void* gu, int in_dtype, void* out, int out_dtype, in
 //   * q goes to q_out [T, H*D], every head padded with zeros from d to D; k into the cache at `slot`
 //     ([pages, page, G, D], zeros from d to D); v with a page's tokens innermost ([pages, G, D, page], zeros
 //     from dv to D).  With v_from_k the values are the keys as projected: before norm and rotation.
-// A work-group per token and four heads (of queries, keys or values, in that order); a wave takes one head, a lane
-// the pairs lane and lane + 64 of it (d <= 256).  A work-group computes the token's cosines and sines once, into LDS.
+// A work-group per token and a share of the heads (of queries, keys or values, in that order); a wave takes one head at a
+// time, a lane the pairs lane and lane + 64 of it (d <= 256).  A work-group computes the token's cosines and sines once, into
+// LDS.  Steps of many tokens leave the values to a kernel of their own (n_units then ends with the keys): written a token at
+// a time they are single numbers a page apart, written for sixteen neighbouring tokens at a time they are runs.
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
     const float* __restrict__ proj, int ldp, const int32_t* __restrict__ pos, const float* __restrict__ wq,
     const float* __restrict__ wk, float eps, const float* __restrict__ freq, float mag, int rot,
     const int32_t* __restrict__ slots, T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache, int H, int G,
-    int d, int dv, int D, int page, int v_from_k, int norm, int halves) {
+    int d, int dv, int D, int page, int v_from_k, int norm, int halves, int n_units) {
     __shared__ float cs[128], sn[128];
     const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const float* row = proj + (size_t)t * ldp;
@@ -684,8 +781,7 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
     __syncthreads();
     const int slot = slots ? slots[t] : -1;
     const size_t pg = slot >= 0 ? (size_t)slot / page : 0, within = slot >= 0 ? (size_t)slot % page : 0;
-    const int units = H + G + (v_from_k ? 0 : G);
-    for (int u = blockIdx.y * 4 + wave; u < units; u += units) {       // one head per wave; written as a loop for its early exits
+    for (int u = blockIdx.y * 4 + wave; u < n_units; u += 4 * gridDim.y) {
         const bool is_q = u < H, is_k = !is_q && u < H + G;
         const int head = is_q ? u : is_k ? u - H : u - H - G;
         const int n = (is_q || is_k) ? d : dv;                   // the values the head has
@@ -745,6 +841,23 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
     }
 }
 
+// The values of sixteen neighbouring rows of the step and one head: a thread has four dimensions of one token, neighbouring
+// lanes neighbouring tokens, so that stores of a page's tokens run together ([pages, G, D, page]).
+template <typename T>
+__global__ __launch_bounds__(256) void head_values_store_kernel(const float* __restrict__ proj, int ldp, int col0, const int32_t* __restrict__ slots,
+                                                                T* __restrict__ v_cache, int n, int G, int dv, int D, int page) {
+    const int t = blockIdx.x * 16 + (threadIdx.x & 15), g = blockIdx.y;
+    if (t >= n) return;
+    const int slot = slots[t];
+    if (slot < 0) return;
+    const size_t base = ((size_t)(slot / page) * G + g) * D * page + slot % page;
+    const float* x = proj + (size_t)t * ldp + col0 + g * dv;
+    for (int c = 4 * (threadIdx.x >> 4); c < D; c += 64)
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            if (c + e < D) v_cache[base + (size_t)(c + e) * page] = tl_from_float<T>(c + e < dv ? x[c + e] : 0.f);
+}
+
 extern "C" int tl_head_norm_rotate_store(const float* proj, int ldp, const int32_t* pos, const float* wq, const float* wk,
                                          float eps, const float* freq, float mag, int rot, const int32_t* slots, void* q_out,
                                          void* k_cache, void* v_cache, int dtype, int T, int H, int G, int d, int dv, int D,
@@ -758,15 +871,25 @@ extern "C" int tl_head_norm_rotate_store(const float* proj, int ldp, const int32
     TL_CHECK_ARG(ldp >= (H + G) * d + (v_from_k ? 0 : G * dv), "tl_head_norm_rotate_store: the projection's rows are too short");
     TL_CHECK_ARG(G == 0 || (slots && k_cache && v_cache), "tl_head_norm_rotate_store: keys need their cache");
     if (T == 0) return 0;
-    dim3 grid(T, tl_ceil_div(H + G + (v_from_k ? 0 : G), 4)), block(256);
+    const bool values_apart = !v_from_k && G > 0 && G <= 65535 && T >= 64;
+    const int units = H + G + (v_from_k || values_apart ? 0 : G);
+    dim3 grid(T, tl_ceil_div(units, T >= 512 ? 16 : 4)), block(256);
     TL_CHECK_ARG(grid.y <= 65535, "tl_head_norm_rotate_store: too many heads");
 #define GO(TT)                                                                                                         \
     hipLaunchKernelGGL(head_norm_rotate_store_kernel<TT>, grid, block, 0, stream, proj, ldp, pos, wq, wk, eps, freq, mag, \
-                       rot, slots, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, H, G, d, dv, D, page, v_from_k, norm, halves)
+                       rot, slots, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, H, G, d, dv, D, page, v_from_k, norm, halves, units)
     if (dtype == TL_F32) GO(float);
     else if (dtype == TL_BF16) GO(bf16_t);
     else return tl_fail("tl_head_norm_rotate_store: unknown dtype %d", dtype);
 #undef GO
+    if (values_apart) {
+        TL_CHECK_LAUNCH("tl_head_norm_rotate_store");
+        dim3 vgrid(tl_ceil_div(T, 16), G);
+        if (dtype == TL_F32)
+            hipLaunchKernelGGL(head_values_store_kernel<float>, vgrid, block, 0, stream, proj, ldp, (H + G) * d, slots, (float*)v_cache, T, G, dv, D, page);
+        else
+            hipLaunchKernelGGL(head_values_store_kernel<bf16_t>, vgrid, block, 0, stream, proj, ldp, (H + G) * d, slots, (bf16_t*)v_cache, T, G, dv, D, page);
+    }
     TL_CHECK_LAUNCH("tl_head_norm_rotate_store");
     return 0;
 }

@@ -12,7 +12,8 @@
 //
 // Decode steps and short portions walk a sequence's tokens in one launch.  Longer portions are cut into chunks of SS_L tokens
 // from a sequence's first row of the step: a state's decay over a chunk is exp(A sum dt), so
-//   1. scan_kernel<LOCAL> gives every chunk's own contribution to the state (from zero) and its sums of dt, all chunks at once;
+//   1. scan_kernel<LOCAL> gives every chunk's own contribution to the state (from zero) and its sums of dt, all chunks at once,
+//      and leaves dt in place of dt_raw;
 //   2. scan_states_kernel walks the chunks per state and leaves what enters each of them in place of its own contribution;
 //   3. scan_kernel<OUTPUT> takes every chunk from the state that enters it; a sequence's last chunk renews its slot.
 // Tokens within a chunk are taken in order by the same instructions in every form, so results agree across cuttings within
@@ -27,7 +28,16 @@
 #define SS_MAX_STATE 256
 #define SS_THREADS 256
 
-__device__ __forceinline__ float ss_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+#define SS_LOG2E 1.4426950408889634f
+#define SS_LN2 0.6931471805599453f
+// softplus(z) = max(z, 0) + ln(1 + w), w = exp(-|z|): ln(1 + w) = ln(u) w / (u - 1) with u the float nearest 1 + w, which takes
+// out what rounding 1 + w lost; w itself where u is 1
+__device__ __forceinline__ float ss_softplus(float z) {
+    const float w = __builtin_amdgcn_exp2f(-SS_LOG2E * fabsf(z)), u = 1.0f + w, d = u - 1.0f;
+    const float l = d == 0.f ? w : SS_LN2 * __builtin_amdgcn_logf(u) * (w * __builtin_amdgcn_rcpf(d));
+    return fmaxf(z, 0.f) + l;
+}
+__device__ __forceinline__ float ss_silu(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-SS_LOG2E * z)); }
 
 enum { SS_WALK = 0, SS_LOCAL = 1, SS_OUTPUT = 2 };
 
@@ -35,7 +45,7 @@ enum { SS_WALK = 0, SS_LOCAL = 1, SS_OUTPUT = 2 };
 // = [B | C]; A2 float [N][inner].
 template <int R, int P, int MODE, typename X>
 __global__ __launch_bounds__(SS_THREADS) void scan_kernel(
-    const float* __restrict__ dt_raw, int lddt, const float* __restrict__ dt_bias, const X* __restrict__ x, int ldx,
+    float* __restrict__ dt_raw, int lddt, const float* __restrict__ dt_bias, const X* __restrict__ x, int ldx,
     const float* __restrict__ z, int ldz, const float* __restrict__ bc, int ldbc, const float* __restrict__ A2,
     const float* __restrict__ D, float* __restrict__ state, long long state_stride, const int32_t* __restrict__ state_slots,
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ chunk_seq, const int32_t* __restrict__ chunk_row,
@@ -56,7 +66,13 @@ __global__ __launch_bounds__(SS_THREADS) void scan_kernel(
         s = chunk_seq[blockIdx.y];
         t0 = chunk_row[blockIdx.y];
         t1 = q_start[s + 1];
-        if (MODE == SS_LOCAL && t1 - t0 <= SS_L) return;          // nothing follows a sequence's last chunk
+        if (MODE == SS_LOCAL && t1 - t0 <= SS_L) {                // nothing follows a sequence's last chunk: its steps only
+            if (p == 0 && ch_ok) {
+                const float bias = dt_bias ? dt_bias[ch] : 0.f;
+                for (int t = t0; t < t1; ++t) dt_raw[(size_t)t * lddt + ch] = ss_softplus(dt_raw[(size_t)t * lddt + ch] + bias);
+            }
+            return;
+        }
         if (t1 - t0 > SS_L) t1 = t0 + SS_L;
     }
     const bool last = MODE != SS_LOCAL && t1 == q_start[s + 1];
@@ -96,8 +112,11 @@ __global__ __launch_bounds__(SS_THREADS) void scan_kernel(
             for (int u = 0; u < SS_AHEAD; ++u) {
                 const int tt = ta + u, t = tb + tt;
                 if (t >= t1) break;
-                const float dt = ss_softplus(dv[u] + bias), dx = dt * xv[u];
-                if (MODE == SS_LOCAL) sum_dt += dt;
+                const float dt = MODE == SS_OUTPUT ? dv[u] : ss_softplus(dv[u] + bias), dx = dt * xv[u];
+                if (MODE == SS_LOCAL) {
+                    sum_dt += dt;
+                    if (p == 0 && ch_ok) dt_raw[(size_t)t * lddt + ch] = dt;
+                }
                 float y0 = 0.f, y1 = 0.f;
 #pragma unroll
                 for (int r4 = 0; r4 < R; r4 += 4) {
@@ -118,7 +137,7 @@ __global__ __launch_bounds__(SS_THREADS) void scan_kernel(
 #pragma unroll
                     for (int off = CW; off < 64; off <<= 1) y += __shfl_xor(y, off, TL_WAVE);
                     y = __builtin_fmaf(skip, xv[u], y);
-                    if (p == 0 && ch_ok) out[(size_t)t * ldo + ch] = tl_from_float<X>(y * (zv[u] / (1.0f + expf(-zv[u]))));
+                    if (p == 0 && ch_ok) out[(size_t)t * ldo + ch] = tl_from_float<X>(y * ss_silu(zv[u]));
                 }
             }
         }
@@ -169,7 +188,7 @@ extern "C" int tl_selective_scan_takes(int N) { return N > 0 && N <= SS_MAX_STAT
 extern "C" int tl_selective_scan_chunk_tokens() { return SS_L; }
 
 template <int MODE, typename X>
-static int ss_launch(const float* dt_raw, int lddt, const float* dt_bias, const void* x, int ldx, const float* z, int ldz,
+static int ss_launch(float* dt_raw, int lddt, const float* dt_bias, const void* x, int ldx, const float* z, int ldz,
                      const float* bc, int ldbc, const float* A2, const float* D, float* state, long long state_stride,
                      const int32_t* state_slots, const int32_t* q_start, const int32_t* chunk_seq, const int32_t* chunk_row,
                      float* ws_state, float* ws_dt, void* out, int ldo, int rows, int inner, int N, hipStream_t stream) {
@@ -188,11 +207,11 @@ static int ss_launch(const float* dt_raw, int lddt, const float* dt_bias, const 
     return 0;
 }
 
-// dt_raw, z float [T, >= inner], bc float [T, >= 2 N] = [B | C], x and out [T, >= inner] of dtype; dt_bias [inner] or null, A2
+// dt_raw (overwritten where NC > 0), z float [T, >= inner], bc float [T, >= 2 N] = [B | C], x and out [T, >= inner] of dtype; dt_bias [inner] or null, A2
 // [N, inner] = A log2 e, D [inner]; state: a request's [N, inner] at state + slot * state_stride.  NC = 0: every sequence's
 // tokens are walked in order.  Else chunk_seq, chunk_row [NC], seq_chunk [S + 1] (chunks of SS_L tokens from a sequence's
 // first row of the step on), ws_state NC * N * inner floats, ws_dt NC * inner floats.
-extern "C" int tl_selective_scan(const float* dt_raw, int lddt, const float* dt_bias, const void* x, int ldx, const float* z, int ldz,
+extern "C" int tl_selective_scan(float* dt_raw, int lddt, const float* dt_bias, const void* x, int ldx, const float* z, int ldz,
                                  const float* bc, int ldbc, const float* A2, const float* D, float* state, long long state_stride,
                                  const int32_t* state_slots, const int32_t* q_start, const int32_t* chunk_seq,
                                  const int32_t* chunk_row, const int32_t* seq_chunk, float* ws_state, float* ws_dt, void* out,

@@ -180,10 +180,10 @@ def _branch_norm_add(x, branch: NormedBranch, weight, eps, out_dtype, rows):
 @dataclass
 class ScaledBranches:
     """Residual branches that join the stream together, with one factor: stands for ``mult * (y1 + y2)`` (``y2`` may
-    be None), still to be added.  The norm that reads the stream next adds it in its own pass
-    (:func:`add_layernorm`)."""
-    y1: torch.Tensor                 # float32 [T, H]
-    y2: torch.Tensor | None
+    be None), still to be added; either may be a product left in its shares of K.  The norm that reads the stream next adds
+    it in its own pass (:func:`add_layernorm`)."""
+    y1: "torch.Tensor | ShareSum"            # float32 [T, H]
+    y2: "torch.Tensor | ShareSum | None"
     mult: float
 
 
@@ -202,13 +202,17 @@ def add_layernorm(x: torch.Tensor, residual: "torch.Tensor | ScaledBranches | No
     if residual is not None and not isinstance(residual, ScaledBranches):
         residual = ScaledBranches(residual, None, 1.0)
     y1, y2, mult = (residual.y1, residual.y2, residual.mult) if residual is not None else (None, None, 1.0)
-    _on_gpu(x, y1, y2, weight, bias, rows)
     _check(x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(), "add_layernorm: x must be contiguous float32 [T, H]")
     T, H = x.shape
+    pieces = []
     for y in (y1, y2):
-        if y is not None:
-            _check(y.dtype == torch.float32 and y.is_contiguous() and tuple(y.shape) == (T, H),
+        t = y.parts if isinstance(y, ShareSum) else y[None] if y is not None else None
+        if t is not None:
+            _check(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape[1:]) == (T, H),
                    "add_layernorm: a branch must be contiguous float32 of x's shape")
+        pieces.append((t, 1 if t is None else t.shape[0], T * H))
+    (y1, n1, st1), (y2, n2, st2) = pieces
+    _on_gpu(x, y1, y2, weight, bias, rows)
     out, n = None, T
     if weight is not None:
         _f32(weight, "add_layernorm weight", H)
@@ -217,7 +221,7 @@ def add_layernorm(x: torch.Tensor, residual: "torch.Tensor | ScaledBranches | No
             _i32(rows, "rows")
             n = rows.numel()
         out = torch.empty(n, H, dtype=out_dtype, device=x.device)
-    _call("tl_add_layernorm", _ptr(x), _ptr(y1), _ptr(y2), ctypes.c_float(mult), _ptr(weight), _ptr(bias), ctypes.c_float(eps),
+    _call("tl_add_layernorm", _ptr(x), _ptr(y1), n1, ctypes.c_longlong(st1), _ptr(y2), n2, ctypes.c_longlong(st2), ctypes.c_float(mult), _ptr(weight), _ptr(bias), ctypes.c_float(eps),
           _ptr(out), _code(out, "add_layernorm out") if out is not None else F32, _ptr(rows), n, H, _stream())
     return out
 
@@ -619,7 +623,7 @@ def swiglu_gate_up(h: torch.Tensor | NormedRows, gate_up_weight: torch.Tensor,
     """``silu(h Wg^T) * (h Wu^T)`` for a fused [2I, K] weight (gate rows first): one kernel for
     few-row bfloat16 batches (it streams the ``shuffled`` copy), product then SiLU-multiply otherwise.
     ``h`` may be :class:`NormedRows` (few-row kernel only).  ``activation`` "gelu_tanh": the tanh form of GELU
-    passes the gate instead of SiLU (in the few-row kernel's epilogue, or by a pass over the float32 product)."""
+    passes the gate instead of SiLU (in the few-row kernel's epilogue, or by a pass over the product)."""
     _check(activation in GLU_ACTIVATIONS, f"swiglu_gate_up: unknown activation {activation!r}")
     if activation != "silu":
         _check(not isinstance(h, NormedRows), "swiglu_gate_up: only SiLU rides on a product that carries a norm")
@@ -635,7 +639,7 @@ def swiglu_gate_up(h: torch.Tensor | NormedRows, gate_up_weight: torch.Tensor,
             na.act = 2
             _call("tl_gemm_skinny_swiglu", _ptr(h), _ptr(shuffled), _ptr(out), M, I, K, lda, I, ctypes.byref(na), _stream())
             return out
-        return glu(linear(h, gate_up_weight, out_dtype=torch.float32, shuffled=shuffled), activation, h.dtype)
+        return glu(linear(h, gate_up_weight, shuffled=shuffled), activation, h.dtype)
     owed = h if isinstance(h, NormedRows) else None
     if owed is not None:
         h = owed.rows
@@ -1434,12 +1438,16 @@ def _check_chunks(chunks: SequenceChunks, num_seqs: int, who: str) -> None:
 
 
 def conv_unit(x: torch.Tensor, taps: torch.Tensor, ctx, state: torch.Tensor, offset: int, unit: int, n_unit: int,
-              n_scaled: int, scale: float, eps: float = 1e-6) -> torch.Tensor:
-    """A short causal convolution per channel and SiLU, as :func:`causal_conv` without bias (``x`` float32 [T, C], ``taps``
-    float32 [K, C], a tap's weights for all channels in a row; the last K - 1 inputs at ``state[slot, offset :]``).  The
+              n_scaled: int, scale: float = 1.0, eps: float = 1e-6, bias: torch.Tensor | None = None,
+              out_dtype: torch.dtype = torch.float32) -> torch.Tensor:
+    """A short causal convolution per channel and SiLU, as :func:`causal_conv` (``x`` float32 [T, C], ``taps`` float32 [K, C], a
+    tap's weights for all channels in a row; the last K - 1 inputs at ``state[slot, offset :]``; a ``bias`` float32 [C] only
+    where no unit is normed).  The
     channels lie in units of ``unit``: the first ``n_unit`` units are then divided by ``sqrt(sum of squares + eps)``, the first
-    ``n_scaled`` of those also multiplied by ``scale``.  Returns float32 [T, C]."""
-    _on_gpu(x, taps, state)
+    ``n_scaled`` of those also multiplied by ``scale``.  Returns [T, C] in ``out_dtype``."""
+    _on_gpu(x, taps, state, bias)
+    if bias is not None:
+        _f32(bias, "conv_unit bias", x.shape[1])
     T, C = x.shape
     K = taps.shape[0]
     _check(x.dtype == torch.float32 and x.stride(1) == 1, "conv_unit: the input must be float32 [T, C]")
@@ -1447,9 +1455,9 @@ def conv_unit(x: torch.Tensor, taps: torch.Tensor, ctx, state: torch.Tensor, off
     _f32(taps, "conv_unit taps")
     _check(offset + (K - 1) * C <= state.shape[1], "conv_unit: the kept inputs do not fit the state")
     kept, stride = _state_ptr(state, offset)
-    out = torch.empty(T, C, dtype=torch.float32, device=x.device)
-    _call("tl_conv_unit", _ptr(x), x.stride(0) if T > 1 else max(C, x.stride(0)), _ptr(taps), kept, ctypes.c_longlong(stride),
-          _ptr(ctx.state_slots), _ptr(ctx.seq_of_token), _ptr(ctx.q_start), _ptr(out), C, T, ctx.num_seqs, C, K, int(unit),
+    out = torch.empty(T, C, dtype=out_dtype, device=x.device)
+    _call("tl_conv_unit", _ptr(x), x.stride(0) if T > 1 else max(C, x.stride(0)), _ptr(taps), _ptr(bias), kept, ctypes.c_longlong(stride),
+          _ptr(ctx.state_slots), _ptr(ctx.seq_of_token), _ptr(ctx.q_start), _ptr(out), _code(out, "conv_unit out"), C, T, ctx.num_seqs, C, K, int(unit),
           int(n_unit), int(n_scaled), ctypes.c_float(scale), ctypes.c_float(eps),
           2 if ctx.facts.decode_only and T == ctx.num_seqs else 1, _stream())
     return out
@@ -1507,7 +1515,8 @@ def selective_scan(dt_raw: torch.Tensor, dt_bias: torch.Tensor | None, x: torch.
     exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n``, result ``(sum_n S[c, n] C_n + skip_c x_c) * silu(z_c)`` in x's dtype.
 
     ``dt_raw``, ``z`` float32 [T, inner], ``x`` [T, inner] float32 or bfloat16, ``bc`` float32 [T, 2 N] = [B | C] (all may be column
-    blocks of wider matrices), ``a2`` float32 [N, inner] = ``A^T log2(e)``, ``skip`` float32 [inner].  S lives at ``state[slot, offset
+    blocks of wider matrices; ``dt_raw`` is used up: with ``chunks`` it holds ``dt`` afterwards), ``a2`` float32 [N, inner] = ``A^T
+    log2(e)``, ``skip`` float32 [inner].  S lives at ``state[slot, offset
     : offset + N * inner]`` as [N, inner].  With ``chunks`` the step's rows are taken in chunks, all at once."""
     _on_gpu(dt_raw, dt_bias, x, z, bc, a2, skip, state)
     T, inner = x.shape

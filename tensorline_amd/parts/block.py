@@ -209,8 +209,8 @@ class ParallelBranchesBlock:
 
         h = norm1(x);  x <- x + m * (mixer(h) + ffn(h))
 
-    with the factor ``m`` = ``LayerSpec.branch_scale``; the feed-forward may be absent.  The branches' outputs are not
-    added at once: they are handed on as :class:`tensorline_amd.ops.kernels.ScaledBranches`, and the norm that reads
+    with the factor ``m`` = ``LayerSpec.branch_scale``; the feed-forward may be absent.  A mixer or feed-forward that sets
+    ``keeps_share_sums`` may leave its last product in its shares of K.  The branches' outputs are not added at once: they are handed on as :class:`tensorline_amd.ops.kernels.ScaledBranches`, and the norm that reads
     the stream next adds both in its own pass.  Where whoever runs next does not take that form
     (``after.scaled_branches``), the block adds them itself and leaves nothing."""
 
@@ -242,8 +242,10 @@ class ParallelBranchesBlock:
 
     def forward(self, x: torch.Tensor, carry, ctx, cache, after: Intake | None = None):
         h = self.norm.forward(x, carry)
-        y = self.mixer.forward(h, ctx, cache)
-        branches = kernels.ScaledBranches(y, self.feed_forward.forward(h, ctx) if self.feed_forward is not None else None, self.scale)
+        shares = lambda part: {"keep_shares": True} if getattr(part, "keeps_share_sums", False) else {}
+        y = self.mixer.forward(h, ctx, cache, **shares(self.mixer))
+        ff = self.feed_forward
+        branches = kernels.ScaledBranches(y, ff.forward(h, ctx, **shares(ff)) if ff is not None else None, self.scale)
         if after is not None and after.scaled_branches:
             return branches
         kernels.add_scaled_branches(x, branches)

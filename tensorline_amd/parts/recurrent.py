@@ -405,10 +405,12 @@ class GatedDeltaRule(Part):
     def input_linear(self) -> Linear:
         return self.proj
 
-    def forward(self, h, ctx, cache):
-        return self.forward_projected(self.proj(h, out_dtype=torch.float32), ctx, cache)
+    keeps_share_sums = True
 
-    def forward_projected(self, proj, ctx, cache):
+    def forward(self, h, ctx, cache, keep_shares: bool = False):
+        return self.forward_projected(self.proj(h, out_dtype=torch.float32), ctx, cache, keep_shares)
+
+    def forward_projected(self, proj, ctx, cache, keep_shares: bool = False):
         """``proj`` float32 [T, q | k | v | g | b | a (| padding)]; rows may be strided."""
         H, C, vs = self.heads, self.conv_channels, self.vs
         qkv = kernels.conv_unit(proj[:, :C], self.conv_w, ctx, cache.state, vs * self.dim, self.dim, 2 * self.kv_heads,
@@ -418,7 +420,7 @@ class GatedDeltaRule(Part):
                                self.dt_bias, ctx, cache.state, H, self.dim, self.vdim, share=H // self.kv_heads,
                                chunks=kernels.step_chunks(ctx))
         y = kernels.gated_group_norm(o, self.norm_w, gate, self.vdim, self.eps, "silu", self.dtype)
-        return self.o_proj(y, out_dtype=torch.float32)
+        return self.o_proj(y, out_dtype=torch.float32, keep_shares=keep_shares)
 
 
 @register_mixer("selective_scan")
@@ -465,7 +467,8 @@ class SelectiveScan(Part):
         for lin in self._linears():
             lin.load(get)
             lin.prepare()
-        self.conv_w, self.conv_b, self.dt_bias, self.skip = get(p + "conv"), get(p + "conv.b"), get(p + "dt.b"), get(p + "D")
+        self.conv_w = get(p + "conv").t().contiguous()              # a tap's weights for all channels in a row
+        self.conv_b, self.dt_bias, self.skip = get(p + "conv.b"), get(p + "dt.b"), get(p + "D")
         # the scan takes powers of two: A log2(e), a state's values for all channels in a row
         self.a2 = (-torch.exp(get(p + "A_log").double()) * math.log2(math.e)).t().to(torch.float32).contiguous()
 
@@ -486,17 +489,19 @@ class SelectiveScan(Part):
     def input_linear(self) -> Linear:
         return self.proj
 
-    def forward(self, h, ctx, cache):
-        return self.forward_projected(self.proj(h, out_dtype=torch.float32), ctx, cache)
+    keeps_share_sums = True
 
-    def forward_projected(self, proj, ctx, cache):
+    def forward(self, h, ctx, cache, keep_shares: bool = False):
+        return self.forward_projected(self.proj(h, out_dtype=torch.float32), ctx, cache, keep_shares)
+
+    def forward_projected(self, proj, ctx, cache, keep_shares: bool = False):
         """``proj`` float32 [T, x | z]; rows may be strided."""
         f32 = torch.float32
-        x = kernels.causal_conv(proj[:, :self.inner], self.conv_w, self.conv_b, ctx, cache.state, self.N * self.inner, act="silu",
-                                out_dtype=self.dtype)
+        x = kernels.conv_unit(proj[:, :self.inner], self.conv_w, ctx, cache.state, self.N * self.inner, 256, 0, 0, bias=self.conv_b,
+                              out_dtype=self.dtype)
         low = self.x_proj(x, out_dtype=f32)
         dt_in = low[:, :self.rank] if self.dtype == f32 else kernels.cast_rows(low[:, :self.rank], self.dtype)
         dt = self.dt_proj(dt_in, out_dtype=f32)
         y = kernels.selective_scan(dt, self.dt_bias, x, proj[:, self.inner:2 * self.inner], low[:, self.rank:], self.a2, self.skip,
                                    ctx, cache.state, 0, chunks=kernels.step_chunks(ctx))
-        return self.o_proj(y, out_dtype=f32)
+        return self.o_proj(y, out_dtype=f32, keep_shares=keep_shares)

@@ -97,7 +97,9 @@ def test_branches_join_the_stream_and_the_layer_norm_reads_it(H, dtype):
     w, b = torch.randn(H), torch.randn(H)
     tol = dict(atol=2e-5, rtol=2e-5) if dtype == torch.float32 else dict(atol=3e-2, rtol=1e-2)
     for branches, total in ((None, x.double()), (kernels.ScaledBranches(y1.to(DEV), y2.to(DEV), 0.35), x.double() + 0.35 * (y1.double() + y2.double())),
-                            (kernels.ScaledBranches(y1.to(DEV), None, -2.0), x.double() - 2.0 * y1.double()), (y1.to(DEV), x.double() + y1.double())):
+                            (kernels.ScaledBranches(y1.to(DEV), None, -2.0), x.double() - 2.0 * y1.double()), (y1.to(DEV), x.double() + y1.double()),
+                            (kernels.ScaledBranches(kernels.ShareSum(torch.stack((y1, y2, x)).to(DEV)), kernels.ShareSum(torch.stack((y2, y2)).to(DEV)), 0.5),
+                             x.double() * 1.5 + 0.5 * y1.double() + 1.5 * y2.double())):
         got_x = x.to(DEV).clone()
         got = kernels.add_layernorm(got_x, branches, w.to(DEV), b.to(DEV), 1e-5, dtype)
         torch.testing.assert_close(got_x.double().cpu(), total, atol=1e-5, rtol=1e-5)
@@ -190,6 +192,29 @@ def test_convolution_into_unit_vectors(case, lens):
         heads[:, :n_scaled] *= 0.3
         want[:, :unit * n_unit] = heads.reshape(-1, unit * n_unit)
         torch.testing.assert_close(torch.cat((outs[0][i], outs[1][i])), want, atol=2e-6, rtol=1e-5)
+
+
+@pytest.mark.parametrize("C,taps", [(88, 4), (50, 6), (300, 1), (1024, 3), (7, 16)])
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_convolution_with_bias_and_without_units(C, taps, dtype):
+    from tensorline_amd.ops import kernels
+    torch.manual_seed(C)
+    wt, bias = torch.randn(C, taps), torch.randn(C)
+    lens = [70, 1, 33]
+    xs = [torch.randn(n + 2, C) for n in lens]
+    state = torch.zeros(4, (taps - 1) * C, device=DEV)
+    outs = [[], [], []]
+    for ls, lo in ((lens, 0), ([2, 2, 2], None), ):
+        step = _Step(ls, False)
+        flat = torch.cat([x[:n] if lo == 0 else x[n:] for x, n in zip(xs, lens)]).to(DEV)
+        out = kernels.conv_unit(flat, wt.t().contiguous().to(DEV), step, state, 0, 256, 0, 0, bias=bias.to(DEV), out_dtype=dtype).double().cpu()
+        at = 0
+        for i, n in enumerate(ls):
+            outs[i].append(out[at:at + n])
+            at += n
+    for i, x in enumerate(xs):
+        want = P.silu(P.causal_conv(x.double(), wt.double(), bias.double()))
+        torch.testing.assert_close(torch.cat(outs[i]), want, **(dict(atol=1e-5, rtol=1e-5) if dtype == torch.float32 else dict(atol=2e-2, rtol=1e-2)))
 
 
 def _plain_delta(q, k, v, b, a, rate_log, bias, S):
