@@ -190,6 +190,19 @@ __device__ __forceinline__ dr_f32x4 dr_mfma4(float4 a, float4 w, dr_f32x4 acc) {
     return acc;
 }
 
+// one of those four products; independent ones are issued in turn (a dependent one waits half as long again)
+template <int E>
+__device__ __forceinline__ dr_f32x4 dr_mfma1(float4 a, float4 w, dr_f32x4 acc) {
+    return __builtin_amdgcn_mfma_f32_16x16x4f32(E == 0 ? a.x : E == 1 ? a.y : E == 2 ? a.z : a.w,
+                                                E == 0 ? w.x : E == 1 ? w.y : E == 2 ? w.z : w.w, acc, 0, 0, 0);
+}
+template <bool V>
+struct DrFlag {
+    static constexpr bool value = V;
+};
+#define DR_EACH4(STEP) STEP(0) STEP(1) STEP(2) STEP(3)
+__device__ __forceinline__ float4 dr_f4(dr_f32x4 v) { return make_float4(v[0], v[1], v[2], v[3]); }
+
 // cs[t] = ln g_1 + .. + ln g_t for the chunk's n tokens (constant beyond), by the first wave
 __device__ __forceinline__ void dr_log_decays(const float* __restrict__ a, int lda, int t0, int n, int h, float rate, float bias,
                                               double* cs) {
@@ -205,62 +218,96 @@ __device__ __forceinline__ void dr_log_decays(const float* __restrict__ a, int l
     }
 }
 
-// A head's keys of the chunk into LDS rows of DP + 4 floats, zeros beyond the chunk's tokens and the head's dk.
+// A head's queries or keys of the chunk: from memory into registers, zeros beyond the chunk's tokens and the head's dk, and
+// from there into LDS rows of DP + 4 floats.
 template <int DP>
-__device__ __forceinline__ void dr_fill_keys(const float* __restrict__ kh, int ldk, int t0, int n, int dk, int vec, float* Ks) {
-    constexpr int PER = DR_L * DP / 4 / DR_THREADS;         // 1, 2, 4 or 8 pieces of four values per thread
+struct DrTile {
+    static constexpr int PER = DR_L * DP / 4 / DR_THREADS;   // 1, 2, 4 or 8 pieces of four values per thread
     float4 r[PER];
+    __device__ __forceinline__ void load(const float* __restrict__ src, int ld, int t0, int n, int dk, int vec) {
 #pragma unroll
-    for (int u = 0; u < PER; ++u) {
-        const int idx = threadIdx.x + u * DR_THREADS, tt = idx / (DP / 4), i = 4 * (idx % (DP / 4));
-        r[u] = tt < n ? dr_load4(kh + (size_t)(t0 + tt) * ldk, i, dk, vec) : make_float4(0.f, 0.f, 0.f, 0.f);
+        for (int u = 0; u < PER; ++u) {
+            const int idx = threadIdx.x + u * DR_THREADS, tt = idx / (DP / 4), i = 4 * (idx % (DP / 4));
+            r[u] = tt < n ? dr_load4(src + (size_t)(t0 + tt) * ld, i, dk, vec) : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
     }
+    __device__ __forceinline__ void stash(float* rows) const {
 #pragma unroll
-    for (int u = 0; u < PER; ++u) {
-        const int idx = threadIdx.x + u * DR_THREADS, tt = idx / (DP / 4), i = 4 * (idx % (DP / 4));
-        *reinterpret_cast<float4*>(&Ks[tt * (DP + 4) + i]) = r[u];
+        for (int u = 0; u < PER; ++u) {
+            const int idx = threadIdx.x + u * DR_THREADS, tt = idx / (DP / 4), i = 4 * (idx % (DP / 4));
+            *reinterpret_cast<float4*>(&rows[tt * (DP + 4) + i]) = r[u];
+        }
     }
-}
+};
 
-// Per (head, chunk): U_0, W [DR_L][DP], the decayed keys transposed [DP][DR_L], the outputs' matrix M_ts = exp(c_t - c_s) (q_t .
-// k_s), s <= t [DR_L][DR_L], exp(c_t) and exp(c_L).  The system is solved in blocks of 16 tokens: the diagonal blocks I + A_ii
-// are inverted by substitution (a lane per column), then X_i = (I + A_ii)^-1 (R_i - sum_(j < i) A_ij X_j) runs on the matrix
-// instruction, 16 columns of a right-hand side at a time: what it leaves in a lane is in the layout it reads its second
-// operand in, so solved blocks are used as they are.  U_0 is kept in that layout, [16 columns][16 tokens][lane][4].
+// Per (head, chunk): U_0, W, the decayed keys transposed, the queries times exp(c_t), the outputs' matrix M_ts = exp(c_t - c_s)
+// (q_t . k_s), s <= t, and exp(c_L); each as the next kernel's operands, in blocks of 16 x 16 laid out [lane][4] as a lane
+// reads them, so that a block is one kilobyte in a row.  (Read row by row, a wave's load of an operand touches sixteen rows
+// in every quarter of it, which takes four times as long.)  The system is solved in blocks of 16 tokens: the diagonal
+// blocks I + A_ii are inverted by substitution (a lane per column), then X_i = (I + A_ii)^-1 (R_i - sum_(j < i) A_ij X_j)
+// runs on the matrix instruction, 16 columns of a right-hand side at a time: what it leaves in a lane is in the layout it
+// reads its second operand in, so solved blocks are used as they are; with its operands exchanged the instruction leaves
+// the transposed block, which is the layout of a first operand, as W is needed.
 template <int DP>
 __global__ __launch_bounds__(DR_THREADS) void delta_prepare_kernel(
     const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk, const float* __restrict__ v, int ldv,
     const float* __restrict__ b, int ldb, const float* __restrict__ a, int lda, const float* __restrict__ rate_log,
     const float* __restrict__ step_bias, int share, const int32_t* __restrict__ q_start, const int32_t* __restrict__ chunk_seq,
     const int32_t* __restrict__ chunk_row, float* __restrict__ ws_u0, float* __restrict__ ws_w, float* __restrict__ ws_kt,
-    float* __restrict__ ws_m, float* __restrict__ ws_in, float* __restrict__ ws_dec, int H, int dk, int dv, int vec) {
+    float* __restrict__ ws_m, float* __restrict__ ws_q, float* __restrict__ ws_dec, int H, int dk, int dv, int vec) {
     constexpr int LDK = DP + 4, NB = DR_L / 16, LDI = 20;
     __shared__ __attribute__((aligned(16))) float Ks[DR_L * LDK];
     __shared__ __attribute__((aligned(16))) float As[DR_L * DR_LDA];      // zeros on and above the diagonal
     __shared__ __attribute__((aligned(16))) float Ti[NB * 16 * LDI];      // the inverted diagonal blocks
     __shared__ double cs[DR_L];
-    __shared__ float bet[DR_L], bin[DR_L];                                // beta_t, beta_t exp(c_t); zero beyond the chunk
+    __shared__ float bet[DR_L], bin[DR_L], into[DR_L];                    // beta_t, beta_t exp(c_t) (zero beyond the chunk), exp(c_t)
     const int h = blockIdx.x, c = blockIdx.y, tid = threadIdx.x;
     const int t0 = chunk_row[c], n = min(DR_L, q_start[chunk_seq[c] + 1] - t0);
     const size_t at = (size_t)c * H + h;
     const int lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
-    float4 qf[DP / 16];
-    {
-        const int tt = wave * 16 + li;
-        const float* qr = q + (size_t)(t0 + (tt < n ? tt : 0)) * ldq + (size_t)(h / share) * dk;
+    DrTile<DP> qt, kt;
+    qt.load(q + (size_t)(h / share) * dk, ldq, t0, n, dk, vec);
+    kt.load(k + (size_t)(h / share) * dk, ldk, t0, n, dk, vec);
+    // the values of this wave's first pair of column blocks are on their way from here on
+    const int vt = (dv + 15) >> 4;
+    dr_f32x4 V[2][NB];
+    auto load_values = [&](int ct) {
 #pragma unroll
-        for (int kk = 0; kk < DP / 16; ++kk)
-            qf[kk] = tt < n ? dr_load4(qr, 16 * kk + 4 * lg, dk, vec) : make_float4(0.f, 0.f, 0.f, 0.f);
-    }
+        for (int x = 0; x < 2; ++x) {
+            const int j = (ct + 4 * x) * 16 + li;
+            const float* vc = v + (size_t)t0 * ldv + (size_t)h * dv + (j < dv ? j : dv - 1);
+#pragma unroll
+            for (int i = 0; i < NB; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int t = 16 * i + 4 * lg + e;
+                    V[x][i][e] = vc[(size_t)(t < n ? t : n - 1) * ldv];    // beyond the chunk beta is zero
+                }
+        }
+    };
+    load_values(wave);
     dr_log_decays(a, lda, t0, n, h, expf(rate_log[h]), step_bias ? step_bias[h] : 0.f, cs);
     if (tid < DR_L) {
         const float beta = tid < n ? dr_sigmoid(b[(size_t)(t0 + tid) * ldb + h]) : 0.f;
         const float in = expf((float)cs[tid]);
         bet[tid] = beta;
         bin[tid] = beta * in;
-        ws_in[at * DR_L + tid] = in;
+        into[tid] = in;
     }
-    dr_fill_keys<DP>(k + (size_t)(h / share) * dk, ldk, t0, n, dk, vec, Ks);
+    // the queries pass through the keys' place
+    qt.stash(Ks);
+    __syncthreads();
+    float4 qf[DP / 16];
+#pragma unroll
+    for (int kk = 0; kk < DP / 16; ++kk) qf[kk] = *reinterpret_cast<const float4*>(&Ks[(wave * 16 + li) * LDK + kk * 16 + 4 * lg]);
+    {
+        const float in = into[wave * 16 + li];
+        float4* dst = reinterpret_cast<float4*>(ws_q + at * (DR_L * DP)) + wave * (DP / 16) * 64 + lane;
+#pragma unroll
+        for (int kk = 0; kk < DP / 16; ++kk) dst[kk * 64] = make_float4(qf[kk].x * in, qf[kk].y * in, qf[kk].z * in, qf[kk].w * in);
+    }
+    __syncthreads();
+    kt.stash(Ks);
     __syncthreads();
     {
         dr_f32x4 ka[NB], qa[NB];
@@ -273,26 +320,47 @@ __global__ __launch_bounds__(DR_THREADS) void delta_prepare_kernel(
             for (int sb = 0; sb < NB; ++sb)
                 if (sb <= wave) {
                     const float4 other = *reinterpret_cast<const float4*>(&Ks[(sb * 16 + li) * LDK + kk * 16 + 4 * lg]);
-                    ka[sb] = dr_mfma4(kf, other, ka[sb]);
-                    qa[sb] = dr_mfma4(qf[kk], other, qa[sb]);
+#define DR_STEP(E)                                   \
+    ka[sb] = dr_mfma1<E>(kf, other, ka[sb]);         \
+    qa[sb] = dr_mfma1<E>(other, qf[kk], qa[sb]);     /* transposed */
+                    DR_EACH4(DR_STEP)
+#undef DR_STEP
                 }
         }
-        float* M = ws_m + at * (DR_L * DR_L);
+        float4* M = reinterpret_cast<float4*>(ws_m + at * (DR_L * DR_L)) + wave * NB * 64 + lane;
 #pragma unroll
-        for (int sb = 0; sb < NB; ++sb)
+        for (int sb = 0; sb < NB; ++sb) {
+            float m[4];
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
-                const int t = wave * 16 + 4 * lg + e, ss = sb * 16 + li;
-                const float f = ss <= t ? expf((float)(cs[t] - cs[ss])) : 0.f;
-                As[t * DR_LDA + ss] = ss < t ? bet[t] * f * ka[sb][e] : 0.f;
-                M[t * DR_L + ss] = f * qa[sb][e];
+                const int t = wave * 16 + 4 * lg + e, ss = sb * 16 + li;                  // this lane of K K^T
+                As[t * DR_LDA + ss] = ss < t ? bet[t] * expf((float)(cs[t] - cs[ss])) * ka[sb][e] : 0.f;
+                const int tq = wave * 16 + li, sq = sb * 16 + 4 * lg + e;                 // this lane of (Q K^T)^T
+                m[e] = sq <= tq ? expf((float)(cs[tq] - cs[sq])) * qa[sb][e] : 0.f;
             }
+            if (sb <= wave) M[sb * 64] = make_float4(m[0], m[1], m[2], m[3]);
+        }
     }
     // the decayed keys, transposed, and the chunk's whole decay
     const double c_end = cs[n - 1];
-    const float out_of = lane < n ? expf((float)(c_end - cs[lane])) : 0.f;        // a thread's token is the same in every pass
-#pragma unroll 8
-    for (int i = wave; i < DP; i += DR_THREADS / 64) ws_kt[at * (DP * DR_L) + i * DR_L + lane] = out_of * Ks[lane * LDK + i];
+    {
+        float out_of[NB][4];
+#pragma unroll
+        for (int kk = 0; kk < NB; ++kk)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int tt = 16 * kk + 4 * lg + e;
+                out_of[kk][e] = tt < n ? expf((float)(c_end - cs[tt])) : 0.f;
+            }
+        float4* dst = reinterpret_cast<float4*>(ws_kt + at * (DP * DR_L)) + lane;
+        for (int it = wave; it < DP / 16; it += DR_THREADS / 64)
+#pragma unroll
+            for (int kk = 0; kk < NB; ++kk) {
+                const float* col = &Ks[(16 * kk + 4 * lg) * LDK + it * 16 + li];
+                dst[(it * NB + kk) * 64] = make_float4(out_of[kk][0] * col[0], out_of[kk][1] * col[LDK], out_of[kk][2] * col[2 * LDK],
+                                                       out_of[kk][3] * col[3 * LDK]);
+            }
+    }
     if (tid == 0) ws_dec[at] = expf((float)c_end);
     __syncthreads();
     {
@@ -320,69 +388,94 @@ __global__ __launch_bounds__(DR_THREADS) void delta_prepare_kernel(
         for (int j = 0; j <= i; ++j)
             af[i][j] = j < i ? *reinterpret_cast<const float4*>(&As[(i * 16 + li) * DR_LDA + j * 16 + 4 * lg])
                              : *reinterpret_cast<const float4*>(&Ti[(i * 16 + li) * LDI + 4 * lg]);
-    const int vt = (dv + 15) >> 4, tiles = vt + DP / 16;
-    for (int ct = wave; ct < tiles; ct += DR_THREADS / 64) {
-        dr_f32x4 X[NB];
-        if (ct < vt) {
-            const int j = ct * 16 + li;
-            const float* vc = v + (size_t)t0 * ldv + (size_t)h * dv + (j < dv ? j : dv - 1);
-#pragma unroll
-            for (int i = 0; i < NB; ++i)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const int t = 16 * i + 4 * lg + e;
-                    X[i][e] = vc[(size_t)(t < n ? t : n - 1) * ldv];       // beyond the chunk beta is zero
-                }
-#pragma unroll
-            for (int i = 0; i < NB; ++i)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) X[i][e] *= bet[16 * i + 4 * lg + e];
-        } else {
-#pragma unroll
-            for (int i = 0; i < NB; ++i)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) X[i][e] = bin[16 * i + 4 * lg + e] * Ks[(16 * i + 4 * lg + e) * LDK + (ct - vt) * 16 + li];
-        }
+    // a pair of blocks of 16 columns at a time: their chains of dependent products are issued in turn
+    auto solve = [&](dr_f32x4 (&X)[2][NB], auto transposed, dr_f32x4 (&Y)[2][NB]) {
 #pragma unroll
         for (int i = 0; i < NB; ++i) {
-            dr_f32x4 r = X[i];
-            if (i > 0) {
-                dr_f32x4 acc = dr_f32x4{0.f, 0.f, 0.f, 0.f};
+            dr_f32x4 a0 = dr_f32x4{0.f, 0.f, 0.f, 0.f}, a1 = a0;
 #pragma unroll
-                for (int j = 0; j < i; ++j) acc = dr_mfma4(af[i][j], make_float4(X[j][0], X[j][1], X[j][2], X[j][3]), acc);
-                r -= acc;
+            for (int j = 0; j < i; ++j) {
+                const float4 x0 = dr_f4(X[0][j]), x1 = dr_f4(X[1][j]);
+#define DR_STEP(E)                              \
+    a0 = dr_mfma1<E>(af[i][j], x0, a0);         \
+    a1 = dr_mfma1<E>(af[i][j], x1, a1);
+                DR_EACH4(DR_STEP)
+#undef DR_STEP
             }
-            X[i] = dr_mfma4(af[i][i], make_float4(r[0], r[1], r[2], r[3]), dr_f32x4{0.f, 0.f, 0.f, 0.f});
+            const float4 r0 = dr_f4(X[0][i] - a0), r1 = dr_f4(X[1][i] - a1);
+            a0 = a1 = dr_f32x4{0.f, 0.f, 0.f, 0.f};
+#define DR_STEP(E)                              \
+    a0 = dr_mfma1<E>(af[i][i], r0, a0);         \
+    a1 = dr_mfma1<E>(af[i][i], r1, a1);
+            DR_EACH4(DR_STEP)
+#undef DR_STEP
+            X[0][i] = a0;
+            X[1][i] = a1;
+            if (transposed.value) {
+                a0 = a1 = dr_f32x4{0.f, 0.f, 0.f, 0.f};
+#define DR_STEP(E)                              \
+    a0 = dr_mfma1<E>(r0, af[i][i], a0);         \
+    a1 = dr_mfma1<E>(r1, af[i][i], a1);
+                DR_EACH4(DR_STEP)
+#undef DR_STEP
+                Y[0][i] = a0;
+                Y[1][i] = a1;
+            }
         }
-        if (ct < vt) {
-            float4* dst = reinterpret_cast<float4*>(ws_u0 + at * (size_t)(vt * 16 * DR_L)) + (size_t)ct * NB * 64 + lane;
+    };
+    dr_f32x4 Y[2][NB];
+    float4* u0 = reinterpret_cast<float4*>(ws_u0 + at * (size_t)(vt * 16 * DR_L)) + lane;
+    for (int ct = wave; ct < vt; ct += 8) {
+        if (ct != wave) load_values(ct);
 #pragma unroll
-            for (int i = 0; i < NB; ++i) dst[i * 64] = make_float4(X[i][0], X[i][1], X[i][2], X[i][3]);
-        } else {
-            float* dst = ws_w + at * (DR_L * DP) + (ct - vt) * 16 + li;
+        for (int x = 0; x < 2; ++x)
 #pragma unroll
             for (int i = 0; i < NB; ++i)
 #pragma unroll
-                for (int e = 0; e < 4; ++e) dst[(16 * i + 4 * lg + e) * DP] = X[i][e];
+                for (int e = 0; e < 4; ++e) V[x][i][e] *= bet[16 * i + 4 * lg + e];
+        solve(V, DrFlag<false>{}, Y);
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+            if (ct + 4 * x < vt) {
+#pragma unroll
+                for (int i = 0; i < NB; ++i) u0[((ct + 4 * x) * NB + i) * 64] = dr_f4(V[x][i]);
+            }
+    }
+    for (int ct = wave; ct < DP / 16; ct += 8) {
+#pragma unroll
+        for (int x = 0; x < 2; ++x) {
+            const int col = ((ct + 4 * x < DP / 16 ? ct + 4 * x : ct) << 4) + li;
+#pragma unroll
+            for (int i = 0; i < NB; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) V[x][i][e] = bin[16 * i + 4 * lg + e] * Ks[(16 * i + 4 * lg + e) * LDK + col];
         }
+        solve(V, DrFlag<true>{}, Y);
+        float4* dst = reinterpret_cast<float4*>(ws_w + at * (DR_L * DP)) + lane;
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+            if (ct + 4 * x < DP / 16) {
+#pragma unroll
+                for (int i = 0; i < NB; ++i) dst[(i * (DP / 16) + ct + 4 * x) * 64] = dr_f4(Y[x][i]);
+            }
     }
 }
 
-// The chunks of a sequence in order, for one head and 16 value columns: U = U_0 - W S, the outputs exp(c_t) S^T q_t + M U, S <-
+// The chunks of a sequence in order, for one head and 16 value columns: U = U_0 - W S, the outputs S^T (exp(c_t) q_t) + M U, S <-
 // exp(c_L) S + (decayed keys)^T U.  S lives in registers in the layout the matrix instruction leaves results in, wave w
 // holding the blocks of 16 key rows w and w + 4, and goes through LDS (as does U) in the layout it reads operands in, which
 // is the same: [block][lane group][lane] of four values.  Wave w has tokens 16 w .. 16 w + 15 of U and of the outputs.  A
 // step's operands are asked for as soon as the step before has used its own, into the same registers.
 template <int NK>
-__global__ __launch_bounds__(DR_THREADS) void delta_states_kernel(
-    const float* __restrict__ q, int ldq, const float* __restrict__ ws_u0, const float* __restrict__ ws_w,
-    const float* __restrict__ ws_kt, const float* __restrict__ ws_m, const float* __restrict__ ws_in,
-    const float* __restrict__ ws_dec, int share, float* __restrict__ state, long long state_stride,
+__global__ __launch_bounds__(DR_THREADS) __attribute__((amdgpu_waves_per_eu(1, 1))) void delta_states_kernel(
+    const float* __restrict__ ws_u0, const float* __restrict__ ws_w, const float* __restrict__ ws_kt,
+    const float* __restrict__ ws_m, const float* __restrict__ ws_q, const float* __restrict__ ws_dec,
+    float* __restrict__ state, long long state_stride,
     const int32_t* __restrict__ state_slots, const int32_t* __restrict__ q_start, const int32_t* __restrict__ seq_chunk,
-    float* __restrict__ out, int ldo, int H, int dk, int dv, int vec) {
+    float* __restrict__ out, int ldo, int H, int dk, int dv) {
     constexpr int DP = NK * 16, NT = (NK + 3) / 4;
     __shared__ float4 Sl[NK * 64], Ul[4 * 64];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), li = lane & 15, lg = lane >> 4;
     // heads vary fastest: with heads a multiple of 8, the column blocks of a head, which read the same W, keys and M, lie on one
     // XCD and share its L2
     const int j = blockIdx.y * 16 + li, h = blockIdx.x, s = blockIdx.z;
@@ -391,7 +484,6 @@ __global__ __launch_bounds__(DR_THREADS) void delta_states_kernel(
     const int row0 = q_start[s], row1 = q_start[s + 1], vt = (dv + 15) >> 4;
     const bool col_ok = j < dv;
     float* st = state + (size_t)state_slots[s] * state_stride + ((size_t)h * dv + (col_ok ? j : 0)) * dk;
-    const float* qh = q + (size_t)(h / share) * dk;
     dr_f32x4 S[NT];
 #pragma unroll
     for (int m = 0; m < NT; ++m) {
@@ -399,42 +491,42 @@ __global__ __launch_bounds__(DR_THREADS) void delta_states_kernel(
 #pragma unroll
         for (int e = 0; e < 4; ++e) S[m][e] = (col_ok && wave + 4 * m < NK && i + e < dk) ? st[i + e] : 0.f;
     }
-    float4 wf[NK], qf[NK], kf[NT][4], mf[4], u0, in;
+    float4 wf[NK], qf[NK], kf[NT][4], mf[4], u0;
     float dec;
-    auto fetch_w = [&](int c) {
-        const float* w = ws_w + ((size_t)c * H + h) * (DR_L * DP) + (wave * 16 + li) * DP + 4 * lg;
+    auto fetch_wq = [&](int c) {
+        const size_t at = (size_t)c * H + h;
+        const float4* w = reinterpret_cast<const float4*>(ws_w + at * (DR_L * DP)) + wave * NK * 64 + lane;
+        const float4* qs = reinterpret_cast<const float4*>(ws_q + at * (DR_L * DP)) + wave * NK * 64 + lane;
 #pragma unroll
-        for (int kk = 0; kk < NK; ++kk) wf[kk] = *reinterpret_cast<const float4*>(w + 16 * kk);
+        for (int kk = 0; kk < NK; ++kk) {
+            wf[kk] = w[kk * 64];
+            qf[kk] = qs[kk * 64];
+        }
     };
     auto fetch_u = [&](int c) {
         const size_t at = (size_t)c * H + h;
         u0 = reinterpret_cast<const float4*>(ws_u0 + at * (size_t)(vt * 16 * DR_L))[((size_t)blockIdx.y * 4 + wave) * 64 + lane];
-        in = *reinterpret_cast<const float4*>(ws_in + at * DR_L + wave * 16 + 4 * lg);
         dec = ws_dec[at];
     };
-    auto fetch_q = [&](int c) {
-        int t = row0 + (c - c0) * DR_L + wave * 16 + li;
-        t = t < row1 ? t : row1 - 1;                          // rows beyond the sequence are computed and not written
-        const float* qr = qh + (size_t)t * ldq;
-#pragma unroll
-        for (int kk = 0; kk < NK; ++kk) qf[kk] = dr_load4(qr, 16 * kk + 4 * lg, dk, vec);
-    };
     auto fetch_k = [&](int c) {
-        const float* kt = ws_kt + ((size_t)c * H + h) * (DP * DR_L) + 4 * lg;
+        const size_t at = (size_t)c * H + h;
+        const float4* kt = reinterpret_cast<const float4*>(ws_kt + at * (DP * DR_L)) + lane;
 #pragma unroll
-        for (int m = 0; m < NT; ++m) {
-            const int it = wave + 4 * m < NK ? wave + 4 * m : NK - 1;
+        for (int kk = 0; kk < 4; ++kk)
 #pragma unroll
-            for (int kk = 0; kk < 4; ++kk) kf[m][kk] = *reinterpret_cast<const float4*>(kt + (it * 16 + li) * DR_L + 16 * kk);
-        }
-        const float* mm = ws_m + ((size_t)c * H + h) * (DR_L * DR_L) + (wave * 16 + li) * DR_L + 4 * lg;
+            for (int m = 0; m < NT; ++m) kf[m][kk] = kt[((wave + 4 * m < NK ? wave + 4 * m : NK - 1) * 4 + kk) * 64];
+        const float4* mm = reinterpret_cast<const float4*>(ws_m + at * (DR_L * DR_L)) + wave * 4 * 64 + lane;
 #pragma unroll
-        for (int kk = 0; kk < 4; ++kk) mf[kk] = *reinterpret_cast<const float4*>(mm + 16 * kk);
+        for (int kk = 0; kk < 4; ++kk)                       // blocks above the diagonal are not kept
+            mf[kk] = kk <= wave ? mm[kk * 64] : make_float4(0.f, 0.f, 0.f, 0.f);
     };
-    fetch_w(c0);
+    // In the order in which a step uses them, here as in the loop: a wait for the first ones is then no wait for the last.
+    fetch_wq(c0);
+    __builtin_amdgcn_sched_barrier(0);
     fetch_u(c0);
-    fetch_q(c0);
+    __builtin_amdgcn_sched_barrier(0);
     fetch_k(c0);
+    __builtin_amdgcn_sched_barrier(0);
     for (int c = c0; c < c1; ++c) {
         const int cn = c + 1 < c1 ? c + 1 : c;
 #pragma unroll
@@ -444,37 +536,53 @@ __global__ __launch_bounds__(DR_THREADS) void delta_states_kernel(
         float4 sf[NK];
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) sf[kk] = Sl[(kk * 4 + lg) * 16 + li];
-        dr_f32x4 p0 = dr_f32x4{0.f, 0.f, 0.f, 0.f}, p1 = p0, y0 = p0, y1 = p0;
+        __builtin_amdgcn_sched_barrier(0);           // all of it asked for before the first product waits
+        // two chains of dependent products in turn, U's first: the others hide the wait for it
+        const dr_f32x4 zero = dr_f32x4{0.f, 0.f, 0.f, 0.f};
+        dr_f32x4 p0 = zero, p1 = zero, y0 = zero, y1 = zero;
 #pragma unroll
-        for (int kk = 0; kk < NK; ++kk) {
-            if (kk & 1) p1 = dr_mfma4(wf[kk], sf[kk], p1);
-            else p0 = dr_mfma4(wf[kk], sf[kk], p0);
+        for (int kk = 0; kk < NK; kk += 2) {
+#define DR_STEP(E)                                           \
+    p0 = dr_mfma1<E>(wf[kk], sf[kk], p0);                    \
+    if (kk + 1 < NK) p1 = dr_mfma1<E>(wf[kk + 1], sf[kk + 1], p1);
+            DR_EACH4(DR_STEP)
+#undef DR_STEP
         }
-        fetch_w(cn);
-        Ul[(wave * 4 + lg) * 16 + li] = make_float4(u0.x - (p0[0] + p1[0]), u0.y - (p0[1] + p1[1]), u0.z - (p0[2] + p1[2]), u0.w - (p0[3] + p1[3]));
+        p0 += p1;
+        Ul[(wave * 4 + lg) * 16 + li] = make_float4(u0.x - p0[0], u0.y - p0[1], u0.z - p0[2], u0.w - p0[3]);
 #pragma unroll
-        for (int kk = 0; kk < NK; ++kk) {
-            if (kk & 1) y1 = dr_mfma4(qf[kk], sf[kk], y1);
-            else y0 = dr_mfma4(qf[kk], sf[kk], y0);
+        for (int kk = 0; kk < NK; kk += 2) {
+#define DR_STEP(E)                                           \
+    y0 = dr_mfma1<E>(qf[kk], sf[kk], y0);                    \
+    if (kk + 1 < NK) y1 = dr_mfma1<E>(qf[kk + 1], sf[kk + 1], y1);
+            DR_EACH4(DR_STEP)
+#undef DR_STEP
         }
-        fetch_q(cn);
-        dr_f32x4 y = y0 + y1;
-        y[0] *= in.x, y[1] *= in.y, y[2] *= in.z, y[3] *= in.w;
+        __builtin_amdgcn_sched_barrier(0);
+        fetch_wq(cn);
+        __builtin_amdgcn_sched_barrier(0);
         const float dec_now = dec;
         fetch_u(cn);
+        __builtin_amdgcn_sched_barrier(0);
         __syncthreads();
         float4 uf[4];
 #pragma unroll
         for (int kk = 0; kk < 4; ++kk) uf[kk] = Ul[(kk * 4 + lg) * 16 + li];
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int m = 0; m < NT; ++m) S[m] *= dec_now;
 #pragma unroll
         for (int kk = 0; kk < 4; ++kk) {
-#pragma unroll
-            for (int m = 0; m < NT; ++m) S[m] = dr_mfma4(kf[m][kk], uf[kk], S[m]);
-            if (kk <= wave) y = dr_mfma4(mf[kk], uf[kk], y);
+#define DR_STEP(E)                                                                                  \
+    _Pragma("unroll") for (int m = 0; m < NT; ++m) S[m] = dr_mfma1<E>(kf[m][kk], uf[kk], S[m]);      \
+    y0 = dr_mfma1<E>(mf[kk], uf[kk], y0);
+            DR_EACH4(DR_STEP)
+#undef DR_STEP
         }
+        const dr_f32x4 y = y0 + y1;
+        __builtin_amdgcn_sched_barrier(0);
         fetch_k(cn);
+        __builtin_amdgcn_sched_barrier(0);
         if (col_ok) {
             const int t = row0 + (c - c0) * DR_L + wave * 16 + 4 * lg;
 #pragma unroll
@@ -498,7 +606,7 @@ extern "C" int tl_delta_chunk_tokens() { return DR_L; }
 // floats of workspace per chunk and head
 extern "C" long long tl_delta_chunked_workspace(int dk, int dv) {
     const long long DP = dr_padded_keys(dk), DV = (dv + 15) / 16 * 16;
-    return 2LL * DR_L * DP + DV * DR_L + DR_L * DR_L + DR_L + 4;
+    return 3LL * DR_L * DP + DV * DR_L + DR_L * DR_L + 4;
 }
 
 // The operands of tl_delta_walk.  chunk_seq, chunk_row [NC]: a chunk's sequence and its first row of the step (a sequence's
@@ -523,17 +631,16 @@ extern "C" int tl_delta_chunked(const float* q, int ldq, const float* k, int ldk
     float* ws_kt = ws_w + nh * DR_L * DP;
     float* ws_m = ws_kt + nh * DR_L * DP;
     float* ws_u0 = ws_m + nh * DR_L * DR_L;
-    float* ws_in = ws_u0 + nh * DV * DR_L;
-    float* ws_dec = ws_in + nh * DR_L;
+    float* ws_q = ws_u0 + nh * DV * DR_L;
+    float* ws_dec = ws_q + nh * DR_L * DP;
 #define GO(NK)                                                                                                                     \
     do {                                                                                                                           \
         hipLaunchKernelGGL(delta_prepare_kernel<16 * NK>, dim3(H, NC), dim3(DR_THREADS), 0, stream, q, ldq, k, ldk, v, ldv, b, ldb, a, lda, \
-                           rate_log, step_bias, share, q_start, chunk_seq, chunk_row, ws_u0, ws_w, ws_kt, ws_m, ws_in, ws_dec, H, dk, \
+                           rate_log, step_bias, share, q_start, chunk_seq, chunk_row, ws_u0, ws_w, ws_kt, ws_m, ws_q, ws_dec, H, dk, \
                            dv, vec);                                                                                                \
         TL_CHECK_LAUNCH("tl_delta_chunked prepare");                                                                               \
-        hipLaunchKernelGGL(delta_states_kernel<NK>, dim3(H, tl_ceil_div(dv, 16), S), dim3(DR_THREADS), 0, stream, q, ldq, ws_u0, ws_w, \
-                           ws_kt, ws_m, ws_in, ws_dec, share, state, state_stride, state_slots, q_start, seq_chunk, out, ldo, H, dk, dv, \
-                           vec);                                                                                                    \
+        hipLaunchKernelGGL(delta_states_kernel<NK>, dim3(H, tl_ceil_div(dv, 16), S), dim3(DR_THREADS), 0, stream, ws_u0, ws_w, ws_kt, ws_m, \
+                           ws_q, ws_dec, state, state_stride, state_slots, q_start, seq_chunk, out, ldo, H, dk, dv);                  \
         TL_CHECK_LAUNCH("tl_delta_chunked states");                                                                                \
     } while (0)
     if (DP == 16) GO(1);
