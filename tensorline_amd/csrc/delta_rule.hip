@@ -89,11 +89,11 @@ __global__ __launch_bounds__(DR_THREADS) void delta_walk_kernel(
     const float* __restrict__ b, int ldb, const float* __restrict__ a, int lda, const float* __restrict__ rate_log,
     const float* __restrict__ step_bias, int share, float* __restrict__ state, long long state_stride,
     const int32_t* __restrict__ state_slots, const int32_t* __restrict__ q_start, float* __restrict__ out, int ldo, int dk,
-    int dv, int vec, int vec_state) {
+    int dv, int vec, int vec_state, int upto) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l = lane & 15;
     const int j = blockIdx.x * 16 + wave * 4 + (lane >> 4), h = blockIdx.y, s = blockIdx.z;
     const int r0 = q_start[s], r1 = q_start[s + 1];
-    if (r1 <= r0) return;
+    if (r1 <= r0 || r1 - r0 > upto) return;
     const bool col_ok = j < dv;
     const int jc = col_ok ? j : dv - 1;
     float* st = state + (size_t)state_slots[s] * state_stride + ((size_t)h * dv + jc) * dk;
@@ -154,11 +154,12 @@ extern "C" int tl_delta_takes(int dk) { return dk > 0 && dk <= DR_MAX_DK ? 1 : 0
 
 // q, k [T, >= (H / share) * dk], v [T, >= H * dv], b, a [T, >= H] float with row strides; rate_log [H], step_bias [H] or
 // null; state: a request's [H, dv, dk] at state + slot * state_stride; out float [T, >= H * dv].  S sequences, rows
-// q_start[s] .. q_start[s + 1].
+// q_start[s] .. q_start[s + 1]; upto > 0: only the sequences that bring at most so many rows are walked.
 extern "C" int tl_delta_walk(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* b, int ldb,
                              const float* a, int lda, const float* rate_log, const float* step_bias, int share, float* state,
                              long long state_stride, const int32_t* state_slots, const int32_t* q_start, float* out, int ldo,
-                             int S, int H, int dk, int dv, hipStream_t stream) {
+                             int S, int H, int dk, int dv, int upto, hipStream_t stream) {
+    if (upto <= 0) upto = 0x7fffffff;
     TL_CHECK_ARG(S >= 0 && H > 0 && dv > 0 && tl_delta_takes(dk), "tl_delta_walk: bad sizes S=%d H=%d dk=%d (at most %d) dv=%d", S, H, dk, DR_MAX_DK, dv);
     TL_CHECK_ARG(share >= 1 && H % share == 0, "tl_delta_walk: %d heads do not share queries and keys in groups of %d", H, share);
     TL_CHECK_ARG(ldq >= H / share * dk && ldk >= H / share * dk && ldv >= H * dv && ldo >= H * dv && ldb >= H && lda >= H, "tl_delta_walk: rows too short");
@@ -170,7 +171,7 @@ extern "C" int tl_delta_walk(const float* q, int ldq, const float* k, int ldk, c
     dim3 grid(tl_ceil_div(dv, 16), H, S), block(DR_THREADS);
 #define GO(M)                                                                                                                  \
     hipLaunchKernelGGL(delta_walk_kernel<M>, grid, block, 0, stream, q, ldq, k, ldk, v, ldv, b, ldb, a, lda, rate_log, step_bias, \
-                       share, state, state_stride, state_slots, q_start, out, ldo, dk, dv, vec, vec_state)
+                       share, state, state_stride, state_slots, q_start, out, ldo, dk, dv, vec, vec_state, upto)
     if (dk <= 64) GO(1);
     else if (dk <= 128) GO(2);
     else GO(4);
@@ -610,7 +611,8 @@ extern "C" long long tl_delta_chunked_workspace(int dk, int dv) {
 }
 
 // The operands of tl_delta_walk.  chunk_seq, chunk_row [NC]: a chunk's sequence and its first row of the step (a sequence's
-// rows in chunks of DR_L from its first row on); seq_chunk [S + 1]: a sequence's first chunk.  ws: NC * H *
+// rows in chunks of DR_L from its first row on); seq_chunk [S + 1]: a sequence's first chunk (a sequence without chunks is
+// left alone).  ws: NC * H *
 // tl_delta_chunked_workspace floats, 16-byte aligned.
 extern "C" int tl_delta_chunked(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* b, int ldb,
                                 const float* a, int lda, const float* rate_log, const float* step_bias, int share, float* state,

@@ -49,7 +49,7 @@ __global__ __launch_bounds__(SS_THREADS) void scan_kernel(
     const float* __restrict__ z, int ldz, const float* __restrict__ bc, int ldbc, const float* __restrict__ A2,
     const float* __restrict__ D, float* __restrict__ state, long long state_stride, const int32_t* __restrict__ state_slots,
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ chunk_seq, const int32_t* __restrict__ chunk_row,
-    float* __restrict__ ws_state, float* __restrict__ ws_dt, X* __restrict__ out, int ldo, int inner, int N) {
+    float* __restrict__ ws_state, float* __restrict__ ws_dt, X* __restrict__ out, int ldo, int inner, int N, int upto) {
     constexpr int NP = R * P, CW = 64 / P, CB = SS_THREADS / P;
     __shared__ __attribute__((aligned(16))) float Bs[SS_TT][NP], Cs[MODE == SS_LOCAL ? 1 : SS_TT][NP];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -61,7 +61,7 @@ __global__ __launch_bounds__(SS_THREADS) void scan_kernel(
         s = blockIdx.y;
         t0 = q_start[s];
         t1 = q_start[s + 1];
-        if (t1 <= t0) return;
+        if (t1 <= t0 || t1 - t0 > upto) return;
     } else {
         s = chunk_seq[blockIdx.y];
         t0 = chunk_row[blockIdx.y];
@@ -191,11 +191,12 @@ template <int MODE, typename X>
 static int ss_launch(float* dt_raw, int lddt, const float* dt_bias, const void* x, int ldx, const float* z, int ldz,
                      const float* bc, int ldbc, const float* A2, const float* D, float* state, long long state_stride,
                      const int32_t* state_slots, const int32_t* q_start, const int32_t* chunk_seq, const int32_t* chunk_row,
-                     float* ws_state, float* ws_dt, void* out, int ldo, int rows, int inner, int N, hipStream_t stream) {
+                     float* ws_state, float* ws_dt, void* out, int ldo, int rows, int inner, int N, int upto,
+                     hipStream_t stream) {
 #define GO(R, P)                                                                                                                      \
     hipLaunchKernelGGL((scan_kernel<R, P, MODE, X>), dim3(tl_ceil_div(inner, SS_THREADS / P), rows), dim3(SS_THREADS), 0, stream, dt_raw, \
                        lddt, dt_bias, (const X*)x, ldx, z, ldz, bc, ldbc, A2, D, state, state_stride, state_slots, q_start, chunk_seq, \
-                       chunk_row, ws_state, ws_dt, (X*)out, ldo, inner, N)
+                       chunk_row, ws_state, ws_dt, (X*)out, ldo, inner, N, upto)
     if (N <= 8) GO(8, 1);
     else if (N <= 16) GO(16, 1);
     else if (N <= 32) GO(16, 2);
@@ -210,12 +211,13 @@ static int ss_launch(float* dt_raw, int lddt, const float* dt_bias, const void* 
 // dt_raw (overwritten where NC > 0), z float [T, >= inner], bc float [T, >= 2 N] = [B | C], x and out [T, >= inner] of dtype; dt_bias [inner] or null, A2
 // [N, inner] = A log2 e, D [inner]; state: a request's [N, inner] at state + slot * state_stride.  NC = 0: every sequence's
 // tokens are walked in order.  Else chunk_seq, chunk_row [NC], seq_chunk [S + 1] (chunks of SS_L tokens from a sequence's
-// first row of the step on), ws_state NC * N * inner floats, ws_dt NC * inner floats.
+// first row of the step on; a sequence without chunks is left to the walk), ws_state NC * N * inner floats, ws_dt NC * inner
+// floats; walk_upto > 0: the sequences that bring at most so many rows are walked beside them.
 extern "C" int tl_selective_scan(float* dt_raw, int lddt, const float* dt_bias, const void* x, int ldx, const float* z, int ldz,
                                  const float* bc, int ldbc, const float* A2, const float* D, float* state, long long state_stride,
                                  const int32_t* state_slots, const int32_t* q_start, const int32_t* chunk_seq,
                                  const int32_t* chunk_row, const int32_t* seq_chunk, float* ws_state, float* ws_dt, void* out,
-                                 int dtype, int ldo, int S, int NC, int inner, int N, hipStream_t stream) {
+                                 int dtype, int ldo, int S, int NC, int inner, int N, int walk_upto, hipStream_t stream) {
     TL_CHECK_ARG(S >= 0 && NC >= 0 && inner > 0 && tl_selective_scan_takes(N), "tl_selective_scan: bad sizes inner=%d state=%d (at most %d)", inner, N, SS_MAX_STATE);
     TL_CHECK_ARG(lddt >= inner && ldx >= inner && ldz >= inner && ldo >= inner && ldbc >= 2 * N, "tl_selective_scan: rows too short");
     TL_CHECK_ARG(A2 && D && state_stride >= (long long)N * inner, "tl_selective_scan: A or D is missing, or the state of a request is too small");
@@ -224,10 +226,14 @@ extern "C" int tl_selective_scan(float* dt_raw, int lddt, const float* dt_bias, 
     if (S == 0) return 0;
 #define GO(MODE, ROWS)                                                                                                              \
     (dtype == TL_BF16 ? ss_launch<MODE, bf16_t>(dt_raw, lddt, dt_bias, x, ldx, z, ldz, bc, ldbc, A2, D, state, state_stride, state_slots, \
-                                                q_start, chunk_seq, chunk_row, ws_state, ws_dt, out, ldo, ROWS, inner, N, stream)    \
+                                                q_start, chunk_seq, chunk_row, ws_state, ws_dt, out, ldo, ROWS, inner, N, walk_upto, stream)    \
                       : ss_launch<MODE, float>(dt_raw, lddt, dt_bias, x, ldx, z, ldz, bc, ldbc, A2, D, state, state_stride, state_slots, \
-                                               q_start, chunk_seq, chunk_row, ws_state, ws_dt, out, ldo, ROWS, inner, N, stream))
-    if (NC == 0) return GO(SS_WALK, S);
+                                               q_start, chunk_seq, chunk_row, ws_state, ws_dt, out, ldo, ROWS, inner, N, walk_upto, stream))
+    if (NC == 0 || walk_upto > 0) {
+        if (NC == 0) walk_upto = 0x7fffffff;
+        const int rc = GO(SS_WALK, S);
+        if (rc || NC == 0) return rc;
+    }
     TL_CHECK_ARG(chunk_seq && chunk_row && seq_chunk && ws_state && ws_dt, "tl_selective_scan: chunk tables or workspace are missing");
     if (int rc = GO(SS_LOCAL, NC)) return rc;
     hipLaunchKernelGGL(scan_states_kernel, dim3(tl_ceil_div(inner, SS_THREADS), N, S), dim3(SS_THREADS), 0, stream, ws_state, ws_dt, A2,

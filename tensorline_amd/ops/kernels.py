@@ -1392,17 +1392,18 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, ctx, st
 # ---------------------------------------------------------------------------------------------
 # Recurrences in chunks of a step's rows: the delta rule and the selective scan
 CHUNK_TOKENS = 64          # tokens per chunk in both kernels
-CHUNKED_FROM = 33          # steps whose sequences bring at most this many tokens less one walk token by token
+WALK_TOKENS = 32           # sequences that bring at most this many tokens are walked token by token
 
 
 @dataclass
 class SequenceChunks:
-    """How the sequences of a step are cut into chunks of ``CHUNK_TOKENS`` rows, each from its first row of the step:
+    """How the longer sequences of a step are cut into chunks of ``CHUNK_TOKENS`` rows, each from its first row of the step:
     ``seq`` and ``row`` (int32 [n]) hold a chunk's sequence and its first row, ``first`` (int32 [S + 1]) a sequence's first
     chunk."""
     seq: torch.Tensor
     row: torch.Tensor
     first: torch.Tensor
+    walked: bool = False             # whether some sequence of the step has no chunks: those of at most WALK_TOKENS rows
 
     @property
     def count(self) -> int:
@@ -1411,12 +1412,12 @@ class SequenceChunks:
 
 def chunk_vectors(facts) -> dict[str, list[int]]:
     """The index vectors of :class:`SequenceChunks` for a step's shape, for the step's upload; none for a step that walks."""
-    if facts.decode_only or facts.max_query_len < CHUNKED_FROM:
+    if facts.decode_only or facts.max_query_len <= WALK_TOKENS:
         return {}
     seq, row, first, at = [], [], [0], 0
     lens = list(facts.q_lens) + [1] * (facts.num_seqs - len(facts.q_lens))      # padding sequences bring one token
     for s, n in enumerate(lens):
-        for lo in range(0, n, CHUNK_TOKENS):
+        for lo in range(0, n if n > WALK_TOKENS else 0, CHUNK_TOKENS):
             seq.append(s)
             row.append(at + lo)
         at += n
@@ -1425,9 +1426,12 @@ def chunk_vectors(facts) -> dict[str, list[int]]:
 
 
 def step_chunks(ctx) -> SequenceChunks | None:
-    """The chunks uploaded with the step, or None: then its tokens are walked one after another."""
+    """The chunks uploaded with the step, or None: then all its sequences are walked token by token."""
     seq = ctx.extra.get("chunks.seq")
-    return None if seq is None else SequenceChunks(seq, ctx.extra["chunks.row"], ctx.extra["chunks.first"])
+    if seq is None:
+        return None
+    lens = ctx.facts.q_lens
+    return SequenceChunks(seq, ctx.extra["chunks.row"], ctx.extra["chunks.first"], min(lens) <= WALK_TOKENS or len(lens) < ctx.num_seqs)
 
 
 def _check_chunks(chunks: SequenceChunks, num_seqs: int, who: str) -> None:
@@ -1476,7 +1480,7 @@ def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b: torch.Tenso
 
     ``q``, ``k`` float32 [T, heads / share * dk] as they enter the rule (the ``share`` consecutive heads of a group read the
     same), ``v`` [T, heads * dv], ``b``, ``a`` [T, heads]; all may be column blocks of wider matrices.  With ``chunks`` (and
-    ``dk`` up to 128) the step's rows are taken in chunks: the same sums in another order.  Returns float32 [T, heads * dv]."""
+    ``dk`` up to 128) the longer sequences' rows are taken in chunks: the same sums in another order.  Returns float32 [T, heads * dv]."""
     _on_gpu(q, k, v, b, a, rate_log, step_bias, state)
     T = q.shape[0]
     share = int(share)
@@ -1500,8 +1504,12 @@ def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b: torch.Tenso
         ws = torch.empty(chunks.count * heads * fn(dk, dv), dtype=torch.float32, device=q.device)
         _call("tl_delta_chunked", *head, _ptr(chunks.seq), _ptr(chunks.row), _ptr(chunks.first), _ptr(ws), _ptr(out), heads * dv,
               ctx.num_seqs, chunks.count, heads, dk, dv, _stream())
-        return out
-    _call("tl_delta_walk", *head, _ptr(out), heads * dv, ctx.num_seqs, heads, dk, dv, _stream())
+        if not chunks.walked:
+            return out
+        walk_upto = WALK_TOKENS
+    else:
+        walk_upto = 0
+    _call("tl_delta_walk", *head, _ptr(out), heads * dv, ctx.num_seqs, heads, dk, dv, walk_upto, _stream())
     return out
 
 
@@ -1517,7 +1525,8 @@ def selective_scan(dt_raw: torch.Tensor, dt_bias: torch.Tensor | None, x: torch.
     ``dt_raw``, ``z`` float32 [T, inner], ``x`` [T, inner] float32 or bfloat16, ``bc`` float32 [T, 2 N] = [B | C] (all may be column
     blocks of wider matrices; ``dt_raw`` is used up: with ``chunks`` it holds ``dt`` afterwards), ``a2`` float32 [N, inner] = ``A^T
     log2(e)``, ``skip`` float32 [inner].  S lives at ``state[slot, offset
-    : offset + N * inner]`` as [N, inner].  With ``chunks`` the step's rows are taken in chunks, all at once."""
+    : offset + N * inner]`` as [N, inner].  With ``chunks`` the longer sequences' rows are taken in
+    chunks, all at once."""
     _on_gpu(dt_raw, dt_bias, x, z, bc, a2, skip, state)
     T, inner = x.shape
     N = a2.shape[0]
@@ -1542,7 +1551,7 @@ def selective_scan(dt_raw: torch.Tensor, dt_bias: torch.Tensor | None, x: torch.
     _call("tl_selective_scan", _ptr(dt_raw), ld(dt_raw), _ptr(dt_bias), _ptr(x), ld(x), _ptr(z), ld(z), _ptr(bc), ld(bc), _ptr(a2),
           _ptr(skip), st, ctypes.c_longlong(stride), _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(seq), _ptr(row), _ptr(first),
           _ptr(ws_s), _ptr(ws_dt), _ptr(out), _code(x, "selective_scan"), inner, ctx.num_seqs,
-          chunks.count if chunks is not None else 0, inner, N, _stream())
+          chunks.count if chunks is not None else 0, inner, N, WALK_TOKENS if chunks is not None and chunks.walked else 0, _stream())
     return out
 
 

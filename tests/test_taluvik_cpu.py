@@ -81,8 +81,9 @@ def test_spec_kinds_run_order_needs_and_names():
 def test_chunks_of_a_step():
     facts = StepFacts(max_context=300, max_query_len=130, num_seqs=4, q_lens=[130, 1, 64], starts=[0, 40, 7])
     v = kernels.chunk_vectors(facts)
-    assert v["chunks.seq"] == [0, 0, 0, 1, 2, 3] and v["chunks.row"] == [0, 64, 128, 130, 131, 195]
-    assert v["chunks.first"] == [0, 3, 4, 5, 6]
+    # the sequence of one token and the padding sequence are walked
+    assert v["chunks.seq"] == [0, 0, 0, 2] and v["chunks.row"] == [0, 64, 128, 131]
+    assert v["chunks.first"] == [0, 3, 3, 4, 4]
     assert kernels.chunk_vectors(StepFacts(max_query_len=1, decode_only=True, num_seqs=2, q_lens=[1, 1], starts=[5, 6])) == {}
     assert kernels.chunk_vectors(StepFacts(max_query_len=32, num_seqs=1, q_lens=[32], starts=[0])) == {}
     # every part that takes chunks asks for the same tables

@@ -83,7 +83,9 @@ class _Step:
         if chunked:
             from tensorline_amd.ops import kernels
             v = kernels.chunk_vectors(StepFacts(max_query_len=10 ** 6, num_seqs=len(lens), q_lens=list(lens)))
-            self.chunks = kernels.SequenceChunks(*(i32(v["chunks." + n]) for n in ("seq", "row", "first")))
+            if v["chunks.seq"]:
+                self.chunks = kernels.SequenceChunks(*(i32(v["chunks." + n]) for n in ("seq", "row", "first")),
+                                                     walked=min(lens) <= kernels.WALK_TOKENS)
 
 
 # ---- every mechanism alone -------------------------------------------------------------------------
@@ -229,7 +231,7 @@ def _plain_delta(q, k, v, b, a, rate_log, bias, S):
 
 
 @pytest.mark.parametrize("chunked", [False, True])
-@pytest.mark.parametrize("lens", [[1, 1, 1], [150, 1, 64, 65], [63, 2], [300]])
+@pytest.mark.parametrize("lens", [[1, 1, 1], [150, 1, 64, 65], [63, 32, 33, 2], [300]])
 @pytest.mark.parametrize("case", [
     # heads, share, dk, dv, what the decays are like
     (4, 2, 24, 40, "mixed"), (3, 3, 9, 13, "mixed"), (2, 1, 128, 64, "long"), (2, 2, 64, 128, "strong"), (1, 1, 16, 5, "none"), (2, 1, 96, 16, "mixed"),
@@ -276,7 +278,7 @@ def test_delta_rule_token_by_token_and_in_chunks(case, lens, chunked):
 
 
 @pytest.mark.parametrize("chunked", [False, True])
-@pytest.mark.parametrize("lens", [[1, 1, 1], [150, 1, 64, 65], [63, 2], [700]])
+@pytest.mark.parametrize("lens", [[1, 1, 1], [150, 1, 64, 65], [63, 32, 33, 2], [700]])
 @pytest.mark.parametrize("inner,N", [(88, 12), (50, 1), (300, 16), (33, 17), (70, 40), (20, 256), (17, 8), (130, 100)])
 def test_selective_scan_token_by_token_and_in_chunks(inner, N, lens, chunked):
     from tensorline_amd.ops import kernels
