@@ -160,10 +160,13 @@ extern "C" int tl_delta_walk(const float* q, int ldq, const float* k, int ldk, c
                              long long state_stride, const int32_t* state_slots, const int32_t* q_start, float* out, int ldo,
                              int S, int H, int dk, int dv, int upto, hipStream_t stream) {
     if (upto <= 0) upto = 0x7fffffff;
-    TL_CHECK_ARG(S >= 0 && H > 0 && dv > 0 && tl_delta_takes(dk), "tl_delta_walk: bad sizes S=%d H=%d dk=%d (at most %d) dv=%d", S, H, dk, DR_MAX_DK, dv);
+    TL_CHECK_ARG(S >= 0 && H > 0 && dv > 0 && tl_delta_takes(dk),
+                 "tl_delta_walk: bad sizes S=%d H=%d dk=%d (at most %d) dv=%d", S, H, dk, DR_MAX_DK, dv);
     TL_CHECK_ARG(share >= 1 && H % share == 0, "tl_delta_walk: %d heads do not share queries and keys in groups of %d", H, share);
-    TL_CHECK_ARG(ldq >= H / share * dk && ldk >= H / share * dk && ldv >= H * dv && ldo >= H * dv && ldb >= H && lda >= H, "tl_delta_walk: rows too short");
-    TL_CHECK_ARG(rate_log && state_stride >= (long long)H * dk * dv, "tl_delta_walk: rates are missing or the state of a request is too small");
+    TL_CHECK_ARG(ldq >= H / share * dk && ldk >= H / share * dk && ldv >= H * dv && ldo >= H * dv && ldb >= H && lda >= H,
+                 "tl_delta_walk: rows too short");
+    TL_CHECK_ARG(rate_log && state_stride >= (long long)H * dk * dv,
+                 "tl_delta_walk: rates are missing or the state of a request is too small");
     TL_CHECK_ARG(H <= 65535 && S <= 65535, "tl_delta_walk: too many heads or sequences for one launch");
     if (S == 0) return 0;
     const int vec = ((uintptr_t)q % 16 == 0 && (uintptr_t)k % 16 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && dk % 4 == 0) ? 1 : 0;
@@ -619,13 +622,17 @@ extern "C" int tl_delta_chunked(const float* q, int ldq, const float* k, int ldk
                                 long long state_stride, const int32_t* state_slots, const int32_t* q_start,
                                 const int32_t* chunk_seq, const int32_t* chunk_row, const int32_t* seq_chunk, float* ws, float* out,
                                 int ldo, int S, int NC, int H, int dk, int dv, hipStream_t stream) {
-    TL_CHECK_ARG(S >= 0 && NC >= 0 && H > 0 && tl_delta_chunked_takes(dk, dv), "tl_delta_chunked: bad sizes S=%d H=%d dk=%d dv=%d", S, H, dk, dv);
+    TL_CHECK_ARG(S >= 0 && NC >= 0 && H > 0 && tl_delta_chunked_takes(dk, dv),
+                 "tl_delta_chunked: bad sizes S=%d H=%d dk=%d dv=%d", S, H, dk, dv);
     TL_CHECK_ARG(share >= 1 && H % share == 0, "tl_delta_chunked: %d heads do not share queries and keys in groups of %d", H, share);
-    TL_CHECK_ARG(ldq >= H / share * dk && ldk >= H / share * dk && ldv >= H * dv && ldo >= H * dv && ldb >= H && lda >= H, "tl_delta_chunked: rows too short");
-    TL_CHECK_ARG(rate_log && state_stride >= (long long)H * dk * dv, "tl_delta_chunked: rates are missing or the state of a request is too small");
+    TL_CHECK_ARG(ldq >= H / share * dk && ldk >= H / share * dk && ldv >= H * dv && ldo >= H * dv && ldb >= H && lda >= H,
+                 "tl_delta_chunked: rows too short");
+    TL_CHECK_ARG(rate_log && state_stride >= (long long)H * dk * dv,
+                 "tl_delta_chunked: rates are missing or the state of a request is too small");
     TL_CHECK_ARG(NC <= 65535 && H <= 65535 && S <= 65535, "tl_delta_chunked: too many chunks, heads or sequences for one launch");
     if (S == 0 || NC == 0) return 0;
-    TL_CHECK_ARG(ws && (uintptr_t)ws % 16 == 0 && chunk_seq && chunk_row && seq_chunk, "tl_delta_chunked: the workspace (16-byte aligned) or the chunk tables are missing");
+    TL_CHECK_ARG(ws && (uintptr_t)ws % 16 == 0 && chunk_seq && chunk_row && seq_chunk,
+                 "tl_delta_chunked: the workspace (16-byte aligned) or the chunk tables are missing");
     const int vec = ((uintptr_t)q % 16 == 0 && (uintptr_t)k % 16 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && dk % 4 == 0) ? 1 : 0;
     const int DP = dr_padded_keys(dk), DV = (dv + 15) / 16 * 16;
     const size_t nh = (size_t)NC * H;

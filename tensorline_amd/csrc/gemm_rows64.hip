@@ -21,6 +21,12 @@
 // tile and its up tile); for a fused q/k/v projection bias, RoPE and the cache write.
 #include "common.h"
 
+// what the gated form passes of a gate: SiLU, or with act 2 the tanh form of GELU
+__device__ __forceinline__ float r64_gate(float v, int act) {
+    if (act == 2) return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
+    return v / (1.0f + expf(-v));
+}
+
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
@@ -186,7 +192,7 @@ __global__ __launch_bounds__(THREADS) void gemm_rows64_kernel(
             float v = owed ? acc[mt][i] * sh_rstd[m] : acc[mt][i];
             if (PAIR) {
                 const float u = owed ? acc2[mt][i] * sh_rstd[m] : acc2[mt][i];
-                C[(size_t)m * ldc + n] = tl_from_float<TO>(v / (1.0f + expf(-v)) * u);
+                C[(size_t)m * ldc + n] = tl_from_float<TO>(r64_gate(v, na.act) * u);
                 continue;
             }
             if (bias) v += bias[n];
@@ -237,7 +243,7 @@ __global__ __launch_bounds__(256) void gemm_rows64_reduce_kernel(const float* __
             if (swiglu) u += p[n_out + n];
         }
         v *= rs;
-        if (swiglu) v = v / (1.0f + expf(-v)) * (u * rs);
+        if (swiglu) v = r64_gate(v, na.act) * (u * rs);
         else if (bias) v += bias[n];
     }
     if (na.resid) {
@@ -390,7 +396,8 @@ static void r64_launch(const R64Plan& p, hipStream_t stream, const bf16_t* A, co
 // [M, I] = silu(gate) * up and bias is not used (with one share I must be a multiple of 16).  norm: null, or an owed
 // normalisation of A's rows and / or a residual sink (TlNormArgs).  With a sink C is not written,
 // swiglu is not allowed, and ss_out gets one partial per row and 16-column tile when shares is 1
-// ([ceil(N/16), M]), per row and 256 columns otherwise ([ceil(N/256), M]).
+// ([ceil(N/16), M]), per row and 256 columns otherwise ([ceil(N/256), M]).  norm->act 2 with swiglu:
+// GELU's tanh form in place of SiLU.
 extern "C" int tl_gemm_rows64(const void* A, const void* Ws, const float* bias, void* C, int c_dtype, float* partial,
                               int M, int N, int K, int lda, int ldc, int shares, int swiglu, const TlNormArgs* norm,
                               hipStream_t stream) {
@@ -408,6 +415,8 @@ extern "C" int tl_gemm_rows64(const void* A, const void* Ws, const float* bias, 
     if (na.ss_in)
         TL_CHECK_ARG(na.ss_n > 0 && na.ss_ld >= M && na.dim > 0.f && na.eps >= 0.f,
                      "tl_gemm_rows64: bad owed-norm arguments (partials %d, stride %d)", na.ss_n, na.ss_ld);
+    TL_CHECK_ARG(na.act == 0 || (na.act == 2 && swiglu), "tl_gemm_rows64: activation %d is not one this product applies",
+                 na.act);
     if (na.resid)
         TL_CHECK_ARG(!swiglu && na.next_weight && na.a_out && na.ss_out && na.resid_ld >= N && na.a_ld >= N &&
                          na.ss_out_ld >= M,

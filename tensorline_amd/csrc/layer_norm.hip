@@ -3,9 +3,9 @@
 //     x[r] += mult * (y1[r] + y2[r])
 //     out[r] = (x[r] - mean) / sqrt(mean((x[r] - mean)^2) + eps) * w + b
 //
-// y1 and y2 may each be absent, and each may come in shares (the K shares of a product, added in ascending order first).  With `rows`: out only, for the sums at rows[r]; x is left as it is.  Without w:
-// the sum only.  Everything is float; the deviations are taken from the row's own mean, never from a difference of
-// two large sums.
+// y1 and y2 may each be absent, and each may come in shares (the K shares of a product, added in ascending order
+// first).  With `rows`: out only, for the sums at rows[r]; x is left as it is.  Without w: the sum only.  Everything is
+// float; the deviations are taken from the row's own mean, never from a difference of two large sums.
 #include "common.h"
 
 #define LN_VPT 4   // float4 per thread at most
@@ -41,7 +41,8 @@ __device__ __forceinline__ float4 ln_branch4(const LnBranch& b, size_t i) {
 
 // Any row length: a thread walks its columns three times.
 template <typename O>
-__global__ __launch_bounds__(1024) void add_layernorm_kernel(float* __restrict__ x, LnBranch b1, LnBranch b2, float mult, const float* __restrict__ w,
+__global__ __launch_bounds__(1024) void add_layernorm_kernel(float* __restrict__ x, LnBranch b1, LnBranch b2, float mult,
+                                                             const float* __restrict__ w,
                                                              const float* __restrict__ b, float eps, O* __restrict__ out,
                                                              const int32_t* __restrict__ rows, int H) {
     __shared__ float red[16];

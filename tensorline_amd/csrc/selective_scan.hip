@@ -208,9 +208,9 @@ static int ss_launch(float* dt_raw, int lddt, const float* dt_bias, const void* 
     return 0;
 }
 
-// dt_raw (overwritten where NC > 0), z float [T, >= inner], bc float [T, >= 2 N] = [B | C], x and out [T, >= inner] of dtype; dt_bias [inner] or null, A2
-// [N, inner] = A log2 e, D [inner]; state: a request's [N, inner] at state + slot * state_stride.  NC = 0: every sequence's
-// tokens are walked in order.  Else chunk_seq, chunk_row [NC], seq_chunk [S + 1] (chunks of SS_L tokens from a sequence's
+// dt_raw (overwritten where NC > 0), z float [T, >= inner], bc float [T, >= 2 N] = [B | C], x and out [T, >= inner] of
+// dtype; dt_bias [inner] or null, A2 [N, inner] = A log2 e, D [inner]; state: a request's [N, inner] at
+// state + slot * state_stride.  NC = 0: every sequence's tokens are walked in order.  Else chunk_seq, chunk_row [NC], seq_chunk [S + 1] (chunks of SS_L tokens from a sequence's
 // first row of the step on; a sequence without chunks is left to the walk), ws_state NC * N * inner floats, ws_dt NC * inner
 // floats; walk_upto > 0: the sequences that bring at most so many rows are walked beside them.
 extern "C" int tl_selective_scan(float* dt_raw, int lddt, const float* dt_bias, const void* x, int ldx, const float* z, int ldz,
@@ -218,9 +218,11 @@ extern "C" int tl_selective_scan(float* dt_raw, int lddt, const float* dt_bias, 
                                  const int32_t* state_slots, const int32_t* q_start, const int32_t* chunk_seq,
                                  const int32_t* chunk_row, const int32_t* seq_chunk, float* ws_state, float* ws_dt, void* out,
                                  int dtype, int ldo, int S, int NC, int inner, int N, int walk_upto, hipStream_t stream) {
-    TL_CHECK_ARG(S >= 0 && NC >= 0 && inner > 0 && tl_selective_scan_takes(N), "tl_selective_scan: bad sizes inner=%d state=%d (at most %d)", inner, N, SS_MAX_STATE);
+    TL_CHECK_ARG(S >= 0 && NC >= 0 && inner > 0 && tl_selective_scan_takes(N),
+                 "tl_selective_scan: bad sizes inner=%d state=%d (at most %d)", inner, N, SS_MAX_STATE);
     TL_CHECK_ARG(lddt >= inner && ldx >= inner && ldz >= inner && ldo >= inner && ldbc >= 2 * N, "tl_selective_scan: rows too short");
-    TL_CHECK_ARG(A2 && D && state_stride >= (long long)N * inner, "tl_selective_scan: A or D is missing, or the state of a request is too small");
+    TL_CHECK_ARG(A2 && D && state_stride >= (long long)N * inner,
+                 "tl_selective_scan: A or D is missing, or the state of a request is too small");
     TL_CHECK_ARG(S <= 65535 && NC <= 65535, "tl_selective_scan: too many sequences or chunks for one launch");
     TL_CHECK_ARG(dtype == TL_F32 || dtype == TL_BF16, "tl_selective_scan: unknown dtype %d", dtype);
     if (S == 0) return 0;

@@ -623,7 +623,7 @@ def swiglu_gate_up(h: torch.Tensor | NormedRows, gate_up_weight: torch.Tensor,
     """``silu(h Wg^T) * (h Wu^T)`` for a fused [2I, K] weight (gate rows first): one kernel for
     few-row bfloat16 batches (it streams the ``shuffled`` copy), product then SiLU-multiply otherwise.
     ``h`` may be :class:`NormedRows` (few-row kernel only).  ``activation`` "gelu_tanh": the tanh form of GELU
-    passes the gate instead of SiLU (in the few-row kernel's epilogue, or by a pass over the product)."""
+    passes the gate instead of SiLU (in the streaming kernels' epilogues, or by a pass over the product)."""
     _check(activation in GLU_ACTIVATIONS, f"swiglu_gate_up: unknown activation {activation!r}")
     if activation != "silu":
         _check(not isinstance(h, NormedRows), "swiglu_gate_up: only SiLU rides on a product that carries a norm")
@@ -639,6 +639,14 @@ def swiglu_gate_up(h: torch.Tensor | NormedRows, gate_up_weight: torch.Tensor,
             na.act = 2
             _call("tl_gemm_skinny_swiglu", _ptr(h), _ptr(shuffled), _ptr(out), M, I, K, lda, I, ctypes.byref(na), _stream())
             return out
+        if _rows64_ok(h, shuffled, M, K, lda) and (I % 16 == 0 or library().tl_gemm_rows64_shares(M, 2 * I, K) > 1):
+            _on_gpu(h, gate_up_weight, shuffled)
+            _check(gate_up_weight.shape[1] == K and gate_up_weight.shape[0] % 2 == 0, "swiglu_gate_up: bad shapes")
+            _check_shuffled(shuffled, 2 * I, K)
+            out = torch.empty(M, I, dtype=h.dtype, device=h.device)
+            na = _NormArgs()
+            na.act = 2
+            return _rows64(h, shuffled, None, out, M, 2 * I, K, lda, I, swiglu=True, norm=ctypes.byref(na))
         return glu(linear(h, gate_up_weight, shuffled=shuffled), activation, h.dtype)
     owed = h if isinstance(h, NormedRows) else None
     if owed is not None:

@@ -210,9 +210,10 @@ class ParallelBranchesBlock:
         h = norm1(x);  x <- x + m * (mixer(h) + ffn(h))
 
     with the factor ``m`` = ``LayerSpec.branch_scale``; the feed-forward may be absent.  A mixer or feed-forward that sets
-    ``keeps_share_sums`` may leave its last product in its shares of K.  The branches' outputs are not added at once: they are handed on as :class:`tensorline_amd.ops.kernels.ScaledBranches`, and the norm that reads
-    the stream next adds both in its own pass.  Where whoever runs next does not take that form
-    (``after.scaled_branches``), the block adds them itself and leaves nothing."""
+    ``keeps_share_sums`` may leave its last product in its shares of K.  The branches' outputs are not added at once:
+    they are handed on as :class:`tensorline_amd.ops.kernels.ScaledBranches`, and the norm that reads the stream next adds
+    both in its own pass.  Where whoever runs next does not take that form (``after.scaled_branches``), the block adds
+    them itself and leaves nothing."""
 
     def __init__(self, spec: LayerSpec, hidden_size: int, dtype, device):
         common = dict(hidden_size=hidden_size, dtype=dtype, device=device)

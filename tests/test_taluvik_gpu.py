@@ -309,6 +309,22 @@ def test_selective_scan_token_by_token_and_in_chunks(inner, N, lens, chunked):
     assert torch.equal(dev_state[:, :off].cpu(), state[:, :off]) and torch.equal(dev_state[len(lens)].cpu(), state[len(lens)])
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("width,ff", [(88, 136), (88, 7), (320, 1024), (1024, 640)])
+def test_feed_forward_alone(width, ff, dtype):
+    """From one row to many: the few-row and the mid-row product with the gate in their epilogues, with and without K cut
+    into shares, and the product with a pass of its own behind it."""
+    cfg = one_layer("mamba1", _mamba(8, 1, 1, 1), ff, width=width)
+    model, w = build(cfg, dtype, seed=3)
+    W = P.as_double(w)
+    for rows in (1, 5, 17, 33, 64, 65, 300):
+        torch.manual_seed(rows)
+        h = torch.randn(rows, width).to(torch.bfloat16).float()
+        got = model.blocks[0].feed_forward.forward(h.to(DEV).to(model.dtype), None).float().cpu()
+        err = _rms_error(got, P.gated_ff(h.double(), W, "l0.mlp.").float())
+        assert err < (1e-5 if dtype == "float32" else 1e-2), f"{rows} rows: {err:.3e}"
+
+
 MIXERS = [
     ("attention", _attn(4, 2, 24, 40, 19, 8)), ("attention", _attn(1, 1, 10, 7, 16, 10, scaling=None, softcap=None)),
     ("attention", _attn(6, 1, 64, 40, 50, 32, softcap=2.0)), ("attention", _attn(2, 2, 128, 96, 0, 128, scale=0.05)),
