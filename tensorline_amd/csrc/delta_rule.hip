@@ -1,6 +1,6 @@
 // The gated delta rule over a matrix state per head, kept per request between steps:
 //
-//     S <- g_t S;   u_t = beta_t (v_t - S^T k_t);   S <- S + k_t u_t^T;   o_t = S^T q_t
+//     u_t = beta_t (v_t - g_t S_(t-1)^T k_t),   S_t = g_t S_(t-1) + k_t u_t^T,   o_t = S_t^T q_t
 //
 // with beta_t = sigmoid(b_t) and g_t = exp(-exp(rate_log) softplus(a_t + step_bias)), one of each per token and head.
 // Queries and keys come as they enter the rule (unit vectors, scaled), shared by the `share` consecutive value heads of a

@@ -1,7 +1,7 @@
-// The selective scan of Mamba (Gu and Dao, "Mamba: Linear-Time Sequence Modeling with Selective State Spaces"): per
-// channel c and state n, with dt = softplus(dt_raw + dt_bias) per token and channel,
+// The selective scan of Mamba (Gu and Dao, "Mamba: Linear-Time Sequence Modeling with Selective State Spaces"): for
+// each channel, with vectors over its N states and the channel's own dt = softplus(dt_raw + dt_bias), x, z at token t,
 //
-//     S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,   y_c = sum_n S[c, n] C_n + D_c x_c,   out_c = y_c silu(z_c)
+//     S_t = exp(dt_t A) S_(t-1) + (dt_t x_t) B_t,   out_t = (C_t . S_t + D x_t) silu(z_t)
 //
 // S of a request is kept in its slot between steps, [state n][channel].  All arithmetic is float; A comes times log2 e, so
 // that a decay is one v_exp_f32.

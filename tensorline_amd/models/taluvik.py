@@ -10,7 +10,7 @@ norm1(x)``, ``x <- x + m (mixer(h) + ff(h))``.  Each layer has one of three mixe
   itself; a learned sink per head in the softmax's denominator.
 
 Feed-forwards are ``W_down (gelu_tanh(W_gate h) * W_up h)`` or absent.  A layer may run on another layer's weights
-(``weights_of``), with a cache or state of its own: the schedule names that layer again.  Embedding rows enter times
+(``weights_of``) and keeps its own cache or state: the schedule names that layer again.  Embedding rows enter times
 ``embedding.scale``; the head is a matrix of its own behind a final layer norm.  Tensor names: ``embed``, ``l<i>.norm1``
 (``.b``), ``l<i>.mix.*``, ``l<i>.mlp.*``, ``final.norm`` (``.b``), ``head``.
 """

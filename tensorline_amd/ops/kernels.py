@@ -1484,7 +1484,8 @@ def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b: torch.Tenso
                state_offset: int = 0, chunks: SequenceChunks | None = None) -> torch.Tensor:
     """The gated delta rule per sequence and head, with S [dk, dv] in the sequence's slot (kept transposed: ``state[slot,
     state_offset : state_offset + heads * dv * dk]``, float32, renewed in place): with ``beta = sigmoid(b)`` and ``g = exp(-exp(
-    rate_log) softplus(a + step_bias))`` per token and head, ``S <- g S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q``.
+    rate_log) softplus(a + step_bias))`` per token and head, ``w_t = beta_t (v_t - g_t S_(t-1)^T k_t)``,
+    ``S_t = g_t S_(t-1) + k_t w_t^T``, ``o_t = S_t^T q_t``.
 
     ``q``, ``k`` float32 [T, heads / share * dk] as they enter the rule (the ``share`` consecutive heads of a group read the
     same), ``v`` [T, heads * dv], ``b``, ``a`` [T, heads]; all may be column blocks of wider matrices.  With ``chunks`` (and
@@ -1527,8 +1528,8 @@ SELECTIVE_SCAN_MAX_STATE = 256
 def selective_scan(dt_raw: torch.Tensor, dt_bias: torch.Tensor | None, x: torch.Tensor, z: torch.Tensor, bc: torch.Tensor,
                    a2: torch.Tensor, skip: torch.Tensor, ctx, state: torch.Tensor, offset: int,
                    chunks: SequenceChunks | None = None) -> torch.Tensor:
-    """Mamba's selective scan per sequence, channel and state, with its gate: ``dt = softplus(dt_raw + dt_bias)``, ``S[c, n] <-
-    exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n``, result ``(sum_n S[c, n] C_n + skip_c x_c) * silu(z_c)`` in x's dtype.
+    """Mamba's selective scan per sequence, channel and state, with its gate: ``dt = softplus(dt_raw + dt_bias)``, per channel
+    ``S_t = exp(dt_t A) S_(t-1) + (dt_t x_t) B_t`` (over the states), result ``(C_t . S_t + skip x_t) silu(z_t)`` in x's dtype.
 
     ``dt_raw``, ``z`` float32 [T, inner], ``x`` [T, inner] float32 or bfloat16, ``bc`` float32 [T, 2 N] = [B | C] (all may be column
     blocks of wider matrices; ``dt_raw`` is used up: with ``chunks`` it holds ``dt`` afterwards), ``a2`` float32 [N, inner] = ``A^T

@@ -329,11 +329,15 @@ class GatedDeltaRule(Part):
     """The mixer of Gated DeltaNet (Yang, Kautz and Hatamizadeh, "Gated Delta Networks: Improving Mamba2 with Delta Rule").
     Parameters: ``heads`` (value heads), ``kv_heads`` (query/key heads; value head h reads number ``h // (heads /
     kv_heads)``), ``dim`` (query/key size), ``vdim``, ``conv`` (taps), ``eps`` of the output norm, ``unit_eps`` inside the
-    root of the unit vectors' length.  q, k and v each pass a causal convolution per channel and SiLU;  q and k are made
-    unit vectors per head, q also times ``dim^(-1/2)``;  beta = sigmoid(W_b h), g = exp(-exp(A_log) softplus(W_a h +
-    dt_bias)) per head;  S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q;  each head's o is divided by its root
-    mean square, times ``norm`` [vdim] that all heads share, times silu(W_g h), and projected.  The request's slot keeps S
-    of every head (transposed, [heads, vdim, dim]) and, behind it, the convolutions' last ``conv`` - 1 inputs.  Everything
+    root of the unit vectors' length.  Per token t: q, k and v leave their projections through a causal convolution per
+    channel and SiLU; each head of q and k is scaled to length one, q besides by ``dim^(-1/2)``; every value head has a write
+    strength beta_t = sigmoid(b_t) and a decay g_t = exp(-exp(A_log) softplus(a_t + dt_bias)), b_t and a_t from the input;
+
+        w_t = beta_t (v_t - g_t S_(t-1)^T k_t),   S_t = g_t S_(t-1) + k_t w_t^T,   o_t = S_t^T q_t;
+
+    o_t of a head is RMS-normed with ``norm`` [vdim], the same for all heads, gated by SiLU of a projection ``g`` of the input
+    and projected.  The request's slot keeps S of every head (transposed, [heads, vdim, dim]) and, behind it, the
+    convolutions' last ``conv`` - 1 inputs.  Everything
     between the projections and the output norm's result is float32 whatever the engine's dtype.  Tensors under the
     prefix: q, q.conv, k, k.conv, v, v.conv, b, a, A_log, dt_bias, g, norm, o."""
 
@@ -426,10 +430,14 @@ class GatedDeltaRule(Part):
 @register_mixer("selective_scan")
 class SelectiveScan(Part):
     """The mixer of Mamba (Gu and Dao, "Mamba: Linear-Time Sequence Modeling with Selective State Spaces").  Parameters:
-    ``inner`` (channels), ``state`` (N states per channel), ``dt_rank``, ``conv`` (taps).  W_in h = [x: inner | z: inner];  x
-    passes a causal convolution per channel (with bias) and SiLU;  W_x x = [low: dt_rank | B: N | C: N];  dt =
-    softplus(W_dt low + bias) per channel, A = -exp(A_log) [inner, N];  S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,
-    y_c = sum_n S[c, n] C_n + D_c x_c;  y * silu(z) is projected.  The request's slot keeps S ([N, inner]) and, behind it,
+    ``inner`` (channels), ``state`` (N states per channel), ``dt_rank``, ``conv`` (taps).  One projection of the input gives x
+    and the gate z; a causal convolution per channel (with bias) and SiLU make the x that a second projection turns into a
+    low-rank step, B and C (N each); the step passes ``dt`` (with bias) and softplus.  With vectors over a channel's states
+    and A = -exp(A_log),
+
+        S_t = exp(dt_t A) S_(t-1) + (dt_t x_t) B_t,   y_t = (C_t . S_t + D x_t) silu(z_t),
+
+    and y is projected.  The request's slot keeps S ([N, inner]) and, behind it,
     the convolution's last ``conv`` - 1 inputs.  Projections and the convolution leave x in the engine's dtype; the steps,
     the decays, the state and the gate are float32.  Tensors under the prefix: in, conv, conv.b, x, dt, dt.b, A_log, D, o."""
 
