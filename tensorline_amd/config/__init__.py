@@ -7,3 +7,4 @@ from tensorline_amd.config.tumitar_config import TumitarConfig  # noqa: F401
 from tensorline_amd.config.zeganex_config import ZeganexConfig  # noqa: F401
 from tensorline_amd.config.kabulix_config import KabulixConfig  # noqa: F401
 from tensorline_amd.config.taluvik_config import TaluvikConfig  # noqa: F401
+from tensorline_amd.config.vubotar_config import VubotarConfig  # noqa: F401

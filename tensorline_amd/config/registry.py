@@ -80,3 +80,4 @@ def _ensure_builtin() -> None:
     import tensorline_amd.models.zeganex  # noqa: F401
     import tensorline_amd.models.kabulix  # noqa: F401
     import tensorline_amd.models.taluvik  # noqa: F401
+    import tensorline_amd.models.vubotar  # noqa: F401

@@ -12,12 +12,14 @@ void tl_attention_generic_bf16(const AgLaunch& a);
 // cover the longest context; ws holds T * nq * nsplit * (d + 2) floats.  sinks: a float per query head
 // (null: none): exp(sinks[h]) is added to head h's softmax denominator (a key that has no value; neither scaled nor
 // capped).  softcap > 0: score -> softcap tanh(score / softcap).  window, chunk, keep_first: which keys a
-// token sees (TlMask).
+// token sees (TlMask).  bias [nq, reach + 1] (null: none): a number per query head and distance, added to the score after
+// scale and cap (TlBias).
 extern "C" int tl_attention_generic(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                     const int32_t* tables, int NB, const int32_t* q_start, const int32_t* pos,
                                     void* out, int out_stride, int dtype, int T, int S, int max_query_len, int nq, int nkv,
                                     int d, int bs, int window, float scale, int nsplit, int split_keys, float* ws,
-                                    const float* sinks, float softcap, int keep_first, int chunk, hipStream_t stream) {
+                                    const float* sinks, float softcap, int keep_first, int chunk,
+                                    const float* bias, int bias_reach, hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && S >= 0 && nq > 0 && nkv > 0 && d > 0 && bs > 0 && NB > 0,
                  "tl_attention_generic: bad sizes T=%d S=%d nq=%d nkv=%d d=%d page=%d NB=%d", T, S, nq, nkv, d, bs, NB);
     TL_CHECK_ARG(nq % nkv == 0, "tl_attention_generic: %d query heads are not a multiple of %d key/value heads", nq, nkv);
@@ -25,6 +27,7 @@ extern "C" int tl_attention_generic(const void* q, int q_stride, const void* k_c
     TL_CHECK_ARG(nkv <= 65535, "tl_attention_generic: too many key/value heads %d", nkv);
     TL_CHECK_ARG(q_stride >= nq * d && out_stride >= nq * d, "tl_attention_generic: row strides too small");
     TL_CHECK_ARG(window >= 0 && keep_first >= 0 && chunk >= 0 && softcap >= 0.f, "tl_attention_generic: negative window, chunk, kept first keys or cap");
+    TL_CHECK_ARG(bias_reach >= 0, "tl_attention_generic: negative reach of the bias");
     TL_CHECK_ARG(max_query_len >= 1 || T == 0, "tl_attention_generic: max_query_len %d", max_query_len);
     if (T == 0 || S == 0) return 0;
     const int G = nq / nkv;
@@ -56,7 +59,7 @@ extern "C" int tl_attention_generic(const void* q, int q_stride, const void* k_c
     a.tiles_per_seq = tiles_per_seq; a.QT = QT; a.GC = GC; a.nq = nq; a.nkv = nkv; a.d = d; a.bs = bs; a.bs_shift = bs_shift;
     a.mask = TlMask{window, chunk, keep_first}; a.nsplit = nsplit; a.split_keys = split_keys; a.scale = scale; a.keys_over_waves = keys_over_waves;
     a.grid = dim3((unsigned)groups, nkv, chunks * nsplit);
-    a.smem = smem; a.stream = stream; a.sinks = sinks; a.softcap = softcap;
+    a.smem = smem; a.stream = stream; a.sinks = sinks; a.softcap = softcap; a.bias = TlBias{bias, bias_reach};
     if (dtype == TL_F32)
         ag_launch_all<float>(a);
     else if (dtype == TL_BF16)

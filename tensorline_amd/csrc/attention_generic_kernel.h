@@ -100,7 +100,7 @@ __global__ __launch_bounds__(AG_THREADS) void attn_generic_kernel(
     const int32_t* __restrict__ tables, int NB, const int32_t* __restrict__ q_start, const int32_t* __restrict__ pos,
     T* __restrict__ out, int out_stride, int tiles_per_seq, int QT, int GC, int nq, int nkv, int bs, int bs_shift,
     TlMask mask, float scale, int nsplit, int split_keys, float* __restrict__ ws_o, float* __restrict__ ws_ml, const float* __restrict__ sinks,
-    float softcap) {
+    float softcap, TlBias bias) {
     constexpr int d = DB * 16;
     constexpr int KT = AG_KT(d, KW);
     extern __shared__ float smem[];
@@ -317,6 +317,18 @@ __global__ __launch_bounds__(AG_THREADS) void attn_generic_kernel(
 #pragma unroll
                     for (int v = 0; v < 4; ++v) sblk[jb][v] = softcap * tanhf(sblk[jb][v] / softcap);
             }
+            if (bias.table) {                              // a bias by distance, one row of numbers per query head
+#pragma unroll
+                for (int v = 0; v < 4; ++v) {
+                    const int row = (KW ? 0 : wave * AG_WROWS) + 4 * lg + v;
+                    const int g = row % GC;
+                    const float* b = bias.table + (size_t)(kvh * G + g0 + (g < gc ? g : 0)) * (bias.reach + 1);
+#pragma unroll
+                    for (int jb = 0; jb < (KW ? 1 : 4); ++jb)
+                        if (KW || jb < key_blocks)
+                            sblk[jb][v] += b[tl_bias_at(my_pos[v] - (k0 + (KW ? wave : jb) * 16 + li), bias.reach)];
+                }
+            }
             // ---- softmax over the tile, per row; rescale what was summed so far ----------------------
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
@@ -522,6 +534,7 @@ struct AgLaunch {
     int q_stride, NB, out_stride, T, tiles_per_seq, QT, GC, nq, nkv, d, bs, bs_shift, nsplit, split_keys;
     const float* sinks;
     TlMask mask;
+    TlBias bias;
     float scale, softcap;
     bool keys_over_waves;
     dim3 grid;
@@ -540,7 +553,7 @@ static void ag_launch_all(const AgLaunch& a) {
     hipLaunchKernelGGL((attn_generic_kernel<TT, DB, KWV>), a.grid, block, a.smem, a.stream, (const TT*)a.q,           \
                        a.q_stride, (const TT*)a.k_cache, (const TT*)a.v_cache, a.tables, a.NB, a.q_start, a.pos,      \
                        (TT*)a.out, a.out_stride, a.tiles_per_seq, a.QT, a.GC, a.nq, a.nkv, a.bs, a.bs_shift, a.mask,   \
-                       a.scale, a.nsplit, a.split_keys, a.ws_o, a.ws_ml, a.sinks, a.softcap)
+                       a.scale, a.nsplit, a.split_keys, a.ws_o, a.ws_ml, a.sinks, a.softcap, a.bias)
 #define AG_CASE(DB)                                                                                                   \
     case DB:                                                                                                          \
         if (a.keys_over_waves) AG_LAUNCH_KW(DB, true); else AG_LAUNCH_KW(DB, false);                                  \

@@ -69,14 +69,14 @@ __device__ __forceinline__ float am_column_max(float v) {
 
 // One block of 32 keys for the NT column tiles of a wave: scores, online softmax, P*V.
 // Scores and the running maximum are kept in the base-2 domain (score * scale * log2 e), so the
-// exponential is one v_exp_f32; sums and accumulators are float.  CAP: the scores are bent by a cap first
-// (tl_capped; scale2 is then its factor into the exponent and cap2 the cap in the base-2 domain).  Masking is skipped when every
+// exponential is one v_exp_f32; sums and accumulators are float.  MODE: how a product becomes a score (tl_score2);
+// in mode 2 `add` holds what is added to the scores of the lane's eight keys.  Masking is skipped when every
 // key of the block is visible to every column of the wave, the rescaling of the accumulator when
 // no running maximum moved.
-template <int DC, int NT, bool CAP>
+template <int DC, int NT, int MODE>
 __device__ __forceinline__ void am_block(const uint4* kf0, const uint4* kf1, const uint4* vf, const uint4 (*qf)[DC],
                                          const int* p_col, const int* lo_col, int first, int kb, int g, float scale2, float cap2,
-                                         float* m_run, float* l_run, f32x4 (*acc)[DC * 2]) {
+                                         const float (*add)[8], float* m_run, float* l_run, f32x4 (*acc)[DC * 2]) {
     constexpr int DB = DC * 2;
     const int key_base = kb + 8 * g;
 #pragma unroll
@@ -90,8 +90,8 @@ __device__ __forceinline__ void am_block(const uint4* kf0, const uint4* kf1, con
         float sv[8];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            sv[i] = CAP ? tl_capped(st0[i], scale2, cap2) : st0[i] * scale2;
-            sv[4 + i] = CAP ? tl_capped(st1[i], scale2, cap2) : st1[i] * scale2;
+            sv[i] = tl_score2<MODE>(st0[i], scale2, cap2, MODE == 2 ? add[j][i] * AM_LOG2E : 0.f);
+            sv[4 + i] = tl_score2<MODE>(st1[i], scale2, cap2, MODE == 2 ? add[j][4 + i] * AM_LOG2E : 0.f);
         }
         const bool edge = (kb + 31 > p_col[j]) || (kb < lo_col[j]);
         if (__any(edge)) {
@@ -143,13 +143,14 @@ __device__ __forceinline__ int am_page_index(int k, int bs, int bs_shift) {
     return bs_shift >= 0 ? k >> bs_shift : k / bs;
 }
 
-template <int DC, int NT, bool CAP>
+template <int DC, int NT, int MODE>
 __global__ __launch_bounds__(256) void attn_mfma_kernel(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int32_t* __restrict__ tables, int NB, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_start, bf16_t* __restrict__ out, int out_stride, float* __restrict__ ws_o,
     float* __restrict__ ws_ml, int nq, int nkv, int bs, int bs_shift, TlMask mask, float scale, int nsplit,
-    int split_blocks, const int32_t* __restrict__ seq_list, int skip_single, const float* __restrict__ sinks, float softcap) {
+    int split_blocks, const int32_t* __restrict__ seq_list, int skip_single, const float* __restrict__ sinks, float softcap,
+    TlBias bias) {
     constexpr int D = DC * 32;
     constexpr int DB = D / 16;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -160,7 +161,7 @@ __global__ __launch_bounds__(256) void attn_mfma_kernel(
     const int widx = blockIdx.z * (blockDim.x >> 6) + wave;    // one to four waves per work-group
     const int tg = widx / nsplit, sp = widx - tg * nsplit;
     const int G = nq / nkv;
-    const float scale2 = CAP ? 2.0f * AM_LOG2E * scale / softcap : scale * AM_LOG2E;   // see am_block
+    const float scale2 = (MODE != 0 && softcap > 0.f) ? 2.0f * AM_LOG2E * scale / softcap : scale * AM_LOG2E;   // see tl_score2
     const float cap2 = softcap * AM_LOG2E;
     const int r0 = q_start[s];
     const int n = q_start[s + 1] - r0;
@@ -270,9 +271,20 @@ __global__ __launch_bounds__(256) void attn_mfma_kernel(
         const int kb = b << 5;
         const int i_next = (i + 1 < n_blocks) ? i + 1 : i;
         const int b_next = i_next < n_head ? ha + i_next : bb + (i_next - n_head);
+        // what the bias adds to this block's scores is asked for ahead of the next block's keys and values, so that
+        // waiting for it does not wait for those (nearly all of it comes from the nearest cache: a few rows of numbers)
+        float add[NT][8];
+        if (MODE == 2) {
+#pragma unroll
+            for (int j = 0; j < NT; ++j) {
+                const float* brow = bias.table + (size_t)head_col[j] * (bias.reach + 1);
+#pragma unroll
+                for (int x = 0; x < 8; ++x) add[j][x] = brow[tl_bias_at(p_col[j] - (kb + 8 * g + x), bias.reach)];
+            }
+        }
         AM_LOAD_BLOCK(b_next, kn0, kn1, vn)
 
-        am_block<DC, NT, CAP>(kf0, kf1, vf, qf, p_col, lo_col, mask.first, kb, g, scale2, cap2, m_run, l_run, acc);
+        am_block<DC, NT, MODE>(kf0, kf1, vf, qf, p_col, lo_col, mask.first, kb, g, scale2, cap2, add, m_run, l_run, acc);
 #pragma unroll
         for (int dc = 0; dc < DC; ++dc) {
             kf0[dc] = kn0[dc];
@@ -323,10 +335,12 @@ __global__ __launch_bounds__(256) void attn_mfma_kernel(
 // take the same unit of 16 consecutive rows, are spread over all banks (at_k_swizzle, at_v_swizzle).
 // All score tiles first, then the softmax of each column tile, then all P*V products, so that key
 // fragments are dead before value fragments are read: few registers are live at once.
-template <int DC, int NT, bool CAP>
+// brow (mode 2): per column tile, where the row of the column's head in the bias table lies in LDS (base-2 domain).
+template <int DC, int NT, int MODE>
 __device__ __forceinline__ void am_block_lds(const uint4* kt, const uint4* vt, int kx, int vx, int half,
                                              const uint4 (*qf)[DC], const int* p_col, const int* lo_col, int first, int kb,
-                                             int c, int g, float scale2, float cap2, float* m_run, float* l_run, f32x4 (*acc)[DC * 2]) {
+                                             int c, int g, float scale2, float cap2, const float* const* brow, int reach, float* m_run,
+                                             float* l_run, f32x4 (*acc)[DC * 2]) {
     constexpr int DB = DC * 2;
     constexpr int UPK = DC * 4;
     const int key_base = kb + 8 * g;
@@ -349,8 +363,9 @@ __device__ __forceinline__ void am_block_lds(const uint4* kt, const uint4* vt, i
         float sv[8];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            sv[i] = CAP ? tl_capped(st0[j][i], scale2, cap2) : st0[j][i] * scale2;
-            sv[4 + i] = CAP ? tl_capped(st1[j][i], scale2, cap2) : st1[j][i] * scale2;
+            const int n = p_col[j] - key_base - i;
+            sv[i] = tl_score2<MODE>(st0[j][i], scale2, cap2, MODE == 2 ? brow[j][tl_bias_at(n, reach)] : 0.f);
+            sv[4 + i] = tl_score2<MODE>(st1[j][i], scale2, cap2, MODE == 2 ? brow[j][tl_bias_at(n - 4, reach)] : 0.f);
         }
         const bool edge = (kb + 31 > p_col[j]) || (kb < lo_col[j]);
         if (__any(edge)) {
@@ -408,10 +423,12 @@ __device__ __forceinline__ void am_block_lds(const uint4* kt, const uint4* vt, i
 // argument, and the LDS reads ahead of the products that use them: the key fragments of two
 // 32-wide slices of the head are in flight while the products of the slice before run, the value
 // fragments of the first 32 keys while the softmax is computed.
-template <int DC, bool CAP>
+// Mode 2: a tile all of whose keys lie `reach` and more away from every column of the wave gets one number per column.
+template <int DC, int MODE>
 __device__ __forceinline__ void am_tile_lds(const uint4* kt, const uint4* vt, int kx, int vx, const uint4* qf,
                                             int p_col, int lo_col, int first, int kb, int c, int g, float scale2, float cap2,
-                                            float& m_run, float& l_run, f32x4* acc) {
+                                            const float* brow, int reach, float& m_run, float& l_run, f32x4* acc) {
+    constexpr bool CAP = MODE != 0;                          // the scores are made ahead of the maximum
     constexpr int DB = DC * 2;
     constexpr int UPK = DC * 4;
     f32x4 st[4];
@@ -438,8 +455,10 @@ __device__ __forceinline__ void am_tile_lds(const uint4* kt, const uint4* vt, in
     // dims, then those of the last 32.  The first four are on their way during the softmax.
     uint4 vf[4];
 #define AM_VFRAG(I) vt[((((I) % DB) * 16 + c) * 8) + ((4 * ((I) / DB) + g) ^ vx)]
+    if (MODE != 2) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) vf[i] = AM_VFRAG(i);
+        for (int i = 0; i < 4; ++i) vf[i] = AM_VFRAG(i);
+    }
     // A vector instruction may read what a matrix-core instruction wrote only a number of cycles
     // later, and the compiler puts that wait before instructions it knows.  The first readers of
     // the scores below are written as assembly (am_max3), which it does not look into: so the first
@@ -455,7 +474,24 @@ __device__ __forceinline__ void am_tile_lds(const uint4* kt, const uint4* vt, in
 #pragma unroll
     for (int r = 0; r < 4; ++r)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) sv[4 * r + i] = CAP ? tl_capped(st[r][i], scale2, cap2) : st[r][i];
+        for (int i = 0; i < 4; ++i) sv[4 * r + i] = MODE == 1 ? tl_capped(st[r][i], scale2, cap2) : st[r][i];
+    if (MODE == 2) {
+        if (__any(p_col - (kb + 63) < reach)) {
+            int away = p_col - kb - 8 * g;                   // the column's distance from the lane's first key
+            asm volatile("" : "+v"(away));                   // made here: sixteen distances kept across tiles would spill
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    sv[4 * r + i] = tl_score2<2>(sv[4 * r + i], scale2, cap2, brow[tl_bias_at(away - 32 * (r >> 1) - 4 * (r & 1) - i, reach)]);
+        } else {
+            const float far = brow[reach];
+#pragma unroll
+            for (int i = 0; i < 16; ++i) sv[i] = tl_score2<2>(sv[i], scale2, cap2, far);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) vf[i] = AM_VFRAG(i);     // only now: their registers are in use until here
+    }
     const bool edge = (kb + 63 > p_col) || (kb < lo_col);
     if (__any(edge)) {
 #pragma unroll
@@ -561,12 +597,12 @@ __device__ __forceinline__ void at_load_to_lds(const void* g, void* lds_base) {
 // work-group per CU (a short portion behind a long context), where the longest walk sets the time and
 // a lone work-group leaves part of its CU unused.  The chains share the barrier, so they pass a
 // tile's phases together and gain less than two work-groups that drift apart would: 10 to 17%.
-template <int DC, int NT, int WAVES, int CH, bool CAP>
+template <int DC, int NT, int WAVES, int CH, int MODE>
 __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int32_t* __restrict__ tables, int NB, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_start, bf16_t* __restrict__ out, int out_stride, int S, int nq, int nkv, int bs,
-    int bs_shift, TlMask mask, float scale, int skip_single, const float* __restrict__ sinks, float softcap) {
+    int bs_shift, TlMask mask, float scale, int skip_single, const float* __restrict__ sinks, float softcap, TlBias bias) {
     constexpr int THREADS = CH * WAVES * 64;
     constexpr int WCOLS = NT * 16;                       // columns of a wave; WAVES * WCOLS = 128 per work-group
     constexpr int D = DC * 32;
@@ -586,10 +622,11 @@ __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
     const uint32_t vs_lds = ks_lds + 2 * TILE * 16;
     int* tab = reinterpret_cast<int*>(at_smem + CH * 4 * TILE);   // page ids of the sequence, as far as needed (NB ints)
     int* qst = tab + NB;                                   // q_start of the step (S + 1 ints)
+    float* bias_lds = reinterpret_cast<float*>(qst + S + 1);   // mode 2: the group's rows of the bias table, times log2 e
     const int c = lane & 15, g = lane >> 4;
     const int kvh = blockIdx.x;                            // fastest: the heads of a group start together
     const int G = nq / nkv;
-    const float scale2 = CAP ? 2.0f * AM_LOG2E * scale / softcap : scale * AM_LOG2E;   // see am_block
+    const float scale2 = (MODE != 0 && softcap > 0.f) ? 2.0f * AM_LOG2E * scale / softcap : scale * AM_LOG2E;   // see tl_score2
     const float cap2 = softcap * AM_LOG2E;
     // Which (sequence, group of 128 columns) this work-group owns: the grid has one work-group per
     // group that exists (a step mixes a long prompt portion with many one-token sequences, and a
@@ -673,10 +710,15 @@ __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
         const int npages = (khi >> bs_shift) + 1;
         for (int i = tid; i < npages; i += THREADS) tab[i] = table[i];
     }
+    if (MODE == 2) {
+        const float* rows = bias.table + (size_t)kvh * G * (bias.reach + 1);
+        for (int i = tid; i < G * (bias.reach + 1); i += THREADS) bias_lds[i] = rows[i] * AM_LOG2E;
+    }
 
     uint4 qf[NT][DC];
     int p_col[NT], lo_col[NT], row_col[NT], head_col[NT];
     bool has_col[NT];
+    const float* brow[NT];
 #pragma unroll
     for (int j = 0; j < NT; ++j) {
         const int col = col0 + j * 16 + c;
@@ -688,6 +730,7 @@ __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
         has_col[j] = valid;
         p_col[j] = valid ? start + tok : AM_NO_COLUMN;
         lo_col[j] = valid ? tl_mask_lo(mask, p_col[j]) : 0;
+        brow[j] = bias_lds + gh * (bias.reach + 1);
         const bf16_t* qp = q + (size_t)row_col[j] * q_stride + (size_t)head_col[j] * D + g * 8;
 #pragma unroll
         for (int dc = 0; dc < DC; ++dc)
@@ -744,13 +787,13 @@ __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
         const uint4* vt = vs + cur * TILE;                                                                    \
         if (NT == 1 && (T) * AT_KEYS + 32 <= wk_hi && (T) * AT_KEYS + 31 >= wk_lo) {                          \
             /* both halves hold keys of the wave: the whole tile at once */                                   \
-            am_tile_lds<DC, CAP>(kt, vt, kx, vx, qf[0], p_col[0], lo_col[0], first_key, (T) * AT_KEYS, c, g, scale2, cap2, \
-                            m_run[0], l_run[0], acc[0]);                                                      \
+            am_tile_lds<DC, MODE>(kt, vt, kx, vx, qf[0], p_col[0], lo_col[0], first_key, (T) * AT_KEYS, c, g, scale2, cap2, \
+                            brow[0], bias.reach, m_run[0], l_run[0], acc[0]);                                 \
         } else {                                                                                              \
             _Pragma("unroll") for (int half = 0; half < 2; ++half) {                                          \
                 const int kb = (T) * AT_KEYS + half * 32;                                                     \
                 if (kb > wk_hi || (kb + 31 < wk_lo && kb >= first_key)) continue; /* the same for the whole wave */ \
-                am_block_lds<DC, NT, CAP>(kt, vt, kx, vx, half, qf, p_col, lo_col, first_key, kb, c, g, scale2, cap2, m_run, l_run, acc); \
+                am_block_lds<DC, NT, MODE>(kt, vt, kx, vx, half, qf, p_col, lo_col, first_key, kb, c, g, scale2, cap2, brow, bias.reach, m_run, l_run, acc); \
             }                                                                                                 \
         }                                                                                                     \
     }
@@ -848,8 +891,9 @@ __global__ __launch_bounds__(CH * WAVES * 64, 32 / WAVES) void attn_tile_kernel(
 // LDS of the tile kernel for head size 32 * DC, a table of `pages` page ids and S sequences: 64 KB of tiles at
 // head size 128, so two work-groups share a CU's 160 KB up to some 8,000 pages per sequence and one
 // work-group has it alone beyond that
-static size_t at_lds_bytes(int DC, int pages, int S, int chains = 1) {
-    return (size_t)chains * (4 * AT_KEYS * DC * 4) * sizeof(uint4) + (size_t)(pages + S + 1) * sizeof(int);
+// (bias_floats: the rows of the bias table of a group of query heads)
+static size_t at_lds_bytes(int DC, int pages, int S, size_t bias_floats, int chains = 1) {
+    return (size_t)chains * (4 * AT_KEYS * DC * 4) * sizeof(uint4) + (size_t)(pages + S + 1) * sizeof(int) + bias_floats * sizeof(float);
 }
 
 // Merge the splits of one (token, head): M = max m_s, out = sum acc_s e^(m_s - M) / sum l_s e^(m_s - M),
@@ -964,20 +1008,22 @@ static void launch_attn(int NT, dim3 grid, int wg_waves, hipStream_t stream, con
                         const bf16_t* vc, const int32_t* tables, int NB, const int32_t* q_start,
                         const int32_t* ctx_start, bf16_t* out, int out_stride, float* ws_o, float* ws_ml, int nq, int nkv,
                         int bs, TlMask mask, float scale, int nsplit, int split_blocks, const int32_t* seq_list,
-                        int skip_single, const float* sinks, float softcap) {
+                        int skip_single, const float* sinks, float softcap, TlBias bias) {
     int bs_shift = -1;                               // pages of a power of two of tokens: a shift finds the page
     if ((bs & (bs - 1)) == 0)
         for (bs_shift = 0; (1 << bs_shift) < bs;) ++bs_shift;
-#define AM_GO(NTV, CAPV)                                                                                                         \
-    hipLaunchKernelGGL((attn_mfma_kernel<DC, NTV, CAPV>), grid, dim3(64 * wg_waves), 0, stream, q, q_stride, kc, vc, tables, NB, \
+#define AM_GO(NTV, MODEV)                                                                                                        \
+    hipLaunchKernelGGL((attn_mfma_kernel<DC, NTV, MODEV>), grid, dim3(64 * wg_waves), 0, stream, q, q_stride, kc, vc, tables, NB, \
                        q_start, ctx_start, out, out_stride, ws_o, ws_ml, nq, nkv, bs, bs_shift, mask, scale, nsplit,           \
-                       split_blocks, seq_list, skip_single, sinks, softcap)
+                       split_blocks, seq_list, skip_single, sinks, softcap, bias)
     if (NT == 1) {
-        if (softcap > 0.f) AM_GO(1, true);
-        else AM_GO(1, false);
+        if (bias.table) AM_GO(1, 2);
+        else if (softcap > 0.f) AM_GO(1, 1);
+        else AM_GO(1, 0);
     } else {
-        if (softcap > 0.f) AM_GO(2, true);
-        else AM_GO(2, false);
+        if (bias.table) AM_GO(2, 2);
+        else if (softcap > 0.f) AM_GO(2, 1);
+        else AM_GO(2, 0);
     }
 #undef AM_GO
 }
@@ -998,14 +1044,15 @@ static void launch_attn(int NT, dim3 grid, int wg_waves, hipStream_t stream, con
 // total_groups128: the sum over the sequences of ceil(n_s * G / 128), that kernel's grid.
 // sinks: a float per query head (null: none): exp(sinks[h]) is added to head h's softmax denominator (a key that has no
 // value; neither scaled nor capped).  softcap > 0: scores are bent, score -> softcap tanh(score / softcap).
-// window, chunk, keep_first: which keys a token sees (TlMask).
+// window, chunk, keep_first: which keys a token sees (TlMask).  bias [nq, bias_reach + 1] (null: none): a number per query
+// head and distance, added to the score after scale and cap (TlBias).
 extern "C" int tl_attention_mfma(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                  const int32_t* tables, int NB, const int32_t* q_start, const int32_t* ctx_start,
                                  const int32_t* pos, void* out, int out_stride, float* ws_o, float* ws_ml, int T, int S,
                                  int nq, int nkv, int d, int bs, int window, float scale, int NT, int max_tile_groups,
                                  int nsplit, int split_blocks, int shared, int total_groups128,
                                  const int32_t* seq_list, int n_list, int skip_single, const float* sinks, float softcap, int keep_first, int chunk,
-                                 hipStream_t stream) {
+                                 const float* bias_table, int bias_reach, hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && S >= 0 && nq > 0 && nkv > 0 && NB > 0, "tl_attention_mfma: bad sizes T=%d S=%d nq=%d nkv=%d NB=%d", T, S, nq, nkv, NB);
     TL_CHECK_ARG(nq % nkv == 0, "tl_attention_mfma: %d query heads are not a multiple of %d key/value heads", nq, nkv);
     TL_CHECK_ARG(d == 32 || d == 64 || d == 128 || d == 256, "tl_attention_mfma: head size %d is not one of 32, 64, 128, 256", d);
@@ -1013,7 +1060,10 @@ extern "C" int tl_attention_mfma(const void* q, int q_stride, const void* k_cach
     TL_CHECK_ARG(NT == 1 || NT == 2, "tl_attention_mfma: NT=%d must be 1 or 2", NT);
     TL_CHECK_ARG(window >= 0 && keep_first >= 0 && chunk >= 0, "tl_attention_mfma: negative window, chunk or kept first keys");
     TL_CHECK_ARG(softcap >= 0.f, "tl_attention_mfma: negative cap %g", (double)softcap);
+    TL_CHECK_ARG(bias_reach >= 0, "tl_attention_mfma: negative reach of the bias");
     const TlMask mask{window, chunk, keep_first};
+    const TlBias bias{bias_table, bias_reach};
+    const size_t bias_floats = bias_table ? (size_t)(nq / nkv) * (bias_reach + 1) : 0;
     TL_CHECK_ARG(nsplit >= 1 && nsplit <= AM_MAX_SPLITS && max_tile_groups >= 1,
                  "tl_attention_mfma: bad split count %d (at most %d) or group count", nsplit, AM_MAX_SPLITS);
     TL_CHECK_ARG(nsplit == 1 || (ws_o && ws_ml && pos && split_blocks >= 1),
@@ -1041,26 +1091,31 @@ extern "C" int tl_attention_mfma(const void* q, int q_stride, const void* k_cach
     // (a head size of 256 has the independent waves only: its tiles of keys and values would not leave
     // LDS for a second work-group per CU)
     if (NT == 2 && nsplit == 1 && shared && pow2 && !seq_list && total_groups128 > 0 && d != 256 &&
-        at_lds_bytes(d / 32, NB, S) <= 160 * 1024) {
+        at_lds_bytes(d / 32, NB, S, bias_floats) <= 160 * 1024) {
         // 128 columns per work-group, keys and values shared through LDS; shared == 2 asks for two
         // chains per work-group where their tiles fit LDS
         int bs_shift = 0;
         while ((1 << bs_shift) < bs) ++bs_shift;
         TL_CHECK_ARG(total_groups128 <= 65535, "tl_attention_mfma: %d column groups are more than a launch takes", total_groups128);
         dim3 sgrid(nkv, (unsigned)total_groups128, 1);
-        const int chains = (shared == 2 && at_lds_bytes(d / 32, NB, S, 2) <= 160 * 1024) ? 2 : 1;
-        const size_t lds = at_lds_bytes(d / 32, NB, S, chains);
-#define TL_TILE_CASE(DCV) do { if (softcap > 0.f) TL_TILE_GO(DCV, true); else TL_TILE_GO(DCV, false); } while (0)
-#define TL_TILE_GO(DCV, CAPV)                                                                                         \
+        const int chains = (shared == 2 && at_lds_bytes(d / 32, NB, S, bias_floats, 2) <= 160 * 1024) ? 2 : 1;
+        const size_t lds = at_lds_bytes(d / 32, NB, S, bias_floats, chains);
+#define TL_TILE_CASE(DCV)                                                                                             \
+    do {                                                                                                              \
+        if (bias_table) TL_TILE_GO(DCV, 2);                                                                           \
+        else if (softcap > 0.f) TL_TILE_GO(DCV, 1);                                                                   \
+        else TL_TILE_GO(DCV, 0);                                                                                      \
+    } while (0)
+#define TL_TILE_GO(DCV, MODEV)                                                                                        \
     do {                                                                                                              \
         if (chains == 2)                                                                                              \
-            hipLaunchKernelGGL((attn_tile_kernel<DCV, AT_NT, 8 / AT_NT, 2, CAPV>), sgrid, dim3(2 * 64 * 8 / AT_NT), lds,    \
+            hipLaunchKernelGGL((attn_tile_kernel<DCV, AT_NT, 8 / AT_NT, 2, MODEV>), sgrid, dim3(2 * 64 * 8 / AT_NT), lds,    \
                                stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride, \
-                               S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap);                                 \
+                               S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap, bias);                              \
         else                                                                                                          \
-            hipLaunchKernelGGL((attn_tile_kernel<DCV, AT_NT, 8 / AT_NT, 1, CAPV>), sgrid, dim3(64 * 8 / AT_NT), lds,        \
+            hipLaunchKernelGGL((attn_tile_kernel<DCV, AT_NT, 8 / AT_NT, 1, MODEV>), sgrid, dim3(64 * 8 / AT_NT), lds,        \
                                stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride, \
-                               S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap);                                 \
+                               S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap, bias);                              \
     } while (0)
         if (d == 32) TL_TILE_CASE(1);
         else if (d == 64) TL_TILE_CASE(2);
@@ -1072,16 +1127,16 @@ extern "C" int tl_attention_mfma(const void* q, int q_stride, const void* k_cach
     }
     if (d == 32)
         launch_attn<1>(NT, grid, wg_waves, stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride,
-                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap);
+                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap, bias);
     else if (d == 64)
         launch_attn<2>(NT, grid, wg_waves, stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride,
-                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap);
+                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap, bias);
     else if (d == 128)
         launch_attn<4>(NT, grid, wg_waves, stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride,
-                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap);
+                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap, bias);
     else
         launch_attn<8>(NT, grid, wg_waves, stream, qq, q_stride, kk, vv, tables, NB, q_start, ctx_start, (bf16_t*)out, out_stride,
-                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap);
+                       ws_o, ws_ml, nq, nkv, bs, mask, scale, nsplit, split_blocks, seq_list, skip_single, sinks, softcap, bias);
     TL_CHECK_LAUNCH("tl_attention_mfma");
     if (nsplit > 1) {
         const int merge_rows = seq_list ? n_list : T;

@@ -161,14 +161,29 @@ __device__ __forceinline__ void t32_weighted_sum(const uint4* vt, const int* vof
 // by more than T32_LAZY, so probabilities stay below 2^T32_LAZY and the accumulator is rescaled in
 // few tiles instead of most.  Sums and accumulators stay relative to the same running maximum, so
 // the result is the same.
-template <bool CAP>
+template <int MODE>
 __device__ __forceinline__ float t32_softmax(const t32_f32x16* sc, bool edge, int p_col, int lo_col, int first, int kb, int h,
-                                             float scale2, float cap2, float& m_run, float& l_run, uint4* pf) {
+                                             float scale2, float cap2, const float* brow, int reach, float& m_run, float& l_run,
+                                             uint4* pf) {
+    constexpr bool CAP = MODE != 0;                          // the scores are made ahead of the maximum
     float sv[32];
 #pragma unroll
     for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int r = 0; r < 16; ++r) sv[16 * t + r] = CAP ? tl_capped(sc[t][r], scale2, cap2) : sc[t][r];
+        for (int r = 0; r < 16; ++r) sv[16 * t + r] = MODE == 1 ? tl_capped(sc[t][r], scale2, cap2) : sc[t][r];
+    if (MODE == 2) {
+        // brow: the row of the column's head in the bias table, in LDS and in the base-2 domain; a tile all of whose keys lie
+        // `reach` and more away from every column of the wave gets one number per column
+        if (__any(p_col - (kb + T32_KEYS - 1) < reach)) {
+#pragma unroll
+            for (int x = 0; x < 32; ++x)
+                sv[x] = tl_score2<2>(sv[x], scale2, cap2, brow[tl_bias_at(p_col - (kb + 16 * (x >> 3) + 8 * h + (x & 7)), reach)]);
+        } else {
+            const float far = brow[reach];
+#pragma unroll
+            for (int x = 0; x < 32; ++x) sv[x] = tl_score2<2>(sv[x], scale2, cap2, far);
+        }
+    }
     if (edge) {                                              // some key of the tile is hidden from some column of the wave
 #pragma unroll
         for (int x = 0; x < 32; ++x) {
@@ -216,12 +231,12 @@ __device__ __forceinline__ float t32_softmax(const t32_f32x16* sc, bool edge, in
 // [S, NB]; q_start [S + 1]; ctx_start [S]; out [T, nq * D] (row stride out_stride).  Grid: (nkv,
 // sum over the sequences of ceil(n_s * G / (32 WAVES))): one work-group per group of columns that
 // exists.  bs = 2^bs_shift >= 8.  skip_single: sequences of one token belong to another launch.
-template <int DC, int WAVES, bool CAP>
+template <int DC, int WAVES, int MODE>
 __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int32_t* __restrict__ tables, int NB, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_start, bf16_t* __restrict__ out, int out_stride, int S, int nq, int nkv, int bs,
-    int bs_shift, TlMask mask, float scale, int skip_single, const float* __restrict__ sinks, float softcap) {
+    int bs_shift, TlMask mask, float scale, int skip_single, const float* __restrict__ sinks, float softcap, TlBias bias) {
     constexpr int THREADS = WAVES * 64;
     constexpr int WGC = WAVES * 32;           // columns of a work-group
     constexpr int D = DC * 32, KS = D / 16, DT = D / 32;
@@ -235,13 +250,14 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
     uint4* vs = t32_smem + 2 * TILE;                       // [2][TILE]
     int* tab = reinterpret_cast<int*>(vs + 2 * TILE);      // page ids of the sequence, as far as needed (NB ints)
     int* qst = tab + NB;                                   // q_start of the step (S + 1 ints)
+    float* bias_lds = reinterpret_cast<float*>(qst + S + 1);   // mode 2: the group's rows of the bias table, times log2 e
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int n32 = lane & 31, h = lane >> 5;
     const int kvh = blockIdx.x;                            // fastest: the heads of a group start together
     const int G = nq / nkv;
     // capped scores: the factor into tl_capped's exponent, and the cap in the base-2 domain
-    const float scale2 = CAP ? 2.0f * T32_LOG2E * scale / softcap : scale * T32_LOG2E;
+    const float scale2 = (MODE != 0 && softcap > 0.f) ? 2.0f * T32_LOG2E * scale / softcap : scale * T32_LOG2E;
     const float cap2 = softcap * T32_LOG2E;
     // Which (sequence, group of WGC columns) this work-group owns.  Within a sequence the groups
     // with the most keys (the last columns) come first.
@@ -303,6 +319,10 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
         const int npages = (khi >> bs_shift) + 1;
         for (int i = tid; i < npages; i += THREADS) tab[i] = table[i];
     }
+    if (MODE == 2) {
+        const float* rows = bias.table + (size_t)kvh * G * (bias.reach + 1);
+        for (int i = tid; i < G * (bias.reach + 1); i += THREADS) bias_lds[i] = rows[i] * T32_LOG2E;
+    }
 
     // Loader.  A K tile is 64 rows x UPK units, a V^T tile D rows x 8 units: UPK wave-loads of 64
     // consecutive units each, wave w issuing numbers w, w + WAVES, ...  Load number L of K holds
@@ -339,6 +359,7 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
     const int row_out = r0 + tok, head = kvh * G + gh;
     const int p_col = valid ? start + tok : T32_NO_COLUMN;
     const int lo_col = valid ? tl_mask_lo(mask, p_col) : 0;
+    const float* brow = bias_lds + gh * (bias.reach + 1);
     uint4 qf[KS];
     {
         const bf16_t* qp = q + (size_t)row_out * q_stride + (size_t)head * D + h * 8;
@@ -407,7 +428,7 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
             t32_f32x16 sc[2];
             uint4 pf[4];
             t32_scores<DC>(ks + cur * TILE, koff, qf, sc);
-            const float factor = t32_softmax<CAP>(sc, edge, p_col, lo_col, mask.first, kb, h, scale2, cap2, m_run, l_run, pf);
+            const float factor = t32_softmax<MODE>(sc, edge, p_col, lo_col, mask.first, kb, h, scale2, cap2, brow, bias.reach, m_run, l_run, pf);
             if (__any(factor != 1.0f)) {                     // some column's maximum moved
 #pragma unroll
                 for (int m = 0; m < DT; ++m)
@@ -441,17 +462,17 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_tile32_kernel(
         }
 }
 
-// LDS of the kernel for head size d, a table of `pages` page ids and S sequences: 64 KB of tiles
-// at a head size of 128
-static size_t t32_lds_bytes(int d, int pages, int S) {
-    return (size_t)(4 * T32_KEYS * (d / 8)) * sizeof(uint4) + (size_t)(pages + S + 1) * sizeof(int);
+// LDS of the kernel for head size d, a table of `pages` page ids, S sequences and bias_floats numbers of a group's rows of
+// the bias table: 64 KB of tiles at a head size of 128
+static size_t t32_lds_bytes(int d, int pages, int S, int bias_floats) {
+    return (size_t)(4 * T32_KEYS * (d / 8)) * sizeof(uint4) + (size_t)(pages + S + 1) * sizeof(int) + (size_t)bias_floats * sizeof(float);
 }
 
 // Whether the kernel takes a step: head size 64 or 128, pages of a power of two of at least 8
-// tokens, and a page table that fits LDS beside the tiles.
-extern "C" int tl_attention_tile32_takes(int d, int bs, int NB, int S, int waves) {
+// tokens, and a page table (and a group's rows of the bias table) that fit LDS beside the tiles.
+extern "C" int tl_attention_tile32_takes(int d, int bs, int NB, int S, int waves, int bias_floats) {
     return (d == 64 || d == 128) && bs >= 8 && (bs & (bs - 1)) == 0 && NB > 0 && S >= 0 && (waves == 4 || waves == 8) &&
-           t32_lds_bytes(d, NB, S) <= 160 * 1024;
+           bias_floats >= 0 && t32_lds_bytes(d, NB, S, bias_floats) <= 160 * 1024;
 }
 
 // Columns of a work-group of `waves` waves (4 or 8): the caller sizes the grid with it (total_groups =
@@ -463,10 +484,13 @@ extern "C" int tl_attention_tile32(const void* q, int q_stride, const void* k_ca
                                    void* out, int out_stride, int T, int S, int nq, int nkv, int d, int bs, int window,
                                    float scale, int waves, int total_groups, int skip_single, const float* sinks,
                                    float softcap, int keep_first,
-                                   int chunk, hipStream_t stream) {
+                                   int chunk, const float* bias_table, int bias_reach, hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && S >= 0 && nq > 0 && nkv > 0 && NB > 0, "tl_attention_tile32: bad sizes T=%d S=%d nq=%d nkv=%d NB=%d", T, S, nq, nkv, NB);
     TL_CHECK_ARG(nq % nkv == 0, "tl_attention_tile32: %d query heads are not a multiple of %d key/value heads", nq, nkv);
-    TL_CHECK_ARG(tl_attention_tile32_takes(d, bs, NB, S, waves),
+    TL_CHECK_ARG(bias_reach >= 0 && (long long)(nq / nkv) * (bias_reach + 1) < (1 << 24), "tl_attention_tile32: bad reach %d of the bias", bias_reach);
+    const int bias_floats = bias_table ? (nq / nkv) * (bias_reach + 1) : 0;
+    const TlBias bias{bias_table, bias_reach};
+    TL_CHECK_ARG(tl_attention_tile32_takes(d, bs, NB, S, waves, bias_floats),
                  "tl_attention_tile32: head size %d, page size %d or a page table of %d entries is not served", d, bs, NB);
     TL_CHECK_ARG(q_stride % 8 == 0 && out_stride % 4 == 0 && q_stride >= nq * d && out_stride >= nq * d,
                  "tl_attention_tile32: bad row strides %d, %d", q_stride, out_stride);
@@ -481,13 +505,13 @@ extern "C" int tl_attention_tile32(const void* q, int q_stride, const void* k_ca
     const TlMask mask{window, chunk, keep_first};
     int bs_shift = 0;
     while ((1 << bs_shift) < bs) ++bs_shift;
-    const size_t lds = t32_lds_bytes(d, NB, S);
+    const size_t lds = t32_lds_bytes(d, NB, S, bias_floats);
     dim3 grid(nkv, (unsigned)total_groups, 1);
     const bf16_t *qq = (const bf16_t*)q, *kk = (const bf16_t*)k_cache, *vv = (const bf16_t*)v_cache;
-#define T32_LAUNCH(DCV, WV) do { if (softcap > 0.f) T32_GO(DCV, WV, true); else T32_GO(DCV, WV, false); } while (0)
-#define T32_GO(DCV, WV, CAPV)                                                                                           \
-    hipLaunchKernelGGL((attn_tile32_kernel<DCV, WV, CAPV>), grid, dim3(64 * WV), lds, stream, qq, q_stride, kk, vv, tables, NB, \
-                       q_start, ctx_start, (bf16_t*)out, out_stride, S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap)
+#define T32_LAUNCH(DCV, WV) do { if (bias_table) T32_GO(DCV, WV, 2); else if (softcap > 0.f) T32_GO(DCV, WV, 1); else T32_GO(DCV, WV, 0); } while (0)
+#define T32_GO(DCV, WV, MODEV)                                                                                          \
+    hipLaunchKernelGGL((attn_tile32_kernel<DCV, WV, MODEV>), grid, dim3(64 * WV), lds, stream, qq, q_stride, kk, vv, tables, NB, \
+                       q_start, ctx_start, (bf16_t*)out, out_stride, S, nq, nkv, bs, bs_shift, mask, scale, skip_single, sinks, softcap, bias)
     if (d == 64 && waves == 4) T32_LAUNCH(2, 4);
     else if (d == 64) T32_LAUNCH(2, 8);
     else if (waves == 4) T32_LAUNCH(4, 4);

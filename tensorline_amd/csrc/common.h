@@ -139,6 +139,31 @@ __device__ __forceinline__ float tl_capped(float raw, float to_exp, float cap_ou
     return __builtin_fmaf(-2.0f * cap_out, __builtin_amdgcn_rcpf(1.0f + e), cap_out);
 }
 
+// ---- a bias by distance ----------------------------------------------------------------------------
+// A learned number per query head and distance n = position of the query - position of the key, added to a score after
+// scale and cap: table [nq, reach + 1], the last column for every distance of `reach` and more; null: none.
+struct TlBias {
+    const float* table;
+    int reach;
+};
+__device__ __forceinline__ int tl_bias_at(int distance, int reach) {
+    return distance < 0 ? 0 : distance < reach ? distance : reach;      // (a key ahead of the query is masked anyway)
+}
+
+// A score in the base-2 domain from the bare product of query and key.  MODE 0: raw * scale2; 1: capped (tl_capped, scale2
+// its factor into the exponent, cap2 the cap in the base-2 domain); 2: capped where cap2 > 0, and `add` (in the base-2
+// domain) on top.
+template <int MODE>
+__device__ __forceinline__ float tl_score2(float raw, float scale2, float cap2, float add) {
+    if (MODE == 0) return raw * scale2;
+    if (MODE == 1) return tl_capped(raw, scale2, cap2);
+    if (cap2 > 0.f) {
+        const float e = __builtin_amdgcn_exp2f(raw * scale2);
+        return __builtin_fmaf(-2.0f * cap2, __builtin_amdgcn_rcpf(1.0f + e), cap2 + add);
+    }
+    return __builtin_fmaf(raw, scale2, add);
+}
+
 // ---- host side -----------------------------------------------------------------------------
 // Every C entry point returns 0 on success.  On failure it returns a non-zero code and leaves a
 // message that tl_last_error() hands out; nothing is launched in that case.

@@ -92,7 +92,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
 // neighbours; a group's score is the sum of its two largest scores (of its one score, for groups of one);
 // only experts of the `keep` best groups can be chosen; of those the `top` with the largest scores are,
 // weighted by their scores divided by the sum of the chosen scores (+ 1e-20).  Among equals the lower index
-// wins, for groups and for experts.  A wave per token: lane l holds the scores of experts l, l + 64, ...
+// wins, for groups and for experts.  With `correction` [E] groups and experts are chosen by score + correction, and the
+// weights are made of the scores alone.  A wave per token: lane l holds the scores of experts l, l + 64, ...
 // (at most 16 of them) and, as lane g, the score of group g (groups <= 64).
 __device__ __forceinline__ void moe_wave_best(float& bv, int& be) {   // the largest value over the wave, the lower index among equals
     const int none = 0x7fffffff;
@@ -109,31 +110,32 @@ __device__ __forceinline__ void moe_wave_best(float& bv, int& be) {   // the lar
 template <int SL>      // scores a lane holds: 1 for up to 64 experts, 4 for up to 256, 16 beyond
 __global__ __launch_bounds__(256) void moe_route_grouped_kernel(const float* __restrict__ logits, int ldl,
                                                                 int32_t* __restrict__ ids, float* __restrict__ weights, int T,
-                                                                int E, int top, int groups, int keep) {
+                                                                int E, int top, int groups, int keep, const float* __restrict__ correction) {
     const int lane = threadIdx.x & 63;
     const int t = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
     if (t >= T) return;
     const float* z = logits + (size_t)t * ldl;
     const int none = 0x7fffffff, per = E / groups;
     const int nsl = (E + 63) >> 6;                         // slots in use: the same for the whole wave
-    float s[SL];
+    float s[SL], pick[SL];                                 // scores, and what is chosen by
     int grp[SL];
 #pragma unroll
     for (int sl = 0; sl < SL; ++sl) {
         const int e = lane + 64 * sl;
         const bool real = sl < nsl && e < E;
         s[sl] = real ? 1.0f / (1.0f + expf(-z[e])) : -1.0f;
+        pick[sl] = real ? (correction ? s[sl] + correction[e] : s[sl]) : -INFINITY;
         grp[sl] = real ? e / per : -1;
     }
     // group scores: per group the two largest scores over the wave (a butterfly over pairs (largest, second);
-    // scores lie in (0, 1), -1 stands for none), lane g keeps group g's
+    // -infinity stands for none), lane g keeps group g's
     float my_group = 0.f;
-    for (int g = 0; g < groups; ++g) {
-        float a1 = -1.0f, a2 = -1.0f;
+    for (int g = 0; groups > 1 && g < groups; ++g) {
+        float a1 = -INFINITY, a2 = -INFINITY;
 #pragma unroll
         for (int sl = 0; sl < SL; ++sl) {
             if (sl < nsl && grp[sl] == g) {
-                const float v = s[sl];
+                const float v = pick[sl];
                 a2 = fmaxf(a2, fminf(a1, v));
                 a1 = fmaxf(a1, v);
             }
@@ -144,11 +146,11 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(const float* __r
             a2 = fmaxf(fminf(a1, b1), fmaxf(a2, b2));
             a1 = fmaxf(a1, b1);
         }
-        if (lane == g) my_group = fmaxf(a1, 0.f) + fmaxf(a2, 0.f);
+        if (lane == g) my_group = a2 > -INFINITY ? a1 + a2 : a1;
     }
     // the best groups
-    unsigned long long kept = 0ull;
-    for (int k = 0; k < keep; ++k) {
+    unsigned long long kept = groups == 1 ? 1ull : 0ull;
+    for (int k = 0; groups > 1 && k < keep; ++k) {
         float bv = my_group;
         int be = (lane < groups && !((kept >> lane) & 1ull)) ? lane : none;
         moe_wave_best(bv, be);
@@ -163,8 +165,8 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(const float* __r
         int be = none;
 #pragma unroll
         for (int sl = 0; sl < SL; ++sl) {
-            if (sl < nsl && grp[sl] >= 0 && !((taken >> sl) & 1u) && ((kept >> grp[sl]) & 1ull) && (be == none || s[sl] > bv)) {
-                bv = s[sl];
+            if (sl < nsl && grp[sl] >= 0 && !((taken >> sl) & 1u) && ((kept >> grp[sl]) & 1ull) && (be == none || pick[sl] > bv)) {
+                bv = pick[sl];
                 be = lane + 64 * sl;
             }
         }
@@ -175,6 +177,7 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(const float* __r
             my_id = be;
         }
     }
+    if (correction && lane < top) my_val = 1.0f / (1.0f + expf(-z[my_id]));      // the chosen score without its correction
     const float sum = tl_wave_sum(lane < top ? my_val : 0.f) + 1e-20f;
     if (lane < top) {
         ids[(size_t)t * top + lane] = my_id;
@@ -183,7 +186,7 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(const float* __r
 }
 
 extern "C" int tl_moe_route_grouped(const float* logits, int ldl, int32_t* ids, float* weights, int T, int E, int top,
-                                    int groups, int keep, hipStream_t stream) {
+                                    int groups, int keep, const float* correction, hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && E > 0 && top > 0 && top <= MOE_MAX_TOP && E <= MOE_MAX_EXPERTS && ldl >= E,
                  "tl_moe_route_grouped: bad sizes E=%d top=%d", E, top);
     TL_CHECK_ARG(groups > 0 && groups <= 64 && E % groups == 0 && keep > 0 && keep <= groups && top <= keep * (E / groups),
@@ -191,7 +194,7 @@ extern "C" int tl_moe_route_grouped(const float* logits, int ldl, int32_t* ids, 
     if (T == 0) return 0;
 #define GO(SLV)                                                                                                     \
     hipLaunchKernelGGL(moe_route_grouped_kernel<SLV>, dim3(tl_ceil_div(T, 4)), dim3(256), 0, stream, logits, ldl, ids, \
-                       weights, T, E, top, groups, keep)
+                       weights, T, E, top, groups, keep, correction)
     if (E <= 64) GO(1);
     else if (E <= 256) GO(4);
     else GO(MOE_MAX_EXPERTS / 64);

@@ -329,8 +329,9 @@ extern "C" int tl_gelu_token_gate(const float* z, const void* table, int dtype, 
 }
 
 // ---- latent attention: between the projections and the attention kernel ---------------------------------
-// proj float [T, ldp] holds per token: H query heads of (d plain + r rotated) columns, then the
-// compressed row of `rank` columns and r columns of the one rotated key part all heads share.
+// q float [T, ldq] holds per token H query heads of (d plain + r rotated) columns, down float [T, ldd] the
+// compressed row of `rank` columns and r columns of the one rotated key part all heads share (both may be
+// columns of one wider matrix).
 // Per token (one work-group):
 //   * the compressed row is divided by its root mean square (eps inside the root) and scaled by
 //     norm_w: the latent c;
@@ -342,14 +343,15 @@ extern "C" int tl_gelu_token_gate(const float* z, const void* table, int dtype, 
 //   * the row [c | rotated key part | zeros] of D columns goes into the cache at `slot`, once token-major
 //     ([pages, page, 1, D]) and once with a page's tokens innermost ([pages, 1, D, page]).
 template <typename T>
-__global__ void latent_prepare_kernel(const float* __restrict__ proj, int ldp, const int32_t* __restrict__ pos,
+__global__ void latent_prepare_kernel(const float* __restrict__ q, int ldq, const float* __restrict__ down, int ldd,
+                                      const int32_t* __restrict__ pos,
                                       const float* __restrict__ freq, float mag, const float* __restrict__ norm_w, float eps,
                                       const int32_t* __restrict__ slots, T* __restrict__ q_plain, T* __restrict__ q_lat,
                                       T* __restrict__ k_cache, T* __restrict__ v_cache, int H, int d, int r, int rank, int D,
                                       int page) {
     __shared__ float red[16];
     const int t = blockIdx.x;
-    const float* row = proj + (size_t)t * ldp;
+    const float* row = q + (size_t)t * ldq;
     const float p = (float)pos[t];
     const int half = r / 2;
     // queries
@@ -370,7 +372,7 @@ __global__ void latent_prepare_kernel(const float* __restrict__ proj, int ldp, c
         q_lat[((size_t)t * H + h) * D + rank + c] = tl_from_float<T>(v);
     }
     // the latent and the shared rotated key part
-    const float* kv = row + H * (d + r);
+    const float* kv = down + (size_t)t * ldd;
     float ss = 0.f;
     for (int c = threadIdx.x; c < rank; c += blockDim.x) ss += kv[c] * kv[c];
     ss = tl_block_sum(ss, red);
@@ -396,20 +398,20 @@ __global__ void latent_prepare_kernel(const float* __restrict__ proj, int ldp, c
     }
 }
 
-extern "C" int tl_latent_prepare(const float* proj, int ldp, const int32_t* pos, const float* freq, float mag,
+extern "C" int tl_latent_prepare(const float* q, int ldq, const float* down, int ldd, const int32_t* pos, const float* freq, float mag,
                                  const float* norm_w, float eps, const int32_t* slots, void* q_plain, void* q_lat,
                                  void* k_cache, void* v_cache, int dtype, int T, int H, int d, int r, int rank, int D, int page,
                                  hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && H > 0 && d > 0 && r >= 0 && r % 2 == 0 && rank > 0 && D >= rank + r && page > 0,
                  "tl_latent_prepare: bad sizes H=%d d=%d r=%d rank=%d D=%d", H, d, r, rank, D);
-    TL_CHECK_ARG(ldp >= H * (d + r) + rank + r, "tl_latent_prepare: the projection's rows are too short");
+    TL_CHECK_ARG(ldq >= H * (d + r) && ldd >= rank + r, "tl_latent_prepare: the projections' rows are too short");
     if (T == 0) return 0;
     dim3 grid(T), block(256);
     if (dtype == TL_F32)
-        hipLaunchKernelGGL(latent_prepare_kernel<float>, grid, block, 0, stream, proj, ldp, pos, freq, mag, norm_w, eps, slots,
+        hipLaunchKernelGGL(latent_prepare_kernel<float>, grid, block, 0, stream, q, ldq, down, ldd, pos, freq, mag, norm_w, eps, slots,
                            (float*)q_plain, (float*)q_lat, (float*)k_cache, (float*)v_cache, H, d, r, rank, D, page);
     else if (dtype == TL_BF16)
-        hipLaunchKernelGGL(latent_prepare_kernel<bf16_t>, grid, block, 0, stream, proj, ldp, pos, freq, mag, norm_w, eps, slots,
+        hipLaunchKernelGGL(latent_prepare_kernel<bf16_t>, grid, block, 0, stream, q, ldq, down, ldd, pos, freq, mag, norm_w, eps, slots,
                            (bf16_t*)q_plain, (bf16_t*)q_lat, (bf16_t*)k_cache, (bf16_t*)v_cache, H, d, r, rank, D, page);
     else return tl_fail("tl_latent_prepare: unknown dtype %d", dtype);
     TL_CHECK_LAUNCH("tl_latent_prepare");
@@ -758,7 +760,8 @@ extern "C" int tl_glu(const void* gu, int in_dtype, void* out, int out_dtype, in
 //     sine are float;
 //   * q goes to q_out [T, H*D], every head padded with zeros from d to D; k into the cache at `slot`
 //     ([pages, page, G, D], zeros from d to D); v with a page's tokens innermost ([pages, G, D, page], zeros
-//     from dv to D).  With v_from_k the values are the keys as projected: before norm and rotation.
+//     from dv to D).  With v_from_k the values are the keys as projected: before norm and rotation.  With `first` (float
+//     [T, >= G*dv], row stride ldf) the values are (1 - lam) v + lam first.
 // A work-group per token and a share of the heads (of queries, keys or values, in that order); a wave takes one head at a
 // time, a lane the pairs lane and lane + 64 of it (d <= 256).  A work-group computes the token's cosines and sines once, into
 // LDS.  Steps of many tokens leave the values to a kernel of their own (n_units then ends with the keys): written a token at
@@ -768,7 +771,7 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
     const float* __restrict__ proj, int ldp, const int32_t* __restrict__ pos, const float* __restrict__ wq,
     const float* __restrict__ wk, float eps, const float* __restrict__ freq, float mag, int rot,
     const int32_t* __restrict__ slots, T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache, int H, int G,
-    int d, int dv, int D, int page, int v_from_k, int norm, int halves, int n_units) {
+    int d, int dv, int D, int page, int v_from_k, int norm, int halves, int n_units, const float* __restrict__ first, int ldf, float lam) {
     __shared__ float cs[128], sn[128];
     const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const float* row = proj + (size_t)t * ldp;
@@ -797,6 +800,14 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
             cb[j] = apart ? i + (rot >> 1) : 2 * i + 1;
             raw[2 * j] = ca[j] < n ? x[ca[j]] : 0.f;
             raw[2 * j + 1] = cb[j] < n ? x[cb[j]] : 0.f;
+        }
+        if (first && !is_q && !is_k) {
+            const float* y0 = first + (size_t)t * ldf + head * dv;
+#pragma unroll
+            for (int j = 0; j < 2; ++j) {
+                raw[2 * j] = (1.0f - lam) * raw[2 * j] + (ca[j] < n ? lam * y0[ca[j]] : 0.f);
+                raw[2 * j + 1] = (1.0f - lam) * raw[2 * j + 1] + (cb[j] < n ? lam * y0[cb[j]] : 0.f);
+            }
         }
         if (!is_q && slot < 0) continue;                         // nothing to write for this token (the same for the wave)
         const float* w = norm == 1 ? (is_q ? wq : is_k ? wk : nullptr) : nullptr;
@@ -845,23 +856,28 @@ __global__ __launch_bounds__(256) void head_norm_rotate_store_kernel(
 // lanes neighbouring tokens, so that stores of a page's tokens run together ([pages, G, D, page]).
 template <typename T>
 __global__ __launch_bounds__(256) void head_values_store_kernel(const float* __restrict__ proj, int ldp, int col0, const int32_t* __restrict__ slots,
-                                                                T* __restrict__ v_cache, int n, int G, int dv, int D, int page) {
+                                                                T* __restrict__ v_cache, int n, int G, int dv, int D, int page,
+                                                                const float* __restrict__ first, int ldf, float lam) {
     const int t = blockIdx.x * 16 + (threadIdx.x & 15), g = blockIdx.y;
     if (t >= n) return;
     const int slot = slots[t];
     if (slot < 0) return;
     const size_t base = ((size_t)(slot / page) * G + g) * D * page + slot % page;
     const float* x = proj + (size_t)t * ldp + col0 + g * dv;
+    const float* y0 = first ? first + (size_t)t * ldf + g * dv : nullptr;
     for (int c = 4 * (threadIdx.x >> 4); c < D; c += 64)
 #pragma unroll
         for (int e = 0; e < 4; ++e)
-            if (c + e < D) v_cache[base + (size_t)(c + e) * page] = tl_from_float<T>(c + e < dv ? x[c + e] : 0.f);
+            if (c + e < D)
+                v_cache[base + (size_t)(c + e) * page] =
+                    tl_from_float<T>(c + e >= dv ? 0.f : y0 ? (1.0f - lam) * x[c + e] + lam * y0[c + e] : x[c + e]);
 }
 
 extern "C" int tl_head_norm_rotate_store(const float* proj, int ldp, const int32_t* pos, const float* wq, const float* wk,
                                          float eps, const float* freq, float mag, int rot, const int32_t* slots, void* q_out,
                                          void* k_cache, void* v_cache, int dtype, int T, int H, int G, int d, int dv, int D,
-                                         int page, int v_from_k, int norm, int halves, hipStream_t stream) {
+                                         int page, int v_from_k, int norm, int halves, const float* first, int ldf, float lam,
+                                         hipStream_t stream) {
     TL_CHECK_ARG(T >= 0 && H > 0 && G >= 0 && d > 0 && dv > 0 && D >= d && D >= dv && D <= 256 && page > 0,
                  "tl_head_norm_rotate_store: bad sizes H=%d G=%d d=%d dv=%d D=%d", H, G, d, dv, D);
     TL_CHECK_ARG(rot >= 0 && rot % 2 == 0 && rot <= d && (rot == 0 || freq), "tl_head_norm_rotate_store: %d turned dimensions of %d", rot, d);
@@ -870,6 +886,7 @@ extern "C" int tl_head_norm_rotate_store(const float* proj, int ldp, const int32
                  "tl_head_norm_rotate_store: queries and keys are normed together or not at all, with weights in form 1");
     TL_CHECK_ARG(ldp >= (H + G) * d + (v_from_k ? 0 : G * dv), "tl_head_norm_rotate_store: the projection's rows are too short");
     TL_CHECK_ARG(G == 0 || (slots && k_cache && v_cache), "tl_head_norm_rotate_store: keys need their cache");
+    TL_CHECK_ARG(!first || (!v_from_k && ldf >= G * dv), "tl_head_norm_rotate_store: mixed values are projected ones, with rows of G * dv");
     if (T == 0) return 0;
     const bool values_apart = !v_from_k && G > 0 && G <= 65535 && T >= 64;
     const int units = H + G + (v_from_k || values_apart ? 0 : G);
@@ -877,7 +894,7 @@ extern "C" int tl_head_norm_rotate_store(const float* proj, int ldp, const int32
     TL_CHECK_ARG(grid.y <= 65535, "tl_head_norm_rotate_store: too many heads");
 #define GO(TT)                                                                                                         \
     hipLaunchKernelGGL(head_norm_rotate_store_kernel<TT>, grid, block, 0, stream, proj, ldp, pos, wq, wk, eps, freq, mag, \
-                       rot, slots, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, H, G, d, dv, D, page, v_from_k, norm, halves, units)
+                       rot, slots, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, H, G, d, dv, D, page, v_from_k, norm, halves, units, first, ldf, lam)
     if (dtype == TL_F32) GO(float);
     else if (dtype == TL_BF16) GO(bf16_t);
     else return tl_fail("tl_head_norm_rotate_store: unknown dtype %d", dtype);
@@ -886,9 +903,9 @@ extern "C" int tl_head_norm_rotate_store(const float* proj, int ldp, const int32
         TL_CHECK_LAUNCH("tl_head_norm_rotate_store");
         dim3 vgrid(tl_ceil_div(T, 16), G);
         if (dtype == TL_F32)
-            hipLaunchKernelGGL(head_values_store_kernel<float>, vgrid, block, 0, stream, proj, ldp, (H + G) * d, slots, (float*)v_cache, T, G, dv, D, page);
+            hipLaunchKernelGGL(head_values_store_kernel<float>, vgrid, block, 0, stream, proj, ldp, (H + G) * d, slots, (float*)v_cache, T, G, dv, D, page, first, ldf, lam);
         else
-            hipLaunchKernelGGL(head_values_store_kernel<bf16_t>, vgrid, block, 0, stream, proj, ldp, (H + G) * d, slots, (bf16_t*)v_cache, T, G, dv, D, page);
+            hipLaunchKernelGGL(head_values_store_kernel<bf16_t>, vgrid, block, 0, stream, proj, ldp, (H + G) * d, slots, (bf16_t*)v_cache, T, G, dv, D, page, first, ldf, lam);
     }
     TL_CHECK_LAUNCH("tl_head_norm_rotate_store");
     return 0;

@@ -130,7 +130,8 @@ class DecoderModel:
             carried = fn() if fn is not None else None
         return Intake(carried, bool(getattr(self.final_norm, "adds_share_sums", False)),
                       bool(getattr(self.final_norm, "adds_normed_branch", False)),
-                      bool(getattr(self.final_norm, "adds_scaled_branches", False)))
+                      bool(getattr(self.final_norm, "adds_scaled_branches", False)),
+                      bool(getattr(self.final_norm, "adds_joined_branches", False)))
 
     def _negotiate(self) -> list[Intake | None]:
         """For every schedule entry the intake of whoever runs after it, or None for a block that

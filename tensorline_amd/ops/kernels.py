@@ -192,6 +192,94 @@ def add_scaled_branches(x: torch.Tensor, branches: ScaledBranches) -> None:
     add_layernorm(x, branches, None, None, 0.0, None)
 
 
+@dataclass
+class ExpertRows:
+    """What the chosen experts of every token gave, not yet added up: stands for ``sum_c weights[t, c] * rows[t * top +
+    c]``.  The norm that reads the stream next adds them in its own pass (:func:`join_norms`)."""
+    rows: torch.Tensor       # float32 [T * top, H]
+    weights: torch.Tensor    # float32 [T, top]
+
+
+@dataclass
+class JoinedBranches:
+    """Two residual branches that join the stream together, each with a factor per channel: stands for ``scale1 * y1 +
+    scale2 * y2`` (``y2`` and the factors may be None), still to be added.  A branch may be a product left in its shares of K or
+    :class:`ExpertRows`.  The norms that read the stream next add it in their own pass (:func:`join_norms`)."""
+    y1: "torch.Tensor | ShareSum | ExpertRows"
+    scale1: torch.Tensor | None
+    y2: "torch.Tensor | ShareSum | ExpertRows | None" = None
+    scale2: torch.Tensor | None = None
+
+
+def _branch_args(y, scale, T: int, H: int):
+    """(tensors to check, ctypes arguments) of one branch of :func:`join_norms`."""
+    if y is None:
+        return [], (_ptr(None), 1, ctypes.c_longlong(0), ctypes.c_longlong(0), _ptr(None), _ptr(None))
+    weights, pieces, piece, token = None, 1, 0, H
+    if isinstance(y, ShareSum):
+        t, pieces, piece = y.parts, y.parts.shape[0], T * H
+        _check(t.dim() == 3 and tuple(t.shape[1:]) == (T, H), "join_norms: shares must be [P, T, H]")
+    elif isinstance(y, ExpertRows):
+        t, weights = y.rows, y.weights
+        pieces, piece, token = weights.shape[1], H, weights.shape[1] * H
+        _check(tuple(t.shape) == (T * pieces, H) and tuple(weights.shape) == (T, pieces), "join_norms: experts' rows must be [T * top, H]")
+        _f32(weights, "join_norms weights")
+    else:
+        t = y
+        _check(tuple(t.shape) == (T, H), "join_norms: a branch must have x's shape")
+    _f32(t, "join_norms branch")
+    if scale is not None:
+        _f32(scale, "join_norms scale", H)
+    return [t, weights, scale], (_ptr(t), pieces, ctypes.c_longlong(piece), ctypes.c_longlong(token), _ptr(weights), _ptr(scale))
+
+
+def join_norms(x: torch.Tensor, residual: "torch.Tensor | ShareSum | JoinedBranches | None", weight1: torch.Tensor | None,
+               weight2: torch.Tensor | None, eps: float, out_dtype: torch.dtype | None,
+               rows: torch.Tensor | None = None) -> tuple[torch.Tensor | None, torch.Tensor | None]:
+    """Without ``rows``: ``x += residual`` in place (float32), returns the RMS norm of each row with ``weight1`` and with
+    ``weight2`` (None: not that one).  With ``rows``: the norms of ``x[rows] + residual[rows]``, ``x`` left alone.  Without
+    weights: only the sum."""
+    if not isinstance(residual, JoinedBranches):
+        residual = JoinedBranches(residual, None)
+    _check(x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(), "join_norms: x must be contiguous float32 [T, H]")
+    T, H = x.shape
+    t1, a1 = _branch_args(residual.y1, residual.scale1, T, H)
+    t2, a2 = _branch_args(residual.y2, residual.scale2, T, H)
+    _on_gpu(x, weight1, weight2, rows, *t1, *t2)
+    n = T
+    if rows is not None:
+        _i32(rows, "rows")
+        n = rows.numel()
+    outs = []
+    for w in (weight1, weight2):
+        if w is not None:
+            _f32(w, "join_norms weight", H)
+        outs.append(torch.empty(n, H, dtype=out_dtype, device=x.device) if w is not None else None)
+    _call("tl_join_norms", _ptr(x), *a1, *a2, _ptr(weight1), _ptr(weight2), ctypes.c_float(eps), _ptr(outs[0]), _ptr(outs[1]),
+          _code(outs[0], "join_norms out") if outs[0] is not None else F32, _ptr(rows), n, H, _stream())
+    return outs[0], outs[1]
+
+
+def norm_rows(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """The RMS norm with ``weight`` of the rows of a float32 [T, n] matrix (may be a block of columns of a wider one)."""
+    _on_gpu(x, weight)
+    _check(x.dtype == torch.float32 and x.dim() == 2 and x.stride(1) == 1, "norm_rows: the input must be float32 [T, n]")
+    T, n = x.shape
+    _f32(weight, "norm_rows weight", n)
+    out = torch.empty(T, n, dtype=out_dtype, device=x.device)
+    _call("tl_norm_rows", _ptr(x), x.stride(0) if T > 1 else max(n, x.stride(0)), _ptr(weight), ctypes.c_float(eps), _ptr(out),
+          _code(out, "norm_rows out"), T, n, _stream())
+    return out
+
+
+def scale_cap(z: torch.Tensor, scale: float, cap: float = 0.0) -> torch.Tensor:
+    """``cap * tanh(scale * z / cap)`` of a float32 tensor, written over it; ``cap`` 0: ``scale * z``."""
+    _on_gpu(z)
+    _f32(z, "scale_cap input")
+    _call("tl_scale_cap", _ptr(z), ctypes.c_longlong(z.numel()), ctypes.c_float(scale), ctypes.c_float(cap), _stream())
+    return z
+
+
 def add_layernorm(x: torch.Tensor, residual: "torch.Tensor | ScaledBranches | None", weight: torch.Tensor | None,
                   bias: torch.Tensor | None, eps: float, out_dtype: torch.dtype | None,
                   rows: torch.Tensor | None = None) -> torch.Tensor | None:
@@ -232,7 +320,10 @@ def add_rmsnorm(x: torch.Tensor, residual: "torch.Tensor | ShareSum | None", wei
     """Without ``rows``: ``x += residual`` in place (float32), returns ``RMSNorm(x) * weight``.
     With ``rows``: returns the norm of ``x[rows] + residual[rows]`` and leaves ``x`` alone.
     ``residual`` may be a :class:`ShareSum`: its shares are added in order, then to ``x``; or a
-    :class:`NormedBranch`: it is normed first, scaled and added."""
+    :class:`NormedBranch`: it is normed first, scaled and added; or :class:`JoinedBranches`."""
+    if isinstance(residual, JoinedBranches):
+        _check(out is None, "add_rmsnorm: joined branches come with an output of its own")
+        return join_norms(x, residual, weight, None, eps, out_dtype, rows)[0]
     if isinstance(residual, NormedBranch):
         _check(out is None, "add_rmsnorm: a normed branch comes with an output of its own")
         return _branch_norm_add(x, residual, weight, eps, out_dtype, rows)
@@ -861,7 +952,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     path: str | None = None, split_keys: int | None = None,
                     single_seqs: torch.Tensor | None = None, route_singles: bool | None = None,
                     sink: torch.Tensor | None = None, keep_first: int = 0, chunk: int = 0,
-                    softcap: float = 0.0) -> torch.Tensor:
+                    softcap: float = 0.0, bias: torch.Tensor | None = None) -> torch.Tensor:
     """Causal attention of each token over the cached keys of its sequence.
 
     ``q``: [T, >= nq*d] with the query heads in the first nq*d columns (row stride free);
@@ -874,7 +965,8 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     begin.  ``softcap`` > 0 bends the
     scores: ``softcap * tanh(s / softcap)``.  ``sink`` (float32 [nq]) adds ``exp(sink_h)`` to the denominator of head h's
     softmax, a key that has no value (its logit is neither scaled nor capped): ``p_j = exp(s_j) / (exp(sink_h) + sum
-    exp(s))``.  Returns [T, nq*d].
+    exp(s))``.  ``bias`` (float32 [nq, reach + 1]) adds ``bias[h, min(i - j, reach)]`` to head h's score of the key at j for
+    the token at i, after scale and cap.  Returns [T, nq*d].
 
     bfloat16 with a head size of 32, 64 or 128 and pages of a multiple of 8 tokens runs on the
     matrix cores; that kernel works per sequence and needs ``q_start`` [S+1], ``ctx_start`` [S]
@@ -896,6 +988,12 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     if sink is not None:
         _f32(sink, "paged_attention sink", num_heads)
     cap = ctypes.c_float(softcap)
+    reach = 0
+    if bias is not None:
+        _on_gpu(q, bias)
+        _check(bias.dim() == 2 and bias.shape[0] == num_heads and bias.shape[1] >= 1, "paged_attention: the bias must be [nq, reach + 1]")
+        _f32(bias, "paged_attention bias")
+        reach = bias.shape[1] - 1
     T = q.shape[0]
     _check(q.dim() == 2 and q.stride(1) == 1 and q.shape[1] >= num_heads * head_dim, "paged_attention: bad query layout")
     _check_caches(k_cache, v_cache, q.dtype, num_kv_heads, head_dim, "paged_attention")
@@ -938,7 +1036,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                       _ptr(q_start), _ptr(ctx_start), _ptr(pos), _ptr(out), o_stride, _ptr(ws[:n_o]), _ptr(ws[n_o:]), T, S,
                       num_heads, num_kv_heads, head_dim, page, int(window), ctypes.c_float(scale), nt1,
                       -(-G // (16 * nt1)), nsplit, max(split_len // 32, 1), 0, 0, _ptr(single_seqs), len(singles), 0,
-                      _ptr(sink), cap, keep_first, chunk, _stream())
+                      _ptr(sink), cap, keep_first, chunk, _ptr(bias), reach, _stream())
                 skip_single = 1
         q_lens = [n for n in plan.q_lens if n > 1] if skip_single else plan.q_lens
         nt = 1 if plan.max_query_len * G <= 16 or head_dim == 256 else 2
@@ -963,21 +1061,22 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
             ws_o, ws_ml = ws[:T * num_heads * nsplit * head_dim], ws[T * num_heads * nsplit * head_dim:]
         waves = 8 if path == "mfma-tile32" else _tile32_waves(plan.q_lens, plan.starts, num_heads) if path in (None, "mfma") else 0
         if (waves and nt == 2 and nsplit == 1 and total128 > 0
-                and library().tl_attention_tile32_takes(head_dim, page, tables.shape[1], S, waves)):
+                and library().tl_attention_tile32_takes(head_dim, page, tables.shape[1], S, waves, G * (reach + 1) if bias is not None else 0)):
             # prompt portions behind many keys, head size 64 or 128: 32 columns per wave on the 32x32
             # matrix-core instruction, work-groups of 256 columns
             cols = 32 * waves
             total = sum(-(-n * G // cols) for n in q_lens) + pads
             _call("tl_attention_tile32", _ptr(q), q_stride, _ptr(k_cache), _ptr(v_cache), _ptr(tables), tables.shape[1],
                   _ptr(q_start), _ptr(ctx_start), _ptr(out), o_stride, T, S, num_heads, num_kv_heads, head_dim, page,
-                  int(window), ctypes.c_float(scale), waves, total, skip_single, _ptr(sink), cap, keep_first, chunk, _stream())
+                  int(window), ctypes.c_float(scale), waves, total, skip_single, _ptr(sink), cap, keep_first, chunk,
+                  _ptr(bias), reach, _stream())
             return out
         _call("tl_attention_mfma", _ptr(q), q_stride, _ptr(k_cache), _ptr(v_cache), _ptr(tables), tables.shape[1],
               _ptr(q_start), _ptr(ctx_start), _ptr(pos), _ptr(out), o_stride, _ptr(ws_o), _ptr(ws_ml), T, S, num_heads,
               num_kv_heads, head_dim, page, int(window), ctypes.c_float(scale), nt, max_groups, nsplit, split_blocks,
               0 if path == "mfma-direct" else _tile16_chains(total128, num_kv_heads, path, plan.max_context), total128,
               _ptr(None), 0,
-              skip_single, _ptr(sink), cap, keep_first, chunk, _stream())
+              skip_single, _ptr(sink), cap, keep_first, chunk, _ptr(bias), reach, _stream())
         return out
     # The any-shape kernel tiles each sequence's tokens: it needs the first row of every sequence and the
     # most tokens one of them brings.  The engine has both; a bare call derives them from seq_of_token.
@@ -1011,7 +1110,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     _call("tl_attention_generic", _ptr(q), q_stride, _ptr(k_cache), _ptr(v_cache), _ptr(tables), tables.shape[1],
           _ptr(q_start), _ptr(pos), _ptr(out), o_stride, _code(q, "paged_attention"), T, S, max(max_query_len, 1), num_heads,
           num_kv_heads, head_dim, page, int(window), ctypes.c_float(scale), nsplit, split_len, _ptr(ws), _ptr(sink), cap,
-          keep_first, chunk, _stream())
+          keep_first, chunk, _ptr(bias), reach, _stream())
     return out
 
 
@@ -1242,10 +1341,11 @@ def gelu_token_gate(z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, col
 
 def latent_prepare(proj: torch.Tensor, pos: torch.Tensor, freq: torch.Tensor, mag: float, norm_weight: torch.Tensor, eps: float,
                    slots: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, heads: int, dim: int, rot: int,
-                   rank: int) -> tuple[torch.Tensor, torch.Tensor]:
+                   rank: int, q: torch.Tensor | None = None) -> tuple[torch.Tensor, torch.Tensor]:
     """What a latent-attention step does between its projections and the attention kernel.  ``proj``
     float32 [T, >= heads * (dim + rot) + rank + rot]: the query heads (plain part, then the part to
-    rotate), the compressed row and the rotated key part all heads share.  The compressed row is RMS
+    rotate), the compressed row and the rotated key part all heads share; with ``q`` (float32 [T, heads * (dim + rot)]) the
+    query heads are there and ``proj`` begins with the compressed row.  The compressed row is RMS
     normed (``norm_weight``, ``eps``), the rotated parts are turned (pair i with i + rot/2, angle
     ``pos * freq[i]``, cosine and sine times ``mag``), and the row [latent | rotated key | zeros] of D =
     the cache's width goes into both cache planes at ``slots``.  Returns (plain query parts [T, heads *
@@ -1261,9 +1361,16 @@ def latent_prepare(proj: torch.Tensor, pos: torch.Tensor, freq: torch.Tensor, ma
     _f32(norm_weight, "latent_prepare norm weight", rank)
     _i32(pos, "pos", T)
     _i32(slots, "slots", T)
+    down = proj if q is not None else proj[:, heads * (dim + rot):]
+    if q is None:
+        q = proj
+    _on_gpu(proj, q)
+    _check(q.dtype == torch.float32 and q.dim() == 2 and q.stride(1) == 1 and q.shape[0] == T, "latent_prepare: the queries must be float32 [T, n]")
+    _check(q.shape[1] >= heads * (dim + rot) and down.shape[1] >= rank + rot, "latent_prepare: the projections' rows are too short")
+    ld = lambda t: t.stride(0) if T > 1 else max(t.shape[1], t.stride(0))
     q_plain = torch.empty(T, heads * dim, dtype=k_cache.dtype, device=proj.device)
     q_lat = torch.empty(T, heads * D, dtype=k_cache.dtype, device=proj.device)
-    _call("tl_latent_prepare", _ptr(proj), proj.stride(0) if T > 1 else proj.shape[1], _ptr(pos), _ptr(freq), ctypes.c_float(mag),
+    _call("tl_latent_prepare", _ptr(q), ld(q), _ptr(down), ld(down), _ptr(pos), _ptr(freq), ctypes.c_float(mag),
           _ptr(norm_weight), ctypes.c_float(eps), _ptr(slots), _ptr(q_plain), _ptr(q_lat), _ptr(k_cache), _ptr(v_cache),
           _code(k_cache, "latent_prepare cache"), T, heads, dim, rot, rank, D, page, _stream())
     return q_plain, q_lat
@@ -1522,6 +1629,63 @@ def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b: torch.Tenso
     return out
 
 
+def matrix_lstm_state(heads: int, dk: int, dv: int) -> int:
+    """Floats of a request's state for :func:`matrix_lstm`: S transposed [heads, dv, dk], then a copy of n [dk] and one of m
+    for every head and block of 16 value columns."""
+    blocks = -(-dv // 16)
+    return heads * (dv * dk + blocks * (dk + 1))
+
+
+MATRIX_LSTM_MAX_KEY = 256
+
+
+def matrix_lstm(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate_in: torch.Tensor, gate_forget: torch.Tensor,
+                bias_in: torch.Tensor | None, bias_forget: torch.Tensor | None, cap: float, ctx, state: torch.Tensor, heads: int,
+                dk: int, dv: int, q_scale: float = 1.0, floor: float = 1e-6, state_offset: int = 0,
+                chunks: SequenceChunks | None = None) -> torch.Tensor:
+    """The matrix memory of xLSTM per sequence and head, with its state in the sequence's slot (``state[slot, state_offset :
+    state_offset + matrix_lstm_state(..)]``, float32, renewed in place): with the log gates ``i = cap tanh((gate_in + bias_in) /
+    cap)`` and ``f = ln sigmoid(cap tanh((gate_forget + bias_forget) / cap))``, ``m_t = max(f_t + m_(t-1), i_t)``, ``S_t =
+    exp(f_t + m_(t-1) - m_t) S_(t-1) + exp(i_t - m_t) k_t v_t^T``, ``n_t`` likewise with ``k_t`` alone, ``o_t = S_t^T q_t / (max(|n_t . q_t|,
+    exp(-m_t)) + floor)``, queries times ``q_scale``.
+
+    ``q``, ``k`` float32 [T, heads * dk], ``v`` [T, heads * dv], the gates [T, heads]; all may be column blocks of wider
+    matrices.  With ``chunks`` the longer sequences' rows are taken in chunks: the same sums in another order.  Returns float32
+    [T, heads * dv]."""
+    _on_gpu(q, k, v, gate_in, gate_forget, bias_in, bias_forget, state)
+    T = q.shape[0]
+    for name, t, n in (("q", q, heads * dk), ("k", k, heads * dk), ("v", v, heads * dv), ("gate_in", gate_in, heads),
+                       ("gate_forget", gate_forget, heads)):
+        _check(t.dtype == torch.float32 and t.dim() == 2 and t.stride(1) == 1 and tuple(t.shape) == (T, n),
+               f"matrix_lstm: {name} must be float32 [T, {n}]")
+    for name, t in (("bias_in", bias_in), ("bias_forget", bias_forget)):
+        if t is not None:
+            _f32(t, "matrix_lstm " + name, heads)
+    _check(state_offset + matrix_lstm_state(heads, dk, dv) <= state.shape[1], "matrix_lstm: the state of a request is too small")
+    st, stride = _state_ptr(state, state_offset)
+    out = torch.empty(T, heads * dv, dtype=torch.float32, device=q.device)
+    ld = lambda t: t.stride(0) if T > 1 else max(t.shape[1], t.stride(0))
+    head = (_ptr(q), ld(q), _ptr(k), ld(k), _ptr(v), ld(v), _ptr(gate_in), ld(gate_in), _ptr(gate_forget), ld(gate_forget), _ptr(bias_in),
+            _ptr(bias_forget), ctypes.c_float(cap), ctypes.c_float(q_scale), ctypes.c_float(floor), st, ctypes.c_longlong(stride),
+            _ptr(ctx.state_slots), _ptr(ctx.q_start))
+    walk_upto = 0
+    if chunks is not None:
+        _check_chunks(chunks, ctx.num_seqs, "matrix_lstm")
+        fn = library().tl_mlstm_workspace
+        fn.restype = ctypes.c_longlong
+        n = chunks.count * heads
+        ws = torch.empty(n * fn(dk, dv), dtype=torch.float32, device=q.device)
+        ws_g = torch.empty(2 * n, dtype=torch.float64, device=q.device)
+        ws_m = torch.empty(n, dtype=torch.float32, device=q.device)
+        _call("tl_mlstm_chunked", *head, _ptr(chunks.seq), _ptr(chunks.row), _ptr(chunks.first), _ptr(ws), _ptr(ws_g), _ptr(ws_m), _ptr(out),
+              heads * dv, ctx.num_seqs, chunks.count, heads, dk, dv, _stream())
+        if not chunks.walked:
+            return out
+        walk_upto = WALK_TOKENS
+    _call("tl_mlstm_walk", *head, _ptr(out), heads * dv, ctx.num_seqs, heads, dk, dv, walk_upto, _stream())
+    return out
+
+
 SELECTIVE_SCAN_MAX_STATE = 256
 
 
@@ -1570,17 +1734,18 @@ ROUTER_WEIGHTINGS = {"softmax_top": 0, "sigmoid": 1, "softmax_all": 2, "sigmoid_
 
 
 def moe_route(logits: torch.Tensor, top: int, weighting: str = "softmax_top", scale: float = 1.0, experts: int | None = None,
-              groups: int = 1, keep: int = 1) -> tuple[torch.Tensor, torch.Tensor]:
+              groups: int = 1, keep: int = 1, correction: torch.Tensor | None = None) -> tuple[torch.Tensor, torch.Tensor]:
     """Per row of float32 ``logits`` [T, E]: the ``top`` largest (lowest index first among equals), as
     int32 ids [T, top], and their weights, float32 [T, top]: the softmax over those alone
     (``weighting`` "softmax_top"), ``scale * sigmoid(logit)`` of each, not renormalised ("sigmoid"), or their
     shares of the softmax over all E logits, not renormalised ("softmax_all").  "sigmoid_grouped": scores are
     ``sigmoid(logit)``; the experts form ``groups`` equal groups of neighbours, a group's score is the sum of its
     two largest scores, only experts of the ``keep`` best groups can be chosen, and the chosen experts' weights are
-    their scores divided by their sum.  ``experts``: the first so many columns of ``logits`` are the router's
+    their scores divided by their sum; with ``correction`` (float32 [E]) groups and experts are chosen by score +
+    correction, the weights made of the scores alone.  ``experts``: the first so many columns of ``logits`` are the router's
     (default: all of them)."""
     _check(weighting in ROUTER_WEIGHTINGS, f"moe_route: unknown weighting {weighting!r}")
-    _on_gpu(logits)
+    _on_gpu(logits, correction)
     T, E = logits.shape
     if experts is not None:
         _check(0 < experts <= E, "moe_route: more experts than columns")
@@ -1589,10 +1754,14 @@ def moe_route(logits: torch.Tensor, top: int, weighting: str = "softmax_top", sc
     ids = torch.empty(T, top, dtype=torch.int32, device=logits.device)
     weights = torch.empty(T, top, dtype=torch.float32, device=logits.device)
     ldl = logits.stride(0) if T > 1 else logits.shape[1]
+    _check(correction is None or weighting == "sigmoid_grouped", "moe_route: a correction comes with the weighting 'sigmoid_grouped'")
+    if correction is not None:
+        _f32(correction, "moe_route correction", E)
     if weighting == "sigmoid_grouped":
         _check(groups > 0 and E % groups == 0 and 0 < keep <= groups and top <= keep * (E // groups) and groups <= 64,
                f"moe_route: {E} experts in {groups} groups of which {keep} are kept do not give {top} choices")
-        _call("tl_moe_route_grouped", _ptr(logits), ldl, _ptr(ids), _ptr(weights), T, E, int(top), int(groups), int(keep), _stream())
+        _call("tl_moe_route_grouped", _ptr(logits), ldl, _ptr(ids), _ptr(weights), T, E, int(top), int(groups), int(keep),
+              _ptr(correction), _stream())
         return ids, weights
     _call("tl_moe_route", _ptr(logits), ldl, _ptr(ids), _ptr(weights), T, E, int(top),
           ROUTER_WEIGHTINGS[weighting], ctypes.c_float(scale), _stream())
@@ -1606,14 +1775,15 @@ def moe_tile_rows(pairs: int, experts: int) -> int:
 
 def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor,
                 limit: float, alpha: float, shared: torch.Tensor | None = None, shift: float = 1.0,
-                gated: bool = True, shared_gate: torch.Tensor | None = None) -> torch.Tensor:
+                gated: bool = True, shared_gate: torch.Tensor | None = None, keep_rows: bool = False) -> "torch.Tensor | ExpertRows":
     """``out[t] = sum_c weights[t, c] * expert_{ids[t, c]}(h[t]) (+ shared[t])`` in float32, where expert
     e is ``down[e] @ act(gate_up[e] @ h)`` with the gated activation ``g' sigmoid(alpha g') (u' + shift)``,
     ``g' = min(g, limit)``, ``u' = clamp(u, -limit, limit)`` (:func:`clamp_glu` has ``shift`` 1; an infinite
     ``limit`` with ``alpha`` 1 and ``shift`` 0 is ``silu(g) * u``).
     ``gate_up`` [E, 2F, K] (gate rows first), ``down`` [E, N, F]; ``h`` [T, K] in the weights' dtype.
     ``gated`` False: experts without gate, ``down[e] @ relu(up[e] @ h)^2`` with ``gate_up`` = up [E, F, K].
-    ``shared_gate`` float32 [T, 1] (rows may be strided): ``shared[t]`` is multiplied by ``sigmoid(shared_gate[t])``."""
+    ``shared_gate`` float32 [T, 1] (rows may be strided): ``shared[t]`` is multiplied by ``sigmoid(shared_gate[t])``.
+    ``keep_rows`` (without a shared expert): the caller takes the experts' rows as they are, as :class:`ExpertRows`."""
     _on_gpu(h, gate_up, down, ids, weights, shared, shared_gate)
     T, K = h.shape
     E, F2, _ = gate_up.shape
@@ -1638,6 +1808,9 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, ids:
     _call("tl_moe_gemm", _ptr(act), _code(act, "moe_experts"), F, _ptr(down), _code(down, "moe_experts weights"), _ptr(y), F32, N,
           _ptr(order), _ptr(tiles), max_tiles, BM, top, N, F, 0, ctypes.c_float(0.0), ctypes.c_float(0.0), ctypes.c_float(0.0),
           _stream())
+    if keep_rows:
+        _check(shared is None, "moe_experts: the experts' rows are handed on without a shared expert only")
+        return ExpertRows(y, weights)
     out = torch.empty(T, N, dtype=torch.float32, device=h.device)
     ldg = 0
     if shared_gate is not None:
@@ -1743,7 +1916,8 @@ def qk_norm_store(proj: torch.Tensor, pos: torch.Tensor, q_weight: torch.Tensor 
 def head_norm_rotate_store(proj: torch.Tensor, pos: torch.Tensor, q_weight: torch.Tensor | None, k_weight: torch.Tensor | None,
                            eps: float, freq: torch.Tensor | None, mag: float, k_cache: torch.Tensor, v_cache: torch.Tensor,
                            slots: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, values_from_keys: bool,
-                           out_dtype: torch.dtype, plain_norm: bool = False, halves: bool = False) -> torch.Tensor:
+                           out_dtype: torch.dtype, plain_norm: bool = False, halves: bool = False,
+                           first_values: torch.Tensor | None = None, mix: float = 0.0) -> torch.Tensor:
     """What lies between a fused q/k(/v) projection and attention, in one pass per token.  ``proj`` float32 [T,
     heads*dim + kv_heads*dim (+ kv_heads*vdim)] (biases added).  Every query head and key head is RMS-normed over
     its ``dim`` values with a weight per dimension that all heads share (float32 [dim]; both None: no norm, or with
@@ -1752,8 +1926,9 @@ def head_norm_rotate_store(proj: torch.Tensor, pos: torch.Tensor, q_weight: torc
     None: no rotation).  A norm without weights comes to the same ahead of a rotation and behind it.  Keys and values go into the cache pages at ``slots`` (``k_cache``
     [pages, page, kv_heads, D], ``v_cache`` [pages, kv_heads, D, page]), heads padded with zeros to D.
     ``values_from_keys``: there are no value columns; a key head's values are its keys as projected, before norm and
-    rotation.  Returns the queries [T, heads * D] in ``out_dtype``."""
-    _on_gpu(proj, pos, q_weight, k_weight, freq, k_cache, v_cache, slots)
+    rotation.  ``first_values`` (float32 [T, kv_heads * vdim], rows may be strided): the values become ``(1 - mix) v + mix *
+    first_values``.  Returns the queries [T, heads * D] in ``out_dtype``."""
+    _on_gpu(proj, first_values, pos, q_weight, k_weight, freq, k_cache, v_cache, slots)
     T = proj.shape[0]
     D, page = k_cache.shape[3], k_cache.shape[1]
     cols = (heads + kv_heads) * dim + (0 if values_from_keys else kv_heads * vdim)
@@ -1773,11 +1948,17 @@ def head_norm_rotate_store(proj: torch.Tensor, pos: torch.Tensor, q_weight: torc
         rot = 2 * freq.numel()
         _f32(freq, "head_norm_rotate_store frequencies", rot // 2)
         _check(0 < rot <= dim, "head_norm_rotate_store: more turned dimensions than a head has")
+    ldf = 0
+    if first_values is not None:
+        _check(not values_from_keys and first_values.dtype == torch.float32 and first_values.stride(1) == 1
+               and tuple(first_values.shape) == (T, kv_heads * vdim), "head_norm_rotate_store: the values mixed in must be float32 [T, kv_heads * vdim]")
+        ldf = first_values.stride(0) if T > 1 else max(first_values.shape[1], first_values.stride(0))
     q = torch.empty(T, heads * D, dtype=out_dtype, device=proj.device)
     _call("tl_head_norm_rotate_store", _ptr(proj), proj.stride(0) if T > 1 else proj.shape[1], _ptr(pos), _ptr(q_weight),
           _ptr(k_weight), ctypes.c_float(eps), _ptr(freq), ctypes.c_float(mag), rot, _ptr(slots), _ptr(q), _ptr(k_cache),
           _ptr(v_cache), _code(q, "head_norm_rotate_store"), T, heads, kv_heads, dim, vdim, D, page,
-          1 if values_from_keys else 0, 1 if q_weight is not None else 2 if plain_norm else 0, 1 if halves else 0, _stream())
+          1 if values_from_keys else 0, 1 if q_weight is not None else 2 if plain_norm else 0, 1 if halves else 0,
+          _ptr(first_values), ldf, ctypes.c_float(mix), _stream())
     return q
 
 

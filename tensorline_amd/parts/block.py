@@ -33,7 +33,7 @@ import torch
 from tensorline_amd.ops import kernels
 from tensorline_amd.parts.base import Part
 from tensorline_amd.parts.registry import build_part, register_block
-from tensorline_amd.parts.spec import Intake, LayerSpec
+from tensorline_amd.parts.spec import Intake, LayerSpec, TensorDecl
 
 
 @register_block("prenorm")
@@ -250,4 +250,84 @@ class ParallelBranchesBlock:
         if after is not None and after.scaled_branches:
             return branches
         kernels.add_scaled_branches(x, branches)
+        return None
+
+
+class ChannelScale(Part):
+    """A learned factor per channel on what a branch adds to the stream."""
+
+    def __init__(self, hidden_size, prefix, dtype, device, name: str):
+        super().__init__(hidden_size, prefix, dtype, device)
+        self.name = prefix + name
+        self.weight: torch.Tensor | None = None
+
+    def tensors(self):
+        return {self.name: TensorDecl((self.hidden_size,), "one_plus_normal", 0.2, "float32")}
+
+    def load(self, get) -> None:
+        self.weight = get(self.name)
+
+    def weight_tensors(self):
+        return [self.weight]
+
+
+@register_block("parallel_normed_branches")
+class ParallelNormedBranchesBlock:
+    """Two branches side by side on the same stream, each behind an RMS norm of its own and with an optional learned factor per
+    channel on its result (``LayerSpec.channel_scales``):
+
+        x <- x + (s1 * mixer(norm1(x)) + s2 * ffn(norm2(x)))
+
+    The feed-forward (with its norm and factor) may be absent.  Both norms divide by the same root mean square, so one kernel
+    adds what the layer before left, and makes both inputs.  The branches' outputs are not added at once: they are handed on as
+    :class:`tensorline_amd.ops.kernels.JoinedBranches` (the feed-forward's as its experts' rows where it can leave them so), and
+    the norms that read the stream next add both in their own pass.  Where whoever runs next does not take that form
+    (``after.joined_branches``), the block adds them itself and leaves nothing."""
+
+    def __init__(self, spec: LayerSpec, hidden_size: int, dtype, device):
+        common = dict(hidden_size=hidden_size, dtype=dtype, device=device)
+        self.spec = spec
+        self.dtype = dtype
+        self.mixer_norm = build_part("norm", spec.mixer_norm, layer_prefix=spec.prefix, **common)
+        self.mixer = build_part("mixer", spec.mixer, layer_prefix=spec.prefix, **common)
+        self.feed_forward_norm = self.feed_forward = self.mixer_scale = self.feed_forward_scale = None
+        scale = lambda i: ChannelScale(prefix=spec.prefix, name=spec.channel_scales[i], **common) if spec.channel_scales else None
+        self.mixer_scale = scale(0)
+        if spec.feed_forward is not None:
+            self.feed_forward_norm = build_part("norm", spec.feed_forward_norm, layer_prefix=spec.prefix, **common)
+            self.feed_forward = build_part("feed_forward", spec.feed_forward, layer_prefix=spec.prefix, **common)
+            self.feed_forward_scale = scale(1)
+        norms = [n for n in (self.mixer_norm, self.feed_forward_norm) if n is not None]
+        if any(not getattr(n, "adds_joined_branches", False) for n in norms) or len({n.eps for n in norms}) != 1:
+            raise ValueError(f"{spec.prefix}: both norms must be RMS norms of one eps: they share a root mean square")
+
+    def parts(self) -> list[Part]:
+        return [p for p in (self.mixer_norm, self.mixer, self.mixer_scale, self.feed_forward_norm, self.feed_forward,
+                            self.feed_forward_scale) if p is not None]
+
+    def cache_need(self):
+        fn = getattr(self.mixer, "cache_need", None)
+        return fn() if fn is not None else None
+
+    def state_need(self):
+        fn = getattr(self.mixer, "state_need", None)
+        return fn() if fn is not None else None
+
+    def intake(self) -> Intake:
+        return Intake(joined_branches=True)
+
+    def forward(self, x: torch.Tensor, carry, ctx, cache, after: Intake | None = None):
+        ff = self.feed_forward
+        h1, h2 = kernels.join_norms(x, carry, self.mixer_norm.weight, self.feed_forward_norm.weight if ff is not None else None,
+                                    self.mixer_norm.eps, self.dtype)
+        keep = lambda part, flag, kw: {kw: True} if getattr(part, flag, False) else {}
+        weight = lambda scale: scale.weight if scale is not None else None
+        y1 = self.mixer.forward(h1, ctx, cache, **keep(self.mixer, "keeps_share_sums", "keep_shares"))
+        y2 = None
+        if ff is not None:
+            y2 = ff.forward(h2, ctx, **keep(ff, "keeps_share_sums", "keep_shares"), **keep(ff, "keeps_expert_rows", "keep_rows"))
+        branches = kernels.JoinedBranches(y1, weight(self.mixer_scale), y2, weight(self.feed_forward_scale))
+        if after is not None and after.joined_branches:
+            return branches
+        kernels.join_norms(x, branches, None, None, 0.0, None)
         return None

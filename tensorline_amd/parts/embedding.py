@@ -13,7 +13,7 @@ the head that turns normed rows into logits.
 
 Reference: ``x = embed_tokens(ids)`` (tensorline/paged.py:240) and ``lm_head`` on the wanted rows
 (paged.py:278-287); a tied head uses the embedding's table (tensorline/manager.py:65).  The
-embedding takes a scale; a bias or a cap on the logits would be other kinds registered beside these.
+embedding takes a scale, the head a scale and a cap on the logits; a bias would be another kind registered beside these.
 """
 from __future__ import annotations
 
@@ -94,11 +94,15 @@ class BigramEmbedding(TokenEmbedding):
 
 @register_head("lm_head")
 class LMHead(Part):
-    """``logits = h W^T`` without bias, in float32.  ``tied``: W is the embedding's table (shared, not copied)."""
+    """``logits = h W^T`` without bias, in float32.  ``tied``: W is the embedding's table (shared, not copied).  ``scale``: a
+    factor on the logits; ``softcap``: then ``softcap * tanh(logits / softcap)`` (None: no cap)."""
 
     def __init__(self, hidden_size, prefix, dtype, device, vocab_size: int, name: str, tied: bool = False,
-                 std: float = 0.02):
+                 std: float = 0.02, scale: float = 1.0, softcap: float | None = None):
         super().__init__(hidden_size, prefix, dtype, device)
+        self.scale, self.softcap = float(scale), float(softcap or 0.0)
+        if self.softcap < 0.0:
+            raise ValueError(f"{prefix}{name}: the cap {softcap} on the logits must be positive")
         self.vocab_size = int(vocab_size)
         self.name = prefix + name
         self.tied = bool(tied)
@@ -127,4 +131,7 @@ class LMHead(Part):
         return self.linear.shuffled is not None
 
     def forward(self, h) -> torch.Tensor:
-        return self.linear(h, out_dtype=torch.float32)
+        logits = self.linear(h, out_dtype=torch.float32)
+        if self.scale != 1.0 or self.softcap:
+            kernels.scale_cap(logits, self.scale, self.softcap)
+        return logits

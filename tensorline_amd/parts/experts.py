@@ -9,9 +9,10 @@ Other designs change the weights (``weighting`` "sigmoid": each chosen expert by
 softmax over all experts, not renormalised), leave the router without bias, use the plain gated
 activation ``silu(g) * u`` (``activation`` "swiglu": no limit, alpha 1, nothing added to u), or have
 experts without gate, ``W_down relu(W_up h)^2`` (``activation`` "relu2": tensors e<i>.up / .down only).
-``weighting`` "sigmoid_grouped": scores are ``sigmoid(z)``; the experts form ``groups`` equal groups of neighbours, a
+``weighting`` "sigmoid_grouped" (with ``groups`` 1: no groups): scores are ``sigmoid(z)``; the experts form ``groups`` equal groups of neighbours, a
 group's score is the sum of its two largest scores, only experts of the ``keep_groups`` best groups can be chosen,
-and the chosen experts' weights are their scores divided by their sum.  A shared expert has the experts' activation
+and the chosen experts' weights are their scores divided by their sum; with ``correction`` a learned number per expert
+(``correction`` [experts]) is added to the scores for the choice, of groups and experts, and not for the weights.  A shared expert has the experts' activation
 (its ``limit`` only with the clamped one) and, with ``shared`` = {ff, gate: True}, is multiplied by
 ``sigmoid(W_sg h)``, one number per token (``shared.sg`` [1, width]), before it is added.
 
@@ -36,12 +37,13 @@ class RoutedExperts(Part):
     """Parameters: ``experts``, ``top``, ``ff`` and ``limit`` of an expert, ``shared`` = {ff, limit} or
     None, ``alpha`` of the gate's sigmoid; ``weighting`` ("softmax_top", "sigmoid" or "softmax_all"),
     ``router_scale``, ``router_bias``, ``activation`` ("clamped_glu", "swiglu" or "relu2"), ``groups`` and ``keep_groups``
-    (with the weighting "sigmoid_grouped").  Tensors under the prefix: router,
+    (with the weighting "sigmoid_grouped"), ``correction`` (likewise).  Tensors under the prefix: router,
     router.b, e<i>.gate / .up / .down, shared.gate / .up / .down / .sg."""
 
     def __init__(self, hidden_size, prefix, dtype, device, experts: int, top: int, ff: int, limit: float | None = None,
                  shared: dict | None = None, alpha: float = 1.702, weighting: str = "softmax_top", router_scale: float = 1.0,
-                 router_bias: bool = True, activation: str = "clamped_glu", groups: int = 1, keep_groups: int | None = None):
+                 router_bias: bool = True, activation: str = "clamped_glu", groups: int = 1, keep_groups: int | None = None,
+                 correction: bool = False):
         super().__init__(hidden_size, prefix, dtype, device)
         if activation not in ("clamped_glu", "swiglu", "relu2") or weighting not in kernels.ROUTER_WEIGHTINGS:
             raise ValueError(f"{prefix}: unknown activation {activation!r} or weighting {weighting!r}")
@@ -62,6 +64,10 @@ class RoutedExperts(Part):
             raise ValueError(f"{prefix}: {experts} experts do not form {groups} equal groups (at most 64) of which {keep_groups} are kept")
         if self.groups > 1 and weighting != "sigmoid_grouped":
             raise ValueError(f"{prefix}: groups of experts come with the weighting 'sigmoid_grouped'")
+        if correction and weighting != "sigmoid_grouped":
+            raise ValueError(f"{prefix}: a correction of the scores comes with the weighting 'sigmoid_grouped'")
+        self.correction_name = prefix + "correction" if correction else None
+        self.correction: torch.Tensor | None = None
         if int(top) > self.keep_groups * (int(experts) // self.groups):
             raise ValueError(f"{prefix}: {top} choices are more than the {self.keep_groups} kept groups hold")
         self.experts, self.top, self.ff, self.limit, self.alpha = int(experts), int(top), int(ff), float(limit), float(alpha)
@@ -86,6 +92,8 @@ class RoutedExperts(Part):
         out = dict(self.router.tensors())
         if self._token_gate is not None:
             out.update(self._token_gate.tensors())
+        if self.correction_name:
+            out[self.correction_name] = TensorDecl((self.experts,), "normal", 0.3, "float32")
         for e in range(self.experts):
             p = f"{self.prefix}e{e}."
             if self.gated:
@@ -99,6 +107,8 @@ class RoutedExperts(Part):
 
     def load(self, get: TensorGetter) -> None:
         self.router.load(get)
+        if self.correction_name:
+            self.correction = get(self.correction_name)
         if self._token_gate is not None:
             # the gate's one row rides on the router's product: logits [T, experts | gate]
             self._token_gate.load(get)
@@ -121,7 +131,7 @@ class RoutedExperts(Part):
             self.shared_down.prepare()
 
     def weight_tensors(self):
-        out = self.router.tensors_kept() + [self.gate_up, self.down]
+        out = self.router.tensors_kept() + [self.gate_up, self.down] + ([self.correction] if self.correction is not None else [])
         if self.shared_down is not None:
             out += self.shared_gate_up.tensors_kept() + self.shared_down.tensors_kept()
         return out
@@ -131,10 +141,16 @@ class RoutedExperts(Part):
             return []
         return [(self.shared_gate_up.weight, self.dtype), (self.shared_down.weight, torch.float32)]
 
-    def forward(self, h, ctx):
+    @property
+    def keeps_expert_rows(self) -> bool:
+        """Whether ``forward`` takes ``keep_rows`` and then leaves the weighted sum of a token's experts to whoever adds the
+        branch to the stream (:class:`tensorline_amd.ops.kernels.ExpertRows`)."""
+        return self.shared_down is None
+
+    def forward(self, h, ctx, keep_rows: bool = False):
         logits = self.router(h, out_dtype=torch.float32)
         ids, weights = kernels.moe_route(logits, self.top, self.weighting, self.router_scale, experts=self.experts,
-                                         groups=self.groups, keep=self.keep_groups)
+                                         groups=self.groups, keep=self.keep_groups, correction=self.correction)
         shared = None
         if self.shared_down is not None:
             if self.activation == "swiglu":       # SiLU rides on the few-row product, as in the dense feed-forward
@@ -144,4 +160,4 @@ class RoutedExperts(Part):
             shared = self.shared_down(act, out_dtype=torch.float32)
         token_gate = logits[:, self.experts:self.experts + 1] if self.shared_gated else None     # applied where it is added
         return kernels.moe_experts(h, self.gate_up, self.down, ids, weights, self.limit, self.alpha, shared, self.shift,
-                                   gated=self.gated, shared_gate=token_gate)
+                                   gated=self.gated, shared_gate=token_gate, keep_rows=keep_rows)

@@ -16,7 +16,13 @@ designs combine around it:
   ``rotary.rotation_frequencies``); None: positions do not enter the scores;
 * ``softcap``: a score s becomes ``softcap * tanh(s / softcap)`` ahead of the softmax; None: it stays;
 * ``sink``: a learned number per query head (``sink`` [heads]) whose exponential joins the softmax's denominator: a key
-  without value, in sight of every token, whose logit is neither scaled nor capped;
+  without value, in sight of every token, whose logit is neither scaled nor capped; ``sink`` "one": the same with the
+  number 0 for every head (a one in the denominator), nothing learned;
+* ``distance_bias`` = {rows, reach}: a learned number per query head and bucket of distances (``rel`` [rows, heads]) is added
+  to a score after scale and cap; see :func:`distance_buckets`;
+* ``value_mix``: "first": the layer leaves its values of the step's tokens for later layers of the step; "mix": its own
+  values become ``(1 - vmix) v + vmix v_first`` with those, before they are cached (``vmix``, a learned scalar; a layer of
+  kind "first" has one too and does not use it); None;
 * ``gate``: "head": head h's output is multiplied by ``sigmoid(W_g h)_h`` (``g`` [heads, width]); "column": every
   output column by its own gate (``g`` [heads * vdim, width]); None.  The gate reads the mixer's input;
 * ``bias``: q, k (and v) carry biases (``.b``).
@@ -28,6 +34,8 @@ request lives (the pages a window or a chunk has passed, but never those of the 
 """
 from __future__ import annotations
 
+import math
+
 import torch
 
 from tensorline_amd.ops import kernels
@@ -38,6 +46,22 @@ from tensorline_amd.parts.rotary import rotation_frequencies
 from tensorline_amd.parts.spec import CacheNeed, TensorDecl, keys_and_values
 
 MASK_KINDS = ("window", "chunk")
+FIRST_VALUES = "masked_attention.first_values"      # the name under which a step keeps the values later layers mix in
+
+
+def distance_buckets(rows: int, reach: int) -> torch.Tensor:
+    """The row of a table of ``rows`` rows for every distance n = 0 .. ``reach`` (farther ones go where ``reach`` goes): one row
+    per distance below h = rows // 2, from there on ``h + floor(ln(n / h) / ln(reach / h) * (rows - h))``, at most the last
+    row: the bucketing of relative positions of T5 (Raffel et al., "Exploring the Limits of Transfer Learning with a Unified
+    Text-to-Text Transformer") for causal attention."""
+    half = rows // 2
+    if half < 1 or reach <= half:
+        raise ValueError(f"a distance table of {rows} rows needs at least two, and a reach of more than {half}, not {reach}")
+    n = torch.arange(reach + 1, dtype=torch.float64)
+    place = torch.log(n.clamp(min=1.0) / half) / math.log(reach / half) * (rows - half)
+    # the nudge keeps a logarithm that is a whole number but for its last digit on the row it belongs to
+    log_rows = (half + torch.floor(place + 1e-9)).clamp(max=rows - 1)
+    return torch.where(n < half, n, log_rows).long()
 
 
 def read_mask(prefix: str, mask: dict | None) -> tuple[int, int, int]:
@@ -58,7 +82,8 @@ class MaskedAttention(Part):
     def __init__(self, hidden_size, prefix, dtype, device, heads: int, kv_heads: int, dim: int, scale: float,
                  vdim: int | None = None, values: str = "proj", mask: dict | None = None, qk_norm: bool | str = False,
                  eps: float = 1e-6, rot: dict | None = None, gate: str | None = None, bias: bool = False,
-                 softcap: float | None = None, sink: bool = False):
+                 softcap: float | None = None, sink: bool | str = False, distance_bias: dict | None = None,
+                 value_mix: str | None = None):
         super().__init__(hidden_size, prefix, dtype, device)
         self.heads, self.kv_heads, self.dim = int(heads), int(kv_heads), int(dim)
         self.vdim = self.dim if vdim is None else int(vdim)
@@ -84,8 +109,19 @@ class MaskedAttention(Part):
         self.softcap = float(softcap) if softcap else 0.0
         if self.softcap < 0.0:
             raise ValueError(f"{prefix}: the score cap {softcap} must be positive")
-        self.sink_name = prefix + "sink" if sink else None
+        if sink not in (True, False, "one"):
+            raise ValueError(f"{prefix}: sink {sink!r} must be True, False or 'one'")
+        self.sink_name = prefix + "sink" if sink is True else None
         self.sink: torch.Tensor | None = None
+        if sink == "one":
+            self.sink = torch.zeros(self.heads, dtype=torch.float32, device=device)
+        self.rel_name, self.distance_bias = None, None
+        if distance_bias:
+            self.rel_name, self.rel_rows = prefix + "rel", int(distance_bias["rows"])
+            self.buckets = distance_buckets(self.rel_rows, int(distance_bias["reach"]))
+        if value_mix not in (None, "first", "mix") or (value_mix and self.values_from_keys):
+            raise ValueError(f"{prefix}: value_mix {value_mix!r} must be 'first', 'mix' or None, with projected values")
+        self.value_mix, self.vmix = value_mix, 0.0
         self.freq, self.mag, self.halves = None, 1.0, False
         if rot:
             dims = int(rot["dims"])
@@ -120,6 +156,10 @@ class MaskedAttention(Part):
             out[self.prefix + "k.norm"] = TensorDecl((self.dim,), "one_plus_normal", 0.1, "float32")
         if self.sink_name:
             out[self.sink_name] = TensorDecl((self.heads,), "normal", 1.0, "float32")
+        if self.rel_name:
+            out[self.rel_name] = TensorDecl((self.rel_rows, self.heads), "normal", 1.0, "float32")
+        if self.value_mix:
+            out[self.prefix + "vmix"] = TensorDecl((), "normal", 0.5, "float32")
         return out
 
     def load(self, get: TensorGetter) -> None:
@@ -147,9 +187,15 @@ class MaskedAttention(Part):
             self.q_norm, self.k_norm = get(self.prefix + "q.norm"), get(self.prefix + "k.norm")
         if self.sink_name:
             self.sink = get(self.sink_name)
+        if self.rel_name:
+            # a number per head and distance up to the reach
+            rel = get(self.rel_name)
+            self.distance_bias = rel.index_select(0, self.buckets.to(rel.device)).t().contiguous()
+        if self.value_mix == "mix":
+            self.vmix = float(get(self.prefix + "vmix"))
 
     def weight_tensors(self):
-        return self.qkv.tensors_kept() + self.o_proj.tensors_kept() + [t for t in (self.q_norm, self.k_norm, self.freq, self.sink) if t is not None]
+        return self.qkv.tensors_kept() + self.o_proj.tensors_kept() + [t for t in (self.q_norm, self.k_norm, self.freq, self.sink, self.distance_bias) if t is not None]
 
     def library_products(self):
         return [(lin.weight, torch.float32) for lin in (self.qkv, self.o_proj) if lin.weight is not None]
@@ -167,13 +213,19 @@ class MaskedAttention(Part):
     def forward(self, h, ctx, cache):
         keys, values = cache.planes["k"], cache.planes["v"]
         proj = self.qkv(h, out_dtype=torch.float32)
+        first = None
+        if self.value_mix == "first":
+            ctx.shared[FIRST_VALUES] = proj[:, self.qkv_cols - self.kv_heads * self.vdim:self.qkv_cols]
+        elif self.value_mix == "mix":
+            first = ctx.shared[FIRST_VALUES]
         q = kernels.head_norm_rotate_store(proj, ctx.pos, self.q_norm, self.k_norm, self.eps, self.freq, self.mag, keys, values,
                                            cache.slots, self.heads, self.kv_heads, self.dim, self.vdim, self.values_from_keys,
-                                           self.dtype, plain_norm=self.plain_norm, halves=self.halves)
+                                           self.dtype, plain_norm=self.plain_norm, halves=self.halves, first_values=first, mix=self.vmix)
         o = kernels.paged_attention(q, keys, values, cache.tables, ctx.seq_of_token, ctx.pos, self.heads, self.kv_heads,
                                     self.kernel_dim, self.scale, window=self.window, keep_first=self.keep_first,
                                     chunk=self.chunk, q_start=ctx.q_start, ctx_start=ctx.ctx_start, plan=ctx.facts,
-                                    single_seqs=ctx.extra.get("attention.single_seqs"), sink=self.sink, softcap=self.softcap)
+                                    single_seqs=ctx.extra.get("attention.single_seqs"), sink=self.sink, softcap=self.softcap,
+                                    bias=self.distance_bias)
         if self.gate:
             kernels.head_gate(o, proj[:, self.qkv_cols:self.qkv_cols + self.gate_cols], self.gate_cols)
         return self.o_proj(o, out_dtype=torch.float32)

@@ -38,6 +38,7 @@ class RMSNorm(Part):
 
     adds_share_sums = True
     adds_normed_branch = True      # ``forward`` takes a kernels.NormedBranch as the residual
+    adds_joined_branches = True    # .. and a kernels.JoinedBranches
 
     def as_branch(self, y: torch.Tensor, mult: float) -> "kernels.NormedBranch":
         """``mult * norm(y)``, left for the norm that reads the stream next to add in its own pass."""

@@ -3,7 +3,7 @@
 The first ones run on one kernel (``kernels.linear_recurrence``): the state S [heads, key dim, value dim]
 lives in float32 in the request's state slot, starts at zero, and is carried from token to token
 and from step to step; a prompt portion is walked token by token in the order of the sequence.
-``ssd``, ``gated_delta`` and ``selective_scan`` take prompt portions in chunks of tokens instead.
+``ssd``, ``gated_delta``, ``selective_scan`` and ``matrix_lstm`` take prompt portions in chunks of tokens instead.
 
 ``lightning_attention``: linear attention with a fixed decay per head.  With q = silu(W_q h), k =
 silu(W_k h), v = silu(W_v h):  S_t = decay_h S_(t-1) + k_t v_t^T,  o_t = S_t^T q_t;  the heads'
@@ -513,3 +513,94 @@ class SelectiveScan(Part):
         y = kernels.selective_scan(dt, self.dt_bias, x, proj[:, self.inner:2 * self.inner], low[:, self.rank:], self.a2, self.skip,
                                    ctx, cache.state, 0, chunks=kernels.step_chunks(ctx))
         return self.o_proj(y, out_dtype=f32, keep_shares=keep_shares)
+
+
+@register_mixer("matrix_lstm")
+class MatrixLSTM(Part):
+    """The matrix memory of xLSTM (mLSTM; Beck et al., "xLSTM: Extended Long Short-Term Memory").  Parameters: ``heads``, ``dim``
+    (query/key size), ``vdim``, ``gate_cap``, ``eps`` of the output norm, ``floor`` (added to the denominator).  Per head, with
+    q scaled by ``dim^(-1/2)`` and the cap bending both gates' logits:
+
+        i_t = cap tanh((W_i h + b_i) / cap),  f_t = ln sigmoid(cap tanh((W_f h + b_f) / cap)),  m_t = max(f_t + m_(t-1), i_t),
+        S_t = exp(f_t + m_(t-1) - m_t) S_(t-1) + exp(i_t - m_t) k_t v_t^T,   n_t likewise with k_t alone,
+        o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + floor),
+
+    S, n and m zero at the start.  Each head's o is divided by its root mean square; the heads side by side times ``norm``, times
+    ``sigmoid(W_g h)``, are projected.  The request's slot keeps S, n and m of every head.  Everything between the projections and
+    the output norm's result is float32 whatever the engine's dtype.  Tensors under the prefix: q, k, v, i, i.b, f, f.b, g,
+    norm, o."""
+
+    def __init__(self, hidden_size, prefix, dtype, device, heads: int, dim: int, vdim: int, gate_cap: float, eps: float = 1e-6,
+                 floor: float = 1e-6):
+        super().__init__(hidden_size, prefix, dtype, device)
+        self.heads, self.dim, self.vdim = int(heads), int(dim), int(vdim)
+        self.cap, self.eps, self.floor = float(gate_cap), float(eps), float(floor)
+        if min(self.heads, self.dim, self.vdim) <= 0 or self.dim > kernels.MATRIX_LSTM_MAX_KEY:
+            raise ValueError(f"{prefix}: {heads} heads of {dim} x {vdim} are not served (key sizes up to {kernels.MATRIX_LSTM_MAX_KEY})")
+        if self.cap <= 0.0:
+            raise ValueError(f"{prefix}: the gates' cap {gate_cap} must be positive")
+        self.qk, self.vs = self.heads * self.dim, self.heads * self.vdim
+        mk = lambda s, n_in, n_out: Linear(prefix + s, n_in, n_out, False, weight_name=prefix + s)
+        self._parts = [mk("q", hidden_size, self.qk), mk("k", hidden_size, self.qk), mk("v", hidden_size, self.vs),
+                       mk("g", hidden_size, self.vs), mk("i", hidden_size, self.heads), mk("f", hidden_size, self.heads)]
+        self.proj: Linear | None = None
+        self.o_proj = mk("o", self.vs, hidden_size)
+        self.bias_in = self.bias_forget = self.norm_w = None
+
+    def tensors(self):
+        out = {}
+        for lin in self._parts + [self.o_proj]:
+            out.update(lin.tensors())
+        p = self.prefix
+        out[p + "i.b"] = TensorDecl((self.heads,), "normal", 1.0, "float32")
+        out[p + "f.b"] = TensorDecl((self.heads,), "normal", 1.0, "float32")
+        out[p + "norm"] = TensorDecl((self.vs,), "one_plus_normal", 0.1, "float32")
+        return out
+
+    def load(self, get: TensorGetter) -> None:
+        p = self.prefix
+        for lin in self._parts + [self.o_proj]:
+            lin.load(get)
+        parts = list(self._parts)
+        spare = -sum(lin.out_features for lin in parts) % 8
+        if spare:                                  # rows of zeros at the end: the product's rows start at 16-byte borders
+            pad = Linear(p + "pad", self.hidden_size, spare, False)
+            pad.weight = parts[0].weight.new_zeros(spare, self.hidden_size)
+            parts.append(pad)
+        self.proj = fuse_linears(p + "qkvgif", parts)
+        for lin in self._parts:
+            lin.weight = None
+        self.o_proj.prepare()
+        self.bias_in, self.bias_forget, self.norm_w = get(p + "i.b"), get(p + "f.b"), get(p + "norm")
+
+    def weight_tensors(self):
+        return self.proj.tensors_kept() + self.o_proj.tensors_kept() + [self.bias_in, self.bias_forget, self.norm_w]
+
+    def library_products(self):
+        return [(lin.weight, torch.float32) for lin in (self.proj, self.o_proj) if lin is not None and lin.weight is not None]
+
+    def cache_need(self):
+        return None
+
+    def state_need(self):
+        return StateNeed((kernels.matrix_lstm_state(self.heads, self.dim, self.vdim),), "float32")
+
+    step_vectors = staticmethod(kernels.chunk_vectors)
+
+    def input_linear(self) -> Linear:
+        return self.proj
+
+    keeps_share_sums = True
+
+    def forward(self, h, ctx, cache, keep_shares: bool = False):
+        return self.forward_projected(self.proj(h, out_dtype=torch.float32), ctx, cache, keep_shares)
+
+    def forward_projected(self, proj, ctx, cache, keep_shares: bool = False):
+        """``proj`` float32 [T, q | k | v | g | i | f (| padding)]; rows may be strided."""
+        H, qk, vs = self.heads, self.qk, self.vs
+        at = 2 * qk + 2 * vs
+        o = kernels.matrix_lstm(proj[:, :qk], proj[:, qk:2 * qk], proj[:, 2 * qk:2 * qk + vs], proj[:, at:at + H], proj[:, at + H:at + 2 * H],
+                                self.bias_in, self.bias_forget, self.cap, ctx, cache.state, H, self.dim, self.vdim,
+                                q_scale=self.dim ** -0.5, floor=self.floor, chunks=kernels.step_chunks(ctx))
+        y = kernels.gated_group_norm(o, self.norm_w, proj[:, 2 * qk + vs:at], self.vdim, self.eps, "sigmoid", self.dtype)
+        return self.o_proj(y, out_dtype=torch.float32, keep_shares=keep_shares)

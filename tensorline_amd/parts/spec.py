@@ -55,6 +55,8 @@ class LayerSpec:
     mixer_post_norm: PartSpec | None = None
     feed_forward_post_norm: PartSpec | None = None
     branch_scale: float = 1.0
+    # for blocks with a learned factor per channel on each branch: the factors' names below the prefix, mixer's first
+    channel_scales: tuple[str, str] | None = None
 
 
 @dataclass(frozen=True)
@@ -73,11 +75,13 @@ class Intake:
     product left in its shares of K (``tensorline_amd.ops.kernels.ShareSum``).  ``normed_branch``: its
     first norm adds a branch output that is still to be normed and scaled
     (``tensorline_amd.ops.kernels.NormedBranch``).  ``scaled_branches``: its first norm adds up to two branch outputs with
-    one factor (``tensorline_amd.ops.kernels.ScaledBranches``)."""
+    one factor (``tensorline_amd.ops.kernels.ScaledBranches``).  ``joined_branches``: its first norm adds two branch outputs
+    with a factor per channel each (``tensorline_amd.ops.kernels.JoinedBranches``)."""
     normed_rows_for: tuple | None = None
     share_sums: bool = False
     normed_branch: bool = False
     scaled_branches: bool = False
+    joined_branches: bool = False
 
 
 @dataclass(frozen=True)
