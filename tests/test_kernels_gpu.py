@@ -373,13 +373,13 @@ def test_product_adds_into_the_residual_and_prepares_the_next_norm(M, N, Kd):
 
 def _attention_case(dtype, nq, nkv, d, bs, lens, q_lens=None, window=0, seed=0, spike=False, path=None, split_keys=None,
                     route_singles=None, pool_pages=None, spike_at=None, sink=False, spike_gain=4.0, score_shift=0.0,
-                    keep_first=0, chunk=0, softcap=0.0):
+                    keep_first=0, chunk=0, softcap=0.0, bias=None):
     """Sequences of context ``lens``; the last ``q_lens[i]`` positions of each are queries.
     pool_pages: the sequences' pages are the last ones of a pool of that many.  ``spike``: the key
     at position 1 (or at ``spike_at(position of the query)``, if that is a key at all) is made to
     match its query, so that it dominates the sum if it is seen.  ``score_shift``: the first dimension of
     every key and query is set so that it takes that much off every score.  ``sink``: True for a logit of 0 in every head, or
-    the heads' logits; ``softcap``: scores bent by that cap."""
+    the heads' logits; ``softcap``: scores bent by that cap; ``bias`` [nq, reach + 1]: added by distance."""
     torch.manual_seed(seed)
     S = len(lens)
     q_lens = q_lens or [1] * S
@@ -432,7 +432,8 @@ def _attention_case(dtype, nq, nkv, d, bs, lens, q_lens=None, window=0, seed=0, 
                               q_start=torch.tensor(qs, dtype=torch.int32, device=DEV),
                               ctx_start=torch.tensor(plan.starts, dtype=torch.int32, device=DEV), plan=plan,
                               path=path, split_keys=split_keys, single_seqs=single_seqs, route_singles=route_singles,
-                              sink=None if logits is None else logits.to(DEV), keep_first=keep_first, chunk=chunk, softcap=softcap)
+                              sink=None if logits is None else logits.to(DEV), keep_first=keep_first, chunk=chunk, softcap=softcap,
+                              bias=None if bias is None else bias.to(DEV))
     if pool_pages:
         kc, vc, tables = kc[first:], vc[first:], tables - first
     kf, vf = kc.double().cpu().view(-1, nkv, d), vc.double().cpu().permute(0, 3, 1, 2).reshape(-1, nkv, d)
@@ -443,8 +444,8 @@ def _attention_case(dtype, nq, nkv, d, bs, lens, q_lens=None, window=0, seed=0, 
         keys = torch.arange(n)
         rows = tcpu[s][keys // bs] * bs + keys % bs
         qs = q[t0:t0 + ql].double().cpu().view(ql, nq, d)
-        if keep_first or chunk or softcap or (logits is not None and bool(logits.any())):
-            want[t0:t0 + ql] = _masked_attention(qs, kf[rows], vf[rows], d ** -0.5, n - ql, window, keep_first, chunk, softcap, logits)
+        if keep_first or chunk or softcap or bias is not None or (logits is not None and bool(logits.any())):
+            want[t0:t0 + ql] = _masked_attention(qs, kf[rows], vf[rows], d ** -0.5, n - ql, window, keep_first, chunk, softcap, logits, bias)
         else:
             want[t0:t0 + ql] = plain.causal_attention(qs, kf[rows], vf[rows], d ** -0.5, window=window, q_offset=n - ql, sink=sink)
         t0 += ql
@@ -641,10 +642,11 @@ def test_attention_one_token_sequences_beside_prompt_portions(heads, d, bs):
     assert torch.equal(short[0], unrouted[0])                 # short contexts stay with the portions
 
 
-def _masked_attention(q, k, v, scale, q_offset, window, keep_first, chunk, softcap=0.0, logits=None):
+def _masked_attention(q, k, v, scale, q_offset, window, keep_first, chunk, softcap=0.0, logits=None, bias=None):
     """q [n, nq, d] at positions q_offset.., k and v [keys, nkv, d]: the query at position i sees key j <= i if it
     lies in the window (i - j < window) or among the first ``keep_first`` keys, and (with ``chunk``) in i's chunk.
-    ``softcap`` bends the scores, ``logits`` [nq] are one more entry of each head's softmax, without a value."""
+    ``softcap`` bends the scores, ``bias`` [nq, reach + 1] is then added by distance (the last column for all farther keys),
+    ``logits`` [nq] are one more entry of each head's softmax, without a value."""
     n, nq, d = q.shape
     nkv = k.shape[1]
     i = (q_offset + torch.arange(n)).view(n, 1)
@@ -660,6 +662,8 @@ def _masked_attention(q, k, v, scale, q_offset, window, keep_first, chunk, softc
         s = (q[:, h] @ k[:, g].T) * scale
         if softcap:
             s = softcap * torch.tanh(s / softcap)
+        if bias is not None:
+            s = s + bias[h].double()[(i - j).clamp(0, bias.shape[1] - 1)]
         s = s.masked_fill(~seen, float("-inf"))
         if logits is not None:
             s = torch.cat((s, torch.full((n, 1), float(logits[h]), dtype=torch.float64)), dim=1)
@@ -979,4 +983,43 @@ def test_capped_scores_with_chunks_in_portions_and_one_token_steps(path, dtype):
         for chunk in (50, 64, 7):
             got, want = _attention_case(dtype, 4, 2, 64, 16, lens, q_lens, seed=chunk, spike=True, path=path, chunk=chunk, spike_gain=6.0,
                                         spike_at=lambda p: (p // chunk) * chunk, softcap=9.0, sink=logits)
+            torch.testing.assert_close(got, want, **tol(dtype, 3e-5, 2e-2))
+
+
+@pytest.mark.parametrize("case", range(len(SINK_CASES)))
+@pytest.mark.parametrize("reach", [0, 1, 40, 700])
+def test_attention_with_a_bias_by_distance_in_every_kernel(case, reach):
+    """A number per head and distance, the last one for all farther keys, of the scores' size and larger: in every kernel and
+    through every merge, with and without cap and sink; tables that fit LDS beside the tiles and ones that do not."""
+    dtype, nq, nkv, d, bs, lens, q_lens, window, path, split = SINK_CASES[case]
+    torch.manual_seed(case + reach)
+    bias = torch.randn(nq, reach + 1) * 3.0
+    kw = dict(window=window, seed=case + 70, path=path, split_keys=split)
+    tol = 2e-5 if dtype == torch.float32 else 2e-2
+    got, want = _attention_case(dtype, nq, nkv, d, bs, lens, q_lens, softcap=4.0, sink=torch.linspace(-2.0, 3.0, nq) if nq > 1 else torch.tensor([1.0]),
+                                bias=bias, **kw)
+    torch.testing.assert_close(got, want, atol=tol, rtol=tol)
+    got, want = _attention_case(dtype, nq, nkv, d, bs, lens, q_lens, bias=bias, **kw)
+    torch.testing.assert_close(got, want, atol=tol, rtol=tol)
+    plain_scores, _ = _attention_case(dtype, nq, nkv, d, bs, lens, q_lens, **kw)
+    if reach >= 40:
+        assert (got - plain_scores).norm() > 0.1 * plain_scores.norm(), "the bias changed nothing where it must"
+
+
+@pytest.mark.parametrize("path,dtype", MASK_PATHS)
+@pytest.mark.parametrize("window,keep_first", [(44, 5), (100, 70), (0, 0)])
+def test_bias_at_every_distance_with_windows_and_kept_keys(path, dtype, window, keep_first):
+    """One distance at a time stands out by so much that the key there carries the sum: the key itself, its neighbour, tiles'
+    and blocks' borders, the distance before the reach, the reach and beyond it; kept first keys count their true distance."""
+    reach = 90
+    for at in (0, 1, 15, 16, 31, 32, 43, 63, 64, 65, 89, 90):
+        if at and window and at >= window and at < reach:
+            continue
+        bias = torch.randn(4, reach + 1, generator=torch.Generator().manual_seed(at)) * 0.5
+        bias[:, at] += 12.0
+        for lens, q_lens in (([300, 99, 160, 9], [130, 1, 60, 9]), ([120, 333, 64], None)):
+            if q_lens is None and path in ("mfma-tile16", "mfma-tile16x2", "mfma-tile32"):
+                continue
+            got, want = _attention_case(dtype, 4, 2, 64, 16, lens, q_lens, seed=at, path=path, window=window, keep_first=keep_first,
+                                        softcap=9.0, sink=True, bias=bias)
             torch.testing.assert_close(got, want, **tol(dtype, 3e-5, 2e-2))
