@@ -609,6 +609,51 @@ def make_taluvik_twin(size: str):
         rope_theta=10000.0, rms_norm_eps=1e-6, tie_word_embeddings=False, max_position_embeddings=32768))
 
 
+# ---- the Vubotar design beside the Kabulix decoder at equal size --------------------------------------
+# Layer sizes that resemble real models of its kinds: matrix memories with heads of 128 keys and 256 values; latent attention
+# with queries through 3/8 of the width, a latent of 192 + 64 rotated dimensions (a cached row of 256); grouped attention with
+# heads of 128 in groups of four, capped, with a bias over 32 buckets of distances up to 128, a window of ``--reach`` tokens
+# (beyond the contexts measured unless asked for) and four kept first tokens; experts of which 6 of 64 (32 at the smallest
+# size) are used.  Four layers (matrix memory, latent, grouped, matrix memory), each beside experts.  The framework's closest
+# other design is Kabulix: ``kabulix`` has the same width, vocabulary, heads, masks, latent and experts, with its own masked
+# attention where this design has matrix memories.
+VUBOTAR_SIZES = {
+    "w1024": dict(width=1024, heads=8, experts=32, top=6, ff=512),
+    "w2048": dict(width=2048, heads=16, experts=64, top=6, ff=1408),
+    "w4096": dict(width=4096, heads=32, experts=64, top=6, ff=2048),
+}
+
+
+def make_vubotar_config(size: str, reach: int = 4096):
+    from tensorline_amd.config import VubotarConfig
+    z = VUBOTAR_SIZES[size]
+    W, H = z["width"], z["heads"]
+    memory = {"heads": H // 2, "dim": 128, "vdim": 256, "gate_cap": 15.0}
+    latent = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": 3 * W // 8, "kv_rank": 192, "scale": 192 ** -0.5,
+              "rot": {"base": 10000.0, "dims": 64}}
+    grouped = {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0, "bias_max": 128,
+               "bias_rows": 32, "mask": {"size": reach, "keep_first": 4}, "v_mix": True}
+    moe = {"kind": "moe", "router": {"experts": z["experts"], "top": z["top"]}, "expert": {"ff": z["ff"]}}
+    layers = [{"type": kind, "mixer": mixer, "mlp": moe} for kind, mixer in
+              (("mlstm", memory), ("latent_attention", latent), ("attention", grouped), ("mlstm", memory))]
+    return VubotarConfig.from_dict({"architecture": "Vubotar", "vocab": HYBRID_VOCAB, "width": W, "norm": {"eps": 1e-6},
+                                    "embedding": {"scale": 1.0}, "logit_scale": 0.5, "logit_softcap": 30.0, "layers": layers})
+
+
+def make_vubotar_twin(size: str, reach: int = 4096):
+    from tensorline_amd.config import KabulixConfig
+    z = VUBOTAR_SIZES[size]
+    W, H = z["width"], z["heads"]
+    windowed = {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                "mask": {"size": reach, "keep_first": 4}, "rot": {"dims": 64, "base": 10000.0}}
+    latent = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 192, "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
+    chunked = {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": reach}}
+    moe = {"kind": "moe", "router": {"experts": z["experts"], "top": z["top"]}, "expert": {"ff": z["ff"]}}
+    layers = [{"type": kind, "mixer": mixer, "mlp": moe} for kind, mixer in
+              (("attention", windowed), ("latent_attention", latent), ("attention", windowed), ("attention_2", chunked))]
+    return KabulixConfig.from_dict({"architecture": "Kabulix", "vocab": HYBRID_VOCAB, "width": W, "norm": {"eps": 1e-6}, "layers": layers})
+
+
 def profile_step(llm, entries_of, seed: int) -> dict:
     """Event time of every kernel of one eager step, summed per entry point (milliseconds), after a
     warm-up step of the same shape."""
@@ -640,7 +685,7 @@ def profile_step(llm, entries_of, seed: int) -> dict:
 def bench_hybrid(args, design: str = "samovik") -> int:
     """Prefill and decode throughput of a design at real layer sizes (``samovik``: HYBRID_SIZES, ``tumitar``:
     TUMITAR_SIZES, ``zeganex``: ZEGANEX_SIZES, ``kabulix``: KABULIX_SIZES, ``taluvik``: TALUVIK_SIZES)
-    beside the dense decoder at equal size, and each step's time by kernel.  One JSON line; the default benchmark is not run."""
+    beside the dense decoder at equal size (``vubotar``: VUBOTAR_SIZES, beside Kabulix), and each step's time by kernel.  One JSON line; the default benchmark is not run."""
     import torch
     table, make, make_twin, model_text = {
         "samovik": (HYBRID_SIZES, make_hybrid_config, make_dense_twin,
@@ -659,7 +704,12 @@ def bench_hybrid(args, design: str = "samovik") -> int:
         "taluvik": (TALUVIK_SIZES, (lambda size: make_taluvik_config(size, args.reach)), make_taluvik_twin,
                     "Taluvik layer sizes (4 layers: delta rule, selective scan, chunked attention with capped scores and sinks, delta "
                     "rule, a dense feed-forward beside each; chunks of %d tokens) beside Qwen2 layers of equal width and weights "
+                    "(4 layers)" % args.reach),
+        "vubotar": (VUBOTAR_SIZES, (lambda size: make_vubotar_config(size, args.reach)), (lambda size: make_vubotar_twin(size, args.reach)),
+                    "Vubotar layer sizes (4 layers: matrix memory, latent attention, capped attention with a bias by distance behind a "
+                    "window of %d tokens, matrix memory, experts beside each) beside Kabulix layers of equal width and experts "
                     "(4 layers)" % args.reach)}[design]
+    other = "kabulix" if design == "vubotar" else "dense"
 
     from tensorline_amd import LLM
     from tensorline_amd.engine.batch import StepEntry
@@ -668,7 +718,7 @@ def bench_hybrid(args, design: str = "samovik") -> int:
     results = {}
     for size in sizes:
         row = {}
-        for which, cfg in (("hybrid", make(size)), ("dense", make_twin(size))):
+        for which, cfg in (("hybrid", make(size)), (other, make_twin(size))):
             max_len = max(context, tokens) + 16
             llm = LLM(config=cfg, seed=args.seed, dtype=args.dtype, device="cuda:0", block_size=page,
                       num_blocks=(batch + 1) * (-(-max_len // page)) + 8, max_num_seqs=batch, max_batched_tokens=max(2048, tokens),
@@ -702,8 +752,8 @@ def bench_hybrid(args, design: str = "samovik") -> int:
             del llm
             gc.collect()
             torch.cuda.empty_cache()
-        row["hybrid_over_dense"] = {"prefill": round(row["hybrid"]["prefill_tok_s"] / row["dense"]["prefill_tok_s"], 3),
-                                    "decode": round(row["hybrid"]["decode_tok_s"] / row["dense"]["decode_tok_s"], 3)}
+        row["hybrid_over_" + other] = {"prefill": round(row["hybrid"]["prefill_tok_s"] / row[other]["prefill_tok_s"], 3),
+                                       "decode": round(row["hybrid"]["decode_tok_s"] / row[other]["decode_tok_s"], 3)}
         results[size] = row
     print(json.dumps({"metric": "hybrid_design_tok_s" if design == "samovik" else design + "_design_tok_s", "unit": "tok/s",
                       "n_gpus": 1, "dtype": args.dtype, "data": "synthetic",
@@ -757,7 +807,10 @@ def main() -> int:
     ap.add_argument("--taluvik", action="store_true",
                     help="the same for the Taluvik design (gated delta rule, selective scan, chunked attention with capped scores "
                          "and sinks, both branches of a layer side by side)")
-    ap.add_argument("--reach", type=int, default=4096, help="with --kabulix and --taluvik: tokens of the windows and chunks")
+    ap.add_argument("--vubotar", action="store_true",
+                    help="the same for the Vubotar design (matrix memories, latent attention with a queries' latent, capped attention "
+                         "with a bias by distance, experts beside every mixer), beside the Kabulix decoder")
+    ap.add_argument("--reach", type=int, default=4096, help="with --kabulix, --taluvik and --vubotar: tokens of the windows and chunks")
     ap.add_argument("--hybrid-sizes", default="", help="which of w1024,w2048,w4096 (default: all)")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -775,6 +828,8 @@ def main() -> int:
         return bench_hybrid(args, "kabulix")
     if args.taluvik:
         return bench_hybrid(args, "taluvik")
+    if args.vubotar:
+        return bench_hybrid(args, "vubotar")
 
     import torch
 

@@ -247,6 +247,19 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_local_kernel(
     const int s = chunks.seq[c], t0 = chunks.row[c];
     const int n = min(ML_L, q_start[s + 1] - t0);
     const int DKP = (dk + 15) & ~15, LD = DKP + 4, nb = (dv + 15) >> 4, kb = DKP >> 4;
+    const int lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), li = lane & 15, lg = lane >> 4;
+    const int jb0 = blockIdx.z * 8 + wave;
+    const float* vb = v + (size_t)t0 * ldv + (size_t)h * dv;
+    float bf[2][4][4];                                     // B: values (asked for ahead of all else), token 16 sb + 4 lg + e, column li
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int sb = 0; sb < 4; ++sb)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int t = 16 * sb + 4 * lg + e, j = (jb0 + 4 * u) * 16 + li;
+                bf[u][sb][e] = t < n && j < dv ? vb[(uint32_t)(t * ldv + j)] : 0.f;
+            }
     float* Ks = ml_smem;
     ml_rows_to_lds(k + (size_t)h * dk, ldk, t0, n, dk, DKP, vec, 1.0f, Ks, LD);
     ml_chunk_gates(gates, t0, n, h, F, g, G);
@@ -264,24 +277,13 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_local_kernel(
     if (blockIdx.z == 0) {
         for (int i = tid; i < DKP; i += ML_THREADS) {
             float sum = 0.f;
+#pragma unroll 16
             for (int t = 0; t < ML_L; ++t) sum = __builtin_fmaf(w[t], Ks[t * LD + i], sum);
             ws_n[at * DKP + i] = sum;
         }
     }
-    const int lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
-    const int jb0 = blockIdx.z * 8 + wave;
     if (jb0 >= nb) return;                                 // no barrier follows
     const bool two = jb0 + 4 < nb;
-    float bf[2][4][4];                                     // B: weighted values, token 16 sb + 4 lg + e, column li
-#pragma unroll
-    for (int u = 0; u < 2; ++u)
-#pragma unroll
-        for (int sb = 0; sb < 4; ++sb)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int t = 16 * sb + 4 * lg + e, j = (jb0 + 4 * u) * 16 + li;
-                bf[u][sb][e] = (t < n && j < dv) ? v[(size_t)(t0 + t) * ldv + (size_t)h * dv + j] : 0.f;
-            }
 #pragma unroll
     for (int sb = 0; sb < 4; ++sb)
 #pragma unroll
@@ -307,6 +309,7 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_local_kernel(
     }
 }
 
+#define ML_RING 4       // fragments of the entering state on their way
 #define ML_AHEAD 4      // chunks whose terms are on their way while the ones before are added
 // Grid (quadruples of state elements / 256, then one block for n; head; sequence).
 __global__ __launch_bounds__(ML_THREADS) void mlstm_scan_kernel(float* __restrict__ ws_s, float* __restrict__ ws_n,
@@ -375,8 +378,9 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_scan_kernel(float* __restric
     if (j < dv) ml_store4(st, i, dk, vec_state, S);
 }
 
-// Grid (chunk, head).  First wave w takes tokens 16 w .. of the matrix, then blocks w, w + 4 of every eight of value columns.
-__global__ __launch_bounds__(ML_THREADS) void mlstm_outputs_kernel(
+// Grid (chunk, head, z): z takes groups z, z + gridDim.z, .. of 8 blocks of value columns.  First wave w takes tokens 16 w .. of the matrix (which every
+// work-group computes for itself), then blocks w and w + 4 of each of its groups.
+__global__ __launch_bounds__(ML_THREADS, 2) void mlstm_outputs_kernel(
     const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk, const float* __restrict__ v, int ldv, MlGates gates,
     float q_scale, float floor_eps, MlChunks chunks, const int32_t* __restrict__ q_start, const float* __restrict__ ws_s,
     const float* __restrict__ ws_n, const float* __restrict__ ws_m, float* __restrict__ out, int ldo, int H, int dk, int dv, int vec) {
@@ -401,7 +405,7 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_outputs_kernel(
         G[tid] = M;                                        // from here on M_t
         into[tid] = expf((float)(m0 - M));
     }
-    const int lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
+    const int lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), li = lane & 15, lg = lane >> 4;
     {
         // n_0 . q_t: four lanes to a token
         const int t = tid >> 2, part = tid & 3;
@@ -431,6 +435,31 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_outputs_kernel(
         ML_EACH(w)
 #undef ML_EACH
     }
+    // What the second half needs from memory is asked for here, ahead of the barriers: the values of this wave's first two blocks
+    // of columns and the first of the entering state's fragments.
+    const float4* S0 = reinterpret_cast<const float4*>(ws_s + at * (size_t)kb * nb * 256);
+    const float* vb = v + (size_t)t0 * ldv + (size_t)h * dv;
+    float bv[2][4][4];                                     // B of the second product: token 16 sb + 4 lg + e, column li
+    float4 ring[ML_RING][2];
+    int jb0 = blockIdx.z * 8 + wave;
+    auto fetch = [&]() {
+#pragma unroll
+        for (int r = 0; r < ML_RING; ++r)
+#pragma unroll
+            for (int u = 0; u < 2; ++u)
+                ring[r][u] = S0[(uint32_t)((min(r, kb - 1) * nb + min(jb0 + 4 * u, nb - 1)) * 64 + lane)];
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int sb = 0; sb < 4; ++sb)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    // (beyond the chunk's tokens the matrix is zero, beyond dv nothing is written: any finite value will do)
+                    const int t = min(16 * sb + 4 * lg + e, n - 1), j = min((jb0 + 4 * u) * 16 + li, dv - 1);
+                    bv[u][sb][e] = vb[(uint32_t)(t * ldv + j)];
+                }
+    };
+    fetch();
     __syncthreads();                                       // the keys are done with; M, into and nq are there
     {
         // this lane holds tokens t = 16 wave + 4 lg + e and s = 16 sb + li
@@ -452,46 +481,38 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_outputs_kernel(
         }
     }
     __syncthreads();
-    const float* S0 = ws_s + at * (size_t)kb * nb * 256;
-    for (int jg = 0; jg < nb; jg += 8) {
-        const int jb0 = jg + wave;
-        if (jb0 >= nb) break;                              // no barrier follows
+    for (; jb0 < nb; jb0 += 8 * gridDim.z) {               // no barrier in here
         const bool two = jb0 + 4 < nb;
-        const int jb1 = two ? jb0 + 4 : jb0;               // a wave with one block computes it twice over
-        float bv[2][4][4];                                 // B of the second product: token 16 sb + 4 lg + e, column li
-#pragma unroll
-        for (int u = 0; u < 2; ++u)
-#pragma unroll
-            for (int sb = 0; sb < 4; ++sb)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const int t = 16 * sb + 4 * lg + e, j = (u ? jb1 : jb0) * 16 + li;
-                    bv[u][sb][e] = (t < n && j < dv) ? v[(size_t)(t0 + t) * ldv + (size_t)h * dv + j] : 0.f;
-                }
+        const int jb1 = jb0 + 4;
         ml_f32x4 y[4][2];
 #pragma unroll
         for (int tb = 0; tb < 4; ++tb) y[tb][0] = y[tb][1] = ml_f32x4{0.f, 0.f, 0.f, 0.f};
-        const float4* f0 = reinterpret_cast<const float4*>(S0) + (size_t)jb0 * 64 + lane;
-        const float4* f1 = reinterpret_cast<const float4*>(S0) + (size_t)jb1 * 64 + lane;
-        float4 s0 = f0[0], s1 = f1[0];
-        for (int ib = 0; ib < kb; ++ib) {
-            const size_t next = (size_t)(ib + 1 < kb ? ib + 1 : ib) * nb * 64;
-            const float4 p0 = f0[next], p1 = f1[next];
-            float4 a[4];
+        for (int base = 0; base < kb; base += ML_RING) {
 #pragma unroll
-            for (int tb = 0; tb < 4; ++tb) a[tb] = *reinterpret_cast<const float4*>(Qs + (tb * 16 + li) * LD + ib * 16 + 4 * lg);
+            for (int r = 0; r < ML_RING; ++r) {
+                const int ib = base + r;
+                if (ib >= kb) break;
+                const float4 s0 = ring[r][0], s1 = ring[r][1];
+                // the place in the ring is taken by the fragment ML_RING steps further on
+                if (ib + ML_RING < kb) {
+                    ring[r][0] = S0[(uint32_t)(((ib + ML_RING) * nb + jb0) * 64 + lane)];
+                    ring[r][1] = S0[(uint32_t)(((ib + ML_RING) * nb + min(jb1, nb - 1)) * 64 + lane)];
+                }
+                float4 a[4];
+#pragma unroll
+                for (int tb = 0; tb < 4; ++tb) a[tb] = *reinterpret_cast<const float4*>(Qs + (tb * 16 + li) * LD + ib * 16 + 4 * lg);
 #define ML_EACH(X)                                                                                             \
     _Pragma("unroll") for (int tb = 0; tb < 4; ++tb) {                                                         \
         y[tb][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[tb].X, s0.X, y[tb][0], 0, 0, 0);                     \
         if (two) y[tb][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[tb].X, s1.X, y[tb][1], 0, 0, 0);            \
     }
-            ML_EACH(x)
-            ML_EACH(y)
-            ML_EACH(z)
-            ML_EACH(w)
+                ML_EACH(x)
+                ML_EACH(y)
+                ML_EACH(z)
+                ML_EACH(w)
 #undef ML_EACH
-            s0 = p0;
-            s1 = p1;
+                __builtin_amdgcn_sched_barrier(0);           // reads of later steps stay there: registers
+            }
         }
 #pragma unroll
         for (int tb = 0; tb < 4; ++tb)
@@ -516,6 +537,7 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_outputs_kernel(
             ML_EACH(z, 2)
             ML_EACH(w, 3)
 #undef ML_EACH
+            __builtin_amdgcn_sched_barrier(0);
         }
         // this lane holds tokens t = 16 tb + 4 lg + e and value column 16 jb + li
 #pragma unroll
@@ -529,6 +551,11 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_outputs_kernel(
                 if (jb0 * 16 + li < dv) o[jb0 * 16 + li] = y[tb][0][e] * d;
                 if (two && jb1 * 16 + li < dv) o[jb1 * 16 + li] = y[tb][1][e] * d;
             }
+        if (jb0 + 8 * (int)gridDim.z < nb) {               // the next blocks' values and fragments
+            jb0 += 8 * gridDim.z;
+            fetch();
+            jb0 -= 8 * gridDim.z;
+        }
     }
 }
 
@@ -595,6 +622,7 @@ extern "C" int tl_mlstm_chunked(const float* q, int ldq, const float* k, int ldk
     const MlGates a{gi, gf, bi, bf, ldi, ldf, cap};
     if (int rc = ml_check("tl_mlstm_chunked", q, ldq, k, ldk, v, ldv, a, state_stride, S, H, dk, dv, ldo)) return rc;
     TL_CHECK_ARG(ws && ws_g && ws_m && (uintptr_t)ws % 16 == 0 && (uintptr_t)ws_g % 8 == 0, "tl_mlstm_chunked: the (16-byte aligned) workspace is missing");
+    TL_CHECK_ARG((long long)ML_L * ldv < (1ll << 31), "tl_mlstm_chunked: rows of %d values are too long", ldv);
     TL_CHECK_ARG(chunk_seq && chunk_row && chunk_first && chunks >= 0, "tl_mlstm_chunked: chunk tables are missing");
     if (S == 0 || chunks == 0) return 0;
     const MlState st{state, state_stride, state_slots};
@@ -614,7 +642,9 @@ extern "C" int tl_mlstm_chunked(const float* q, int ldq, const float* k, int ldk
     hipLaunchKernelGGL(mlstm_scan_kernel, dim3(s_blocks + 1, H, S), dim3(ML_THREADS), 0, stream, ws, ws_n, ws_g, ws_m, st, ch, H, dk, dv,
                        s_blocks, vs);
     TL_CHECK_LAUNCH("tl_mlstm_chunked scan");
-    hipLaunchKernelGGL(mlstm_outputs_kernel, dim3(chunks, H), dim3(ML_THREADS), lds_c, stream, q, ldq, k, ldk, v, ldv, a, q_scale, floor_eps,
+    // few chunks and heads: the groups of value columns to work-groups of their own; many: one after another in one
+    const int groups = (long long)chunks * H < 512 ? (nb + 7) / 8 : 1;
+    hipLaunchKernelGGL(mlstm_outputs_kernel, dim3(chunks, H, groups), dim3(ML_THREADS), lds_c, stream, q, ldq, k, ldk, v, ldv, a, q_scale, floor_eps,
                        ch, q_start, ws, ws_n, ws_m, out, ldo, H, dk, dv, vec);
     TL_CHECK_LAUNCH("tl_mlstm_chunked outputs");
     return 0;

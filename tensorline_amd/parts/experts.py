@@ -93,7 +93,7 @@ class RoutedExperts(Part):
         if self._token_gate is not None:
             out.update(self._token_gate.tensors())
         if self.correction_name:
-            out[self.correction_name] = TensorDecl((self.experts,), "normal", 0.3, "float32")
+            out[self.correction_name] = TensorDecl((self.experts,), "normal", 0.02, "float32")
         for e in range(self.experts):
             p = f"{self.prefix}e{e}."
             if self.gated:

@@ -99,6 +99,8 @@ def spread(w: dict) -> None:
             t.add_(3.0)
         if name.endswith(".rel"):
             t.mul_(1.5)
+        if name.endswith(".correction"):
+            t.mul_(15.0)
     for name in [n for n in w if n.endswith("mix.i.b")]:
         q, k = w[name[:-3] + "q"], w[name[:-3] + "k"]
         q.mul_(0.5).add_(k)
