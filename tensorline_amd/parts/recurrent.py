@@ -525,9 +525,9 @@ class MatrixLSTM(Part):
         S_t = exp(f_t + m_(t-1) - m_t) S_(t-1) + exp(i_t - m_t) k_t v_t^T,   n_t likewise with k_t alone,
         o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + floor),
 
-    S, n and m zero at the start.  Each head's o is divided by its root mean square; the heads side by side times ``norm``, times
-    ``sigmoid(W_g h)``, are projected.  The request's slot keeps S, n and m of every head.  Everything between the projections and
-    the output norm's result is float32 whatever the engine's dtype.  Tensors under the prefix: q, k, v, i, i.b, f, f.b, g,
+    S, n and m zero at the start.  The heads' outputs are RMS-normed one by one, scaled per channel by ``norm``, gated by the sigmoid
+    of a projection ``g`` of the input and projected.  The request's slot keeps S, n and m of every head.  Everything between the
+    projections and the output norm's result is float32 whatever the engine's dtype.  Tensors under the prefix: q, k, v, i, i.b, f, f.b, g,
     norm, o."""
 
     def __init__(self, hidden_size, prefix, dtype, device, heads: int, dim: int, vdim: int, gate_cap: float, eps: float = 1e-6,
